@@ -275,6 +275,10 @@ class CacheManager:
             return 0
         return max(0, num_cached - window + 1) // self.block_size
 
+    def _first_free_page(self, group: CacheGroup) -> int:
+        """Index of the first page a window may ever pass: those before it hold tokens that stay for good."""
+        return pages_needed(group.requirement.keep_first, self.block_size)
+
     def pages_short(self, request_id, num_new: int) -> List[int]:
         """Per group: pages that `reserve(request_id, num_new)` would have to take."""
         entry = self._requests.get(request_id)
@@ -338,7 +342,7 @@ class CacheManager:
                 continue
             table = entry.tables[g]
             stop = min(self._first_needed_page(group, entry.num_cached), len(table))
-            begin = entry.passed[g]
+            begin = max(entry.passed[g], self._first_free_page(group))
             if stop > begin:
                 passed = [table[i] for i in range(begin, stop) if table[i] != GONE]
                 if passed:

@@ -14,6 +14,7 @@ from .model_config import ConfigError, ModelSpec, Qwen2Config, read_config_json
 from .dufelix_config import DufelixConfig
 from .duparax_config import DuparaxConfig
 from .musutar_config import MusutarConfig
+from .netovik_config import NetovikConfig
 from .sekazen_config import SekazenConfig
 
 _ARCHITECTURES: Dict[str, Any] = {}
@@ -75,3 +76,4 @@ register_architecture(MusutarConfig.architecture, MusutarConfig)
 register_architecture(DuparaxConfig.architecture, DuparaxConfig)
 register_architecture(SekazenConfig.architecture, SekazenConfig)
 register_architecture(DufelixConfig.architecture, DufelixConfig)
+register_architecture(NetovikConfig.architecture, NetovikConfig)

@@ -7,6 +7,7 @@
 // A step is a flattened batch: token t belongs to request token_request[t], whose new tokens are rows
 // cu_q[b] .. cu_q[b+1]-1 and whose state is row state_slots[b] of a state tensor.
 #include "common.h"
+#include "vector_values.h"
 
 namespace {
 
@@ -37,68 +38,6 @@ __device__ __forceinline__ float activate(float z, int kind) {   // the kinds of
 // residual are read once, up front and together, and wait in LDS too (rows of up to NORM_HELD_MAX columns); else
 // they are read again where they are needed.
 constexpr int NORM_HELD_MAX = 8192;
-
-// V values at p as floats: V = 4 takes one 16-byte (float32) or 8-byte (bfloat16) load, V = 8 two or one of 16 bytes
-template <int V, typename T>
-__device__ __forceinline__ void load_values(const T* __restrict__ p, float out[V]) {
-  if constexpr (V == 8 && sizeof(T) == 4) {
-    load_values<4>(p, out);
-    load_values<4>(p + 4, out + 4);
-  } else if constexpr (V == 8) {
-    const uint4 v = *reinterpret_cast<const uint4*>(p);
-    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
-#pragma unroll
-    for (int k = 0; k < 4; ++k) out[2 * k] = __uint_as_float(w[k] << 16), out[2 * k + 1] = __uint_as_float(w[k] & 0xffff0000u);
-  } else if constexpr (V == 4 && sizeof(T) == 4) {
-    const float4 v = *reinterpret_cast<const float4*>(p);
-    out[0] = v.x, out[1] = v.y, out[2] = v.z, out[3] = v.w;
-  } else if constexpr (V == 4) {
-    const uint2 v = *reinterpret_cast<const uint2*>(p);
-    out[0] = __uint_as_float(v.x << 16), out[1] = __uint_as_float(v.x & 0xffff0000u);
-    out[2] = __uint_as_float(v.y << 16), out[3] = __uint_as_float(v.y & 0xffff0000u);
-  } else {
-#pragma unroll
-    for (int k = 0; k < V; ++k) out[k] = to_float(p[k]);
-  }
-}
-
-template <int V, typename T>
-__device__ __forceinline__ void store_values(T* __restrict__ p, const float v[V]) {
-  const auto word = [](float lo, float hi) {
-    return static_cast<uint32_t>(__builtin_bit_cast(uint16_t, static_cast<bf16_t>(lo))) |
-           (static_cast<uint32_t>(__builtin_bit_cast(uint16_t, static_cast<bf16_t>(hi))) << 16);
-  };
-  if constexpr (V == 8 && sizeof(T) == 4) {
-    store_values<4>(p, v);
-    store_values<4>(p + 4, v + 4);
-  } else if constexpr (V == 8) {
-    *reinterpret_cast<uint4*>(p) = uint4{word(v[0], v[1]), word(v[2], v[3]), word(v[4], v[5]), word(v[6], v[7])};
-  } else if constexpr (V == 4 && sizeof(T) == 4) {
-    *reinterpret_cast<float4*>(p) = float4{v[0], v[1], v[2], v[3]};
-  } else if constexpr (V == 4) {
-    *reinterpret_cast<uint2*>(p) = uint2{word(v[0], v[1]), word(v[2], v[3])};
-  } else {
-#pragma unroll
-    for (int k = 0; k < V; ++k) p[k] = from_float<T>(v[k]);
-  }
-}
-
-// the sum of `slices` vectors that lie `stride` elements apart, added in order; eight slices' loads under way together
-template <int V, typename T>
-__device__ __forceinline__ void sum_values(const T* __restrict__ p, int slices, int64_t stride, float out[V]) {
-  load_values<V>(p, out);
-  for (int s = 1; s < slices; s += 8) {
-    float a[8][V];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) load_values<V>(p + min(s + u, slices - 1) * stride, a[u]);
-#pragma unroll
-    for (int u = 0; u < 8; ++u)
-      if (s + u < slices) {
-#pragma unroll
-        for (int k = 0; k < V; ++k) out[k] += a[u][k];
-      }
-  }
-}
 
 template <int V, typename A, typename B, typename O>
 __global__ void norm_chain_kernel(const A* __restrict__ t0, int slices0, int64_t stride0, const float* __restrict__ w0,
@@ -765,22 +704,31 @@ __global__ void lru_chunk_apply_kernel(const float* __restrict__ a, const float*
 constexpr int ROUTE_MAX_EXPERTS = 1024;
 constexpr int ROUTE_MAX_TOP = 32;
 
-// the weights of the chosen experts from their logits (largest first): softmax over those alone, or each one's own sigmoid
-__device__ __forceinline__ void write_route_weights(const float* chosen, float* __restrict__ out, int top, int sigmoid) {
-  if (sigmoid) {
+// the weights of the chosen experts from their logits (largest first): softmax over those alone (scoring 0), each one's
+// own sigmoid (1), or the softmax over all experts (2; `rest`: the sum of exp(z - the largest z) over those not chosen)
+__device__ __forceinline__ void write_route_weights(const float* chosen, float* __restrict__ out, int top, int scoring,
+                                                    float rest) {
+  if (scoring == 1) {
     for (int k = 0; k < top; ++k) out[k] = 1.f / (1.f + expf(-chosen[k]));
     return;
   }
   const float peak = chosen[0];
-  float total = 0.f;
+  float total = scoring == 2 ? rest : 0.f;
   for (int k = 0; k < top; ++k) total += expf(chosen[k] - peak);
   for (int k = 0; k < top; ++k) out[k] = expf(chosen[k] - peak) / total;
+}
+
+// by one wave, once the chosen experts' logits have been taken out of z (they are -inf there by then)
+__device__ __forceinline__ float rest_of_softmax(const float* z, int E, int lane, float peak) {
+  float sum = 0.f;
+  for (int e = lane; e < E; e += 64) sum += expf(z[e] - peak);
+  return wave_sum(sum);
 }
 
 template <typename X, typename W>
 __global__ void __launch_bounds__(256)
 route_topk_kernel(const X* __restrict__ x, const W* __restrict__ weight, const float* __restrict__ bias,
-                  int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int sigmoid) {
+                  int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int scoring) {
   extern __shared__ float xs[];                       // the token's row as float32
   __shared__ float z[ROUTE_MAX_EXPERTS];
   __shared__ float chosen[ROUTE_MAX_TOP];
@@ -804,6 +752,7 @@ route_topk_kernel(const X* __restrict__ x, const W* __restrict__ weight, const f
   }
   __syncthreads();
   if (wave != 0) return;
+  float peak = 0.f;                                   // the largest logit
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -819,13 +768,16 @@ route_topk_kernel(const X* __restrict__ x, const W* __restrict__ weight, const f
       if (other > best || (other == best && other_at < at)) best = other, at = other_at;
     }
     if (at == 0x7fffffff) at = k;                     // (unreachable for finite logits)
+    if (k == 0) peak = best;
     if (lane == 0) {
       experts[t * top + k] = at;
       chosen[k] = best;
     }
     if (at % 64 == lane) z[at] = -INFINITY;           // the lane that reads this place takes it out itself
   }
-  if (lane == 0) write_route_weights(chosen, gates + t * top, top, sigmoid);
+  float rest = 0.f;
+  if (scoring == 2) rest = rest_of_softmax(z, E, lane, peak);
+  if (lane == 0) write_route_weights(chosen, gates + t * top, top, scoring, rest);
 }
 
 // The same for bfloat16 rows and weights whose width is a multiple of 8: a thread takes 16-byte pieces of the token's
@@ -854,7 +806,7 @@ struct RouteScratch {
 
 template <int GROUP>                                   // experts worked on side by side: 16, or 8 where there are no more
 __device__ __forceinline__ void route_row_bf16(const bf16_t* __restrict__ x_row, const bf16_t* __restrict__ weight,
-                                               const float* __restrict__ bias, int C, int E, int top, int sigmoid,
+                                               const float* __restrict__ bias, int C, int E, int top, int scoring,
                                                RouteScratch& lds) {
   static_assert(GROUP <= ROUTE_GROUP, "the scratch holds ROUTE_GROUP sums a wave");
   const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
@@ -891,6 +843,7 @@ __device__ __forceinline__ void route_row_bf16(const bf16_t* __restrict__ x_row,
     __syncthreads();
   }
   if (wave == 0) {
+    float peak = 0.f;
     for (int k = 0; k < top; ++k) {
       float best = -INFINITY;
       int at = 0x7fffffff;
@@ -905,26 +858,29 @@ __device__ __forceinline__ void route_row_bf16(const bf16_t* __restrict__ x_row,
         if (other > best || (other == best && other_at < at)) best = other, at = other_at;
       }
       if (at == 0x7fffffff) at = k;
+      if (k == 0) peak = best;
       if (lane == 0) {
         lds.ids[k] = at;
         lds.chosen[k] = best;
       }
       if (at % 64 == lane) lds.z[at] = -INFINITY;
     }
-    if (lane == 0) write_route_weights(lds.chosen, lds.weights, top, sigmoid);
+    float rest = 0.f;
+    if (scoring == 2) rest = rest_of_softmax(lds.z, E, lane, peak);
+    if (lane == 0) write_route_weights(lds.chosen, lds.weights, top, scoring, rest);
   }
   __syncthreads();
 }
 
 __global__ void __launch_bounds__(256)
 route_topk_bf16_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ weight, const float* __restrict__ bias,
-                       int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int sigmoid) {
+                       int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int scoring) {
   __shared__ RouteScratch lds;
   const int64_t t = blockIdx.x;
   if (E <= 8) {
-    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, sigmoid, lds);
+    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, lds);
   } else {
-    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, sigmoid, lds);
+    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, lds);
   }
   if (threadIdx.x < top) {
     experts[t * top + threadIdx.x] = lds.ids[threadIdx.x];
@@ -1038,7 +994,7 @@ __global__ void route_glu_kernel(const X* __restrict__ gate_up, int64_t ld, int 
 template <int V, typename X, typename O>
 __global__ void __launch_bounds__(256)
 route_topk_glu_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ weight, const float* __restrict__ bias, int C,
-                      int E, int top, int sigmoid, const X* __restrict__ gate_up, int64_t ld, int slices, int64_t stride,
+                      int E, int top, int scoring, const X* __restrict__ gate_up, int64_t ld, int slices, int64_t stride,
                       int F, int width, float limit, float slope, float up_shift, int on_input, O* __restrict__ out) {
   __shared__ RouteScratch lds;
   const int64_t t = blockIdx.y;
@@ -1051,9 +1007,9 @@ route_topk_glu_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w
     sum_values<V>(gate_up + t * ld + width + c, slices, stride, u);
   }
   if (E <= 8) {
-    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, sigmoid, lds);
+    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, lds);
   } else {
-    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, sigmoid, lds);
+    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, lds);
   }
   if (c >= width) return;
   const int e = c / F;
@@ -1266,17 +1222,18 @@ extern "C" int distie_lru_scan_chunked(const float* a, const float* x, float* st
   return launch_status();
 }
 
+// scoring: 0 softmax over the chosen, 1 sigmoid, 2 softmax over all experts
 extern "C" int distie_route_topk(const void* x, int x_dtype, const void* weight, int w_dtype, const float* bias,
-                                 int32_t* experts, float* gates, int T, int C, int E, int top, int sigmoid,
+                                 int32_t* experts, float* gates, int T, int C, int E, int top, int scoring,
                                  hipStream_t stream) {
   if (T <= 0) return 0;
-  if (C < 1 || E < 1 || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP ||
+  if (C < 1 || E < 1 || scoring < 0 || scoring > 2 || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP ||
       static_cast<size_t>(C) * sizeof(float) > 96 * 1024)
     return DISTIE_BAD_ARGUMENT;
   if (x_dtype == DISTIE_BF16 && w_dtype == DISTIE_BF16 && C % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(weight) % 16 == 0) {
     route_topk_bf16_kernel<<<T, 256, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(weight), bias,
-                                                  experts, gates, C, E, top, sigmoid);
+                                                  experts, gates, C, E, top, scoring);
     return launch_status();
   }
   const size_t lds = static_cast<size_t>(C) * sizeof(float);
@@ -1286,7 +1243,7 @@ extern "C" int distie_route_topk(const void* x, int x_dtype, const void* weight,
                             hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
       return DISTIE_BAD_ARGUMENT;
     route_topk_kernel<X, W><<<T, 256, lds, stream>>>(static_cast<const X*>(x), static_cast<const W*>(weight), bias,
-                                                     experts, gates, C, E, top, sigmoid);
+                                                     experts, gates, C, E, top, scoring);
   }));
   return launch_status();
 }
@@ -1341,12 +1298,12 @@ extern "C" int distie_route_glu(const void* gate_up, int dtype, int64_t ld, int 
 }
 
 // `distie_route_topk` (bfloat16 rows and weights) and `distie_route_glu` in one launch; for steps of few rows.
-extern "C" int distie_route_topk_glu(const void* x, const void* weight, const float* bias, int C, int sigmoid,
+extern "C" int distie_route_topk_glu(const void* x, const void* weight, const float* bias, int C, int scoring,
                                      const void* gate_up, int dtype, int64_t ld, int slices, int T, int top, int E, int F,
                                      float limit, float slope, float up_shift, int on_input, void* out, int out_dtype,
                                      hipStream_t stream) {
   if (T <= 0) return 0;
-  if (C < 8 || C % 8 || E < 1 || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP || F < 1 || slices < 1 ||
+  if (C < 8 || scoring < 0 || scoring > 2 || C % 8 || E < 1 || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP || F < 1 || slices < 1 ||
       T > 65535 || (slices > 1 && dtype != DISTIE_F32) || ld < 2 * static_cast<int64_t>(E) * F ||
       reinterpret_cast<uintptr_t>(x) % 16 != 0 || reinterpret_cast<uintptr_t>(weight) % 16 != 0)
     return DISTIE_BAD_ARGUMENT;
@@ -1357,7 +1314,7 @@ extern "C" int distie_route_topk_glu(const void* x, const void* weight, const fl
   const dim3 grid((width / V + 255) / 256, T);
 #define DISTIE_ROUTE_TOPK_GLU(V)                                                                                          \
   DISTIE_DISPATCH(dtype, X, DISTIE_DISPATCH(out_dtype, O, (route_topk_glu_kernel<V, X, O><<<grid, 256, 0, stream>>>(       \
-      static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(weight), bias, C, E, top, sigmoid,                        \
+      static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(weight), bias, C, E, top, scoring,                        \
       static_cast<const X*>(gate_up), ld, slices, stride, F, width, limit, slope, up_shift, on_input, static_cast<O*>(out)))))
   if (V == 8) {
     DISTIE_ROUTE_TOPK_GLU(8);

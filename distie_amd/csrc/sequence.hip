@@ -279,7 +279,7 @@ __global__ void conv_rope_kv_write_kernel(const X* __restrict__ product, int64_t
                                           const int32_t* __restrict__ state_slots, int H, int G, int D, int E, int DP,
                                           int block_size, int has_kv, int write, const int32_t* __restrict__ positions,
                                           float temp_coef, int temp_every, const float* __restrict__ q_norm,
-                                          const float* __restrict__ k_norm, float norm_eps, int slices, int64_t stride) {
+                                          const float* __restrict__ k_norm, float norm_eps, int slices, int64_t stride, int v_base) {
   // slices > 1 (taps 0 only): the product is partial sums that lie `stride` elements apart, added in order while read
   const int64_t t = blockIdx.x;
   const int head = blockIdx.y;
@@ -310,11 +310,11 @@ __global__ void conv_rope_kv_write_kernel(const X* __restrict__ product, int64_t
   if (head >= H + G) {                                   // a v head
     if (!write) {
       if (single && taps > 1)
-        for (int e = threadIdx.x; e < E; e += blockDim.x) (void)value((H + G) * D + (head - H - G) * E + e);
+        for (int e = threadIdx.x; e < E; e += blockDim.x) (void)value(v_base + (head - H - G) * E + e);
       return;
     }
     for (int e = threadIdx.x; e < E; e += blockDim.x) {
-      const float v = value((H + G) * D + (head - H - G) * E + e);
+      const float v = value(v_base + (head - H - G) * E + e);
       v_cache[((page * G + (head - H - G)) * DP + e) * block_size + offset] = from_float<C>(to_float(from_float<Q>(v)));
     }
     return;
@@ -380,13 +380,14 @@ __global__ void sigmoid_gate_kernel(const X* __restrict__ x, int ldh, int E, con
 // out = x / sqrt(mean(x^2) + eps) * weight * sigmoid(gate): the norm over all heads together, then the gate.
 // V channels a thread at a time (4: 16-byte loads of x, every load of a row under way before the sum).
 // A row of x may be one group of a wider row (blockIdx.y: the group, `ld` columns a row, the weight shared by the
-// groups); `silu`: the gate is g * sigmoid(g).
+// groups, or every column's own with `own_weights`); `silu`: the gate is g * sigmoid(g).
 template <int V, typename W, typename G, typename O>
 __global__ void rmsnorm_gate_kernel(const float* __restrict__ x, const W* __restrict__ weight, float eps,
                                     const G* __restrict__ gates, int64_t ldg, O* __restrict__ out, int N, int64_t ld,
-                                    int silu) {
+                                    int silu, int own_weights) {
   __shared__ float scratch[16];
   const int64_t t = blockIdx.x;
+  if (own_weights) weight += static_cast<int64_t>(blockIdx.y) * N;
   const float* row = x + t * ld + static_cast<int64_t>(blockIdx.y) * N;
   if (gates != nullptr) gates += static_cast<int64_t>(blockIdx.y) * N;
   out += t * (ld - N) + static_cast<int64_t>(blockIdx.y) * N;
@@ -869,7 +870,7 @@ head_norm_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ product, int64_t 
                                     int D, int E, int DP, int block_size, int has_kv, int write,
                                     const int32_t* __restrict__ positions, float temp_coef, int temp_every,
                                     const float* __restrict__ q_norm, const float* __restrict__ k_norm, float norm_eps,
-                                    int qk_blocks, int lanes) {
+                                    int qk_blocks, int lanes, int v_base) {
   if (static_cast<int>(blockIdx.x) >= qk_blocks) {
     const int t0 = (static_cast<int>(blockIdx.x) - qk_blocks) / G * VGROUP;
     const int g = (static_cast<int>(blockIdx.x) - qk_blocks) % G;
@@ -882,7 +883,7 @@ head_norm_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ product, int64_t 
     const uint16_t* rows = reinterpret_cast<const uint16_t*>(product);
     uint16_t* cache = reinterpret_cast<uint16_t*>(v_cache);
     for (int e = threadIdx.x; e < E; e += blockDim.x) {
-      const int c = (H + G) * D + g * E + e;
+      const int c = v_base + g * E + e;
       uint32_t bits[VGROUP];
 #pragma unroll
       for (int k = 0; k < VGROUP; ++k) bits[k] = k < n ? rows[static_cast<int64_t>(t0 + k) * ld + c] : 0u;
@@ -1363,6 +1364,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
                                          const float* k_norm, float norm_eps, int slices, int q_dtype, hipStream_t stream) {
   // slices > 1: `product` is float32 partial sums [slices, T, ld] (no convolution then); q_out is of `q_dtype`
   // temp_every >= 1: q of the token at position p times 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)
+  // has_kv 2: the product holds no columns of v; the values are the columns of k as they are (E is D, no convolution)
   // q_norm / k_norm (float32 [D], null: none): every q / k head goes through x / sqrt(mean(x^2) + norm_eps) * weight
   // over its D values, behind the convolution and in front of the rotation
   if (T <= 0) return 0;
@@ -1371,6 +1373,9 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
   if (H < 1 || G < 1 || D < 1 || E < 1 || DP < D || DP < E || block_size < 1 || pairs < 0 || 2 * pairs > D ||
       taps < 0 || taps > MAX_TAPS)
     return DISTIE_BAD_ARGUMENT;
+  const bool tied = has_kv == 2;
+  if (tied && (E != D || taps > 0)) return DISTIE_BAD_ARGUMENT;
+  const int v_base = tied ? H * D : (H + G) * D;         // the first column of v
   if ((pairs > 0 && table == nullptr) || (taps > 1 && state == nullptr) || (taps >= 1 && weight == nullptr))
     return DISTIE_BAD_ARGUMENT;
   if (has_kv && write && (k_cache == nullptr || v_cache == nullptr || slots == nullptr)) return DISTIE_BAD_ARGUMENT;
@@ -1379,7 +1384,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
   const int64_t stride = static_cast<int64_t>(T) * ld;
   const bool normed = q_norm != nullptr || k_norm != nullptr;
   const int norm_items = (has_kv ? H + G : H) * ((DP - pairs) / 8);
-  if ((!normed || (static_cast<size_t>(norm_items) * sizeof(float) <= 48 * 1024 && D % 8 == 0 && pairs % 4 == 0 &&
+  if ((!tied || (normed && DP <= 512)) && (!normed || (static_cast<size_t>(norm_items) * sizeof(float) <= 48 * 1024 && D % 8 == 0 && pairs % 4 == 0 &&
                    reinterpret_cast<uintptr_t>(q_norm) % 16 == 0 && reinterpret_cast<uintptr_t>(k_norm) % 16 == 0)) &&
       dtype == DISTIE_BF16 && q_dtype == DISTIE_BF16 && (weight == nullptr || w_dtype == DISTIE_BF16) && (!write || cache_dtype == DISTIE_BF16) &&
       T >= 32 && D % 8 == 0 && E % 8 == 0 && DP % 8 == 0 && pairs % 8 == 0 && ld % 8 == 0 &&
@@ -1398,7 +1403,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
       head_norm_rope_kv_write_bf16_kernel<<<qk_blocks + v_only, 256, 0, stream>>>(
           static_cast<const bf16_t*>(product), ld, static_cast<const float2*>(table), pairs, magnitude,
           static_cast<bf16_t*>(q_out), static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), slots, T, H, G, D, E, DP,
-          block_size, has_kv, write, positions, temp_coef, temp_every, q_norm, k_norm, norm_eps, qk_blocks, lanes);
+          block_size, has_kv, write, positions, temp_coef, temp_every, q_norm, k_norm, norm_eps, qk_blocks, lanes, v_base);
       return launch_status();
     }
 #define DISTIE_CONV_ROPE_BF16(NORM, LDS)                                                                                 \
@@ -1427,7 +1432,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
             static_cast<const float*>(product), ld, nullptr, taps, state, static_cast<const float2*>(table),
             pairs, magnitude, static_cast<Q*>(q_out), static_cast<C*>(k_cache), static_cast<C*>(v_cache), slots, cu_q,
             token_request, state_slots, H, G, D, E, DP, block_size, has_kv, write, positions, temp_coef, temp_every,
-            q_norm, k_norm, norm_eps, slices, stride)));
+            q_norm, k_norm, norm_eps, slices, stride, v_base)));
     return launch_status();
   }
   DISTIE_DISPATCH(dtype, X, DISTIE_DISPATCH(w_dtype, W, DISTIE_DISPATCH(cache_dtype, C,
@@ -1435,7 +1440,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
           static_cast<const X*>(product), ld, static_cast<const W*>(weight), taps, state, static_cast<const float2*>(table),
           pairs, magnitude, static_cast<X*>(q_out), static_cast<C*>(k_cache), static_cast<C*>(v_cache), slots, cu_q,
           token_request, state_slots, H, G, D, E, DP, block_size, has_kv, write, positions, temp_coef, temp_every,
-          q_norm, k_norm, norm_eps, slices, stride))));
+          q_norm, k_norm, norm_eps, slices, stride, v_base))));
   return launch_status();
 }
 
@@ -1463,7 +1468,7 @@ extern "C" int distie_sigmoid_gate(const void* x, int x_dtype, int ldh, int E, c
 
 extern "C" int distie_rmsnorm_gate(const float* x, const void* weight, int w_dtype, float eps, const void* gates,
                                    int g_dtype, int64_t ldg, void* out, int out_dtype, int T, int N, int groups, int silu,
-                                   hipStream_t stream) {
+                                   int own_weights, hipStream_t stream) {
   // N: columns of one norm; a row of x, of the gates and of out holds `groups` of them side by side
   if (T <= 0) return 0;
   if (N < 1 || groups < 1 || (gates != nullptr && ldg < static_cast<int64_t>(N) * groups)) return DISTIE_BAD_ARGUMENT;
@@ -1478,7 +1483,7 @@ extern "C" int distie_rmsnorm_gate(const float* x, const void* weight, int w_dty
 #define DISTIE_NORM_GATE(V)                                                                                  \
   DISTIE_DISPATCH(w_dtype, W, DISTIE_DISPATCH(g_dtype, G, DISTIE_DISPATCH(out_dtype, O,                      \
       rmsnorm_gate_kernel<V, W, G, O><<<grid, threads, 0, stream>>>(                                         \
-          x, static_cast<const W*>(weight), eps, static_cast<const G*>(gates), ldg, static_cast<O*>(out), N, ld, silu))))
+          x, static_cast<const W*>(weight), eps, static_cast<const G*>(gates), ldg, static_cast<O*>(out), N, ld, silu, own_weights))))
   if (wide) {
     DISTIE_NORM_GATE(4);
   } else {

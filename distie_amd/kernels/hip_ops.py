@@ -314,7 +314,7 @@ class HipOps(Ops):
         o.distie_conv_rope_kv_write.argtypes = [_P, _I, _L, _P, _I, _I, _P, _P, _I, _F, _P, _P, _P, _I, _P, _P, _P, _P,
                                                 _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _F, _I, _P, _P, _F, _I, _I, _P]
         o.distie_sigmoid_gate.argtypes = [_P, _I, _I, _I, _P, _I, _L, _P, _I, _I, _I, _P]
-        o.distie_rmsnorm_gate.argtypes = [_P, _P, _I, _F, _P, _I, _L, _P, _I, _I, _I, _I, _I, _P]
+        o.distie_rmsnorm_gate.argtypes = [_P, _P, _I, _F, _P, _I, _L, _P, _I, _I, _I, _I, _I, _I, _P]
         o.distie_norm_chain.argtypes = [_P, _I, _I, _P, _P, _I, _I, _P, _F, _F, _P, _F, _P, _P, _F, _P, _I, _P, _I, _I, _P]
         o.distie_gated_decay_scan.argtypes = [_P, _I, _L, _P, _P, _L, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _F, _F, _P]
         o.distie_gated_decay_scan_chunked.argtypes = [_P, _I, _L, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _P]
@@ -341,6 +341,13 @@ class HipOps(Ops):
                                               _I, _I, _P]
         o.distie_gate_rmsnorm.argtypes = [_P, _P, _I, _F, _P, _I, _L, _P, _I, _I, _I, _I, _I, _P]
         o.distie_glu_mul.argtypes = [_P, _I, _I, _P, _I, _I, _I, _I, _P]
+        o.distie_group_chain.argtypes = [_P, _I, _I, _P, _F, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P]
+        o.distie_token_shift.argtypes = [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _P]
+        o.distie_wkv_scan.argtypes = [_P, _P, _P, _P, _I, _L, _P, _I, _L, _I, _P, _P, _P, _P, _P, _F, _P, _I, _P, _P, _I, _I,
+                                      _I, _P]
+        o.distie_tanh_f32.argtypes = [_P, _L, _P, _I, _I, _P]
+        o.distie_mixed_attention_generic.argtypes = [_P, _I, _L, _P, _P, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _F,
+                                                     _I, _I, _F, _P, _I, _P, _P, _P]
         o.distie_argmax.argtypes = [_P, _P, _I, _I, _P, _P, _P]
         o.distie_argmax_parts.argtypes = [_I, _I]
         o.distie_sample.argtypes = [_P, _P, _P, _P, _P, _I, _I, _P, _P, _P, _P]
@@ -929,7 +936,6 @@ class HipOps(Ops):
             raise KernelError(f"paged_attention: the scale of the scores must be positive, not {scale}")
         qkv = self.dense(qkv)
         self._own(qkv, k_cache, v_cache)
-        lib = self.attention_library(head_dim)
         T = qkv.shape[0]
         table = meta.groups[group].block_table
         self._check_cache(k_cache, v_cache, num_kv_heads, meta.block_size, head_dim)
@@ -948,6 +954,11 @@ class HipOps(Ops):
                 if vector.dtype != torch.float32 or tuple(vector.shape) != (num_heads,):
                     raise KernelError(f"paged_attention: {name} must be float32 [num_heads]")
         sinks_ptr = sinks.data_ptr() if sinks is not None else None
+        if extras is not None and extras.mixes_heads:
+            self._mixed_attention(qkv, meta, table, rows_ptr, k_cache, v_cache, out, num_heads, num_kv_heads, head_dim, scale,
+                                  window, extras)
+            return out
+        lib = self.attention_library(head_dim)
         bf16 = qkv.dtype == torch.bfloat16 and k_cache.dtype == torch.bfloat16
         if plain and bf16 and meta.block_size % 16 == 0 and head_dim % 16 == 0 and head_dim <= self.LARGEST_MATRIX_CORE_HEAD:
             # how the step is launched, and its buffers for partial results, are the same for every layer
@@ -1003,6 +1014,31 @@ class HipOps(Ops):
             out.data_ptr(), T, num_heads, num_kv_heads, meta.block_size, float(scale), int(window or 0),
             slopes.data_ptr() if slopes is not None else None, cap, sinks_ptr, self._stream()), "attention_generic")
         return out
+
+    def _mixed_attention(self, q, meta: BatchMeta, table, rows_ptr, k_cache, v_cache, out, num_heads, num_kv_heads, head_dim,
+                         scale, window, extras) -> None:
+        """Attention for layers whose heads see each other's scores (csrc/mixed_attention.hip)."""
+        if extras.head_slopes is not None:
+            raise KernelError("paged_attention: slopes do not go with mixed heads")
+        bias, mix = extras.distance_bias, extras.head_mix
+        for name, t, rows in (("distance_bias", bias, num_heads), ("head_mix", mix, num_heads)):
+            if t is not None:
+                self._own(t)
+                if t.dtype != torch.float32 or t.dim() != 2 or t.shape[0] != rows:
+                    raise KernelError(f"paged_attention: {name} must be float32 with a row a head")
+        if mix is not None and mix.shape[1] != num_heads:
+            raise KernelError("paged_attention: head_mix must be [num_heads, num_heads]")
+        if q.shape[1] != num_heads * head_dim:
+            raise KernelError("paged_attention: mixed heads take q alone")
+        if not self._ops.distie_mixed_attention_fits(num_heads, head_dim):
+            raise KernelError(f"paged_attention: {num_heads} mixed heads of {head_dim} do not fit the LDS of a compute unit")
+        ptr = lambda t: t.data_ptr() if t is not None else None
+        _check(self._ops.distie_mixed_attention_generic(
+            q.data_ptr(), _code(q), q.shape[1], k_cache.data_ptr(), v_cache.data_ptr(), _code(k_cache),
+            meta.positions.data_ptr(), meta.token_request.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr,
+            out.data_ptr(), q.shape[0], num_heads, num_kv_heads, head_dim, meta.block_size, float(scale), int(window or 0),
+            int(extras.keep_first) if window else 0, float(extras.score_cap or 0.0), ptr(bias),
+            bias.shape[1] if bias is not None else 0, ptr(mix), ptr(extras.sinks), self._stream()), "mixed_attention_generic")
 
     def _attention_plan(self, lib, meta: BatchMeta, T, num_heads, num_kv_heads, head_dim, window) -> dict:
         group = num_heads // num_kv_heads
@@ -1174,7 +1210,8 @@ class HipOps(Ops):
                               f"[slots, {taps - 1}, {channels}]")
 
     def conv_rope_kv_write(self, product, conv_weight, state, meta, group, k_cache, v_cache, inv_freq, magnitude,
-                           num_heads, num_kv_heads, dim, value_dim, padded_dim, has_kv, write, q_temp=None, qk_norm=None):
+                           num_heads, num_kv_heads, dim, value_dim, padded_dim, has_kv, write, q_temp=None, qk_norm=None,
+                           keys_are_values=False):
         # without a filter the kernel adds up a product's partial sums itself while it reads them
         slices, q_dtype = 1, None
         if isinstance(product, PartialSums) and conv_weight is None:
@@ -1194,7 +1231,9 @@ class HipOps(Ops):
                 raise KernelError("conv_rope_kv_write: a norm on the heads needs a weight for q, and for k where there are keys")
         self._own(product, conv_weight, state, k_cache, v_cache, inv_freq)
         T, W = product.shape[0] // slices, product.shape[1]
-        channels = num_heads * dim + (num_kv_heads * (dim + value_dim) if has_kv else 0)
+        if keys_are_values and (not has_kv or conv_weight is not None or value_dim != dim):
+            raise KernelError("conv_rope_kv_write: values that are the keys go with keys, one head size and no filter")
+        channels = num_heads * dim + (num_kv_heads * (dim if keys_are_values else dim + value_dim) if has_kv else 0)
         taps = 0 if conv_weight is None else conv_weight.shape[1]
         if T != meta.num_tokens or W < channels:
             raise KernelError("conv_rope_kv_write: the product does not match the batch or the head counts")
@@ -1216,7 +1255,7 @@ class HipOps(Ops):
             ptr(k_cache) if write else None, ptr(v_cache) if write else None, _code(k_cache) if write else _code(product),
             meta.groups[group].slots.data_ptr() if write else None, meta.cu_q.data_ptr(), meta.token_request.data_ptr(),
             meta.state_slots.data_ptr(), T, num_heads, num_kv_heads, dim, value_dim, padded_dim, meta.block_size,
-            1 if has_kv else 0, 1 if write else 0, meta.positions.data_ptr(), float(q_temp[0]) if q_temp else 0.0,
+            2 if keys_are_values else (1 if has_kv else 0), 1 if write else 0, meta.positions.data_ptr(), float(q_temp[0]) if q_temp else 0.0,
             int(q_temp[1]) if q_temp else 0, ptr(q_norm), ptr(k_norm) if has_kv else None, float(norm_eps),
             slices, _CODES[q_dtype], self._stream()), "conv_rope_kv_write")
         if taps > 1:
@@ -1307,10 +1346,10 @@ class HipOps(Ops):
         self._own(x, weight)
         if gate not in ("sigmoid", "silu"):
             raise KernelError(f"rmsnorm_gate: no gate named {gate!r}")
-        if gate_first or (group is not None and x.dim() == 2 and tuple(weight.shape) == (x.shape[1],) and group != x.shape[1]):
+        if gate_first:
             # the gate in front of the norm, every column with a weight of its own
-            if not gate_first or gates is None:
-                raise KernelError("rmsnorm_gate: a weight for every column of grouped norms goes with the gate in front")
+            if gates is None:
+                raise KernelError("rmsnorm_gate: no gate to put in front of the norm")
             if x.dtype != torch.float32 or x.dim() != 2 or tuple(weight.shape) != (x.shape[1],) or \
                     (group is not None and (group < 1 or x.shape[1] % group)):
                 raise KernelError("rmsnorm_gate: x must be float32 [T, N], weight [N], N a multiple of the group")
@@ -1323,7 +1362,7 @@ class HipOps(Ops):
                                                  1 if gate == "silu" else 0, self._stream()), "gate_rmsnorm")
             return out
         if x.dtype != torch.float32 or x.dim() != 2 or (group is not None and (group < 1 or x.shape[1] % group)) or \
-                tuple(weight.shape) != (group or x.shape[1],):
+                tuple(weight.shape) not in ((group or x.shape[1],), (x.shape[1],)):
             raise KernelError("rmsnorm_gate: x must be float32 [T, N], weight [N] (or [group], N a multiple of it)")
         T, N = x.shape
         g_ptr, g_ld, g_code = None, 0, _F32
@@ -1334,7 +1373,8 @@ class HipOps(Ops):
         size = group or N
         _check(self._ops.distie_rmsnorm_gate(x.data_ptr(), weight.data_ptr(), _code(weight), float(eps), g_ptr, g_code,
                                              g_ld, out.data_ptr(), _code(out), T, size, N // size,
-                                             1 if gate == "silu" else 0, self._stream()), "rmsnorm_gate")
+                                             1 if gate == "silu" else 0, 1 if weight.shape[0] != size else 0,
+                                             self._stream()), "rmsnorm_gate")
         return out
 
     # ---- norms behind sub-layers, mixers side by side, gated states, routers (csrc/recurrent.hip)
@@ -1478,6 +1518,93 @@ class HipOps(Ops):
         _mark_written(state)
         return out
 
+    # ---- time mixing with a token shift, norms in groups, averages over the depth (csrc/time_mixing.hip, csrc/depth.hip)
+    def token_shift(self, x, mu, state, meta):
+        x = self.dense(x)
+        self._own(x, mu, state)
+        T, C = x.shape
+        if T != meta.num_tokens or mu.dtype != torch.float32 or mu.dim() != 2 or mu.shape[1] != C:
+            raise KernelError("token_shift: x are the step's rows, mu float32 [mixes, C]")
+        if state.dtype != torch.float32 or tuple(state.shape[1:]) != (C,):
+            raise KernelError("token_shift: the state is float32 [slots, C]")
+        out = torch.empty((mu.shape[0], T, C), dtype=x.dtype, device=self.device)
+        _check(self._ops.distie_token_shift(x.data_ptr(), _code(x), mu.data_ptr(), mu.shape[0], state.data_ptr(),
+                                            out.data_ptr(), meta.cu_q.data_ptr(), meta.token_request.data_ptr(),
+                                            meta.state_slots.data_ptr(), T, C, self._stream()), "token_shift")
+        _mark_written(state)
+        return out
+
+    def wkv_decay_logits(self, low, up, up_bias):
+        low = low if low.dtype == torch.float32 else low.float()
+        ptr, ld = self._rows_view(low, up.shape[1])
+        bent = torch.empty(low.shape, dtype=torch.float32, device=self.device)
+        _check(self._ops.distie_tanh_f32(ptr, ld, bent.data_ptr(), low.shape[0], low.shape[1], self._stream()), "tanh_f32")
+        return self.linear_f32out(bent, up, up_bias)
+
+    def wkv_mix(self, r, k, v, gates, low, up, up_bias, bonus, state, meta, num_heads, dim, norm_weight, eps, out_dtype):
+        N, T, rank = num_heads * dim, r.shape[0], up.shape[1]
+        self._own(up, up_bias, bonus, state, norm_weight)
+        views = [self._rows_view(t, N) for t in (r, k, v, gates)]
+        ld = views[0][1]
+        if T != meta.num_tokens or any(t.dtype != r.dtype or t.shape[0] != T for t in (k, v, gates)) or \
+                any(view[1] != ld for view in views) or low.shape[0] != T:
+            raise KernelError("wkv_mix: r, k, v and gates are the step's rows, of one dtype and row stride")
+        for name, t, shape in (("up", up, (N, rank)), ("up_bias", up_bias, (N,)), ("bonus", bonus, (N,)),
+                               ("norm_weight", norm_weight, (N,))):
+            if t.dtype != torch.float32 or tuple(t.shape) != shape:
+                raise KernelError(f"wkv_mix: {name} must be float32 {list(shape)}")
+        if state.dtype != torch.float32 or tuple(state.shape[1:]) != (num_heads, dim, dim):
+            raise KernelError("wkv_mix: the state is float32 [slots, heads, dim, dim]")
+        if dim > self._ops.distie_wkv_scan_max_dim() or rank > self._ops.distie_wkv_scan_max_rank():
+            raise KernelError(f"wkv_mix: heads of up to {self._ops.distie_wkv_scan_max_dim()} and decays through up to "
+                              f"{self._ops.distie_wkv_scan_max_rank()} dimensions")
+        low_ptr, low_ld = self._rows_view(low, rank)
+        out = torch.empty((T, N), dtype=out_dtype, device=self.device)
+        _check(self._ops.distie_wkv_scan(
+            views[0][0], views[1][0], views[2][0], views[3][0], _code(r), ld, low_ptr, _code(low), low_ld, rank, up.data_ptr(),
+            up_bias.data_ptr(), bonus.data_ptr(), state.data_ptr(), norm_weight.data_ptr(), float(eps), out.data_ptr(),
+            _code(out), meta.cu_q.data_ptr(), meta.state_slots.data_ptr(), meta.num_requests, num_heads, dim,
+            self._stream()), "wkv_scan")
+        _mark_written(state)
+        return out
+
+    def group_rmsnorm(self, x, weight, eps, groups, out_dtype):
+        return self._group_chain(x, weight, eps, groups, None, None, None, out_dtype)
+
+    def _group_chain(self, delta, weight, eps, groups, residual, into, history, out_dtype):
+        delta, slices = self._term(delta)
+        T, C = delta.shape[-2:]
+        self._own(weight, residual, into)
+        if weight.dtype != torch.float32 or tuple(weight.shape) != (C,) or groups < 1 or C % groups:
+            raise KernelError("norm in groups: weight float32 [C], C a multiple of the groups")
+        for t in (residual, into):
+            if t is not None and (t.dtype != torch.float32 or tuple(t.shape) != (T, C)):
+                raise KernelError("norm in groups: the residual is float32 [T, C]")
+        first = rest = weights = None
+        index = 0
+        if history is not None:
+            first, rest, index, weights = history
+            self._own(first, rest, weights)
+            if first.dtype != torch.float32 or rest.dtype != torch.float32 or tuple(first.shape) != (T, C) or \
+                    rest.dim() != 3 or tuple(rest.shape[1:]) != (T, C) or not 0 <= index < rest.shape[0] or \
+                    weights.dtype != torch.float32 or tuple(weights.shape) != (index + 2,):
+                raise KernelError("average over the depth: X_0 float32 [T, C], the others [layers, T, C], a weight for each")
+        out = torch.empty((T, C), dtype=out_dtype, device=self.device) if out_dtype is not None else None
+        ptr = lambda t: t.data_ptr() if t is not None else None
+        _check(self._ops.distie_group_chain(
+            delta.data_ptr(), _code(delta), slices, weight.data_ptr(), float(eps), int(groups), ptr(residual), ptr(into),
+            ptr(first), ptr(rest), int(index), ptr(weights), ptr(out), _code(out) if out is not None else _F32, T, C,
+            self._stream()), "group_chain")
+        if into is not None:
+            _mark_written(into)
+        return out
+
+    def add_group_normed(self, residual, delta, weight, eps, groups, out_dtype, in_place=True, history=None):
+        into = residual if in_place else torch.empty_like(residual)
+        read = self._group_chain(delta, weight, eps, groups, residual, into, history,
+                                 None if out_dtype == torch.float32 else out_dtype)
+        return into, into if out_dtype == torch.float32 else read
+
     def lru_gates(self, u, recur_weight, recur_bias, input_weight, input_bias, lam, rate):
         u = self.dense(u)
         self._own(recur_weight, recur_bias, input_weight, input_bias, lam)
@@ -1533,8 +1660,10 @@ class HipOps(Ops):
         _mark_written(state)
         return out
 
+    SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_all": 2}
+
     def route_topk(self, x, weight, bias, top, scoring="softmax"):
-        if scoring not in ("softmax", "sigmoid"):
+        if scoring not in self.SCORINGS:
             raise KernelError(f"route_topk: no scoring named {scoring!r}")
         x = self.dense(x)
         self._own(x, weight, bias)
@@ -1546,7 +1675,7 @@ class HipOps(Ops):
         gates = torch.empty((T, top), dtype=torch.float32, device=self.device)
         _check(self._ops.distie_route_topk(x.data_ptr(), _code(x), weight.data_ptr(), _code(weight),
                                            bias.data_ptr() if bias is not None else None, experts.data_ptr(),
-                                           gates.data_ptr(), T, C, E, int(top), 1 if scoring == "sigmoid" else 0,
+                                           gates.data_ptr(), T, C, E, int(top), self.SCORINGS[scoring],
                                            self._stream()), "route_topk")
         return experts, gates
 
@@ -1581,7 +1710,7 @@ class HipOps(Ops):
 
     def route_experts_glu(self, x, router_weight, router_bias, top, scoring, gate_up, num_experts, width, limit, slope,
                           up_shift, on_input):
-        if scoring not in ("softmax", "sigmoid"):
+        if scoring not in self.SCORINGS:
             raise KernelError(f"route_experts_glu: no scoring named {scoring!r}")
         x = self.dense(x)
         T, C = x.shape
@@ -1604,7 +1733,7 @@ class HipOps(Ops):
         out = torch.empty((T, num_experts * width), dtype=dtype, device=self.device)
         _check(self._ops.distie_route_topk_glu(
             x.data_ptr(), router_weight.data_ptr(), router_bias.data_ptr() if router_bias is not None else None, C,
-            1 if scoring == "sigmoid" else 0, source.data_ptr(), _code(source), gate_up.shape[1], slices, T, int(top),
+            self.SCORINGS[scoring], source.data_ptr(), _code(source), gate_up.shape[1], slices, T, int(top),
             num_experts, width, float(limit or 0.0), float(slope), float(up_shift), 1 if on_input else 0, out.data_ptr(),
             _code(out), self._stream()), "route_topk_glu")
         return out

@@ -70,11 +70,19 @@ class ScoreExtras:
     + s[h] * (j - i), a bias by the distance to the key with a slope of the head's own (a position
     encoding that needs no rotation). With `sinks` z: the softmax's denominator holds exp(z[h]) beside the
     visible keys' terms, weight(i, j) = exp(score(i, j)) / (exp(z[h]) + sum_j' exp(score(i, j'))); the sink is
-    not scaled, has no value and counts once for every query, whatever its window."""
+    not scaled, has no value and counts once for every query, whatever its window.
+
+    With `distance_bias` b: + b[h, min(i - j, N - 1)] behind the cap, a learned bias by the distance to the key. With
+    `head_mix` M: the heads' scores of every pair of query and key are then mixed, score_h <- sum_g M[h, g] score_g,
+    in front of mask and softmax. With `keep_first` n: a windowed layer also sees the keys 0 .. n - 1 whatever their
+    distance."""
 
     head_slopes: Optional[torch.Tensor] = None      # float32 [H] on the device
     score_cap: Optional[float] = None               # > 0
     sinks: Optional[torch.Tensor] = None            # float32 [H] on the device
+    distance_bias: Optional[torch.Tensor] = None    # float32 [H, N] on the device
+    head_mix: Optional[torch.Tensor] = None         # float32 [H, H] on the device
+    keep_first: int = 0
 
     def __post_init__(self):
         if self.score_cap is not None and not self.score_cap > 0:
@@ -82,12 +90,18 @@ class ScoreExtras:
 
     @property
     def plain(self) -> bool:
-        return self.head_slopes is None and self.score_cap is None and self.sinks is None
+        return not self.bends_scores and self.sinks is None and not self.mixes_heads
 
     @property
     def bends_scores(self) -> bool:
         """Something changes the scores themselves (a sink does not: it only joins the denominator)."""
         return self.head_slopes is not None or self.score_cap is not None
+
+    @property
+    def mixes_heads(self) -> bool:
+        """A bias by distance, scores mixed between the heads or keys kept ahead of the window: what the kernels that
+        work on all heads of a token together compute."""
+        return self.distance_bias is not None or self.head_mix is not None or self.keep_first > 0
 
 
 class Ops(abc.ABC):
@@ -229,7 +243,7 @@ class Ops(abc.ABC):
                            k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor],
                            inv_freq: Optional[torch.Tensor], magnitude: float, num_heads: int, num_kv_heads: int,
                            dim: int, value_dim: int, padded_dim: int, has_kv: bool, write: bool,
-                           q_temp=None, qk_norm=None) -> torch.Tensor:
+                           q_temp=None, qk_norm=None, keys_are_values: bool = False) -> torch.Tensor:
         """Behind attention's stacked projection. The first columns of `product` (act [T, W]) are q (num_heads x
         dim) and, if `has_kv`, k (num_kv_heads x dim) and v (num_kv_heads x value_dim); further columns are left
         alone. Each of these channels goes through `causal_conv` (no residual; `conv_weight` [channels, taps],
@@ -242,7 +256,9 @@ class Ops(abc.ABC):
         1 + coef * ln(floor((p + 1) / every) + 1), computed in float32 (None: none).
         `qk_norm` = (q_weight float32 [dim], k_weight float32 [dim] or None without keys, eps): behind the convolution
         and in front of the rotation every q and k head becomes x / sqrt(mean(x^2) + eps) * weight over its `dim`
-        values, in float32 (None: none)."""
+        values, in float32 (None: none).
+        `keys_are_values`: there are no columns of v; the values are the k columns as they are in the product, in front
+        of norm and rotation (value_dim is dim; no convolution)."""
         raise NotImplementedError(f"{type(self).__name__} has no convolution over time")
 
     def sigmoid_gate(self, x: torch.Tensor, num_heads: int, head_stride: int, width: int,
@@ -386,6 +402,58 @@ class Ops(abc.ABC):
         low, up, bias = decay_low
         return self.linear_f32out(low.contiguous(), up, bias)
 
+    # ---- time mixing with a token shift, norms in groups, averages over the depth
+    def token_shift(self, x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, meta: BatchMeta) -> torch.Tensor:
+        """x act [T, C], mu float32 [n, C] -> act [n, T, C]: x_t + (x_(t-1) - x_t) * mu[k] for every k, in float32 in front
+        of the rounding. The row before a request's first of the step comes from `state` (float32 [slots + 1, C], rows
+        by `meta.state_slots`), which is left holding the request's last row."""
+        raise NotImplementedError(f"{type(self).__name__} has no token shift")
+
+    def linear_each(self, xs: torch.Tensor, weights, unrounded=()):
+        """xs act [n, T, K] and n weights [N_k, K] -> xs[k] times weights[k] transposed, a tensor [T, N_k] or a column
+        view with a row stride each: act, or float32 for the indexes in `unrounded`. An implementation may run them
+        as one product, and may then leave all of them unrounded."""
+        return [self.linear_f32out(xs[k], w) if k in unrounded else self.dense(self.linear(xs[k], w))
+                for k, w in enumerate(weights)]
+
+    def prepare_linear_each(self, weights) -> None:
+        """Called once for the weights of a `linear_each` after they are loaded, as `prepare_linear`."""
+        for w in weights:
+            self.prepare_linear(w, role="qkv")
+
+    def wkv_decay_logits(self, low: torch.Tensor, up: torch.Tensor, up_bias: torch.Tensor) -> torch.Tensor:
+        """up tanh(low) + up_bias -> float32 [T, N]: low float32 [T, rank] (or a column view), up float32 [N, rank],
+        up_bias float32 [N]; tanh and product in float32."""
+        return self.linear_f32out(torch.tanh(low.float()).contiguous(), up, up_bias)
+
+    def wkv_mix(self, r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gates: torch.Tensor, low: torch.Tensor,
+                up: torch.Tensor, up_bias: torch.Tensor, bonus: torch.Tensor, state: torch.Tensor, meta: BatchMeta,
+                num_heads: int, dim: int, norm_weight: torch.Tensor, eps: float, out_dtype) -> torch.Tensor:
+        """Time mixing with a decay per key channel and token and a bonus for the current token. r, k, v [T, H * dim]
+        (tensors or column views, one dtype). With z = `wkv_decay_logits(low, up, up_bias)` and w = exp(-exp(z)), per head
+
+            o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T r_t,        S_t = diag(w_t) S_(t-1) + k_t v_t^T;
+
+        every head's o is divided by sqrt(mean(o^2) + eps), and the heads side by side are multiplied by `norm_weight`
+        [H * dim] and silu(gates) (gates [T, H * dim], of r's dtype) -> `out_dtype` [T, H * dim]. `bonus` float32
+        [H * dim]; `state` float32 [slots + 1, H, dim, dim] (key channel, value column; rows by `meta.state_slots`) is
+        read and left as the step's last row leaves it. Decay, state, sums, norm and gate in float32."""
+        raise NotImplementedError(f"{type(self).__name__} has no time mixing")
+
+    def group_rmsnorm(self, x: torch.Tensor, weight: torch.Tensor, eps: float, groups: int, out_dtype) -> torch.Tensor:
+        """float32 [T, C]: every one of `groups` equal consecutive parts of a row divided by sqrt(mean(part^2) + eps), the
+        whole times `weight` (float32 [C]) -> `out_dtype` [T, C]; statistics in float32."""
+        raise NotImplementedError(f"{type(self).__name__} has no norm in groups")
+
+    def add_group_normed(self, residual: torch.Tensor, delta, weight: torch.Tensor, eps: float, groups: int, out_dtype,
+                         in_place: bool = True, history=None):
+        """x = residual + group_rmsnorm(delta) (float32 [T, C]; `delta` act [T, C] or what `linear` returned) -> (x, x in
+        `out_dtype`: None for an `out_dtype` of None, x itself for float32). x is `residual`'s own tensor if `in_place`.
+        `history` = (first, rest, index, weights): an average over the depth. first float32 [T, C] is X_0, rest float32
+        [layers, T, C] holds X_1 .. X_index in its first rows; x is stored as X_(index + 1) (rest[index]) and what is
+        returned and left in the residual is sum_j weights[j] X_j, j = 0 .. index + 1 (weights float32 [index + 2])."""
+        raise NotImplementedError(f"{type(self).__name__} has no norm in groups")
+
     def lru_gates(self, u: torch.Tensor, recur_weight: torch.Tensor, recur_bias: torch.Tensor,
                   input_weight: torch.Tensor, input_bias: torch.Tensor, lam: torch.Tensor, rate: float):
         """The coefficients of a real-gated linear recurrent unit. u act [T, R] in B equal parts; the gates'
@@ -405,7 +473,8 @@ class Ops(abc.ABC):
     def route_topk(self, x, weight: torch.Tensor, bias: Optional[torch.Tensor], top: int, scoring: str = "softmax"):
         """The router of a mixture of experts: z = weight x + bias in float32 (x act [T, C], weight [E, C], bias
         float32 [E] or None); for every row the `top` largest z (the lower index among equals) and, as weights,
-        softmax over those alone (`scoring` "softmax") or sigmoid(z) of each, not renormalised ("sigmoid")
+        softmax over those alone (`scoring` "softmax"), over all experts and not renormalised ("softmax_all"), or
+        sigmoid(z) of each, not renormalised ("sigmoid")
         -> (experts int32 [T, top], their weights float32 [T, top]), largest first."""
         raise NotImplementedError(f"{type(self).__name__} has no router")
 

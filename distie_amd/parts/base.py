@@ -41,7 +41,7 @@ from ..config.model_config import PartSpec
 @dataclass(frozen=True)
 class ParamSpec:
     shape: Tuple[int, ...]
-    init: str = "normal"   # "normal" | "ones" | "zeros" | "int" | "eye" (a square matrix: the identity)
+    init: str = "normal"   # "normal" | "ones" | "zeros" | "int" | "eye" (a square matrix: the identity) | "last_one" (a vector: 0 .. 0 1)
 
 
 PAGE = -1      # stands for the page size in the shape of a paged tensor
@@ -59,12 +59,13 @@ class TensorDecl:
 
 @dataclass(frozen=True)
 class PagedTensors:
-    """A mixer that keeps something for every token (or for the last `window` tokens), in pages:
+    """A mixer that keeps something for every token (or for the last `window` tokens and the first `keep_first`), in pages:
     for each declared tensor the cache holds `[pages + 1, *shape]` per layer, addressed through the
     request's block table of the layer's group. Mixers with equal declarations share a group of pages."""
 
     tensors: Tuple[TensorDecl, ...]
     window: Optional[int] = None
+    keep_first: int = 0              # with a window: so many of a request's first tokens stay readable for good
 
     def page_shape(self, decl: TensorDecl, block_size: int) -> Tuple[int, ...]:
         return tuple(block_size if s == PAGE else s for s in decl.shape)

@@ -256,7 +256,90 @@ class BranchNormResidual(Block):
         stream.lanes["pending"] = (y, self.feed_forward_post_norm)
 
 
+class DepthAveragedBranchNorm(Block):
+    """A norm on each sub-layer's result only (norms in groups), and behind every layer a weighted average over the
+    depth ("depth-weighted averaging"):
+
+        x <- x + mixer_post_norm(mixer(x));   x <- x + feed_forward_post_norm(feed_forward(x));   X_(i+1) = x
+        x <- sum over j = 0 .. i+1 of dwa[j] X_j                    (X_0: the embedding output; tensor `dwa` [i + 2])
+
+    for layer i (`index` of `layers`). A layer may have no feed-forward. Everything is float32 but what a sub-layer
+    reads, which is the residual rounded to the activations' precision. X_0 .. X_L live for one step: X_0 is the
+    embedding's own tensor, the others rows of one slab. A sub-layer's result stays pending with its norm (and,
+    behind the layer's last one, with the average); the next read adds it, all in one kernel
+    (`Ops.add_group_normed`)."""
+
+    CHILDREN = {"mixer": "mixer", "mixer_post_norm": "norm", "feed_forward": "feed_forward",
+                "feed_forward_post_norm": "norm"}
+    OPTIONAL = ("feed_forward", "feed_forward_post_norm")
+
+    def __init__(self, spec, parts) -> None:
+        super().__init__(spec, parts)
+        self.index, self.layers = int(spec.params["index"]), int(spec.params["layers"])
+        if not 0 <= self.index < self.layers:
+            raise ValueError("a depth-averaged layer's index is below the number of layers")
+        if (self.feed_forward is None) != (self.feed_forward_post_norm is None):
+            raise ValueError("a feed-forward and its norm come together")
+        for norm in (self.mixer_post_norm, self.feed_forward_post_norm):
+            if norm is not None and getattr(norm, "fused_kind", None) != "group_rms":
+                raise ValueError("the depth-averaged arrangement takes RMS norms in groups")
+        self.depth_weights = None
+
+    def param_specs(self):
+        return {"dwa": ParamSpec((self.index + 2,), "last_one")}
+
+    def load(self, tensors) -> None:
+        self.depth_weights = tensors["dwa"].float().contiguous()
+
+    @staticmethod
+    def _close(ops, stream: ResidualStream, act_dtype):
+        """Add what is pending, through its norm and with the average where one is due; -> the residual in
+        `act_dtype` (None: nobody reads it)."""
+        delta, norm, average = stream.lanes["pending"]
+        stream.lanes["pending"] = None
+        history = None
+        if average is not None:
+            index, weights = average
+            history = (stream.lanes["first"], stream.lanes["rest"], index, weights)
+        # X_0 is read again by every average: the first sum goes to a tensor of its own
+        in_place = stream.hidden is not stream.lanes["first"]
+        stream.hidden, read = ops.add_group_normed(stream.hidden, delta, norm.weight, norm.eps, norm.groups, act_dtype,
+                                                   in_place, history)
+        return read
+
+    @staticmethod
+    def _settle(ops, stream: ResidualStream) -> None:
+        if stream.lanes and stream.lanes["pending"] is not None:
+            DepthAveragedBranchNorm._close(ops, stream, None)
+        stream.lanes = None
+
+    def _read(self, ops, stream: ResidualStream, act_dtype):
+        if stream.pending is not None:
+            raise ValueError("the depth-averaged arrangement starts from a residual with nothing pending on it")
+        if stream.lanes is None:
+            first = stream.hidden
+            stream.lanes = {"first": first, "pending": None,
+                            "rest": torch.empty((self.layers, *first.shape), dtype=first.dtype, device=first.device)}
+            stream.settle = self._settle
+        if stream.lanes["pending"] is None:
+            return ops.read_residual(stream.hidden, act_dtype)
+        return self._close(ops, stream, act_dtype)
+
+    def forward(self, ops, stream: ResidualStream, ctx: StepContext, cache, writes_cache: bool) -> None:
+        average = (self.index, self.depth_weights)
+        h = self._read(ops, stream, ctx.act_dtype)
+        y = self.mixer.forward(ops, h, ctx, cache["mixer"], writes_cache)
+        if self.feed_forward is None:
+            stream.lanes["pending"] = (y, self.mixer_post_norm, average)
+            return
+        stream.lanes["pending"] = (y, self.mixer_post_norm, None)
+        h = self._read(ops, stream, ctx.act_dtype)
+        y = self.feed_forward.forward(ops, h, ctx)
+        stream.lanes["pending"] = (y, self.feed_forward_post_norm, average)
+
+
 register_part("block", "prenorm_residual", PreNormResidual)
 register_part("block", "branch_norm_residual", BranchNormResidual)
+register_part("block", "depth_averaged_branch_norm", DepthAveragedBranchNorm)
 register_part("block", "sandwich_residual", SandwichResidual)
 register_part("block", "hyper_connections", HyperConnections)

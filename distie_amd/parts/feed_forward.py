@@ -86,10 +86,12 @@ class RoutedExperts(FeedForward):
 
     Variants, each a parameter: `router_bias` False: no `router.b`. `scoring` "sigmoid": an expert's weight is
     sigmoid(z) of its own logit, not renormalised over the chosen (the `top` largest scores are the `top` largest
-    logits). `weight_on` "input": the weight multiplies what the expert reads, expert(w x), instead of what it
+    logits). `scoring` "softmax_all": the softmax over all experts' logits, not renormalised over the chosen either. `weight_on` "input": the weight multiplies what the expert reads, expert(w x), instead of what it
     returns. `activation` "clamped_glu": with g = min(gate x, limit) and u = clamp(up x, -limit, limit) the hidden
     values are g * sigmoid(slope * g) * (u + up_shift). Since gate and up are linear, gate (w x) = w (gate x): the
-    weight is applied to the stacked product's columns, in float32, in front of the clamps.
+    weight is applied to the stacked product's columns, in float32, in front of the clamps. `route_in_hidden` (no shared
+    expert): the plain activation too goes through the kernel that knows the routing, behind the stacked product,
+    instead of the product's own epilogue and a scaling behind it.
 
     All experts' gate and up weights are stacked into one matrix (the shared expert's behind them), all down weights
     side by side into another: one product gives every expert's hidden values for every token, those of the experts a
@@ -111,13 +113,13 @@ class RoutedExperts(FeedForward):
         self.scoring = str(p.get("scoring", "softmax"))
         self.weight_on = str(p.get("weight_on", "output"))
         self.activation = str(p.get("activation", "silu_glu"))
-        if self.scoring not in ("softmax", "sigmoid") or self.weight_on not in ("input", "output") or \
+        if self.scoring not in ("softmax", "softmax_all", "sigmoid") or self.weight_on not in ("input", "output") or \
                 self.activation not in ("silu_glu", "clamped_glu"):
-            raise ValueError("routed experts: scoring is softmax or sigmoid, weight_on input or output, activation "
+            raise ValueError("routed experts: scoring is softmax, softmax_all or sigmoid, weight_on input or output, activation "
                              "silu_glu or clamped_glu")
-        self.plain = self.activation == "silu_glu" and self.weight_on == "output"
+        self.plain = self.activation == "silu_glu" and self.weight_on == "output" and not p.get("route_in_hidden", False)
         if not self.plain and self.shared_size:
-            raise ValueError("routed experts: a shared expert goes with the plain gated activation only")
+            raise ValueError("routed experts: a shared expert goes with the plain gated activation (and without route_in_hidden) only")
         self.limit = float(p.get("limit") or 0.0)
         self.slope = float(p.get("slope", 1.0))
         self.up_shift = float(p.get("up_shift", 0.0))

@@ -38,6 +38,36 @@ class RMSNorm(Norm):
         return ops.add_rmsnorm(residual, delta, self.weight, self.eps, out_dtype)
 
 
+class GroupRMSNorm(Norm):
+    """RMS norm in groups: a row is cut into `groups` equal consecutive parts, each is divided by its own root mean
+    square, and the whole is multiplied by the weight; statistics in float32."""
+
+    fused_kind = "group_rms"
+
+    def __init__(self, spec) -> None:
+        super().__init__(spec)
+        self.size = int(spec.params["size"])
+        self.eps = float(spec.params["eps"])
+        self.groups = int(spec.params.get("groups") or 1)
+        if self.groups < 1 or self.size % self.groups:
+            raise ValueError("a norm's groups must divide its size")
+        self.weight_name = spec.params.get("weight_name", "weight")
+        self.weight = None
+
+    def param_specs(self):
+        return {self.weight_name: ParamSpec((self.size,), "ones")}
+
+    def load(self, tensors) -> None:
+        self.weight = tensors[self.weight_name].float().contiguous()
+
+    def apply(self, ops, x, out_dtype):
+        return ops.group_rmsnorm(x, self.weight, self.eps, self.groups, out_dtype)
+
+    def add_apply(self, ops, residual, delta, out_dtype):
+        residual += ops.dense(delta)
+        return self.apply(ops, residual, out_dtype)
+
+
 class LayerNorm(Norm):
     """Centred norm with a weight and no bias: y = (x - mean) / sqrt(var + eps) * weight, where var is the mean of
     the squared deviations; statistics in float32."""
@@ -68,4 +98,5 @@ class LayerNorm(Norm):
 
 
 register_part("norm", "rmsnorm", RMSNorm)
+register_part("norm", "group_rmsnorm", GroupRMSNorm)
 register_part("norm", "layernorm", LayerNorm)

@@ -1,0 +1,74 @@
+"""Time mixing with a data-dependent decay (the recurrence of RWKV-6: Peng et al., "Eagle and Finch: RWKV with
+Matrix-Valued States and Dynamic Recurrence").
+
+h is the mixer's input and h' the token before's (zeros in front of a request's first token). Each of r, k, v, g, w reads
+a mix of its own, m_s = h + (h' - h) * mu_s:
+
+    r = W_r m_r,  k = W_k m_k,  v = W_v m_v  (heads x dim each),   gate = silu(W_g m_g)
+    w = exp(-exp(W_w2 tanh(W_w1 m_w) + w0))         a factor in (0, 1) for every head and key channel
+
+and per head, with a bonus u that only the current token gets,
+
+    o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,      S_t = diag(w_t) S_(t-1) + k_t v_t^T.
+
+Every head's o is divided by its root mean square, the heads side by side are multiplied by a weight and the gate and
+projected by W_o. A request's state is S (float32 [heads, dim, dim], zero at the start) and its last h (float32). The
+decay, its exponentials, S and its sums, norm and gate are float32 in either precision.
+"""
+
+from __future__ import annotations
+
+import torch
+
+from ..config.model_config import PartSpec
+from .base import FixedState, Mixer, ParamSpec, TensorDecl, register_part
+
+
+class WKV(Mixer):
+    MIXES = ("r", "k", "v", "g", "w")
+
+    def __init__(self, spec: PartSpec) -> None:
+        super().__init__(spec)
+        p = spec.params
+        self.hidden_size = int(p["hidden_size"])
+        self.num_heads = int(p["num_heads"])
+        self.head_dim = int(p["head_dim"])
+        self.decay_rank = int(p["decay_rank"])
+        self.eps = float(p["eps"])
+        if self.decay_rank < 1:
+            raise ValueError("the decay's projection has at least one dimension")
+        self.inner = self.num_heads * self.head_dim
+        self.mu = self.weights = self.up_weight = self.up_bias = self.bonus = self.norm_weight = self.out_weight = None
+
+    def cache_requirement(self):
+        return FixedState((TensorDecl("state", (self.num_heads, self.head_dim, self.head_dim), torch.float32),
+                           TensorDecl("last", (self.hidden_size,), torch.float32)))
+
+    def param_specs(self):
+        C, N, R = self.hidden_size, self.inner, self.decay_rank
+        return {**{f"mu.{name}": ParamSpec((C,)) for name in self.MIXES},
+                **{name: ParamSpec((N, C)) for name in "rkvg"},
+                "w1": ParamSpec((R, C)), "w2": ParamSpec((N, R)), "w0": ParamSpec((N,)),
+                "u": ParamSpec((self.num_heads, self.head_dim)), "norm": ParamSpec((N,), "ones"), "o": ParamSpec((C, N))}
+
+    def load(self, tensors) -> None:
+        self.mu = torch.stack([tensors[f"mu.{name}"].float() for name in self.MIXES]).contiguous()
+        self.weights = tuple(tensors[name].contiguous() for name in ("r", "k", "v", "g", "w1"))
+        self.up_weight, self.up_bias = tensors["w2"].float().contiguous(), tensors["w0"].float().contiguous()
+        self.bonus = tensors["u"].float().reshape(-1).contiguous()
+        self.norm_weight = tensors["norm"].float().contiguous()
+        self.out_weight = tensors["o"].contiguous()
+
+    def prepare(self, ops) -> None:
+        ops.prepare_linear_each(self.weights)
+        ops.prepare_linear(self.out_weight, role="attn_out")
+
+    def forward(self, ops, x, ctx, cache, writes_cache: bool):
+        mixes = ops.token_shift(x, self.mu, cache["last"], ctx.meta)
+        r, k, v, gates, low = ops.linear_each(mixes, self.weights, unrounded=(4,))
+        mixed = ops.wkv_mix(r, k, v, gates, low, self.up_weight, self.up_bias, self.bonus, cache["state"], ctx.meta,
+                            self.num_heads, self.head_dim, self.norm_weight, self.eps, ctx.act_dtype)
+        return ops.linear(mixed, self.out_weight)
+
+
+register_part("mixer", "wkv", WKV)

@@ -79,6 +79,8 @@ class TorchOps(Ops):
                 pos = int(meta.positions[t])
                 first = 0 if window is None else max(0, pos - window + 1)
                 keys = torch.arange(first, pos + 1, device=qkv.device)
+                if extras is not None and extras.keep_first:
+                    keys = torch.cat([torch.arange(min(extras.keep_first, first), device=qkv.device), keys])
                 pages = table[b, keys // P]
                 assert (pages >= 0).all(), "attention would read a page that was given back"
                 k = k_cache[pages, :, keys % P].float()          # [n, KH, D]
@@ -90,6 +92,10 @@ class TorchOps(Ops):
                     s = extras.score_cap * torch.tanh(s / extras.score_cap)
                 if extras is not None and extras.head_slopes is not None:
                     s = s + extras.head_slopes.float()[:, None] * (keys - pos).float()[None, :]
+                if extras is not None and extras.distance_bias is not None:
+                    s = s + extras.distance_bias[:, (pos - keys).clamp(max=extras.distance_bias.shape[1] - 1)]
+                if extras is not None and extras.head_mix is not None:
+                    s = extras.head_mix @ s
                 if extras is not None and extras.sinks is not None:
                     w = torch.softmax(torch.cat([s, extras.sinks.float()[:, None]], -1), -1)[:, :-1]
                 else:
@@ -147,8 +153,11 @@ class TorchOps(Ops):
         return (y if act is None else self.activation(y, act)).to(x.dtype)
 
     def conv_rope_kv_write(self, product, conv_weight, state, meta, group, k_cache, v_cache, inv_freq, magnitude,
-                           num_heads, num_kv_heads, dim, value_dim, padded_dim, has_kv, write, q_temp=None, qk_norm=None):
+                           num_heads, num_kv_heads, dim, value_dim, padded_dim, has_kv, write, q_temp=None, qk_norm=None,
+                           keys_are_values=False):
         T = product.shape[0]
+        if keys_are_values:
+            product = torch.cat([product, product[:, num_heads * dim:(num_heads + num_kv_heads) * dim]], 1)
         channels = num_heads * dim + (num_kv_heads * (dim + value_dim) if has_kv else 0)
         u = product[:, :channels]
         u = self._conv(u, conv_weight, state, meta, False) if conv_weight is not None else u.float()
@@ -328,6 +337,53 @@ class TorchOps(Ops):
             state[slots[b]] = s
         return out.view(T, H * E)
 
+    # ---- time mixing with a token shift, norms in groups, averages over the depth
+    def token_shift(self, x, mu, state, meta):
+        h = x.float()
+        before = torch.cat([torch.zeros_like(h[:1]), h[:-1]])
+        cu, slots = meta.cu_q.tolist(), meta.state_slots.tolist()
+        for b in range(meta.num_requests):
+            if cu[b] < cu[b + 1]:
+                before[cu[b]] = state[slots[b]]
+                state[slots[b]] = h[cu[b + 1] - 1]
+        return (h + (before - h) * mu[:, None, :]).to(x.dtype)
+
+    def wkv_mix(self, r, k, v, gates, low, up, up_bias, bonus, state, meta, num_heads, dim, norm_weight, eps, out_dtype):
+        T = r.shape[0]
+        z = self.wkv_decay_logits(low, up, up_bias)
+        decay = torch.exp(-torch.exp(z)).view(T, num_heads, dim)
+        r, k, v = (t.float().reshape(T, num_heads, dim) for t in (r, k, v))
+        u = bonus.view(num_heads, dim)
+        out = torch.zeros(T, num_heads, dim, dtype=torch.float32, device=r.device)
+        cu, slots = meta.cu_q.tolist(), meta.state_slots.tolist()
+        for b in range(meta.num_requests):
+            s = state[slots[b]]
+            for t in range(cu[b], cu[b + 1]):
+                pair = k[t][:, :, None] * v[t][:, None, :]
+                out[t] = ((s + u[:, :, None] * pair) * r[t][:, :, None]).sum(1)
+                s = decay[t][:, :, None] * s + pair
+            state[slots[b]] = s
+        g = gates.float()
+        normed = out / torch.sqrt((out ** 2).mean(-1, keepdim=True) + eps)
+        return (normed.view(T, num_heads * dim) * norm_weight * g * torch.sigmoid(g)).to(out_dtype)
+
+    def group_rmsnorm(self, x, weight, eps, groups, out_dtype):
+        T, C = x.shape
+        v = x.float().view(T, groups, C // groups)
+        return ((v / torch.sqrt((v ** 2).mean(-1, keepdim=True) + eps)).view(T, C) * weight).to(out_dtype)
+
+    def add_group_normed(self, residual, delta, weight, eps, groups, out_dtype, in_place=True, history=None):
+        x = residual + self.group_rmsnorm(delta, weight, eps, groups, torch.float32)
+        if history is not None:
+            first, rest, index, weights = history
+            rest[index] = x
+            x = weights[0] * first
+            for j in range(index + 1):
+                x = x + weights[j + 1] * rest[j]
+        if in_place:
+            x = residual.copy_(x)
+        return x, None if out_dtype is None else (x if out_dtype == x.dtype else x.to(out_dtype))
+
     def lru_gates(self, u, recur_weight, recur_bias, input_weight, input_bias, lam, rate):
         T, R = u.shape
         B = recur_weight.shape[0]
@@ -356,6 +412,8 @@ class TorchOps(Ops):
             z = z + bias.float()
         order = torch.sort(z, dim=-1, descending=True, stable=True).indices[:, :top]
         chosen = torch.gather(z, 1, order)
+        if scoring == "softmax_all":
+            return order.to(torch.int32), torch.gather(torch.softmax(z, -1), 1, order)
         return order.to(torch.int32), torch.sigmoid(chosen) if scoring == "sigmoid" else torch.softmax(chosen, -1)
 
     def route_glu(self, gate_up, experts, gates, num_experts, width, limit, slope, up_shift, on_input):
