@@ -17,7 +17,7 @@ serves it), points at batch 1 and 32, and a cache that takes the card's memory u
 the time to the first token and the time per output token after it, defined as the reference's load
 generator defines them (benchmarks/load/stats.py:29-34, 67-86).
 
-`--design musutar|duparax|sekazen|dufelix [--size w1024|w2048|w4096]`: prefill and decode of that decoder beside a Qwen2
+`--design musutar|duparax|sekazen|dufelix|netovik [--size w1024|w2048|w4096]`: prefill and decode of that decoder beside a Qwen2
 decoder of equal width, depth, heads and weights, at layer sizes of real models; one JSON line with both for every size.
 
 Random weights N(0, 0.02), seeded uniform token ids.
@@ -304,6 +304,28 @@ def dufelix_config(size):
             "embedding": {"scale": 8.0}, "layers": layers}
 
 
+def netovik_config(size):
+    """Groups of four layers: time mixing (heads of 64 on the whole width, a decay through a thirty-second of it), time
+    mixing again, windowed attention with mixed heads, kept first keys and a table of distance biases, and time mixing;
+    dense feed-forwards alternate with mixtures of eight experts of a quarter of the dense size, two a token; norms in
+    four groups, an average over the depth behind every layer."""
+    z = DESIGN_SIZES[size]
+    layers = []
+    for i in range(z["layers"]):
+        mlp = {"kind": "dense", "ff": z["ff"]} if i % 2 == 0 else \
+            {"kind": "moe", "router": {"experts": 8, "top": 2}, "expert": {"ff": z["ff"] // 4}}
+        if i % 4 == 2:
+            mixer = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"], "softcap": 30.0,
+                     "scale": z["dim"] ** -0.5, "bias_max": 512, "bias_rows": 32,
+                     "mask": {"size": z["window"], "keep_first": 64}}
+            layers.append({"type": "attention", "mixer": mixer, "mlp": mlp})
+        else:
+            layers.append({"type": "wkv", "mlp": mlp,
+                           "mixer": {"heads": z["width"] // 64, "dim": 64, "rank": z["width"] // 32}})
+    return {"architecture": "Netovik", "vocab": DESIGN_VOCAB, "width": z["width"], "norm": {"eps": 1e-6, "groups": 4},
+            "embedding": {"scale": 8.0}, "layers": layers}
+
+
 def qwen2_of_weights(size, layer_weights):
     """The Qwen2 decoder with the same width, depth and heads and a feed-forward sized so that its layers hold as many
     weights as the other design's layers do on average."""
@@ -322,7 +344,8 @@ def design_pair(design, size):
     from distie_amd.config import config_from_dict
     from distie_amd.engine.model import Model
 
-    config = {"sekazen": sekazen_config, "duparax": duparax_config, "dufelix": dufelix_config}[design](size)
+    config = {"sekazen": sekazen_config, "duparax": duparax_config, "dufelix": dufelix_config,
+              "netovik": netovik_config}[design](size)
     total = 0
     for name, spec in Model.declare(config_from_dict(config).model_spec()).items():
         if name.startswith("l"):
@@ -394,7 +417,7 @@ def main() -> int:
                         help="size the cache from free memory (the default for --shape 32b and --serve: 0.9)")
     parser.add_argument("--packed-weights", default=None, metavar="ROLES",
                         help="packed copies only for these products (qkv,attn_out,gate_up,down,head); 'none' for no copies")
-    parser.add_argument("--design", default=None, choices=["musutar", "duparax", "sekazen", "dufelix"],
+    parser.add_argument("--design", default=None, choices=["musutar", "duparax", "sekazen", "dufelix", "netovik"],
                         help="instead of the workload above: this design beside a Qwen2 decoder of equal size, prefill and decode")
     parser.add_argument("--size", default=None, choices=sorted(DESIGN_SIZES), help="with --design: one size instead of all")
     args = parser.parse_args()

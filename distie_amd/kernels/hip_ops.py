@@ -345,6 +345,8 @@ class HipOps(Ops):
         o.distie_token_shift.argtypes = [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _P]
         o.distie_wkv_scan.argtypes = [_P, _P, _P, _P, _I, _L, _P, _I, _L, _I, _P, _P, _P, _P, _P, _F, _P, _I, _P, _P, _I, _I,
                                       _I, _P]
+        o.distie_wkv_scan_chunked.argtypes = [_P, _P, _P, _P, _I, _L, _P, _P, _P, _P, _F, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I,
+                                              _I, _P]
         o.distie_tanh_f32.argtypes = [_P, _L, _P, _I, _I, _P]
         o.distie_mixed_attention_generic.argtypes = [_P, _I, _L, _P, _P, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _F,
                                                      _I, _I, _F, _P, _I, _P, _P, _P]
@@ -1560,6 +1562,19 @@ class HipOps(Ops):
                               f"{self._ops.distie_wkv_scan_max_rank()} dimensions")
         low_ptr, low_ld = self._rows_view(low, rank)
         out = torch.empty((T, N), dtype=out_dtype, device=self.device)
+        if not self.captured and meta.host_cu_q is not None and meta.max_q >= self.SCAN_CHUNKED_MIN_ROWS and \
+                dim <= self._ops.distie_wkv_chunked_max_dim():
+            # portions of prompts: chunks of rows side by side instead of one row after the other
+            z = self.wkv_decay_logits(low, up, up_bias)
+            count, packed, scratch = self._scan_chunks(meta, self._ops.distie_wkv_chunk_rows(), num_heads, dim, dim)
+            totals = torch.empty((count, num_heads, dim), dtype=torch.float32, device=self.device)
+            _check(self._ops.distie_wkv_scan_chunked(
+                views[0][0], views[1][0], views[2][0], views[3][0], _code(r), ld, z.data_ptr(), bonus.data_ptr(),
+                state.data_ptr(), norm_weight.data_ptr(), float(eps), out.data_ptr(), _code(out), scratch.data_ptr(),
+                totals.data_ptr(), packed.data_ptr(), packed.data_ptr() + 16 * count, meta.state_slots.data_ptr(), count,
+                meta.num_requests, num_heads, dim, self._stream()), "wkv_scan_chunked")
+            _mark_written(state)
+            return out
         _check(self._ops.distie_wkv_scan(
             views[0][0], views[1][0], views[2][0], views[3][0], _code(r), ld, low_ptr, _code(low), low_ld, rank, up.data_ptr(),
             up_bias.data_ptr(), bonus.data_ptr(), state.data_ptr(), norm_weight.data_ptr(), float(eps), out.data_ptr(),
