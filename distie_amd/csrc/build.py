@@ -1,12 +1,13 @@
 """Building and finding the native libraries.
 
-Four kinds of shared library, all built from the sources beside this file:
+Five kinds of shared library, all built from the sources beside this file:
 
 * `core`  - the id pool of the cache manager (C++, host only, g++);
 * `ops`   - the HIP kernels that do not depend on the head size (hipcc, gfx950);
 * `library` - the calls of the vendor's matrix-product library for large products (hipcc, linked with hipBLASLt);
 * `attn_d<D>` - the attention kernels for head size D (hipcc, `-DDISTIE_HEAD_DIM=D`; the matrix-core
-  kernels for multiples of 16 up to 256, the wave-per-token kernel for every even size up to 1024).
+  kernels for multiples of 16 up to 256, the wave-per-token kernel for every even size up to 1024);
+* `mixattn_d<D>` - the matrix-core kernels of attention with mixed heads for head size D (a multiple of 32 up to 256).
 
 A library's file name carries a hash of its sources and flags, so a stale build is never
 loaded. Libraries live in `distie_amd/_lib/` (in-tree); if that folder cannot be written,
@@ -39,6 +40,7 @@ CXX_FLAGS = ["-O2", "-fPIC", "-std=c++17", "-pthread"]
 OPS_SOURCES = ["elementwise.hip", "gemm.hip", "gemv.hip", "decode_products.hip", "sampling.hip", "sequence.hip", "recurrent.hip", "latent.hip", "ssm.hip",
                "depth.hip", "time_mixing.hip", "mixed_attention.hip"]
 ATTN_SOURCES = ["attention.hip"]
+MIXED_ATTN_SOURCES = ["mixed_attention_mc.hip"]
 LIBRARY_SOURCES = ["library_products.hip"]
 LINK_LIBS = {"library": ["-lhipblaslt"]}
 HEADERS = ["common.h"]
@@ -78,6 +80,11 @@ def _spec(name: str):
         if dim < 2 or dim > 1024 or dim % 2:
             raise BuildError(f"attention kernels are built for even head sizes up to 1024, not {dim}")
         return list(ATTN_SOURCES), _hipcc(), list(HIP_FLAGS) + [f"-DDISTIE_HEAD_DIM={dim}"]
+    if name.startswith("mixattn_d"):
+        dim = int(name[len("mixattn_d"):])
+        if dim < 32 or dim > 256 or dim % 32:
+            raise BuildError(f"the kernels of attention with mixed heads are built for multiples of 32 up to 256, not {dim}")
+        return list(MIXED_ATTN_SOURCES), _hipcc(), list(HIP_FLAGS) + [f"-DDISTIE_HEAD_DIM={dim}"]
     raise BuildError(f"no native library named {name}")
 
 
@@ -197,12 +204,15 @@ def ensure(name: str) -> Path:
 
 
 DEFAULT_HEAD_DIMS = (16, 32, 40, 48, 64, 80, 96, 112, 128, 192, 256, 288)
+DEFAULT_MIXED_HEAD_DIMS = (32, 64, 96, 128, 160)
 
 
 def build_all(head_dims=DEFAULT_HEAD_DIMS, force: bool = True) -> List[Path]:
     out = [build("core", force), build("ops", force), build("library", force)]
     for d in head_dims:
         out.append(build(f"attn_d{d}", force))
+    for d in DEFAULT_MIXED_HEAD_DIMS:
+        out.append(build(f"mixattn_d{d}", force))
     return out
 
 

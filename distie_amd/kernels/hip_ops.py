@@ -221,6 +221,9 @@ class HipOps(Ops):
     # length are cut as before). Everywhere else it is level or behind (32 requests: 30 -> 33 us).
     DECODE_SHARED_BELOW = 0.8
     DECODE_MAX_RUNS = 256
+    # attention with mixed heads: from so many tokens a step on a workgroup takes 16 queries instead of 8 (fewer would
+    # leave compute units without one)
+    MIXED_WIDE_TOKENS = 6144
     # the matrix-core attention kernels take heads up to 256; wider ones (a latent that all heads share) run on the
     # wave-per-token kernel, in either precision
     LARGEST_MATRIX_CORE_HEAD = 256
@@ -254,6 +257,7 @@ class HipOps(Ops):
         self._ops = ctypes.CDLL(str(build.ensure("ops")))
         self._declare()
         self._attn: Dict[int, ctypes.CDLL] = {}
+        self._mixed: Dict[int, ctypes.CDLL] = {}
         # pinned staging buffers for `upload`, used in turn: [host tensor, its numpy view, event of the last copy]
         self._uploads = [[None, None, None] for _ in range(self.UPLOAD_BUFFERS)]
         self._next_upload = 0
@@ -392,6 +396,18 @@ class HipOps(Ops):
             if lib.distie_attention_head_dim() != head_dim:
                 raise KernelError("attention library was built for another head size")
             self._attn[head_dim] = lib
+        return lib
+
+    def mixed_attention_library(self, head_dim: int) -> ctypes.CDLL:
+        lib = self._mixed.get(head_dim)
+        if lib is None:
+            lib = ctypes.CDLL(str(build.ensure(f"mixattn_d{head_dim}")))
+            lib.distie_mixed_fits.argtypes = [_I, _I]
+            lib.distie_mixed_attention_bf16.argtypes = [_P, _L, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I,
+                                                        _F, _P, _I, _P, _P, _I, _I, _I, _I, _P, _P, _P]
+            if lib.distie_mixed_head_dim() != head_dim:
+                raise KernelError("the library of attention with mixed heads was built for another head size")
+            self._mixed[head_dim] = lib
         return lib
 
     def _own(self, *tensors) -> None:
@@ -1032,15 +1048,57 @@ class HipOps(Ops):
             raise KernelError("paged_attention: head_mix must be [num_heads, num_heads]")
         if q.shape[1] != num_heads * head_dim:
             raise KernelError("paged_attention: mixed heads take q alone")
+        ptr = lambda t: t.data_ptr() if t is not None else None
+        keep = int(extras.keep_first) if window else 0
+        if q.dtype == torch.bfloat16 and k_cache.dtype == torch.bfloat16 and meta.block_size % 16 == 0 and \
+                head_dim % 32 == 0 and head_dim <= self.LARGEST_MATRIX_CORE_HEAD:
+            lib = self.mixed_attention_library(head_dim)
+            queries = lib.distie_mixed_fits(num_heads, num_kv_heads)
+            if queries:
+                key = ("mixed_attention", int(window or 0), keep, num_heads, head_dim, meta.max_kv, meta.all_decode,
+                       meta.singles_bound)
+                plan = meta.scratch.get(key)
+                if plan is None or plan["cu_q"] is not meta.host_cu_q:
+                    plan = meta.scratch[key] = self._mixed_plan(lib, meta, num_heads, head_dim, window, keep)
+                if queries == 16 and q.shape[0] < self.MIXED_WIDE_TOKENS:
+                    queries = 8
+                _check(lib.distie_mixed_attention_bf16(
+                    q.data_ptr(), q.shape[1], k_cache.data_ptr(), v_cache.data_ptr(), meta.positions.data_ptr(),
+                    meta.cu_q.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr, out.data_ptr(), q.shape[0],
+                    meta.num_requests, num_heads, num_kv_heads, meta.block_size, float(scale), int(window or 0), keep,
+                    float(extras.score_cap or 0.0), ptr(bias), bias.shape[1] if bias is not None else 0, ptr(mix),
+                    ptr(extras.sinks), 1 if plan["prefill"] else 0, queries, 1 if plan["decode"] else 0, plan["splits"],
+                    ptr(plan["partial_o"]), ptr(plan["partial_ml"]), self._stream()), "mixed_attention_bf16")
+                return
         if not self._ops.distie_mixed_attention_fits(num_heads, head_dim):
             raise KernelError(f"paged_attention: {num_heads} mixed heads of {head_dim} do not fit the LDS of a compute unit")
-        ptr = lambda t: t.data_ptr() if t is not None else None
         _check(self._ops.distie_mixed_attention_generic(
             q.data_ptr(), _code(q), q.shape[1], k_cache.data_ptr(), v_cache.data_ptr(), _code(k_cache),
             meta.positions.data_ptr(), meta.token_request.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr,
             out.data_ptr(), q.shape[0], num_heads, num_kv_heads, head_dim, meta.block_size, float(scale), int(window or 0),
-            int(extras.keep_first) if window else 0, float(extras.score_cap or 0.0), ptr(bias),
-            bias.shape[1] if bias is not None else 0, ptr(mix), ptr(extras.sinks), self._stream()), "mixed_attention_generic")
+            keep, float(extras.score_cap or 0.0), ptr(bias), bias.shape[1] if bias is not None else 0, ptr(mix),
+            ptr(extras.sinks), self._stream()), "mixed_attention_generic")
+
+    def _mixed_plan(self, lib, meta: BatchMeta, num_heads, head_dim, window, keep) -> dict:
+        """Which of the mixed heads' kernels a step needs, and the buffers for partial results of single tokens (one
+        for every run of keys a token may see): the same for every layer with these sizes."""
+        singles = meta.num_requests if meta.all_decode else 0
+        if not meta.all_decode and meta.singles_bound is not None:
+            singles = meta.singles_bound
+        elif not meta.all_decode and meta.host_cu_q is not None:
+            singles = int((meta.host_cu_q[1:] - meta.host_cu_q[:-1] == 1).sum())
+        run = lib.distie_mixed_decode_keys()
+        plan = {"cu_q": meta.host_cu_q, "decode": singles > 0, "splits": 0, "partial_o": None, "partial_ml": None,
+                "prefill": singles < meta.num_requests or (meta.singles_bound is not None and not meta.all_decode)}
+        if plan["decode"]:
+            splits = -(-meta.max_kv // run)
+            if window:
+                splits = min(splits, -(-keep // run) + (int(window) + run - 2) // run + 1)
+            plan["splits"] = max(1, splits)
+            shape = (meta.num_requests, plan["splits"], num_heads)
+            plan["partial_o"] = torch.empty((*shape, head_dim), dtype=torch.float32, device=self.device)
+            plan["partial_ml"] = torch.empty((*shape, 2), dtype=torch.float32, device=self.device)
+        return plan
 
     def _attention_plan(self, lib, meta: BatchMeta, T, num_heads, num_kv_heads, head_dim, window) -> dict:
         group = num_heads // num_kv_heads
