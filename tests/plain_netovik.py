@@ -47,7 +47,7 @@ def wkv_scan(r, k, v, decay, u):
     return out
 
 
-def wkv(h, w, p, m, eps):
+def wkv(h, w, p, m, eps, watch=None):
     T = h.shape[0]
     H, D = int(m["heads"]), int(m["dim"])
     before = token_shift(h)
@@ -56,6 +56,8 @@ def wkv(h, w, p, m, eps):
     gate = silu(mix["g"] @ w[p + "g"].T)
     decay = wkv_decay(mix["w"], w[p + "w1"], w[p + "w2"], w[p + "w0"]).view(T, H, D)
     o = wkv_scan(r, k, v, decay, w[p + "u"])
+    if watch is not None:
+        watch("heads", o, wkv_scan(r ** 2, k ** 2, v ** 2, decay ** 2, w[p + "u"] ** 2))     # and its terms' squares, summed
     return (rms(o, eps).reshape(T, H * D) * w[p + "norm"] * gate) @ w[p + "o"].T
 
 
@@ -120,8 +122,10 @@ def route(h, router, top):
     return order.indices[:, :top], order.values[:, :top]
 
 
-def mixture(h, w, p, mlp):
+def mixture(h, w, p, mlp, watch=None):
     chosen, scores = route(h, w[p + "router"], int(mlp["router"]["top"]))
+    if watch is not None:
+        watch("router", h @ w[p + "router"].T, int(mlp["router"]["top"]))
     out = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for e, s in zip(chosen[t].tolist(), scores[t]):
@@ -129,16 +133,17 @@ def mixture(h, w, p, mlp):
     return out
 
 
-def feed_forward(h, w, p, mlp):
-    return gated(h, w, p) if mlp["kind"] == "dense" else mixture(h, w, p, mlp)
+def feed_forward(h, w, p, mlp, watch=None):
+    return gated(h, w, p) if mlp["kind"] == "dense" else mixture(h, w, p, mlp, watch)
 
 
 def depth_average(results, weights):
     return sum(weights[j] * x for j, x in enumerate(results))
 
 
-def forward(cfg, weights, ids):
-    """-> (float64 logits [T, vocab], the averaged residual behind every layer)."""
+def forward(cfg, weights, ids, watch=None):
+    """-> (float64 logits [T, vocab], the averaged residual behind every layer). `watch(what, ...)` is shown the heads'
+    outputs in front of their norms and the routers' logits."""
     w = {name: t.double() for name, t in weights.items()}
     eps, groups = float(cfg["norm"]["eps"]), int(cfg["norm"].get("groups") or 1)
     ids = torch.as_tensor(ids, dtype=torch.long)
@@ -146,10 +151,13 @@ def forward(cfg, weights, ids):
     results, after = [x], []
     for i, layer in enumerate(cfg["layers"]):
         p = f"l{i}."
-        mixer = wkv if layer["type"] == "wkv" else attention
-        x = x + group_norm(mixer(x, w, p + "mix.", layer["mixer"], eps), w[p + "norm1"], groups, eps)
+        if layer["type"] == "wkv":
+            y = wkv(x, w, p + "mix.", layer["mixer"], eps, watch)
+        else:
+            y = attention(x, w, p + "mix.", layer["mixer"], eps)
+        x = x + group_norm(y, w[p + "norm1"], groups, eps)
         if layer.get("mlp"):
-            x = x + group_norm(feed_forward(x, w, p + "mlp.", layer["mlp"]), w[p + "norm2"], groups, eps)
+            x = x + group_norm(feed_forward(x, w, p + "mlp.", layer["mlp"], watch), w[p + "norm2"], groups, eps)
         results.append(x)
         x = depth_average(results, w[p + "dwa"])
         after.append(x.clone())
