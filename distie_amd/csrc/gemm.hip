@@ -522,6 +522,72 @@ extern "C" int distie_gemm_packed_bf16(const void* x, const void* w_packed, cons
   return launch_status();
 }
 
+// Several products side by side, each with an input of its own (x: [count, M, K]) and weights of its own: the packed copies
+// one behind the other, every weight's rows rounded up to whole row blocks. blockIdx.x: row block; blockIdx.z: a group of 16
+// rows of x. The WAVES waves of a workgroup share the k tiles and add their sums through LDS, so nothing is cut across
+// workgroups: y [M, ld] in float32, row block b in the columns 16 b .. 16 b + 15.
+constexpr int EACH_MAX = 8;
+struct EachBlocks {
+  int count;
+  int end[EACH_MAX];           // row blocks up to and with each product's last
+};
+
+template <int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void gemm_packed_each_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
+                                                                      float* __restrict__ y, int M, int K, int ld,
+                                                                      EachBlocks blocks) {
+  __shared__ float part[WAVES][4][64];
+  const int lane = threadIdx.x % 64, wave = threadIdx.x / 64, r = lane % 16, g = lane / 16;
+  int product = 0;
+#pragma unroll
+  for (int j = 0; j < EACH_MAX - 1; ++j)
+    if (j + 1 < blocks.count && static_cast<int>(blockIdx.x) >= blocks.end[j]) product = j + 1;
+  const int m0 = 16 * blockIdx.z, rows = min(16, M - m0);
+  const int k_tiles = (K + 31) / 32;
+  const int per_wave = ((k_tiles + WAVES - 1) / WAVES + 3) / 4 * 4;
+  const int t_begin = min(k_tiles, wave * per_wave), t_end = min(k_tiles, t_begin + per_wave);
+  const bf16_t* wp = w + static_cast<int64_t>(blockIdx.x) * k_tiles * PK_TILE + lane * 8;
+  const bf16_t* xp = x + (static_cast<int64_t>(product) * M + m0 + min(r, rows - 1)) * K + 8 * g;
+  const floatx4 acc = packed_accumulate(wp, xp, t_begin, t_end, K, g, blockIdx.x + wave);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) part[wave][i][lane] = acc[i];
+  __syncthreads();
+  // wave i % WAVES adds up the sums of the lane's row i
+  for (int i = wave; i < 4; i += WAVES) {
+    float sum = 0.f;
+#pragma unroll
+    for (int v = 0; v < WAVES; ++v) sum += part[v][i][lane];
+    if (r < rows) y[static_cast<int64_t>(m0 + r) * ld + 16 * static_cast<int64_t>(blockIdx.x) + 4 * g + i] = sum;
+  }
+}
+
+// ends: `count` numbers on the host, the row blocks up to and with each product's last; y: float32 [M, 16 * ends[count - 1]]
+extern "C" int distie_gemm_packed_each_bf16(const void* x, const void* w_packed, float* y, int M, int K, int count,
+                                            const int32_t* ends, hipStream_t stream) {
+  if (M <= 0) return 0;
+  if (M > 256 || K <= 0 || K % 8 != 0 || count < 1 || count > EACH_MAX) return DISTIE_BAD_ARGUMENT;
+  EachBlocks blocks = {};
+  blocks.count = count;
+  for (int j = 0; j < count; ++j) {
+    if (ends[j] < 1 || (j > 0 && ends[j] <= ends[j - 1])) return DISTIE_BAD_ARGUMENT;
+    blocks.end[j] = ends[j];
+  }
+  const int all = blocks.end[count - 1];
+  const dim3 grid(all, 1, (M + 15) / 16);
+  const bf16_t* xb = static_cast<const bf16_t*>(x);
+  const bf16_t* wb = static_cast<const bf16_t*>(w_packed);
+  const int waves = std::min(packed_waves(K), 8);
+#define EACH(WAVES) gemm_packed_each_kernel<WAVES><<<grid, 64 * WAVES, 0, stream>>>(xb, wb, y, M, K, 16 * all, blocks)
+  switch (waves) {
+    case 8: EACH(8); break;
+    case 4: EACH(4); break;
+    case 2: EACH(2); break;
+    default: EACH(1); break;
+  }
+#undef EACH
+  return launch_status();
+}
+
 // ---------------------------------------------------------------- packed weights, up to 96 rows of x a pass
 // A workgroup of WAVES waves owns as many row blocks (one a wave) and one slice of K. Per k-step of 128 the
 // weights go straight into registers, some k-steps ahead; the x tile ([16 MB rows, 128 k], the same for

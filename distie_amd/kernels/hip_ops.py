@@ -308,6 +308,7 @@ class HipOps(Ops):
         o.distie_gemm_packed_wide_slices.argtypes = [_I, _I]
         o.distie_gemm_packed_wide_qkv_bf16.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
         o.distie_gemm_packed_rotary_bf16.argtypes = [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
+        o.distie_gemm_packed_each_bf16.argtypes = [_P, _P, _P, _I, _I, _I, _P, _P]
         o.distie_decode_norm_fits.argtypes = [_I]
         o.distie_decode_product_residual.argtypes = [_P, _P, _P, _P, _I, _I, _I, _P]
         o.distie_decode_norm_product.argtypes = [_P, _P, _F, _P, _P, _P, _I, _I, _I, _I, _P, _P, _P, _P,
@@ -1593,6 +1594,52 @@ class HipOps(Ops):
                                             meta.state_slots.data_ptr(), T, C, self._stream()), "token_shift")
         _mark_written(state)
         return out
+
+    EACH_MAX_ROWS = 32        # up to so many rows several products with inputs of their own run as one launch
+
+    def prepare_linear_each(self, weights):
+        """One packed copy for all, kept on the first weight: the weights one behind the other, each rounded up to whole
+        row blocks (the projections of few rows); beside it nothing, as more rows go to the library."""
+        first = weights[0]
+        if (self.packed_roles is not None and "qkv" not in self.packed_roles) or not self.packed_weights or \
+                any(w.dtype != torch.bfloat16 or w.dim() != 2 or w.shape[1] != first.shape[1] for w in weights) or \
+                first.shape[1] % 8 or len(weights) > 8 or hasattr(first, "_distie_each"):
+            return
+        K = first.shape[1]
+        blocks = [-(-w.shape[0] // 16) for w in weights]
+        free, total = torch.cuda.mem_get_info(self.device)
+        if free - 2 * sum(blocks) * -(-K // 32) * 512 < self.PACKED_KEEPS_FREE * total:
+            self._packed_left_out += 1
+            return
+        packed = torch.empty(sum(blocks) * -(-K // 32) * 512, dtype=torch.bfloat16, device=self.device)
+        at, maps = 0, []
+        for w, count in zip(weights, blocks):
+            self._own(w)
+            row_map = self._row_map(w.shape[0], False, None).to(device=self.device, dtype=torch.int32)
+            maps.append(row_map)
+            size = count * -(-K // 32) * 512
+            _check(self._ops.distie_pack_rows(w.data_ptr(), packed[at:at + size].data_ptr(), row_map.data_ptr(), count, K,
+                                              self._stream()), "pack_rows")
+            at += size
+        torch.cuda.current_stream(self.device).synchronize()      # the row maps are freed on return
+        first._distie_each = (packed, np.cumsum(np.asarray(blocks, dtype=np.int32)).astype(np.int32))
+
+    def linear_each(self, xs, weights, unrounded=()):
+        held = getattr(weights[0], "_distie_each", None)
+        if held is None or xs.dtype != torch.bfloat16 or xs.shape[1] > self.EACH_MAX_ROWS:
+            return super().linear_each(xs, weights, unrounded)
+        self._own(xs)
+        packed, ends = held
+        count, M, K = xs.shape
+        if count != len(weights) or any(w.shape[1] != K for w in weights) or \
+                [int(e) for e in np.diff(ends, prepend=0)] != [-(-w.shape[0] // 16) for w in weights] or \
+                packed.numel() != int(ends[-1]) * -(-K // 32) * 512:
+            raise KernelError("linear_each: an input [rows, K] for every weight [N, K], the weights it was prepared for")
+        out = torch.empty((M, 16 * int(ends[-1])), dtype=torch.float32, device=self.device)
+        _check(self._ops.distie_gemm_packed_each_bf16(xs.data_ptr(), packed.data_ptr(), out.data_ptr(), M, K, count,
+                                                      ends.ctypes.data, self._stream()), "gemm_packed_each_bf16")
+        starts = [0] + [16 * int(e) for e in ends[:-1]]
+        return [out[:, at:at + w.shape[0]] for at, w in zip(starts, weights)]
 
     def wkv_decay_logits(self, low, up, up_bias):
         low = low if low.dtype == torch.float32 else low.float()
