@@ -7,8 +7,8 @@
 //    to the waves. Scale, cap and bias, then into LDS, float32. (2) A wave owns queries: for each, the heads' scores of 16 keys
 //    are mixed as a float32 matrix product (heads x heads times heads x keys), masked, and their softmax is carried on; the
 //    weights go to LDS in bfloat16. (3) The waves add weights times values to the columns of (1), which they keep.
-//  * mixed_decode: one token a request; a workgroup owns 64 keys of it. A wave scores and mixes 16 keys for all heads, the
-//    waves agree on the maxima, and the sums over the 64 keys go to memory as a partial result.
+//  * mixed_decode: one token a request; a workgroup of sixteen waves owns 64 keys of it. Four waves share 16 keys: they score
+//    and mix them for all heads, all agree on the maxima, and the sums over the 64 keys go to memory as a partial result.
 //  * mixed_reduce: puts a token's partial results together.
 #include "common.h"
 
@@ -43,7 +43,7 @@ struct MixedArgs {
   const float* sinks;            // [H] or null
   float* partial_o;              // decode: [B, splits, H, D]
   float* partial_ml;             // decode: [B, splits, H, 2]
-  int table_width, bias_len, requests, H, G, block_size, window, keep, splits, skip_singles;
+  int table_width, bias_len, requests, H, G, block_size, window, keep, splits, skip_singles, all_single;
   float scale, cap;
 };
 
@@ -169,35 +169,73 @@ mixed_prefill_kernel(MixedArgs p) {
     for (int d = 0; d < D / 16; ++d) o[n][d] = floatx4{0.f, 0.f, 0.f, 0.f};
   }
 
-  const auto next_step = [&](int c) { return c >= keep && c + KT - 1 < first ? first / KT * KT : c; };
-  int c = next_step(0), buffer = 0;
-  stage_bias(c, buffer);
-  __syncthreads();
-  while (c <= last) {
-    // the pages of the step's two runs of 16 keys; a run that nobody sees takes the other's (its weights are zero)
+  // Where the registers allow it, a step's keys are asked for while the step before is mixed, and its values before its own
+  // scores are made: what is left of a trip to memory then hides behind the other phases.
+  constexpr bool AHEAD = NT * D <= 128;
+  bf16x8 keys[AHEAD ? NT : 1][2][D / 32];
+  // the pages of a step's two runs of 16 keys; a run that nobody sees takes the other's (its weights are zero)
+  const auto pages_of = [&](int at, int page[2]) {
     bool seen[2];
-    int page[2];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
-      const int k0 = c + 16 * u;
+      const int k0 = at + 16 * u;
       seen[u] = k0 <= last && (k0 + 15 >= first || k0 < keep);
       page[u] = seen[u] ? table[k0 / bs] : -1;
     }
     if (!seen[0]) page[0] = page[1];
     if (!seen[1]) page[1] = page[0];
+  };
+  const auto keys_at = [&](int at, int page, int u, int n) {
+    const int k0 = at + 16 * u;
+    return p.k_cache + ((static_cast<int64_t>(page) * G + kh[n]) * bs + k0 % bs + i) * D + 8 * g;
+  };
+  const auto load_keys = [&](int at, const int page[2]) {
+    if constexpr (AHEAD) {
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          const bf16_t* src = keys_at(at, page[u], u, n);
+#pragma unroll
+          for (int s = 0; s < D / 32; ++s) keys[n][u][s] = *reinterpret_cast<const bf16x8*>(src + 32 * s);
+        }
+    }
+  };
+  const auto next_step = [&](int c) { return c >= keep && c + KT - 1 < first ? first / KT * KT : c; };
+  int c = next_step(0), buffer = 0;
+  stage_bias(c, buffer);
+  int page[2];
+  pages_of(c, page);                           // (the first step holds key 0 or the window's first: somebody sees it)
+  load_keys(c, page);
+  __syncthreads();
+  while (c <= last) {
+    bf16x8 values[AHEAD ? NT : 1][D / 16];
+    const auto values_at = [&](int n) {
+      return p.v_cache + ((static_cast<int64_t>(g < 2 ? page[0] : page[1]) * G + kh[n]) * D + i) * bs + (c + 8 * g) % bs;
+    };
+    if constexpr (AHEAD) {
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int d = 0; d < D / 16; ++d)
+          values[n][d] = *reinterpret_cast<const bf16x8*>(values_at(n) + static_cast<int64_t>(16 * d) * bs);
+    }
     // (1) raw scores of this wave's columns
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       if (!have[n]) continue;
 #pragma unroll
       for (int u = 0; u < 2; ++u) {
-        if (!seen[u]) continue;
-        const int k0 = c + 16 * u;
-        const bf16_t* src = p.k_cache + ((static_cast<int64_t>(page[u]) * G + kh[n]) * bs + k0 % bs + i) * D + 8 * g;
+        const bf16_t* src = keys_at(c, page[u], u, n);
         floatx4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int s = 0; s < D / 32; ++s)
-          acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(src + 32 * s), q[n][s], acc, 0, 0, 0);
+        for (int s = 0; s < D / 32; ++s) {
+          if constexpr (AHEAD) {
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(keys[n][u][s], q[n][s], acc, 0, 0, 0);
+          } else {
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(src + 32 * s), q[n][s], acc, 0, 0, 0);
+          }
+        }
         float v[4];
         const float* by_distance = bias_s + (buffer * H + head[n]) * BW + query[n] - (16 * u + 4 * g) + KT - 1;
 #pragma unroll
@@ -211,7 +249,12 @@ mixed_prefill_kernel(MixedArgs p) {
     __syncthreads();
     // (2) this wave's queries: mix the heads, mask, carry the softmax on
     const int following = next_step(c + KT);
-    if (following <= last) stage_bias(following, 1 - buffer);
+    int page_next[2] = {page[0], page[1]};
+    if (following <= last) {
+      pages_of(following, page_next);
+      load_keys(following, page_next);
+      stage_bias(following, 1 - buffer);
+    }
     for (int y = wave; y < nq; y += PF_WAVES) {
       const int pos = pos0 + y;
       const int from = p.window > 0 ? max(0, pos - p.window + 1) : 0;
@@ -258,14 +301,18 @@ mixed_prefill_kernel(MixedArgs p) {
         for (int d = 0; d < D / 16; ++d) o[n][d] *= alpha;
       }
       const bf16x8 weights = *reinterpret_cast<const bf16x8*>(P + at * PP + 8 * g);
-      const int k0 = c + 8 * g;
-      const bf16_t* src = p.v_cache + ((static_cast<int64_t>(g < 2 ? page[0] : page[1]) * G + kh[n]) * D + i) * bs + k0 % bs;
 #pragma unroll
-      for (int d = 0; d < D / 16; ++d)
-        o[n][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(src + static_cast<int64_t>(16 * d) * bs),
-                                                          weights, o[n][d], 0, 0, 0);
+      for (int d = 0; d < D / 16; ++d) {
+        if constexpr (AHEAD) {
+          o[n][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(values[n][d], weights, o[n][d], 0, 0, 0);
+        } else {
+          o[n][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              *reinterpret_cast<const bf16x8*>(values_at(n) + static_cast<int64_t>(16 * d) * bs), weights, o[n][d], 0, 0, 0);
+        }
+      }
     }
     c = following;
+    page[0] = page_next[0], page[1] = page_next[1];
     buffer = 1 - buffer;
   }
 #pragma unroll
@@ -288,15 +335,17 @@ mixed_prefill_kernel(MixedArgs p) {
 }
 
 // ------------------------------------------------------------------------------------------------ single tokens
-constexpr int DC_WAVES = 4;
+constexpr int DC_WAVES = 16;
 constexpr int DC_KEYS = 64;
+constexpr int DC_RUNS = DC_KEYS / 16;    // runs of 16 keys; DC_WAVES / DC_RUNS waves share a run's heads
+constexpr int RD_WAVES = 4;              // of the kernel that puts partial results together
 constexpr int DC_SP = DC_KEYS + 16;      // floats between the heads' scores
 constexpr int DC_PP = DC_KEYS + 8;       // bfloat16 values between the heads' weights
-constexpr int MAX_HEAD_TILES = 4;
+constexpr int MAX_HEAD_TILES = DC_WAVES / DC_RUNS;
 
 size_t decode_lds(int H) {
   const int HP = (H + 15) / 16 * 16;
-  return sizeof(float) * static_cast<size_t>(HP) * (DC_SP + HP + 4 + 2 * DC_WAVES) + sizeof(bf16_t) * static_cast<size_t>(HP) * DC_PP;
+  return sizeof(float) * static_cast<size_t>(HP) * (DC_SP + HP + 4 + 2 * DC_RUNS) + sizeof(bf16_t) * static_cast<size_t>(HP) * DC_PP;
 }
 
 // which runs of 64 keys the token at `pos` sees: those with kept first keys ahead of the window's, then the window's
@@ -313,17 +362,20 @@ struct VisibleRuns {
 
 __global__ void __launch_bounds__(64 * DC_WAVES)
 mixed_decode_kernel(MixedArgs p) {
+  constexpr int PARTS = DC_WAVES / DC_RUNS;
+  constexpr int AHEAD = 2;                                 // tiles of values a wave asks for before the scores are made
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int H = p.H, G = p.G, group = H / G, HP = heads_padded(H), bs = p.block_size;
   bf16_t* P = reinterpret_cast<bf16_t*>(lds);              // [HP][DC_PP]
   float* S = lds + HP * DC_PP / 2;                         // [HP][DC_SP]
   float* M = S + HP * DC_SP;                               // [HP][HP + 4]
-  float* wave_top = M + HP * (HP + 4);                     // [DC_WAVES][HP]
-  float* wave_total = wave_top + DC_WAVES * HP;            // [DC_WAVES][HP]
+  float* run_top = M + HP * (HP + 4);                      // [DC_RUNS][HP]
+  float* run_total = run_top + DC_RUNS * HP;               // [DC_RUNS][HP]
   const int lane = threadIdx.x % 64, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64), i = lane % 16, g = lane / 16;
+  const int run = wave % DC_RUNS, part = wave / DC_RUNS;
   const int request = blockIdx.y, split = blockIdx.x;
-  const int64_t t = p.cu_q[request];
-  if (p.cu_q[request + 1] - t != 1) return;
+  const int64_t t = p.all_single ? request : p.cu_q[request];
+  if (!p.all_single && p.cu_q[request + 1] - t != 1) return;
   const int pos = p.positions[t];
   const VisibleRuns runs(pos, p.window, p.keep);
   if (split >= runs.total) return;
@@ -332,127 +384,153 @@ mixed_decode_kernel(MixedArgs p) {
   const int keep = p.window > 0 ? p.keep : 0;
   const int32_t* table = p.block_table + static_cast<int64_t>(p.table_rows != nullptr ? p.table_rows[request] : request) * p.table_width;
   const float bend = p.cap > 0.f ? 2.f * LOG2E / p.cap : 0.f;
-  int page[DC_KEYS / 16], some = 0;
+  int page[DC_RUNS], some = 0, mine = -1;
 #pragma unroll
-  for (int u = 0; u < DC_KEYS / 16; ++u) {
+  for (int u = 0; u < DC_RUNS; ++u) {
     const int k0 = c + 16 * u;
     const bool seen = k0 <= pos && (k0 + 15 >= first || k0 < keep);
     page[u] = seen ? table[k0 / bs] : -1;
     if (seen) some = page[u];
+    if (u == run) mine = page[u];
   }
-  const int k0 = c + 16 * wave;
-  int mine = -1;
 #pragma unroll
-  for (int u = 0; u < DC_KEYS / 16; ++u)
-    if (u == wave) mine = page[u];
-#pragma unroll
-  for (int u = 0; u < DC_KEYS / 16; ++u)
+  for (int u = 0; u < DC_RUNS; ++u)
     if (page[u] < 0) page[u] = some;                       // keys that are not seen have weight zero: any page will do
+  const int tiles = (group + 15) / 16;                     // column tiles of a key/value head's query heads
+  const int k0 = c + 16 * run;
+  // (a) raw scores of the run's keys, the column tiles dealt to the run's waves; the values of the first tiles of (c)
+  const int value_tiles = G * tiles * (D / 16);
+  bf16x8 values[AHEAD][DC_KEYS / 32];
+  const auto values_at = [&](int tile, int m) {
+    const int d = tile % (D / 16), kh = tile / (D / 16) / tiles;
+    const int at = g < 2 ? page[2 * m] : page[2 * m + 1];
+    return p.v_cache + ((static_cast<int64_t>(at) * G + kh) * D + 16 * d + i) * bs + (c + 32 * m + 8 * g) % bs;
+  };
+  for (int kc = part; kc < G * tiles; kc += PARTS) {
+    const int kh = kc / tiles, hg = kc % tiles * 16 + i;
+    const int head = kh * group + min(hg, group - 1);
+    const bf16_t* k = p.k_cache + ((static_cast<int64_t>(mine < 0 ? some : mine) * G + kh) * bs + k0 % bs + i) * D + 8 * g;
+    const bf16_t* q = p.q + t * p.q_stride + static_cast<int64_t>(head) * D + 8 * g;
+    bf16x8 kf[D / 32], qf[D / 32];
+#pragma unroll
+    for (int s = 0; s < D / 32; ++s) {
+      kf[s] = *reinterpret_cast<const bf16x8*>(k + 32 * s);
+      qf[s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
+    }
+    float by_distance[4] = {};
+    if (p.bias != nullptr) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        by_distance[r] = p.bias[static_cast<int64_t>(head) * p.bias_len + min(max(pos - (k0 + 4 * g + r), 0), p.bias_len - 1)];
+    }
+    if (kc == part) {
+#pragma unroll
+      for (int x = 0; x < AHEAD; ++x)
+#pragma unroll
+        for (int m = 0; m < DC_KEYS / 32; ++m)
+          values[x][m] = *reinterpret_cast<const bf16x8*>(values_at(min(wave + x * DC_WAVES, value_tiles - 1), m));
+    }
+    floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < D / 32; ++s) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], acc, 0, 0, 0);
+    float v[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = capped(acc[r], p.scale, p.cap, bend) + by_distance[r];
+    if (hg < group) *reinterpret_cast<float4*>(S + head * DC_SP + 16 * run + 4 * g) = float4{v[0], v[1], v[2], v[3]};
+  }
+  if (part >= G * tiles) {
+#pragma unroll
+    for (int x = 0; x < AHEAD; ++x)
+#pragma unroll
+      for (int m = 0; m < DC_KEYS / 32; ++m)
+        values[x][m] = *reinterpret_cast<const bf16x8*>(values_at(min(wave + x * DC_WAVES, value_tiles - 1), m));
+  }
   stage_mix(p, HP, M);
   for (int x = threadIdx.x; x < (HP - H) * DC_SP; x += blockDim.x) S[H * DC_SP + x] = 0.f;
-  const int tiles = (group + 15) / 16;
-  if (mine >= 0) {
-    for (int kc = 0; kc < G * tiles; ++kc) {
-      const int kh = kc / tiles, hg = kc % tiles * 16 + i;
-      const int head = kh * group + min(hg, group - 1);
-      const bf16_t* k = p.k_cache + ((static_cast<int64_t>(mine) * G + kh) * bs + k0 % bs + i) * D + 8 * g;
-      const bf16_t* q = p.q + t * p.q_stride + static_cast<int64_t>(head) * D + 8 * g;
-      floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int s = 0; s < D / 32; ++s)
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(k + 32 * s),
-                                                      *reinterpret_cast<const bf16x8*>(q + 32 * s), acc, 0, 0, 0);
-      float v[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        v[r] = capped(acc[r], p.scale, p.cap, bend);
-        if (p.bias != nullptr)
-          v[r] += p.bias[static_cast<int64_t>(head) * p.bias_len + min(max(pos - (k0 + 4 * g + r), 0), p.bias_len - 1)];
-      }
-      if (hg < group) *reinterpret_cast<float4*>(S + head * DC_SP + 16 * wave + 4 * g) = float4{v[0], v[1], v[2], v[3]};
-    }
-  }
   __syncthreads();
+  // (b) mixed and masked scores of 16 heads and the run's keys a wave, the maxima of all runs, weights and their sums
   const int key = k0 + i;
   const bool see = mine >= 0 && key <= pos && (key >= first || key < keep);
-  floatx4 mixed[MAX_HEAD_TILES];
-#pragma unroll
-  for (int ht = 0; ht < MAX_HEAD_TILES; ++ht) {
-    if (16 * ht >= HP) break;
-    floatx4 a = {0.f, 0.f, 0.f, 0.f};
-    const float* rows_of_m = M + (16 * ht + i) * (HP + 4) + g;
-    const float* scores = S + g * DC_SP + 16 * wave + i;
+  const bool mixes = 16 * part < HP;                       // (a wave has one tile of heads at most: PARTS >= MAX_HEAD_TILES)
+  floatx4 mixed = {0.f, 0.f, 0.f, 0.f};
+  if (mixes) {
+    const float* rows_of_m = M + (16 * part + i) * (HP + 4) + g;
+    const float* scores = S + g * DC_SP + 16 * run + i;
     for (int s = 0; s < HP; s += 4)
-      a = __builtin_amdgcn_mfma_f32_16x16x4f32(rows_of_m[s], scores[s * DC_SP], a, 0, 0, 0);
+      mixed = __builtin_amdgcn_mfma_f32_16x16x4f32(rows_of_m[s], scores[s * DC_SP], mixed, 0, 0, 0);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      if (!see) a[r] = -INFINITY;
-      const float top = row_max(a[r]);
-      if (i == 0) wave_top[wave * HP + 16 * ht + 4 * g + r] = top;
+      if (!see) mixed[r] = -INFINITY;
+      const float top = row_max(mixed[r]);
+      if (i == 0) run_top[run * HP + 16 * part + 4 * g + r] = top;
     }
-    mixed[ht] = a;
   }
   __syncthreads();
-#pragma unroll
-  for (int ht = 0; ht < MAX_HEAD_TILES; ++ht) {
-    if (16 * ht >= HP) break;
+  if (mixes) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int head = 16 * ht + 4 * g + r;
-      float top = wave_top[head];
+      const int head = 16 * part + 4 * g + r;
+      float top = run_top[head];
 #pragma unroll
-      for (int w = 1; w < DC_WAVES; ++w) top = fmaxf(top, wave_top[w * HP + head]);
-      const float weight = see ? exponential(mixed[ht][r] - top) : 0.f;
+      for (int u = 1; u < DC_RUNS; ++u) top = fmaxf(top, run_top[u * HP + head]);
+      const float weight = see ? exponential(mixed[r] - top) : 0.f;
       const float total = row_sum(weight);
-      P[head * DC_PP + 16 * wave + i] = static_cast<bf16_t>(weight);
-      if (i == 0) wave_total[wave * HP + head] = total;
+      P[head * DC_PP + 16 * run + i] = static_cast<bf16_t>(weight);
+      if (i == 0) run_total[run * HP + head] = total;
     }
   }
   __syncthreads();
+  // (c) the partial result
   const int64_t place = (static_cast<int64_t>(request) * p.splits + split) * H;
   for (int h = threadIdx.x; h < H; h += blockDim.x) {
-    float top = wave_top[h], total = wave_total[h];
-    for (int w = 1; w < DC_WAVES; ++w) top = fmaxf(top, wave_top[w * HP + h]), total += wave_total[w * HP + h];
+    float top = run_top[h], total = run_total[h];
+#pragma unroll
+    for (int u = 1; u < DC_RUNS; ++u) top = fmaxf(top, run_top[u * HP + h]), total += run_total[u * HP + h];
     p.partial_ml[(place + h) * 2] = top;
     p.partial_ml[(place + h) * 2 + 1] = total;
   }
-  for (int tile = wave; tile < G * tiles * (D / 16); tile += DC_WAVES) {
+  const auto finish = [&](int tile, const bf16x8 v[DC_KEYS / 32]) {
     const int d = tile % (D / 16), kc = tile / (D / 16), kh = kc / tiles, hg = kc % tiles * 16 + i;
     const int head = kh * group + min(hg, group - 1);
     floatx4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int m = 0; m < DC_KEYS / 32; ++m) {
-      const int at = (g < 2 ? page[2 * m] : page[2 * m + 1]);
-      const bf16_t* v = p.v_cache + ((static_cast<int64_t>(at) * G + kh) * D + 16 * d + i) * bs + (c + 32 * m + 8 * g) % bs;
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(v),
-                                                    *reinterpret_cast<const bf16x8*>(P + head * DC_PP + 32 * m + 8 * g), acc, 0, 0, 0);
-    }
+    for (int m = 0; m < DC_KEYS / 32; ++m)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v[m], *reinterpret_cast<const bf16x8*>(P + head * DC_PP + 32 * m + 8 * g), acc, 0, 0, 0);
     if (hg < group)
       *reinterpret_cast<float4*>(p.partial_o + (place + head) * D + 16 * d + 4 * g) = float4{acc[0], acc[1], acc[2], acc[3]};
+  };
+#pragma unroll
+  for (int x = 0; x < AHEAD; ++x)
+    if (wave + x * DC_WAVES < value_tiles) finish(wave + x * DC_WAVES, values[x]);
+  for (int tile = wave + AHEAD * DC_WAVES; tile < value_tiles; tile += DC_WAVES) {
+    bf16x8 v[DC_KEYS / 32];
+#pragma unroll
+    for (int m = 0; m < DC_KEYS / 32; ++m) v[m] = *reinterpret_cast<const bf16x8*>(values_at(tile, m));
+    finish(tile, v);
   }
 }
 
 // one block a (request, head): the waves deal the partial results, a lane owns dimensions lane, lane + 64, ...
-__global__ void __launch_bounds__(64 * DC_WAVES)
+__global__ void __launch_bounds__(64 * RD_WAVES)
 mixed_reduce_kernel(MixedArgs p) {
-  __shared__ float sums[DC_WAVES][D], tops[DC_WAVES], totals[DC_WAVES];
+  __shared__ float sums[RD_WAVES][D], tops[RD_WAVES], totals[RD_WAVES];
   const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
   const int request = blockIdx.x, head = blockIdx.y;
-  const int64_t t = p.cu_q[request];
-  if (p.cu_q[request + 1] - t != 1) return;
+  const int64_t t = p.all_single ? request : p.cu_q[request];
+  if (!p.all_single && p.cu_q[request + 1] - t != 1) return;
   const VisibleRuns runs(p.positions[t], p.window, p.keep);
   const int64_t place = static_cast<int64_t>(request) * p.splits * p.H + head;
   float top = -INFINITY, total = 0.f, acc[(D + 63) / 64];
 #pragma unroll
   for (int x = 0; x < (D + 63) / 64; ++x) acc[x] = 0.f;
-  for (int s = wave; s < runs.total; s += DC_WAVES) top = fmaxf(top, p.partial_ml[(place + static_cast<int64_t>(s) * p.H) * 2]);
+  for (int s = wave; s < runs.total; s += RD_WAVES) top = fmaxf(top, p.partial_ml[(place + static_cast<int64_t>(s) * p.H) * 2]);
   if (lane == 0) tops[wave] = top;
   __syncthreads();
   const float sink = p.sinks != nullptr ? p.sinks[head] : -INFINITY;
   top = sink;
 #pragma unroll
-  for (int w = 0; w < DC_WAVES; ++w) top = fmaxf(top, tops[w]);
-  for (int s = wave; s < runs.total; s += DC_WAVES) {
+  for (int w = 0; w < RD_WAVES; ++w) top = fmaxf(top, tops[w]);
+  for (int s = wave; s < runs.total; s += RD_WAVES) {
     const int64_t at = place + static_cast<int64_t>(s) * p.H;
     const float weight = expf(p.partial_ml[at * 2] - top);
     total += p.partial_ml[at * 2 + 1] * weight;
@@ -467,11 +545,11 @@ mixed_reduce_kernel(MixedArgs p) {
   __syncthreads();
   float all = sink == -INFINITY ? 0.f : expf(sink - top);
 #pragma unroll
-  for (int w = 0; w < DC_WAVES; ++w) all += totals[w];
+  for (int w = 0; w < RD_WAVES; ++w) all += totals[w];
   for (int d = threadIdx.x; d < D; d += blockDim.x) {
     float v = 0.f;
 #pragma unroll
-    for (int w = 0; w < DC_WAVES; ++w) v += sums[w][d];
+    for (int w = 0; w < RD_WAVES; ++w) v += sums[w][d];
     p.out[(t * p.H + head) * D + d] = static_cast<bf16_t>(v / all);
   }
 }
@@ -521,8 +599,8 @@ extern "C" int distie_mixed_fits(int H, int G) {
 
 extern "C" int distie_mixed_decode_keys() { return DC_KEYS; }
 
-// prefill: T rows of B requests in workgroups of `queries` (8 or 16); `decode`: the requests that bring one token, `splits`
-// partial results each (at least as many as runs of 64 keys any of them sees)
+// prefill: T rows of B requests in workgroups of `queries` (8 or 16); `decode`: the requests that bring one token (2: all do,
+// row b is request b's), `splits` partial results each (at least as many as runs of 64 keys any of them sees)
 extern "C" int distie_mixed_attention_bf16(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                                            const int32_t* positions, const int32_t* cu_q, const int32_t* block_table,
                                            int table_width, const int32_t* table_rows, void* out, int T, int B, int H, int G,
@@ -543,6 +621,7 @@ extern "C" int distie_mixed_attention_bf16(const void* q, int64_t q_stride, cons
   p.partial_o = partial_o, p.partial_ml = partial_ml;
   p.table_width = table_width, p.bias_len = bias_len, p.requests = B, p.H = H, p.G = G, p.block_size = block_size;
   p.window = window, p.keep = keep, p.splits = splits, p.skip_singles = decode ? 1 : 0;
+  p.all_single = decode == 2 ? 1 : 0;
   p.scale = scale, p.cap = cap;
   if (decode) {
     if (splits < 1 || splits > 65535 || B > 65535 || H > 65535 || partial_o == nullptr || partial_ml == nullptr ||
@@ -555,7 +634,7 @@ extern "C" int distie_mixed_attention_bf16(const void* q, int64_t q_stride, cons
     mixed_decode_kernel<<<dim3(splits, B), 64 * DC_WAVES, lds, stream>>>(p);
     int status = launch_status();
     if (status != 0) return status;
-    mixed_reduce_kernel<<<dim3(B, H), 64 * DC_WAVES, 0, stream>>>(p);
+    mixed_reduce_kernel<<<dim3(B, H), 64 * RD_WAVES, 0, stream>>>(p);
     if ((status = launch_status()) != 0) return status;
   }
   if (prefill) {

@@ -20,15 +20,15 @@ __global__ void token_shift_kernel(const X* __restrict__ x, const float* __restr
   const int64_t t = blockIdx.x;
   const int c = V * static_cast<int>(blockIdx.y * blockDim.x + threadIdx.x);
   if (c >= C) return;
-  const int b = token_request[t];
-  const int64_t first = cu_q[b];
+  const int b = token_request != nullptr ? token_request[t] : static_cast<int>(t);     // null: a row a request
+  const int64_t first = token_request != nullptr ? cu_q[b] : t;
   float h[V], before[V];
   load_values<V>(x + t * C + c, h);
   if (t > first) {
     load_values<V>(x + (t - 1) * C + c, before);
   } else {
     float* own = state + static_cast<int64_t>(state_slots[b]) * C + c;
-    const int64_t last = cu_q[b + 1] - 1;
+    const int64_t last = token_request != nullptr ? cu_q[b + 1] - 1 : t;
     float keep[V];
     load_values<V>(own, before);
     load_values<V>(x + last * C + c, keep);

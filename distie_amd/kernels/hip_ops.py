@@ -1068,7 +1068,7 @@ class HipOps(Ops):
                     meta.cu_q.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr, out.data_ptr(), q.shape[0],
                     meta.num_requests, num_heads, num_kv_heads, meta.block_size, float(scale), int(window or 0), keep,
                     float(extras.score_cap or 0.0), ptr(bias), bias.shape[1] if bias is not None else 0, ptr(mix),
-                    ptr(extras.sinks), 1 if plan["prefill"] else 0, queries, 1 if plan["decode"] else 0, plan["splits"],
+                    ptr(extras.sinks), 1 if plan["prefill"] else 0, queries, (2 if meta.all_decode else 1) if plan["decode"] else 0, plan["splits"],
                     ptr(plan["partial_o"]), ptr(plan["partial_ml"]), self._stream()), "mixed_attention_bf16")
                 return
         if not self._ops.distie_mixed_attention_fits(num_heads, head_dim):
@@ -1590,7 +1590,7 @@ class HipOps(Ops):
             raise KernelError("token_shift: the state is float32 [slots, C]")
         out = torch.empty((mu.shape[0], T, C), dtype=x.dtype, device=self.device)
         _check(self._ops.distie_token_shift(x.data_ptr(), _code(x), mu.data_ptr(), mu.shape[0], state.data_ptr(),
-                                            out.data_ptr(), meta.cu_q.data_ptr(), meta.token_request.data_ptr(),
+                                            out.data_ptr(), meta.cu_q.data_ptr(), None if meta.all_decode else meta.token_request.data_ptr(),
                                             meta.state_slots.data_ptr(), T, C, self._stream()), "token_shift")
         _mark_written(state)
         return out
