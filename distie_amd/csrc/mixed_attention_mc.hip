@@ -101,7 +101,7 @@ size_t prefill_lds(int H) {
          sizeof(bf16_t) * static_cast<size_t>(HP) * QT * PP;
 }
 
-template <int QT, int NT>
+template <int QT, int NT, bool ONE>                         // ONE: up to 16 heads, one tile of the mixing product
 __global__ void __launch_bounds__(64 * PF_WAVES)
 mixed_prefill_kernel(MixedArgs p) {
   constexpr int HS = scores_stride<QT>(), BW = QT + KT;
@@ -139,12 +139,25 @@ mixed_prefill_kernel(MixedArgs p) {
   for (int x = threadIdx.x; x < (HP - H) * HS; x += blockDim.x) S[H * HS + x] = 0.f;
   for (int x = threadIdx.x; x < HP * QT; x += blockDim.x) m_s[x] = -INFINITY, l_s[x] = 0.f;
   for (int x = threadIdx.x; x < HP * QT * PP / 2; x += blockDim.x) reinterpret_cast<uint32_t*>(P)[x] = 0u;
-  auto stage_bias = [&](int c, int buffer) {
+  // the biases of a step's distances: asked for by `load_bias` (the first two of a thread), in LDS after `stage_bias`
+  float bias_held[2] = {0.f, 0.f};
+  const auto bias_at = [&](int c, int x) {
+    return p.bias[static_cast<int64_t>(x / BW) * p.bias_len + min(max(pos0 - c + x % BW - (KT - 1), 0), p.bias_len - 1)];
+  };
+  const auto load_bias = [&](int c) {
     if (p.bias == nullptr) return;
-    for (int x = threadIdx.x; x < H * BW; x += blockDim.x) {
-      const int distance = min(max(pos0 - c + x % BW - (KT - 1), 0), p.bias_len - 1);
-      bias_s[buffer * H * BW + x] = p.bias[static_cast<int64_t>(x / BW) * p.bias_len + distance];
+#pragma unroll
+    for (int k = 0; k < 2; ++k) bias_held[k] = bias_at(c, min(static_cast<int>(threadIdx.x) + k * 64 * PF_WAVES, H * BW - 1));
+  };
+  const auto stage_bias = [&](int c, int buffer) {
+    if (p.bias == nullptr) return;
+    float* to = bias_s + buffer * H * BW;
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int x = threadIdx.x + k * 64 * PF_WAVES;
+      if (x < H * BW) to[x] = bias_held[k];
     }
+    for (int x = threadIdx.x + 2 * 64 * PF_WAVES; x < H * BW; x += 64 * PF_WAVES) to[x] = bias_at(c, x);
   };
 
   // this wave's columns: tile n holds 16 pairs of a query and a head of key/value head kh[n]
@@ -203,11 +216,26 @@ mixed_prefill_kernel(MixedArgs p) {
   };
   const auto next_step = [&](int c) { return c >= keep && c + KT - 1 < first ? first / KT * KT : c; };
   int c = next_step(0), buffer = 0;
-  stage_bias(c, buffer);
-  int page[2];
+  load_bias(c);
+  int page[2], page_next[2];
   pages_of(c, page);                           // (the first step holds key 0 or the window's first: somebody sees it)
   load_keys(c, page);
+  int following = next_step(c + KT);
+  page_next[0] = page[0], page_next[1] = page[1];
+  if (following <= last) pages_of(following, page_next);
+  stage_bias(c, buffer);
   __syncthreads();
+  // running maxima and sums of this wave's queries, lane (i, g) with heads 4 g .. 4 g + 3 of a tile, for all i alike: in
+  // registers where there is one tile, else in m_s and l_s
+  constexpr int QW = QT / PF_WAVES;
+  float top_of[QW][4], total_of[QW][4];
+#pragma unroll
+  for (int w = 0; w < QW; ++w)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) top_of[w][r] = -INFINITY, total_of[w][r] = 0.f;
+  float mix_rows[4];                           // ONE: this lane's part of the mixing matrix
+#pragma unroll
+  for (int s = 0; s < 4; ++s) mix_rows[s] = ONE ? M[i * (HP + 4) + g + 4 * s] : 0.f;
   while (c <= last) {
     bf16x8 values[AHEAD ? NT : 1][D / 16];
     const auto values_at = [&](int n) {
@@ -220,6 +248,11 @@ mixed_prefill_kernel(MixedArgs p) {
         for (int d = 0; d < D / 16; ++d)
           values[n][d] = *reinterpret_cast<const bf16x8*>(values_at(n) + static_cast<int64_t>(16 * d) * bs);
     }
+    // what the step after the next and the next one will need: pages and biases
+    const int later = next_step(following + KT);
+    int page_later[2] = {page_next[0], page_next[1]};
+    if (later <= last) pages_of(later, page_later);
+    if (following <= last) load_bias(following);
     // (1) raw scores of this wave's columns
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
@@ -248,44 +281,60 @@ mixed_prefill_kernel(MixedArgs p) {
     }
     __syncthreads();
     // (2) this wave's queries: mix the heads, mask, carry the softmax on
-    const int following = next_step(c + KT);
-    int page_next[2] = {page[0], page[1]};
     if (following <= last) {
-      pages_of(following, page_next);
       load_keys(following, page_next);
       stage_bias(following, 1 - buffer);
     }
-    for (int y = wave; y < nq; y += PF_WAVES) {
+#pragma unroll
+    for (int w = 0; w < QW; ++w) {
+      const int y = wave + w * PF_WAVES;
+      if (y >= nq) break;
       const int pos = pos0 + y;
       const int from = p.window > 0 ? max(0, pos - p.window + 1) : 0;
       const int key_a = c + i, key_b = key_a + 16;
       const bool see_a = key_a <= pos && (key_a >= from || key_a < keep);
       const bool see_b = key_b <= pos && (key_b >= from || key_b < keep);
-      for (int h0 = 0; h0 < HP; h0 += 16) {
+      const float* scores = S + g * HS + y * KP + i;
+      for (int h0 = 0; h0 < (ONE ? 16 : HP); h0 += 16) {
         floatx4 a = {0.f, 0.f, 0.f, 0.f}, b = {0.f, 0.f, 0.f, 0.f};
-        const float* rows_of_m = M + (h0 + i) * (HP + 4) + g;
-        const float* scores = S + g * HS + y * KP + i;
-        for (int s = 0; s < HP; s += 4) {
-          const float w = rows_of_m[s];
-          a = __builtin_amdgcn_mfma_f32_16x16x4f32(w, scores[s * HS], a, 0, 0, 0);
-          b = __builtin_amdgcn_mfma_f32_16x16x4f32(w, scores[s * HS + 16], b, 0, 0, 0);
+        if constexpr (ONE) {
+#pragma unroll
+          for (int s = 0; s < 4; ++s) {
+            a = __builtin_amdgcn_mfma_f32_16x16x4f32(mix_rows[s], scores[4 * s * HS], a, 0, 0, 0);
+            b = __builtin_amdgcn_mfma_f32_16x16x4f32(mix_rows[s], scores[4 * s * HS + 16], b, 0, 0, 0);
+          }
+        } else {
+          const float* rows_of_m = M + (h0 + i) * (HP + 4) + g;
+          for (int s = 0; s < HP; s += 4) {
+            const float weight = rows_of_m[s];
+            a = __builtin_amdgcn_mfma_f32_16x16x4f32(weight, scores[s * HS], a, 0, 0, 0);
+            b = __builtin_amdgcn_mfma_f32_16x16x4f32(weight, scores[s * HS + 16], b, 0, 0, 0);
+          }
         }
+        float alpha[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int at = (h0 + 4 * g + r) * QT + y;
           const float va = see_a ? a[r] : -INFINITY, vb = see_b ? b[r] : -INFINITY;
-          const float old = m_s[at];
+          const int at = (h0 + 4 * g + r) * QT + y;
+          const float old = ONE ? top_of[w][r] : m_s[at];
           const float top = fmaxf(old, row_max(fmaxf(va, vb)));
           const float pa = see_a ? exponential(va - top) : 0.f, pb = see_b ? exponential(vb - top) : 0.f;
-          const float sum = row_sum(pa + pb);
-          const float alpha = old == top ? 1.f : exponential(old - top);
-          P[at * PP + i] = static_cast<bf16_t>(pa);
-          P[at * PP + 16 + i] = static_cast<bf16_t>(pb);
-          if (i == 0) {
+          alpha[r] = old == top ? 1.f : exponential(old - top);
+          const float total = (ONE ? total_of[w][r] : l_s[at]) * alpha[r] + row_sum(pa + pb);
+          if constexpr (ONE) {
+            total_of[w][r] = total;
+            top_of[w][r] = top;
+          } else if (i == 0) {
             m_s[at] = top;
-            l_s[at] = l_s[at] * alpha + sum;
-            a_s[at] = alpha;
+            l_s[at] = total;
           }
+          bf16_t* to = P + at * PP + i;
+          to[0] = static_cast<bf16_t>(pa);
+          to[16] = static_cast<bf16_t>(pb);
+        }
+        if (i == 0) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) a_s[(h0 + 4 * g + r) * QT + y] = alpha[r];
         }
       }
     }
@@ -311,10 +360,22 @@ mixed_prefill_kernel(MixedArgs p) {
         }
       }
     }
-    c = following;
+    c = following, following = later;
     page[0] = page_next[0], page[1] = page_next[1];
+    page_next[0] = page_later[0], page_next[1] = page_later[1];
     buffer = 1 - buffer;
   }
+  if (ONE && i == 0) {
+#pragma unroll
+    for (int w = 0; w < QW; ++w)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int at = (4 * g + r) * QT + wave + w * PF_WAVES;
+        m_s[at] = top_of[w][r];
+        l_s[at] = total_of[w][r];
+      }
+  }
+  __syncthreads();
 #pragma unroll
   for (int n = 0; n < NT; ++n) {
     if (!column[n] || query[n] >= nq) continue;
@@ -564,26 +625,26 @@ bool prefill_fits(int H, int G, int QT) {
          (QT == 16 ? prefill_lds<16>(H) : prefill_lds<8>(H)) <= static_cast<size_t>(LDS_LIMIT);
 }
 
-template <int QT, int NT>
+template <int QT, int NT, bool ONE>
 int launch_prefill(const MixedArgs& p, int blocks, hipStream_t stream) {
   const size_t lds = prefill_lds<QT>(p.H);
-  if (lds > 48 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(mixed_prefill_kernel<QT, NT>),
+  if (lds > 48 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(mixed_prefill_kernel<QT, NT, ONE>),
                                              hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
     return DISTIE_BAD_ARGUMENT;
-  mixed_prefill_kernel<QT, NT><<<blocks, 64 * PF_WAVES, lds, stream>>>(p);
+  mixed_prefill_kernel<QT, NT, ONE><<<blocks, 64 * PF_WAVES, lds, stream>>>(p);
   return launch_status();
 }
 
-template <int QT>
+template <int QT, bool ONE>
 int launch_prefill_tiles(const MixedArgs& p, int blocks, hipStream_t stream) {
   const int each = (column_tiles(p.H, p.G, QT) + PF_WAVES - 1) / PF_WAVES;
-  if (each == 1) return launch_prefill<QT, 1>(p, blocks, stream);
+  if (each == 1) return launch_prefill<QT, 1, ONE>(p, blocks, stream);
   if constexpr (MAX_TILES >= 2)
-    if (each == 2) return launch_prefill<QT, 2>(p, blocks, stream);
+    if (each == 2) return launch_prefill<QT, 2, ONE>(p, blocks, stream);
   if constexpr (MAX_TILES >= 4)
-    if (each <= 4) return launch_prefill<QT, 4>(p, blocks, stream);
+    if (each <= 4) return launch_prefill<QT, 4, ONE>(p, blocks, stream);
   if constexpr (MAX_TILES >= 8)
-    if (each <= 8) return launch_prefill<QT, 8>(p, blocks, stream);
+    if (each <= 8) return launch_prefill<QT, 8, ONE>(p, blocks, stream);
   return DISTIE_BAD_ARGUMENT;
 }
 
@@ -640,7 +701,10 @@ extern "C" int distie_mixed_attention_bf16(const void* q, int64_t q_stride, cons
   if (prefill) {
     if ((queries != 8 && queries != 16) || !prefill_fits(H, G, queries)) return DISTIE_BAD_ARGUMENT;
     const int blocks = T / queries + B + 1;
-    return queries == 16 ? launch_prefill_tiles<16>(p, blocks, stream) : launch_prefill_tiles<8>(p, blocks, stream);
+    if (H <= 16)
+      return queries == 16 ? launch_prefill_tiles<16, true>(p, blocks, stream) : launch_prefill_tiles<8, true>(p, blocks, stream);
+    return queries == 16 ? launch_prefill_tiles<16, false>(p, blocks, stream)
+                         : launch_prefill_tiles<8, false>(p, blocks, stream);
   }
   return 0;
 }
