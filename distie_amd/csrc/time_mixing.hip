@@ -67,7 +67,7 @@ wkv_scan_kernel(const X* __restrict__ r_in, const X* __restrict__ k_in, const X*
   constexpr int SUB = THREADS / (PARTS * ROWS);            // threads that share a channel's decay (4 at least, a power of two)
   const int b = blockIdx.x, head = blockIdx.y;
   const int e = threadIdx.x % COLS, part = threadIdx.x / COLS;
-  const int first = cu_q[b], last = cu_q[b + 1];
+  const int first = cu_q != nullptr ? cu_q[b] : b, last = cu_q != nullptr ? cu_q[b + 1] : b + 1;     // null: a row a request
   if (first >= last) return;
   float* own = state + (static_cast<int64_t>(state_slots[b]) * H + head) * D * D;
   float s[ROWS];

@@ -346,7 +346,7 @@ class HipOps(Ops):
                                               _I, _I, _P]
         o.distie_gate_rmsnorm.argtypes = [_P, _P, _I, _F, _P, _I, _L, _P, _I, _I, _I, _I, _I, _P]
         o.distie_glu_mul.argtypes = [_P, _I, _I, _P, _I, _I, _I, _I, _P]
-        o.distie_group_chain.argtypes = [_P, _I, _I, _P, _F, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P]
+        o.distie_group_chain.argtypes = [_P, _I, _I, _P, _F, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P, _I, _P, _P, _P]
         o.distie_token_shift.argtypes = [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _P]
         o.distie_wkv_scan.argtypes = [_P, _P, _P, _P, _I, _L, _P, _I, _L, _I, _P, _P, _P, _P, _P, _F, _P, _I, _P, _P, _I, _I,
                                       _I, _P]
@@ -1683,15 +1683,15 @@ class HipOps(Ops):
         _check(self._ops.distie_wkv_scan(
             views[0][0], views[1][0], views[2][0], views[3][0], _code(r), ld, low_ptr, _code(low), low_ld, rank, up.data_ptr(),
             up_bias.data_ptr(), bonus.data_ptr(), state.data_ptr(), norm_weight.data_ptr(), float(eps), out.data_ptr(),
-            _code(out), meta.cu_q.data_ptr(), meta.state_slots.data_ptr(), meta.num_requests, num_heads, dim,
-            self._stream()), "wkv_scan")
+            _code(out), None if meta.all_decode else meta.cu_q.data_ptr(), meta.state_slots.data_ptr(), meta.num_requests,
+            num_heads, dim, self._stream()), "wkv_scan")
         _mark_written(state)
         return out
 
     def group_rmsnorm(self, x, weight, eps, groups, out_dtype):
         return self._group_chain(x, weight, eps, groups, None, None, None, out_dtype)
 
-    def _group_chain(self, delta, weight, eps, groups, residual, into, history, out_dtype):
+    def _group_chain(self, delta, weight, eps, groups, residual, into, history, out_dtype, shift=None):
         delta, slices = self._term(delta)
         T, C = delta.shape[-2:]
         self._own(weight, residual, into)
@@ -1709,12 +1709,24 @@ class HipOps(Ops):
                     rest.dim() != 3 or tuple(rest.shape[1:]) != (T, C) or not 0 <= index < rest.shape[0] or \
                     weights.dtype != torch.float32 or tuple(weights.shape) != (index + 2,):
                 raise KernelError("average over the depth: X_0 float32 [T, C], the others [layers, T, C], a weight for each")
-        out = torch.empty((T, C), dtype=out_dtype, device=self.device) if out_dtype is not None else None
+        mu = state = slots = None
+        if shift is not None:
+            mu, state, slots = shift
+            self._own(mu, state, slots)
+            if mu.dtype != torch.float32 or mu.dim() != 2 or mu.shape[1] != C or slots.shape[0] != T or \
+                    state.dtype != torch.float32 or tuple(state.shape[1:]) != (C,):
+                raise KernelError("norm in groups with a token shift: mu float32 [mixes, C], the state float32 [slots, C], a row "
+                                  "a request")
+        out = None
+        if out_dtype is not None:
+            out = torch.empty((T, C) if mu is None else (mu.shape[0], T, C), dtype=out_dtype, device=self.device)
         ptr = lambda t: t.data_ptr() if t is not None else None
         _check(self._ops.distie_group_chain(
             delta.data_ptr(), _code(delta), slices, weight.data_ptr(), float(eps), int(groups), ptr(residual), ptr(into),
-            ptr(first), ptr(rest), int(index), ptr(weights), ptr(out), _code(out) if out is not None else _F32, T, C,
-            self._stream()), "group_chain")
+            ptr(first), ptr(rest), int(index), ptr(weights), ptr(out), _code(out) if out is not None else _F32, T, C, ptr(mu),
+            mu.shape[0] if mu is not None else 0, ptr(state), ptr(slots), self._stream()), "group_chain")
+        if state is not None:
+            _mark_written(state)
         if into is not None:
             _mark_written(into)
         return out
@@ -1724,6 +1736,15 @@ class HipOps(Ops):
         read = self._group_chain(delta, weight, eps, groups, residual, into, history,
                                  None if out_dtype == torch.float32 else out_dtype)
         return into, into if out_dtype == torch.float32 else read
+
+    def add_group_normed_shift(self, residual, delta, weight, eps, groups, out_dtype, in_place, history, mu, state, meta):
+        if not meta.all_decode:
+            return super().add_group_normed_shift(residual, delta, weight, eps, groups, out_dtype, in_place, history, mu, state,
+                                                  meta)
+        # a row a request: the block that owns a row shifts it too
+        into = residual if in_place else torch.empty_like(residual)
+        return into, self._group_chain(delta, weight, eps, groups, residual, into, history, out_dtype,
+                                       (mu, state, meta.state_slots))
 
     def lru_gates(self, u, recur_weight, recur_bias, input_weight, input_bias, lam, rate):
         u = self.dense(u)

@@ -454,6 +454,12 @@ class Ops(abc.ABC):
         returned and left in the residual is sum_j weights[j] X_j, j = 0 .. index + 1 (weights float32 [index + 2])."""
         raise NotImplementedError(f"{type(self).__name__} has no norm in groups")
 
+    def add_group_normed_shift(self, residual: torch.Tensor, delta, weight: torch.Tensor, eps: float, groups: int, out_dtype,
+                               in_place: bool, history, mu: torch.Tensor, state: torch.Tensor, meta: BatchMeta):
+        """`add_group_normed`, then `token_shift` of what it hands out -> (x, the mixes); an implementation may fuse the two."""
+        x, read = self.add_group_normed(residual, delta, weight, eps, groups, out_dtype, in_place, history)
+        return x, self.token_shift(read, mu, state, meta)
+
     def lru_gates(self, u: torch.Tensor, recur_weight: torch.Tensor, recur_bias: torch.Tensor,
                   input_weight: torch.Tensor, input_bias: torch.Tensor, lam: torch.Tensor, rate: float):
         """The coefficients of a real-gated linear recurrent unit. u act [T, R] in B equal parts; the gates'

@@ -292,9 +292,9 @@ class DepthAveragedBranchNorm(Block):
         self.depth_weights = tensors["dwa"].float().contiguous()
 
     @staticmethod
-    def _close(ops, stream: ResidualStream, act_dtype):
+    def _close(ops, stream: ResidualStream, act_dtype, shift=None):
         """Add what is pending, through its norm and with the average where one is due; -> the residual in
-        `act_dtype` (None: nobody reads it)."""
+        `act_dtype` (None: nobody reads it), or with `shift` (mu, state, meta) its mixes with the tokens before."""
         delta, norm, average = stream.lanes["pending"]
         stream.lanes["pending"] = None
         history = None
@@ -303,8 +303,11 @@ class DepthAveragedBranchNorm(Block):
             history = (stream.lanes["first"], stream.lanes["rest"], index, weights)
         # X_0 is read again by every average: the first sum goes to a tensor of its own
         in_place = stream.hidden is not stream.lanes["first"]
-        stream.hidden, read = ops.add_group_normed(stream.hidden, delta, norm.weight, norm.eps, norm.groups, act_dtype,
-                                                   in_place, history)
+        common = (stream.hidden, delta, norm.weight, norm.eps, norm.groups, act_dtype, in_place, history)
+        if shift is None:
+            stream.hidden, read = ops.add_group_normed(*common)
+        else:
+            stream.hidden, read = ops.add_group_normed_shift(*common, *shift)
         return read
 
     @staticmethod
@@ -313,7 +316,7 @@ class DepthAveragedBranchNorm(Block):
             DepthAveragedBranchNorm._close(ops, stream, None)
         stream.lanes = None
 
-    def _read(self, ops, stream: ResidualStream, act_dtype):
+    def _read(self, ops, stream: ResidualStream, act_dtype, shift=None):
         if stream.pending is not None:
             raise ValueError("the depth-averaged arrangement starts from a residual with nothing pending on it")
         if stream.lanes is None:
@@ -322,13 +325,19 @@ class DepthAveragedBranchNorm(Block):
                             "rest": torch.empty((self.layers, *first.shape), dtype=first.dtype, device=first.device)}
             stream.settle = self._settle
         if stream.lanes["pending"] is None:
-            return ops.read_residual(stream.hidden, act_dtype)
-        return self._close(ops, stream, act_dtype)
+            read = ops.read_residual(stream.hidden, act_dtype)
+            return read if shift is None else ops.token_shift(read, *shift)
+        return self._close(ops, stream, act_dtype, shift)
 
     def forward(self, ops, stream: ResidualStream, ctx: StepContext, cache, writes_cache: bool) -> None:
         average = (self.index, self.depth_weights)
-        h = self._read(ops, stream, ctx.act_dtype)
-        y = self.mixer.forward(ops, h, ctx, cache["mixer"], writes_cache)
+        if hasattr(self.mixer, "shift"):
+            # the mixer reads its input mixed with the token before: made along with the read of the residual
+            mixes = self._read(ops, stream, ctx.act_dtype, (*self.mixer.shift(cache["mixer"]), ctx.meta))
+            y = self.mixer.forward_mixed(ops, mixes, ctx, cache["mixer"])
+        else:
+            h = self._read(ops, stream, ctx.act_dtype)
+            y = self.mixer.forward(ops, h, ctx, cache["mixer"], writes_cache)
         if self.feed_forward is None:
             stream.lanes["pending"] = (y, self.mixer_post_norm, average)
             return

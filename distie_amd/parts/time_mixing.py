@@ -63,8 +63,15 @@ class WKV(Mixer):
         ops.prepare_linear_each(self.weights)
         ops.prepare_linear(self.out_weight, role="attn_out")
 
+    def shift(self, cache):
+        """What the token shift in front of this mixer takes, for an arrangement that runs it along with its own read of
+        the residual (`forward_mixed` is handed the result): (mu, the state it keeps)."""
+        return self.mu, cache["last"]
+
     def forward(self, ops, x, ctx, cache, writes_cache: bool):
-        mixes = ops.token_shift(x, self.mu, cache["last"], ctx.meta)
+        return self.forward_mixed(ops, ops.token_shift(x, *self.shift(cache), ctx.meta), ctx, cache)
+
+    def forward_mixed(self, ops, mixes, ctx, cache):
         r, k, v, gates, low = ops.linear_each(mixes, self.weights, unrounded=(4,))
         mixed = ops.wkv_mix(r, k, v, gates, low, self.up_weight, self.up_bias, self.bonus, cache["state"], ctx.meta,
                             self.num_heads, self.head_dim, self.norm_weight, self.eps, ctx.act_dtype)
