@@ -80,6 +80,10 @@ wkv_scan_kernel(const X* __restrict__ r_in, const X* __restrict__ k_in, const X*
   const int channel = threadIdx.x / SUB, sub = threadIdx.x % SUB;      // the channel whose decay it helps to make
   const float* up_row = up + static_cast<int64_t>(head * D + min(channel, D - 1)) * rank;
   const float z0 = up_bias[head * D + min(channel, D - 1)];
+  constexpr int UP_HELD = 16;                              // of the channel's row, kept for all tokens
+  float up_held[UP_HELD];
+#pragma unroll
+  for (int i = 0; i < UP_HELD; ++i) up_held[i] = sub + i * SUB < rank ? up_row[sub + i * SUB] : 0.f;
   if (d_own < D) u_s[d_own] = bonus[head * D + d_own];
   const float weight = e < D ? norm_weight[head * D + e] : 0.f;
   float nr = 0.f, nk = 0.f, nv = 0.f, ng = 0.f, nl = 0.f;
@@ -99,7 +103,9 @@ wkv_scan_kernel(const X* __restrict__ r_in, const X* __restrict__ k_in, const X*
     if (t + 1 < last) fetch(t + 1);
     __syncthreads();
     float z = 0.f;
-    for (int i = sub; i < rank; i += SUB) z += up_row[i] * low_s[i];
+#pragma unroll
+    for (int i = 0; i < UP_HELD; ++i) z += up_held[i] * (sub + i * SUB < rank ? low_s[sub + i * SUB] : 0.f);
+    for (int i = sub + UP_HELD * SUB; i < rank; i += SUB) z += up_row[i] * low_s[i];
 #pragma unroll
     for (int o = SUB / 2; o > 0; o >>= 1) z += __shfl_xor(z, o, 64);
     if (sub == 0 && channel < D) w_s[channel] = expf(-expf(z + z0));
