@@ -432,7 +432,7 @@ class Ops(abc.ABC):
         """Time mixing with a decay per key channel and token and a bonus for the current token. r, k, v [T, H * dim]
         (tensors or column views, one dtype). With z = `wkv_decay_logits(low, up, up_bias)` and w = exp(-exp(z)), per head
 
-            o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T r_t,        S_t = diag(w_t) S_(t-1) + k_t v_t^T;
+            o[e] = sum_d r[d] (S[d][e] + bonus[d] k[d] v[e]),     then S[d][e] <- w[d] S[d][e] + k[d] v[e];
 
         every head's o is divided by sqrt(mean(o^2) + eps), and the heads side by side are multiplied by `norm_weight`
         [H * dim] and silu(gates) (gates [T, H * dim], of r's dtype) -> `out_dtype` [T, H * dim]. `bonus` float32

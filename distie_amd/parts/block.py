@@ -261,7 +261,7 @@ class DepthAveragedBranchNorm(Block):
     depth ("depth-weighted averaging"):
 
         x <- x + mixer_post_norm(mixer(x));   x <- x + feed_forward_post_norm(feed_forward(x));   X_(i+1) = x
-        x <- sum over j = 0 .. i+1 of dwa[j] X_j                    (X_0: the embedding output; tensor `dwa` [i + 2])
+        x <- dwa[0] X_0 + dwa[1] X_1 + ... + dwa[i+1] X_(i+1)     (X_0: the embedding output; tensor `dwa` [i + 2])
 
     for layer i (`index` of `layers`). A layer may have no feed-forward. Everything is float32 but what a sub-layer
     reads, which is the residual rounded to the activations' precision. X_0 .. X_L live for one step: X_0 is the

@@ -8,8 +8,8 @@ et al., "Talking-Heads Attention"), with a learned bias by distance and values t
     weight = exp(score) / (exp(sink_score) + sum over the visible keys of exp(score))
 
 Key j is visible to query i iff j <= i and (i - j < window or j < keep_first); without a window all j <= i are. The
-distance n falls into bucket n up to half of the table's B rows, then into logarithmically wider ones:
-min(B - 1, B/2 + floor(ln(n / (B/2)) / ln(bias_max / (B/2)) * (B - B/2))). The table is spread at load to one value
+distance n falls into bucket n up to half of the table's rows, `half` = rows / 2, then into logarithmically wider ones that
+reach the table's end at bias_max: half + floor((rows - half) * log_(bias_max / half)(n / half)), at most rows - 1. The table is spread at load to one value
 a distance, up to the distance from which on the last row holds (`distance_bias`). Scores, cap, bias, mixing and
 softmax are float32 in either precision.
 

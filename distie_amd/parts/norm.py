@@ -39,8 +39,8 @@ class RMSNorm(Norm):
 
 
 class GroupRMSNorm(Norm):
-    """RMS norm in groups: a row is cut into `groups` equal consecutive parts, each is divided by its own root mean
-    square, and the whole is multiplied by the weight; statistics in float32."""
+    """RMS norm in groups: `groups` runs of neighbouring columns, as many in each, have a root mean square of their own; the
+    weight is one for every column of the row. Statistics in float32."""
 
     fused_kind = "group_rms"
 

@@ -1,19 +1,18 @@
 """Time mixing with a data-dependent decay (the recurrence of RWKV-6: Peng et al., "Eagle and Finch: RWKV with
 Matrix-Valued States and Dynamic Recurrence").
 
-h is the mixer's input and h' the token before's (zeros in front of a request's first token). Each of r, k, v, g, w reads
-a mix of its own, m_s = h + (h' - h) * mu_s:
+x_t is what the mixer reads (x_(-1) = 0). The five projections read it blended with the row in front of it, every channel
+at a rate of its own: b_s = (1 - mu_s) x_t + mu_s x_(t-1) for s = r, k, v, g, w. With [H, D] vectors
 
-    r = W_r m_r,  k = W_k m_k,  v = W_v m_v  (heads x dim each),   gate = silu(W_g m_g)
-    w = exp(-exp(W_w2 tanh(W_w1 m_w) + w0))         a factor in (0, 1) for every head and key channel
+    r = R b_r,   k = K b_k,   v = V b_v,   gate = silu(G b_g),   keep = exp(-exp(w0 + W2 tanh(W1 b_w)))
 
-and per head, with a bonus u that only the current token gets,
+(keep in (0, 1), one for every head and key channel d) a head computes, a column e of its state M at a time,
 
-    o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,      S_t = diag(w_t) S_(t-1) + k_t v_t^T.
+    y[e] = sum_d r[d] (M[d][e] + u[d] k[d] v[e])        the current token counts with a bonus u
+    M[d][e] <- keep[d] M[d][e] + k[d] v[e]
 
-Every head's o is divided by its root mean square, the heads side by side are multiplied by a weight and the gate and
-projected by W_o. A request's state is S (float32 [heads, dim, dim], zero at the start) and its last h (float32). The
-decay, its exponentials, S and its sums, norm and gate are float32 in either precision.
+y / sqrt(mean(y^2) + eps), all heads side by side, times a weight and the gate, is projected back to the width. A request's state is M
+(float32 [heads, dim, dim], zero at the start) and its last x (float32). The decay, its exponentials, M and its sums, norm and gate are float32 in either precision.
 """
 
 from __future__ import annotations
