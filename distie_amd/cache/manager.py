@@ -1,14 +1,14 @@
 """The cache manager: pages of keys and values with a block table for each request, and
 slots for per-request state of fixed size.
 
-A mixer declares what it keeps (`PagedTensors`: tensors per page and a window, or `FixedState`:
+A mixer declares what it keeps (`PagedTensors`: tensors per page and a window or chunk, or `FixedState`:
 tensors per request); the manager allocates what is declared and knows nothing of what the tensors
 mean. Mixers are put into *groups* by their declaration: attention layers that keep every key form one
 group, those that keep a window of the same length another. Every group has pages of its own: its own
 id pool, for each declared tensor a slab `[mixers of the group, pages + 1, *shape of a page]` (the last
 page is a sink that is never handed out: padding rows of a captured decode step write there, as in
 worker/src/inference/torch_engine.py:439-446) and, for each request, its own block table. A table is addressed by position: entry i holds the page of positions
-i*block_size .. (i+1)*block_size - 1, or -1 once a window has passed that page and it
+i*block_size .. (i+1)*block_size - 1, or -1 once a window (or the end of a chunk) has passed that page and it
 was given back. Pages are handed out when a step needs them (`reserve`), given back when
 a request ends (`release`), is preempted (`reset`), or a window has passed them
 (`commit`), and are used again with their stale contents, which no kernel may read.
@@ -270,10 +270,7 @@ class CacheManager:
 
     def _first_needed_page(self, group: CacheGroup, num_cached: int) -> int:
         """Index of the first page a query at position >= num_cached can still read."""
-        window = group.requirement.window
-        if window is None:
-            return 0
-        return max(0, num_cached - window + 1) // self.block_size
+        return group.requirement.first_readable(num_cached) // self.block_size
 
     def _first_free_page(self, group: CacheGroup) -> int:
         """Index of the first page a window may ever pass: those before it hold tokens that stay for good."""
@@ -338,7 +335,7 @@ class CacheManager:
         entry = self._requests[request_id]
         entry.num_cached += num_new
         for g, group in enumerate(self.groups):
-            if group.requirement.window is None:
+            if group.requirement.window is None and group.requirement.chunk is None:
                 continue
             table = entry.tables[g]
             stop = min(self._first_needed_page(group, entry.num_cached), len(table))

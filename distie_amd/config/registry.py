@@ -13,6 +13,7 @@ from typing import Any, Dict, Mapping
 from .model_config import ConfigError, ModelSpec, Qwen2Config, read_config_json
 from .dufelix_config import DufelixConfig
 from .duparax_config import DuparaxConfig
+from .mepapel_config import MepapelConfig
 from .musutar_config import MusutarConfig
 from .netovik_config import NetovikConfig
 from .sekazen_config import SekazenConfig
@@ -77,3 +78,4 @@ register_architecture(DuparaxConfig.architecture, DuparaxConfig)
 register_architecture(SekazenConfig.architecture, SekazenConfig)
 register_architecture(DufelixConfig.architecture, DufelixConfig)
 register_architecture(NetovikConfig.architecture, NetovikConfig)
+register_architecture(MepapelConfig.architecture, MepapelConfig)

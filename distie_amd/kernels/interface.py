@@ -75,7 +75,7 @@ class ScoreExtras:
     With `distance_bias` b: + b[h, min(i - j, N - 1)] behind the cap, a learned bias by the distance to the key. With
     `head_mix` M: the heads' scores of every pair of query and key are then mixed, score_h <- sum_g M[h, g] score_g,
     in front of mask and softmax. With `keep_first` n: a windowed layer also sees the keys 0 .. n - 1 whatever their
-    distance."""
+    distance. With `chunk` c (and no window): query i sees the keys j <= i with floor(j / c) = floor(i / c)."""
 
     head_slopes: Optional[torch.Tensor] = None      # float32 [H] on the device
     score_cap: Optional[float] = None               # > 0
@@ -83,14 +83,17 @@ class ScoreExtras:
     distance_bias: Optional[torch.Tensor] = None    # float32 [H, N] on the device
     head_mix: Optional[torch.Tensor] = None         # float32 [H, H] on the device
     keep_first: int = 0
+    chunk: int = 0                                  # 0: none
 
     def __post_init__(self):
+        if self.chunk < 0 or (self.chunk and self.keep_first):
+            raise ValueError("a chunk is at least one position, and has no kept first keys")
         if self.score_cap is not None and not self.score_cap > 0:
             raise ValueError("score_cap must be positive")
 
     @property
     def plain(self) -> bool:
-        return not self.bends_scores and self.sinks is None and not self.mixes_heads
+        return not self.bends_scores and self.sinks is None and not self.mixes_heads and not self.chunk
 
     @property
     def bends_scores(self) -> bool:
@@ -102,6 +105,24 @@ class ScoreExtras:
         """A bias by distance, scores mixed between the heads or keys kept ahead of the window: what the kernels that
         work on all heads of a token together compute."""
         return self.distance_bias is not None or self.head_mix is not None or self.keep_first > 0
+
+
+@dataclass(frozen=True)
+class RouteRule:
+    """How a router with the scoring "sigmoid_share" chooses and weighs, and whether one more row of its weight gates a
+    shared expert (with any scoring).
+
+    s = sigmoid(z); choice score = s + correction. With `groups` > 1 the experts form that many groups of neighbours; a
+    group counts by the sum of its two largest choice scores (of its only one), and experts outside the `kept` strongest
+    groups are never chosen. The `top` experts with the largest choice scores are weighted by scale * s / (sum of the chosen
+    experts' s + 1e-20). `shared`: the router's weight has one row more than there are experts, and the sigmoid of its
+    logit is handed out behind the chosen experts' weights."""
+
+    correction: Optional[torch.Tensor] = None       # float32 [E] on the device
+    groups: int = 1
+    kept: int = 1
+    scale: float = 1.0
+    shared: bool = False
 
 
 class Ops(abc.ABC):
@@ -243,7 +264,8 @@ class Ops(abc.ABC):
                            k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor],
                            inv_freq: Optional[torch.Tensor], magnitude: float, num_heads: int, num_kv_heads: int,
                            dim: int, value_dim: int, padded_dim: int, has_kv: bool, write: bool,
-                           q_temp=None, qk_norm=None, keys_are_values: bool = False) -> torch.Tensor:
+                           q_temp=None, qk_norm=None, keys_are_values: bool = False,
+                           neighbours: bool = False) -> torch.Tensor:
         """Behind attention's stacked projection. The first columns of `product` (act [T, W]) are q (num_heads x
         dim) and, if `has_kv`, k (num_kv_heads x dim) and v (num_kv_heads x value_dim); further columns are left
         alone. Each of these channels goes through `causal_conv` (no residual; `conv_weight` [channels, taps],
@@ -258,7 +280,7 @@ class Ops(abc.ABC):
         and in front of the rotation every q and k head becomes x / sqrt(mean(x^2) + eps) * weight over its `dim`
         values, in float32 (None: none).
         `keys_are_values`: there are no columns of v; the values are the k columns as they are in the product, in front
-        of norm and rotation (value_dim is dim; no convolution)."""
+        of norm and rotation (value_dim is dim; no convolution). `neighbours`: the pairs of the rotation are (2i, 2i + 1)."""
         raise NotImplementedError(f"{type(self).__name__} has no convolution over time")
 
     def sigmoid_gate(self, x: torch.Tensor, num_heads: int, head_stride: int, width: int,
@@ -269,10 +291,13 @@ class Ops(abc.ABC):
         raise NotImplementedError(f"{type(self).__name__} has no gates")
 
     def decay_scan(self, product: torch.Tensor, state: torch.Tensor, decay: torch.Tensor, meta: BatchMeta,
-                   num_heads: int, dim: int, value_dim: int) -> torch.Tensor:
+                   num_heads: int, dim: int, value_dim: int, act: Optional[str] = "silu", k_scale: float = 1.0,
+                   inv_freq: Optional[torch.Tensor] = None, neighbours: bool = False) -> torch.Tensor:
         """Linear attention with a decay per head, as a recurrence over each request's rows: with q = silu(.),
         k = silu(.) (num_heads x dim each) and v = silu(.) (num_heads x value_dim) taken from the first columns of
-        `product` (act [T, W]), S <- decay[h] * S + k v^T and o = S^T q. `state` float32 [slots + 1, num_heads,
+        `product` (act [T, W]), S <- decay[h] * S + k v^T and o = S^T q. `act` None: the columns as they are instead of
+        their silu; then the first 2 * len(inv_freq) dimensions of every q and k head may be turned by the token's position
+        (`neighbours`: pairs (2i, 2i + 1), else (i, i + len(inv_freq))) and k is multiplied by `k_scale`. `state` float32 [slots + 1, num_heads,
         dim, value_dim] (rows by `meta.state_slots`) is read and left as the step's last row leaves it.
         -> float32 [T, num_heads * value_dim]. Everything behind the activations in float32."""
         raise NotImplementedError(f"{type(self).__name__} has no decayed state")
@@ -301,6 +326,20 @@ class Ops(abc.ABC):
         `state` float32 [slots + 1, H, N, P] (rows by `meta.state_slots`) is read and left as the step's last row
         leaves it. -> float32 [T, H * P]. Softplus, exponentials, the state, its products and sums in float32."""
         raise NotImplementedError(f"{type(self).__name__} has no state-space recurrence")
+
+    def delta_scan(self, qkv: torch.Tensor, beta: torch.Tensor, decay: torch.Tensor, a_log: torch.Tensor,
+                   dt_bias: torch.Tensor, state: torch.Tensor, meta: BatchMeta, num_heads: int, num_kv_heads: int, dim: int,
+                   value_dim: int, q_scale: float, unit_eps: float) -> torch.Tensor:
+        """The gated delta rule, over each request's rows in order. `qkv` act [T, 2 * G * dim + H * value_dim] (or a view of
+        columns): q, k (G heads of dim each; head h of H uses h // (H / G)), v. `beta` and `decay` act [T, H] (or views):
+        the logits b and a of the write strength and of the decay. q and k become x / sqrt(sum(x^2) + unit_eps) by head, q
+        times `q_scale` besides; with w = sigmoid(b) and f = exp(-exp(a_log) * softplus(a + dt_bias)), per head
+
+            S <- f S,    u = w * (v - S^T k),    S <- S + k u^T,    o = S^T q.
+
+        `a_log`, `dt_bias` float32 [H]; `state` float32 [slots + 1, H, dim, value_dim] (rows by `meta.state_slots`) is read
+        and left as the step's last row leaves it. -> float32 [T, H * value_dim]; everything in float32."""
+        raise NotImplementedError(f"{type(self).__name__} has no delta rule")
 
     def ssm_scan_captures(self, state_size: int) -> bool:
         """Whether `ssm_scan` at this state size can run inside a captured step (its launches then must not hang on the
@@ -476,30 +515,36 @@ class Ops(abc.ABC):
         one of `activation`'s names or None for mul itself; `mul` None: h)."""
         raise NotImplementedError(f"{type(self).__name__} has no gated linear recurrent unit")
 
-    def route_topk(self, x, weight: torch.Tensor, bias: Optional[torch.Tensor], top: int, scoring: str = "softmax"):
+    def route_topk(self, x, weight: torch.Tensor, bias: Optional[torch.Tensor], top: int, scoring: str = "softmax",
+                   rule: Optional[RouteRule] = None):
         """The router of a mixture of experts: z = weight x + bias in float32 (x act [T, C], weight [E, C], bias
         float32 [E] or None); for every row the `top` largest z (the lower index among equals) and, as weights,
         softmax over those alone (`scoring` "softmax"), over all experts and not renormalised ("softmax_all"), or
-        sigmoid(z) of each, not renormalised ("sigmoid")
-        -> (experts int32 [T, top], their weights float32 [T, top]), largest first."""
+        sigmoid(z) of each, not renormalised ("sigmoid"), or as `rule` says ("sigmoid_share")
+        -> (experts int32 [T, top], their weights float32 [T, top]), largest first. With `rule.shared` weight and bias have
+        one row more, and the weights are [T, top + 1], the last the sigmoid of that row's logit."""
         raise NotImplementedError(f"{type(self).__name__} has no router")
 
     def route_glu(self, gate_up, experts: torch.Tensor, gates: torch.Tensor, num_experts: int, width: int,
-                  limit: Optional[float], slope: float, up_shift: float, on_input: bool) -> torch.Tensor:
+                  limit: Optional[float], slope: float, up_shift: float, on_input: bool,
+                  shared_width: int = 0) -> torch.Tensor:
         """The hidden values of routed gated experts from the stacked product. `gate_up` act [T, 2 * num_experts *
         width] (or what `linear` returned): every expert's gate columns, expert after expert, then every expert's up
         columns. For expert e of a row with weight w (zero result if the row did not choose e):
         g, u = gate and up columns, times w if `on_input`; with `limit`: g <- min(g, limit), u <- clamp(u, -limit,
         limit); hidden = g * sigmoid(slope * g) * (u + up_shift), times w unless `on_input`
-        -> act [T, num_experts * width], in float32 behind the product's rounding."""
+        -> act [T, num_experts * width], in float32 behind the product's rounding. `shared_width` > 0: both halves of
+        `gate_up` end with that many columns of an expert that every row uses, with the weight in gates[:, top] (gates
+        [T, top + 1]); its hidden values stand behind the others'."""
         raise NotImplementedError(f"{type(self).__name__} has no routed feed-forward")
 
     def route_experts_glu(self, x, router_weight: torch.Tensor, router_bias: Optional[torch.Tensor], top: int,
                           scoring: str, gate_up, num_experts: int, width: int, limit: Optional[float], slope: float,
-                          up_shift: float, on_input: bool) -> torch.Tensor:
+                          up_shift: float, on_input: bool, rule: Optional[RouteRule] = None,
+                          shared_width: int = 0) -> torch.Tensor:
         """`route_topk` of x, then `route_glu` of `gate_up` with what it chose; an implementation may fuse the two."""
-        experts, gates = self.route_topk(x, router_weight, router_bias, top, scoring)
-        return self.route_glu(gate_up, experts, gates, num_experts, width, limit, slope, up_shift, on_input)
+        experts, gates = self.route_topk(x, router_weight, router_bias, top, scoring, rule)
+        return self.route_glu(gate_up, experts, gates, num_experts, width, limit, slope, up_shift, on_input, shared_width)
 
     def softcap(self, x: torch.Tensor, cap: float) -> torch.Tensor:
         """float32 [R, N] (in place) -> cap * tanh(x / cap)."""
@@ -532,6 +577,15 @@ class Ops(abc.ABC):
         if kind == "silu":
             return self.linear_silu_mul(x, gate_up_weight)
         return self.glu_mul(self.linear(x, gate_up_weight), kind)
+
+    def clamped_glu(self, gate_up, limit: float, slope: float, up_shift: float) -> torch.Tensor:
+        """[T, 2I] (or what `linear` returned) -> [T, I]: with g = min(first half, limit) and u = clamp(second half, -limit,
+        limit), g * sigmoid(slope * g) * (u + up_shift), in float32 behind the product's rounding."""
+        raise NotImplementedError(f"{type(self).__name__} has no clamped gated activation")
+
+    def linear_clamped_glu(self, x, gate_up_weight: torch.Tensor, limit: float, slope: float, up_shift: float) -> torch.Tensor:
+        """clamped_glu(linear(x, gate_up_weight), ...); an implementation may fuse the two."""
+        return self.clamped_glu(self.linear(x, gate_up_weight), limit, slope, up_shift)
 
     @abc.abstractmethod
     def silu_mul(self, gate_up: torch.Tensor) -> torch.Tensor:

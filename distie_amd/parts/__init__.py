@@ -1,4 +1,4 @@
-from . import (attention, block, conv_attention, embedding, feed_forward, latent_attention, linear_attention, mixed_attention,  # noqa: F401  (registration)
+from . import (attention, block, conv_attention, delta_rule, embedding, feed_forward, latent_attention, linear_attention, mixed_attention,  # noqa: F401  (registration)
                norm, parallel, position, recurrent, state_space, time_mixing)
 from .attention import PagedKV
 from .base import (PAGE, Block, Borrowed, CacheNeeds, Embedding, FeedForward, FixedState, Head, Mixer, Norm, PagedTensors, ParamSpec, Part,

@@ -22,12 +22,13 @@ from ..kernels.interface import ScoreExtras
 from .base import PAGE, Mixer, PagedTensors, ParamSpec, TensorDecl, build_part, register_part
 
 
-def PagedKV(num_kv_heads: int, head_dim: int, window: Optional[int] = None, keep_first: int = 0) -> PagedTensors:
+def PagedKV(num_kv_heads: int, head_dim: int, window: Optional[int] = None, keep_first: int = 0,
+            chunk: Optional[int] = None) -> PagedTensors:
     """What attention keeps for every token, in the layout its kernels read: keys as
     `[kv_heads, page, head_dim]` per page, values transposed inside a page, `[kv_heads, head_dim, page]`,
     so that the key index is contiguous for the matrix cores."""
     return PagedTensors((TensorDecl("k", (num_kv_heads, PAGE, head_dim)),
-                         TensorDecl("v", (num_kv_heads, head_dim, PAGE))), window, keep_first)
+                         TensorDecl("v", (num_kv_heads, head_dim, PAGE))), window, keep_first, chunk)
 
 
 def context_classes(limit: int, first: int = 1024) -> Tuple[int, ...]:

@@ -59,13 +59,26 @@ class TensorDecl:
 
 @dataclass(frozen=True)
 class PagedTensors:
-    """A mixer that keeps something for every token (or for the last `window` tokens and the first `keep_first`), in pages:
+    """A mixer that keeps something for every token (or for the last `window` tokens and the first `keep_first`, or for the
+    tokens of the current `chunk`), in pages:
     for each declared tensor the cache holds `[pages + 1, *shape]` per layer, addressed through the
     request's block table of the layer's group. Mixers with equal declarations share a group of pages."""
 
     tensors: Tuple[TensorDecl, ...]
     window: Optional[int] = None
     keep_first: int = 0              # with a window: so many of a request's first tokens stay readable for good
+    chunk: Optional[int] = None      # instead of a window: only the tokens of the same run of so many positions (counted
+    #                                  from position 0) stay readable; a run is given back when the next one begins
+
+    def __post_init__(self):
+        if self.chunk is not None and (self.window is not None or self.keep_first or self.chunk < 1):
+            raise ValueError("a chunk is at least one position, and takes the place of a window")
+
+    def first_readable(self, position: int) -> int:
+        """The first position (kept ones aside) that a query at `position` or behind it may still read."""
+        if self.chunk is not None:
+            return position // self.chunk * self.chunk
+        return 0 if self.window is None else max(0, position - self.window + 1)
 
     def page_shape(self, decl: TensorDecl, block_size: int) -> Tuple[int, ...]:
         return tuple(block_size if s == PAGE else s for s in decl.shape)

@@ -9,7 +9,12 @@
 * an output gate: the concatenated heads times sigmoid(W_g h), h being the mixer's input, before the output projection
   (`output_gate` True: a gate for every value column, `g` [heads * value_dim, C]; "head": one number for each head,
   `g` [heads, C]);
-* biases on q, k and v (`bias`: tensors `<q|k|v>.b`, added in the projection);
+* biases on q, k and v (`bias`: tensors `<q|k|v>.b`, added in the projection) and on the output projection (`out_bias`:
+  `o.b`);
+* rotation of neighbouring dimensions (`rotate` "neighbours": dimension 2i is paired with 2i + 1) instead of halves
+  ("halves": i with i + dims / 2);
+* chunks (`chunk`): position i sees only the keys j <= i of its own run of `chunk` positions, counted from position 0 of
+  the sequence, instead of a window;
 * a query temperature by position (`q_temp` = {coef, every}): q at position p is multiplied by
   1 + coef * ln(floor((p + 1) / every) + 1), in float32, so that later queries weigh their keys more sharply;
 * a norm on every head of q and k (`qk_norm` = {eps, offset}): RMS norm over the head's `head_dim` values with the
@@ -60,6 +65,11 @@ class ConvGatedAttention(Mixer):
         self.value_dim = int(p.get("value_dim") or self.head_dim)
         self.conv_taps = int(p.get("conv_taps") or 0)
         self.window = p.get("window")
+        self.chunk = p.get("chunk")
+        if self.chunk is not None and (self.window is not None or int(self.chunk) < 1 or p.get("kv_from") is not None):
+            raise ValueError("a chunk is at least one position, takes the place of a window, and goes with keys of the layer's own")
+        self.neighbours = {"halves": False, "neighbours": True}[str(p.get("rotate", "halves"))]
+        self.out_bias = bool(p.get("out_bias", False))
         self.keep = p.get("keep", self.window)          # how far back the cache must reach (None: everything)
         self.scale = float(p.get("scale", self.head_dim ** -0.5))
         gate = p.get("output_gate", True)
@@ -84,14 +94,14 @@ class ConvGatedAttention(Mixer):
         self.conv_channels = q + (k + v if self.has_kv else 0)
         self.out_width = self.num_heads * self.value_dim
         self.gate_width = self.num_heads if self.gate_per_head else self.out_width
-        self.in_weight = self.in_bias = self.conv_weight = self.out_weight = None
+        self.in_weight = self.in_bias = self.conv_weight = self.out_weight = self.out_bias_t = None
 
     def _projections(self):
         q, k, v = self.num_heads * self.head_dim, self.num_kv_heads * self.head_dim, self.num_kv_heads * self.value_dim
         return [("q", q)] + ([("k", k), ("v", v)] if self.has_kv else [])
 
     def cache_requirement(self):
-        paged = PagedKV(self.num_kv_heads, self.padded_dim, self.keep) if self.has_kv else Borrowed(int(self.kv_from))
+        paged = PagedKV(self.num_kv_heads, self.padded_dim, self.keep, chunk=self.chunk) if self.has_kv else Borrowed(int(self.kv_from))
         state = None
         if self.conv_taps > 1:
             state = FixedState((TensorDecl("conv", (self.conv_taps - 1, self.conv_channels), torch.float32),))
@@ -117,6 +127,8 @@ class ConvGatedAttention(Mixer):
         if self.output_gate:
             specs["g"] = ParamSpec((self.gate_width, self.hidden_size))
         specs["o"] = ParamSpec((self.hidden_size, self.out_width))
+        if self.out_bias:
+            specs["o.b"] = ParamSpec((self.hidden_size,))
         return specs
 
     def load(self, tensors) -> None:
@@ -131,12 +143,15 @@ class ConvGatedAttention(Mixer):
         if self.conv_taps:
             self.conv_weight = torch.cat([tensors[name + ".conv"] for name, _ in self._projections()], dim=0).contiguous()
         self.out_weight = tensors["o"].contiguous()
+        if self.out_bias:
+            self.out_bias_t = tensors["o.b"].float().contiguous()
         if self.qk_norm is not None:
             self.q_norm_weight = (tensors["q.norm"].float() + self.qk_norm[1]).contiguous()
             if self.has_kv:
                 self.k_norm_weight = (tensors["k.norm"].float() + self.qk_norm[1]).contiguous()
-        if self.sink:
-            self.extras = ScoreExtras(sinks=tensors["sink"].float().contiguous())
+        if self.sink or self.chunk is not None:
+            self.extras = ScoreExtras(sinks=tensors["sink"].float().contiguous() if self.sink else None,
+                                      chunk=int(self.chunk or 0))
         self.position.to_device(self.out_weight.device)
 
     def prepare(self, ops) -> None:
@@ -157,7 +172,8 @@ class ConvGatedAttention(Mixer):
                                    self.position.rotary(), self.position.rotary_magnitude(), self.num_heads,
                                    self.num_kv_heads, self.head_dim, self.value_dim, self.padded_dim, self.has_kv,
                                    writes_cache and self.has_kv, self.q_temp,
-                                   None if self.qk_norm is None else (self.q_norm_weight, self.k_norm_weight, self.qk_norm[0]))
+                                   None if self.qk_norm is None else (self.q_norm_weight, self.k_norm_weight, self.qk_norm[0]),
+                                   neighbours=self.neighbours)
         mixed = ops.paged_attention(q, ctx.meta, cache.group, k_cache, v_cache, self.num_heads, self.num_kv_heads,
                                     self.padded_dim, self.scale, self.window, self.extras)
         if self.output_gate:
@@ -168,7 +184,7 @@ class ConvGatedAttention(Mixer):
                 mixed = ops.sigmoid_gate(mixed, self.num_heads, self.padded_dim, self.value_dim, gates)
         elif self.padded_dim != self.value_dim:
             mixed = ops.sigmoid_gate(mixed, self.num_heads, self.padded_dim, self.value_dim, None)
-        return ops.linear(mixed, self.out_weight)
+        return ops.linear(mixed, self.out_weight, self.out_bias_t)
 
 
 register_part("mixer", "conv_gated_attention", ConvGatedAttention)

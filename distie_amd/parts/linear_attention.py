@@ -15,7 +15,7 @@ from __future__ import annotations
 import torch
 
 from ..config.model_config import PartSpec
-from .base import FixedState, Mixer, ParamSpec, register_part
+from .base import FixedState, Mixer, ParamSpec, build_part, register_part
 
 
 class DecayLinearAttention(Mixer):
@@ -59,6 +59,71 @@ class DecayLinearAttention(Mixer):
         first = self.num_heads * (2 * self.head_dim + self.value_dim)
         gates = product[:, first:first + self.num_heads * self.value_dim]
         normed = ops.rmsnorm_gate(mixed, self.norm_weight, self.eps, gates, ctx.act_dtype)
+        return ops.linear(normed, self.out_weight)
+
+
+class Retention(Mixer):
+    """Linear attention with a fixed decay per head and rotated queries and keys ("retention": Sun et al., "Retentive
+    Network: A Successor to Transformer for Large Language Models"), as a state that is carried from token to token.
+
+    q = W_q h, k = W_k h (heads x dim), v = W_v h (heads x value_dim), no activation; the first dimensions of every q and k
+    head are turned by the token's position (`position`: the frequencies; `rotate` "halves": dimension i is paired with i +
+    dims / 2, "neighbours": 2i with 2i + 1), and k is multiplied by `k_scale` (dim^(-1/2)) behind that. Per head
+
+        S_t = decay_h * S_(t-1) + k_t v_t^T,        o_t = S_t^T q_t.
+
+    Every head's o is divided by its root mean square (no weight), the heads side by side are multiplied by silu(W_g h) and
+    projected by W_o. The state starts at zero and is float32 [heads, dim, value_dim] for each request; rotation, scale,
+    state, sums and norm are float32 in either precision. The four projections are one matrix product: their weights
+    are stacked at load."""
+
+    def __init__(self, spec: PartSpec) -> None:
+        super().__init__(spec)
+        p = spec.params
+        self.hidden_size = int(p["hidden_size"])
+        self.num_heads = int(p["num_heads"])
+        self.head_dim = int(p["head_dim"])
+        self.value_dim = int(p.get("value_dim") or self.head_dim)
+        self.eps = float(p["eps"])
+        self.k_scale = float(p.get("k_scale", self.head_dim ** -0.5))
+        self.neighbours = {"halves": False, "neighbours": True}[str(p.get("rotate", "halves"))]
+        self.position = build_part("position", p.get("position") or PartSpec("none"))
+        self.decay_values = tuple(float(d) for d in p["decay"])
+        if len(self.decay_values) != self.num_heads:
+            raise ValueError(f"{len(self.decay_values)} decays for {self.num_heads} heads")
+        self.in_weight = self.out_weight = self.unit_weight = self.decay = None
+
+    def cache_requirement(self):
+        return FixedState.of((self.num_heads, self.head_dim, self.value_dim))
+
+    def param_specs(self):
+        qk, v = self.num_heads * self.head_dim, self.num_heads * self.value_dim
+        return {"q": ParamSpec((qk, self.hidden_size)), "k": ParamSpec((qk, self.hidden_size)),
+                "v": ParamSpec((v, self.hidden_size)), "g": ParamSpec((v, self.hidden_size)),
+                "o": ParamSpec((self.hidden_size, v))}
+
+    def load(self, tensors) -> None:
+        stacked = [tensors[name] for name in "qkvg"]
+        dtype = torch.float32 if any(t.dtype == torch.float32 for t in stacked) else stacked[0].dtype
+        self.in_weight = torch.cat([t.to(dtype) for t in stacked], dim=0).contiguous()
+        self.out_weight = tensors["o"].contiguous()
+        device = self.out_weight.device
+        self.unit_weight = torch.ones(self.value_dim, dtype=torch.float32, device=device)
+        self.decay = torch.tensor(self.decay_values, dtype=torch.float64).to(torch.float32).to(device)
+        self.position.to_device(device)
+
+    def prepare(self, ops) -> None:
+        ops.prepare_linear(self.in_weight, role="qkv")
+        ops.prepare_linear(self.out_weight, role="attn_out")
+
+    def forward(self, ops, x, ctx, cache, writes_cache: bool):
+        product = ops.dense(ops.linear(x, self.in_weight))
+        mixed = ops.decay_scan(product, cache["state"], self.decay, ctx.meta, self.num_heads, self.head_dim,
+                               self.value_dim, act=None, k_scale=self.k_scale, inv_freq=self.position.rotary(),
+                               neighbours=self.neighbours)
+        first = self.num_heads * (2 * self.head_dim + self.value_dim)
+        gates = product[:, first:first + self.num_heads * self.value_dim]
+        normed = ops.rmsnorm_gate(mixed, self.unit_weight, self.eps, gates, ctx.act_dtype, group=self.value_dim, gate="silu")
         return ops.linear(normed, self.out_weight)
 
 
@@ -134,3 +199,4 @@ class GatedLinearAttention(Mixer):
 
 register_part("mixer", "decay_linear_attention", DecayLinearAttention)
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
+register_part("mixer", "retention", Retention)

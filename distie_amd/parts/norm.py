@@ -11,7 +11,9 @@ from .base import Norm, ParamSpec, register_part
 
 class RMSNorm(Norm):
     """`offset`: what is added to the stored weight (1 for designs whose files hold the weight minus one:
-    y = x / rms(x) * (1 + w)); the sum is made once at load, in float32, and is the weight from then on."""
+    y = x / rms(x) * (1 + w)). `gain`: what the weight is multiplied by (a factor on a sub-layer's normed result, for
+    designs that add a part of it only). Both are applied once at load, in float32, and the result is the weight from
+    then on."""
 
     fused_kind = "rms"          # what `Ops.hyper_step` calls this norm when it computes it while reading the streams
 
@@ -21,6 +23,7 @@ class RMSNorm(Norm):
         self.eps = float(spec.params["eps"])
         self.weight_name = spec.params.get("weight_name", "weight")      # the tensor's name behind the prefix
         self.offset = float(spec.params.get("offset") or 0.0)
+        self.gain = float(spec.params.get("gain", 1.0))
         self.weight = None
 
     def param_specs(self):
@@ -28,8 +31,8 @@ class RMSNorm(Norm):
 
     def load(self, tensors) -> None:
         self.weight = tensors[self.weight_name].contiguous()
-        if self.offset:
-            self.weight = (self.weight.float() + self.offset).contiguous()
+        if self.offset or self.gain != 1.0:
+            self.weight = ((self.weight.float() + self.offset) * self.gain).contiguous()
 
     def apply(self, ops, x, out_dtype):
         return ops.rmsnorm(x, self.weight, self.eps, out_dtype)

@@ -78,6 +78,8 @@ class TorchOps(Ops):
             for t in range(cu[b], cu[b + 1]):
                 pos = int(meta.positions[t])
                 first = 0 if window is None else max(0, pos - window + 1)
+                if extras is not None and extras.chunk:
+                    first = pos // extras.chunk * extras.chunk
                 keys = torch.arange(first, pos + 1, device=qkv.device)
                 if extras is not None and extras.keep_first:
                     keys = torch.cat([torch.arange(min(extras.keep_first, first), device=qkv.device), keys])
@@ -154,7 +156,7 @@ class TorchOps(Ops):
 
     def conv_rope_kv_write(self, product, conv_weight, state, meta, group, k_cache, v_cache, inv_freq, magnitude,
                            num_heads, num_kv_heads, dim, value_dim, padded_dim, has_kv, write, q_temp=None, qk_norm=None,
-                           keys_are_values=False):
+                           keys_are_values=False, neighbours=False):
         T = product.shape[0]
         if keys_are_values:
             product = torch.cat([product, product[:, num_heads * dim:(num_heads + num_kv_heads) * dim]], 1)
@@ -166,11 +168,8 @@ class TorchOps(Ops):
         def turned(x):
             if inv_freq is None:
                 return x
-            pairs = inv_freq.shape[0]
-            ang = meta.positions.float()[:, None] * inv_freq.float()[None, :]
-            cos, sin = (ang.cos() * magnitude)[:, None, :], (ang.sin() * magnitude)[:, None, :]
-            a, b = x[..., :pairs], x[..., pairs:2 * pairs]
-            return torch.cat([a * cos - b * sin, b * cos + a * sin, x[..., 2 * pairs:]], -1)
+            turn = 2 * inv_freq.shape[0]
+            return torch.cat([self._turn(x[..., :turn], meta.positions, inv_freq, magnitude, neighbours), x[..., turn:]], -1)
 
         def normed(x, weight):
             if qk_norm is None:
@@ -201,12 +200,18 @@ class TorchOps(Ops):
             kept = kept * (g[:, :, None] if per_head else g.view(T, num_heads, width))
         return kept.reshape(T, num_heads * width).to(x.dtype)
 
-    def decay_scan(self, product, state, decay, meta, num_heads, dim, value_dim):
+    def decay_scan(self, product, state, decay, meta, num_heads, dim, value_dim, act="silu", k_scale=1.0, inv_freq=None,
+                   neighbours=False):
         T = product.shape[0]
-        act = lambda z: z * torch.sigmoid(z)
+        plain = act is None
+        act = lambda z: z if plain else z * torch.sigmoid(z)
         q = act(product[:, :num_heads * dim].float()).view(T, num_heads, dim)
         k = act(product[:, num_heads * dim:2 * num_heads * dim].float()).view(T, num_heads, dim)
         v = act(product[:, 2 * num_heads * dim:num_heads * (2 * dim + value_dim)].float()).view(T, num_heads, value_dim)
+        if inv_freq is not None:
+            n = 2 * inv_freq.shape[0]
+            q, k = (torch.cat([self._turn(z[..., :n], meta.positions, inv_freq, 1.0, neighbours), z[..., n:]], -1) for z in (q, k))
+        k = k * k_scale
         out = torch.zeros(T, num_heads, value_dim, dtype=torch.float32, device=product.device)
         cu = meta.cu_q.tolist()
         slots = meta.state_slots.tolist()
@@ -253,6 +258,27 @@ class TorchOps(Ops):
                 out[t] = torch.einsum("hnp,hn->hp", s, C[t]) + skip.float()[:, None] * x[t]
             state[slots[b]] = s
         return out.view(T, H * P)
+
+    def delta_scan(self, qkv, beta, decay, a_log, dt_bias, state, meta, num_heads, num_kv_heads, dim, value_dim, q_scale,
+                   unit_eps):
+        T, H, G, D, E = qkv.shape[0], num_heads, num_kv_heads, dim, value_dim
+        unit = lambda z: z / torch.sqrt((z * z).sum(-1, keepdim=True) + unit_eps)
+        own = lambda z: unit(z.float().reshape(T, G, D)).repeat_interleave(H // G, dim=1)
+        q, k = own(qkv[:, :G * D]) * q_scale, own(qkv[:, G * D:2 * G * D])
+        v = qkv[:, 2 * G * D:2 * G * D + H * E].float().reshape(T, H, E)
+        strength = torch.sigmoid(beta.float())
+        f = torch.exp(-torch.exp(a_log) * torch.nn.functional.softplus(decay.float() + dt_bias, threshold=80.0))
+        out = torch.zeros(T, H, E, dtype=torch.float32, device=qkv.device)
+        cu, slots = meta.cu_q.tolist(), meta.state_slots.tolist()
+        for b in range(meta.num_requests):
+            s = state[slots[b]]
+            for t in range(cu[b], cu[b + 1]):
+                s = f[t][:, None, None] * s
+                u = strength[t][:, None] * (v[t] - torch.einsum("hde,hd->he", s, k[t]))
+                s = s + k[t][:, :, None] * u[:, None, :]
+                out[t] = torch.einsum("hde,hd->he", s, q[t])
+            state[slots[b]] = s
+        return out.view(T, H * E)
 
     @staticmethod
     def _turn(x, positions, inv_freq, magnitude, neighbours):
@@ -406,18 +432,44 @@ class TorchOps(Ops):
             out = out * (mul.float() if mul_act is None else self.activation(mul.float(), mul_act))
         return out.to(out_dtype)
 
-    def route_topk(self, x, weight, bias, top, scoring="softmax"):
+    def route_topk(self, x, weight, bias, top, scoring="softmax", rule=None):
         z = x.float() @ weight.float().T
         if bias is not None:
             z = z + bias.float()
+        if rule is not None and rule.shared:
+            experts, gates = self._chosen(z[:, :-1], top, scoring, rule)
+            return experts, torch.cat([gates, torch.sigmoid(z[:, -1:])], 1)
+        return self._chosen(z, top, scoring, rule)
+
+    @staticmethod
+    def _chosen(z, top, scoring, rule):
+        if scoring == "sigmoid_share":
+            s = torch.sigmoid(z)
+            choice = s if rule.correction is None else s + rule.correction
+            if rule.groups > 1:
+                parts = choice.view(z.shape[0], rule.groups, -1)
+                strength = parts.sort(-1, descending=True).values[..., :2].sum(-1)
+                kept = torch.sort(strength, dim=-1, descending=True, stable=True).indices[:, :rule.kept]
+                closed = torch.ones_like(strength, dtype=torch.bool).scatter_(1, kept, False)
+                choice = parts.masked_fill(closed[..., None], -math.inf).view_as(choice)
+            order = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
+            own = torch.gather(s, 1, order)
+            return order.to(torch.int32), own / (own.sum(-1, keepdim=True) + 1e-20) * rule.scale
         order = torch.sort(z, dim=-1, descending=True, stable=True).indices[:, :top]
         chosen = torch.gather(z, 1, order)
         if scoring == "softmax_all":
             return order.to(torch.int32), torch.gather(torch.softmax(z, -1), 1, order)
         return order.to(torch.int32), torch.sigmoid(chosen) if scoring == "sigmoid" else torch.softmax(chosen, -1)
 
-    def route_glu(self, gate_up, experts, gates, num_experts, width, limit, slope, up_shift, on_input):
+    def route_glu(self, gate_up, experts, gates, num_experts, width, limit, slope, up_shift, on_input, shared_width=0):
         T = gate_up.shape[0]
+        if shared_width:
+            E = num_experts * width
+            gate, up = gate_up.split(E + shared_width, 1)
+            routed = self.route_glu(torch.cat([gate[:, :E], up[:, :E]], 1), experts, gates[:, :-1], num_experts, width, limit,
+                                    slope, up_shift, on_input)
+            own = gates[:, -1:] * gate[:, E:].float() * torch.sigmoid(slope * gate[:, E:].float()) * (up[:, E:].float() + up_shift)
+            return torch.cat([routed, own.to(gate_up.dtype)], 1)
         factor = torch.zeros(T, num_experts, dtype=torch.float32, device=gate_up.device)
         factor.scatter_(1, experts.long(), gates.float())
         chosen = torch.zeros(T, num_experts, dtype=torch.bool, device=gate_up.device)
@@ -459,6 +511,11 @@ class TorchOps(Ops):
         else:
             raise ValueError(kind)
         return r.to(x.dtype)
+
+    def clamped_glu(self, gate_up, limit, slope, up_shift):
+        inter = gate_up.shape[1] // 2
+        g, u = gate_up[:, :inter].float().clamp(max=limit), gate_up[:, inter:].float().clamp(-limit, limit)
+        return (g * torch.sigmoid(slope * g) * (u + up_shift)).to(gate_up.dtype)
 
     def silu_mul(self, gate_up):
         inter = gate_up.shape[1] // 2
