@@ -2,7 +2,8 @@
 // matrix-core kernels exist for multiples of 16 only, the wave-per-token kernel for every even size).
 //
 // out[t, h] = softmax_j(q[t, h] . k[j, h / G] * scale) v[j, h / G] over the keys j that token t may see:
-// first(t) <= j <= position(t), first = 0, or position - window + 1 on a windowed layer. Keys and values
+// first(t) <= j <= position(t): first = 0 (window 0), position - window + 1 (window > 0), or the start of the run of
+// -window positions that the token lies in, counted from position 0 (window < 0: chunks that see only themselves). Keys and values
 // are read through the block table of the token's request (row table_rows[request] of block_table, or row
 // `request` itself when table_rows is null): key j lives in page table[j / P] at offset
 // j % P of a cache laid out k [pages, kv_heads, P, D], v [pages, kv_heads, D, P]. The new tokens of the step are
@@ -29,6 +30,12 @@ constexpr int D = DISTIE_HEAD_DIM;
 constexpr int DIMS_PER_LANE = (D + DISTIE_WAVE - 1) / DISTIE_WAVE;
 
 extern "C" int distie_attention_head_dim() { return D; }
+
+// the first key that the token at position `pos` sees (`window`: see above; never falls as the position grows)
+__device__ __forceinline__ int first_visible(int pos, int window) {
+  if (window > 0) return max(0, pos - window + 1);
+  return window < 0 ? pos - pos % -window : 0;
+}
 
 template <typename C>
 __device__ __forceinline__ float dot_row(const float* q, const C* k);
@@ -114,7 +121,7 @@ __global__ __launch_bounds__(DISTIE_WAVE * WAVES) void attn_generic_kernel(
   for (int d = threadIdx.x; d < D; d += DISTIE_WAVE * WAVES) q_s[d] = to_float(q[d]);
   __syncthreads();
 
-  const int first = window > 0 ? max(0, q_pos - window + 1) : 0;
+  const int first = first_visible(q_pos, window);
   const int last = q_pos;   // inclusive
   const bool by_page = block_size % 4 == 0 && DISTIE_WAVE % block_size == 0;
   const float slope = head_slopes != nullptr ? head_slopes[h] : 0.f;
@@ -263,7 +270,7 @@ __global__ __launch_bounds__(DISTIE_WAVE * WAVES) void attn_grouped_f32_kernel(
       q_r[g][d] = v.x; q_r[g][d + 1] = v.y; q_r[g][d + 2] = v.z; q_r[g][d + 3] = v.w;
     }
   }
-  const int first = window > 0 ? max(0, q_pos - window + 1) : 0;
+  const int first = first_visible(q_pos, window);
   const int last = q_pos;   // inclusive
   float m[G], l[G];
   float acc[G][DIMS_PER_LANE];
@@ -422,7 +429,7 @@ __global__ __launch_bounds__(DISTIE_WAVE * WAVES) void attn_grouped_f32_kernel(
   }
 }
 
-// qkv: [T, q_stride] with q of head h at columns h*D; out: [T, heads*D]. window = 0: every earlier key.
+// qkv: [T, q_stride] with q of head h at columns h*D; out: [T, heads*D]. window: see the head of the file.
 // head_slopes (float32 [heads], may be null): score += slope[h] * (key - position); score_cap > 0: the scaled score
 // goes through cap * tanh(score / cap) first. Only this kernel takes the two. sinks (float32 [heads], may be null): the
 // softmax's denominator holds exp(sinks[h]) beside the keys' terms; every kernel of this file takes them.
@@ -433,7 +440,7 @@ extern "C" int distie_attention_generic(const void* qkv, int dtype, int64_t q_st
                                         int block_size, float scale, int window, const float* head_slopes,
                                         float score_cap, const float* sinks, hipStream_t stream) {
   if (tokens <= 0) return 0;
-  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size < 1 || table_width < 1 || window < 0 ||
+  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size < 1 || table_width < 1 ||
       score_cap < 0.f)
     return DISTIE_BAD_ARGUMENT;
   const bool plain_scores = head_slopes == nullptr && score_cap == 0.f;
@@ -535,7 +542,7 @@ struct KeyRuns {
 // than a short one; the caller made it long enough for the longest request to fit max_splits runs.
 __device__ __forceinline__ KeyRuns key_runs(int q_pos, int window, int max_splits, int run_len = 0) {
   KeyRuns runs;
-  runs.first = window > 0 ? max(0, q_pos - window + 1) : 0;
+  runs.first = first_visible(q_pos, window);
   runs.origin = runs.first / RUN_STEP * RUN_STEP;
   const int span = q_pos - runs.origin + 1;
   const int step = max_splits * RUN_STEP;
@@ -950,10 +957,10 @@ extern "C" int distie_attention_decode_bf16(const void* qkv, int64_t q_stride, c
                                             const int32_t* shared_run_len, const float* sinks, hipStream_t stream) {
   if (num_requests <= 0) return 0;
   const int group = kv_heads > 0 ? heads / kv_heads : 0;
-  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size % 16 != 0 || table_width < 1 || window < 0 ||
+  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size % 16 != 0 || table_width < 1 ||
       split_hint < RUN_STEP || split_hint % RUN_STEP != 0 || max_splits < 1 || max_splits > RD_MAX_RUNS ||
       group > 16 * DECODE_MAX_MB || kv_heads > 65535 || num_requests > 65535 || heads > 65535 ||
-      (shared_run_len != nullptr && (window > 0 || !dense_rows)))
+      (shared_run_len != nullptr && (window != 0 || !dense_rows)))
     return DISTIE_BAD_ARGUMENT;
   const dim3 grid = shared_run_len != nullptr ? dim3(kv_heads, num_requests, max_splits) : dim3(max_splits, kv_heads, num_requests);
   const bf16_t* q = static_cast<const bf16_t*>(qkv);
@@ -1059,7 +1066,7 @@ __global__ __launch_bounds__(PF_THREADS, (D <= 128) ? 2 : 1) void attn_prefill_k
   const int token0 = begin + tile * PF_BM;
   const int columns = min(PF_BM, end - token0);           // of the workgroup
   const int pos0 = positions[token0];                     // the tokens of a portion have consecutive positions
-  const int key_begin = window > 0 ? max(0, pos0 - window + 1) : 0;
+  const int key_begin = first_visible(pos0, window);
   const int key_end = pos0 + columns - 1;
   const int32_t* table = block_table + static_cast<int64_t>(table_rows != nullptr ? table_rows[request] : request) * table_width;
 
@@ -1071,10 +1078,11 @@ __global__ __launch_bounds__(PF_THREADS, (D <= 128) ? 2 : 1) void attn_prefill_k
   const int wave_col0 = wave * PF_WAVE_COLS;
   const int wave_cols = max(0, min(PF_WAVE_COLS, columns - wave_col0));
   const int wave_last = pos0 + wave_col0 + wave_cols - 1;
-  const int wave_first = window > 0 ? max(0, pos0 + wave_col0 - window + 1) : 0;
+  const int wave_first = first_visible(pos0 + wave_col0, window);
+  const int wave_open = first_visible(max(wave_last, 0), window);      // from here on every column of the wave sees (up to its own position)
   const int col = min(wave_col0 + c, columns - 1);        // columns past the end repeat the last; dropped later
   const int col_last = pos0 + col;                        // the last key the column sees, and the first
-  const int col_first = window > 0 ? max(0, col_last - window + 1) : 0;
+  const int col_first = first_visible(col_last, window);
   bf16x8 q_reg[PF_DK];
   {
     const bf16_t* q = qkv + (token0 + col) * q_stride + static_cast<int64_t>(head) * D;
@@ -1190,7 +1198,7 @@ __global__ __launch_bounds__(PF_THREADS, (D <= 128) ? 2 : 1) void attn_prefill_k
     // ---- softmax step of the lane's column. A tile whose keys every column of the wave sees needs no mask:
     // that is every tile but those on the diagonal and at a window's edge.
     const bool tile_open = k0 + PF_BN - 1 <= pos0 + wave_col0 &&
-                           (window <= 0 || k0 >= pos0 + wave_col0 + wave_cols - window);
+                           k0 >= wave_open;
     if (!tile_open) {
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb)
@@ -1405,7 +1413,7 @@ extern "C" int distie_attention_prefill_bf16(const void* qkv, int64_t q_stride, 
   // splits > 1: the keys are walked in that many parts side by side (worth it for long portions), with
   // part_o (float32 [splits, tokens, heads, D]) and part_ml (float32 [splits, tokens, heads, 2]) in between.
   if (tokens <= 0) return 0;
-  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size % 16 != 0 || table_width < 1 || window < 0 ||
+  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size % 16 != 0 || table_width < 1 ||
       num_requests < 1 || heads > 65535 || min_q_len < 1 || splits < 1 || splits > PF_MAX_SPLITS || !(scale > 0.f) ||
       (splits > 1 && (part_o == nullptr || part_ml == nullptr || token_request == nullptr)))
     return DISTIE_BAD_ARGUMENT;
@@ -1471,17 +1479,18 @@ __global__ __launch_bounds__(PF_THREADS, 1) void attn_prefill_f32_kernel(
   const int token0 = begin + tile * PF_BM;
   const int columns = min(PF_BM, end - token0);
   const int pos0 = positions[token0];
-  const int key_begin = window > 0 ? max(0, pos0 - window + 1) : 0;
+  const int key_begin = first_visible(pos0, window);
   const int key_end = pos0 + columns - 1;
   const int32_t* table = block_table + static_cast<int64_t>(table_rows != nullptr ? table_rows[request] : request) * table_width;
 
   const int wave_col0 = wave * PF_WAVE_COLS;
   const int wave_cols = max(0, min(PF_WAVE_COLS, columns - wave_col0));
   const int wave_last = pos0 + wave_col0 + wave_cols - 1;
-  const int wave_first = window > 0 ? max(0, pos0 + wave_col0 - window + 1) : 0;
+  const int wave_first = first_visible(pos0 + wave_col0, window);
+  const int wave_open = first_visible(max(wave_last, 0), window);      // from here on every column of the wave sees (up to its own position)
   const int col = min(wave_col0 + c, columns - 1);
   const int col_last = pos0 + col;
-  const int col_first = window > 0 ? max(0, col_last - window + 1) : 0;
+  const int col_first = first_visible(col_last, window);
   float4 q_reg[D / 8];                                    // of the lane's column: d = 8 g + 4 h + (0..3)
   {
     const float* q = qkv + (token0 + col) * q_stride + static_cast<int64_t>(head) * D;
@@ -1578,7 +1587,7 @@ __global__ __launch_bounds__(PF_THREADS, 1) void attn_prefill_f32_kernel(
       __builtin_amdgcn_sched_group_barrier(0x008, 4 * PF32_AHEAD, 0);
     }
     const bool tile_open = k0 + PF_BN - 1 <= pos0 + wave_col0 &&
-                           (window <= 0 || k0 >= pos0 + wave_col0 + wave_cols - window);
+                           k0 >= wave_open;
     if (!tile_open) {
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb)
@@ -1692,7 +1701,7 @@ extern "C" int distie_attention_prefill_f32(const void* qkv, int64_t q_stride, c
                                             int splits, const float* sinks, hipStream_t stream) {
 #if (DISTIE_HEAD_DIM % 32 == 0) && (DISTIE_HEAD_DIM <= 128)
   if (tokens <= 0) return 0;
-  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size % 16 != 0 || table_width < 1 || window < 0 ||
+  if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || block_size % 16 != 0 || table_width < 1 ||
       num_requests < 1 || heads > 65535 || min_q_len < 1 || splits < 1 || splits > PF_MAX_SPLITS || !(scale > 0.f) ||
       q_stride % 4 != 0 ||
       (splits > 1 && (part_o == nullptr || part_ml == nullptr || token_request == nullptr)))

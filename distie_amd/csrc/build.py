@@ -38,7 +38,7 @@ HIP_FLAGS = ["-O3", f"--offload-arch={ARCH}", "-fPIC", "-std=c++17",
 CXX_FLAGS = ["-O2", "-fPIC", "-std=c++17", "-pthread"]
 
 OPS_SOURCES = ["elementwise.hip", "gemm.hip", "gemv.hip", "decode_products.hip", "sampling.hip", "sequence.hip", "recurrent.hip", "latent.hip", "ssm.hip",
-               "depth.hip", "time_mixing.hip", "mixed_attention.hip"]
+               "depth.hip", "time_mixing.hip", "mixed_attention.hip", "delta.hip"]
 ATTN_SOURCES = ["attention.hip"]
 MIXED_ATTN_SOURCES = ["mixed_attention_mc.hip"]
 LIBRARY_SOURCES = ["library_products.hip"]

@@ -1,0 +1,482 @@
+// The gated delta rule: a state per head that forgets by a factor computed from the token and corrects what it holds under
+// the token's key.
+//
+// qkv [T, ld] holds q (G heads of D), k (G heads of D), v (H heads of E); head h reads q/k head h / (H / G). b and a: one
+// logit a head and row. With q^ = q / sqrt(sum(q^2) + unit_eps) * q_scale, k^ = k / sqrt(sum(k^2) + unit_eps),
+// w = sigmoid(b), ln f = -exp(a_log) * softplus(a + dt_bias), per head
+//     S <- f S (D x E, float32),   u = w (v - S^T k^),   S <- S + k^ u^T,   o = S^T q^.
+// state float32 [slots, H, D, E]. Unit norms, w, f, the state and every sum are float32 in either precision.
+//
+// A step is a flattened batch: request b's new tokens are rows cu_q[b] .. cu_q[b+1]-1, its state row state_slots[b].
+#include "common.h"
+
+namespace {
+
+__device__ __forceinline__ float sigmoidf(float x) { return 1.f / (1.f + expf(-x)); }
+__device__ __forceinline__ float softplusf(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
+// ---------------------------------------------------------------------------------------------------
+// Row after row. A block owns 64 columns e of one head of one request; wave `part` keeps the state's rows d = part * ROWS
+// .. + ROWS - 1 of its lanes' columns in registers. Every wave fetches all of q and k (lane: dimensions lane, lane + 64,
+// ...), so it has the sums of their squares and their product without a barrier, and keeps them in rows of LDS of its own.
+// With S the state in front of the row: S^T k^ and S^T q^ are summed in one walk, their parts meet in LDS (two sets of
+// places in turn: one barrier a row), and o = f S^T q^ + (k^ . q^) u. The next row's inputs are asked for before this row's
+// are used.
+template <typename X, int PARTS, int ROWS>
+__global__ void __launch_bounds__(64 * PARTS)
+delta_scan_kernel(const X* __restrict__ qkv, int64_t ld, const X* __restrict__ beta, int64_t ldb, const X* __restrict__ decay,
+                  int64_t lda, const float* __restrict__ a_log, const float* __restrict__ dt_bias, float* __restrict__ state,
+                  float* __restrict__ out, const int32_t* __restrict__ cu_q, const int32_t* __restrict__ state_slots, int H,
+                  int G, int D, int E, float q_scale, float unit_eps) {
+  constexpr int PER = PARTS * ROWS / 64;                 // dimensions of q and k a lane fetches
+  __shared__ float q_s[PARTS][PARTS * ROWS], k_s[PARTS][PARTS * ROWS];
+  __shared__ float partial[2][PARTS][2][64];
+  const int b = blockIdx.x, head = blockIdx.y;
+  const int lane = threadIdx.x % 64, part = threadIdx.x / 64;
+  const int e = blockIdx.z * 64 + lane;
+  const int first = cu_q[b], last = cu_q[b + 1];
+  if (first >= last) return;
+  const int shared_head = head / (H / G);
+  const float rate = -expf(a_log[head]), bias = dt_bias[head];
+  const int64_t q_at = static_cast<int64_t>(shared_head) * D, k_at = static_cast<int64_t>(G + shared_head) * D;
+  const int64_t v_at = 2 * static_cast<int64_t>(G) * D + static_cast<int64_t>(head) * E + e;
+  float* own = state + (static_cast<int64_t>(state_slots[b]) * H + head) * D * E;
+  const int d0 = part * ROWS;
+  float s[ROWS];
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) s[r] = (d0 + r < D && e < E) ? own[static_cast<int64_t>(d0 + r) * E + e] : 0.f;
+  float nq[PER], nk[PER], nv = 0.f, nb = 0.f, na = 0.f;
+  auto fetch = [&](int t) {
+    const X* row = qkv + static_cast<int64_t>(t) * ld;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int d = lane + 64 * i;
+      nq[i] = d < D ? to_float(row[q_at + d]) : 0.f;
+      nk[i] = d < D ? to_float(row[k_at + d]) : 0.f;
+    }
+    nv = e < E ? to_float(row[v_at]) : 0.f;
+    nb = to_float(beta[static_cast<int64_t>(t) * ldb + head]);
+    na = to_float(decay[static_cast<int64_t>(t) * lda + head]);
+  };
+  fetch(first);
+  for (int t = first; t < last; ++t) {
+    float qq = 0.f, kk = 0.f, qk = 0.f;
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      q_s[part][lane + 64 * i] = nq[i];
+      k_s[part][lane + 64 * i] = nk[i];
+      qq += nq[i] * nq[i];
+      kk += nk[i] * nk[i];
+      qk += nq[i] * nk[i];
+    }
+    __builtin_amdgcn_wave_barrier();
+    const float v = nv, w = sigmoidf(nb), f = expf(rate * softplusf(na + bias));
+    if (t + 1 < last) fetch(t + 1);
+    const float q_unit = q_scale / sqrtf(wave_sum(qq) + unit_eps), k_unit = 1.f / sqrtf(wave_sum(kk) + unit_eps);
+    const float both = wave_sum(qk) * q_unit * k_unit;
+    float by_k = 0.f, by_q = 0.f;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) {
+      by_k += s[r] * k_s[part][d0 + r];
+      by_q += s[r] * q_s[part][d0 + r];
+    }
+    float(*place)[2][64] = partial[t & 1];
+    place[part][0][lane] = by_k;
+    place[part][1][lane] = by_q;
+    __syncthreads();
+    float all_k = 0.f, all_q = 0.f;
+#pragma unroll
+    for (int p = 0; p < PARTS; ++p) all_k += place[p][0][lane], all_q += place[p][1][lane];
+    const float u = w * (v - f * (all_k * k_unit));
+    const float ku = k_unit * u;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) s[r] = f * s[r] + k_s[part][d0 + r] * ku;
+    if (part == 0 && e < E) out[(static_cast<int64_t>(t) * H + head) * E + e] = f * (all_q * q_unit) + both * u;
+  }
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r)
+    if (d0 + r < D && e < E) own[static_cast<int64_t>(d0 + r) * E + e] = s[r];
+}
+
+// ---------------------------------------------------------------------------------------------------
+// Portions of prompts, in chunks of L = 64 rows. With l_i the running sum of ln f inside the chunk (falling, <= 0) and S
+// the state in front of it, the chunk's corrections u solve a triangular system,
+//     u_i + sum_{j<i} A_ij u_j = w_i (v_i - exp(l_i) S^T k^_i),      A_ij = w_i exp(l_i - l_j) (k^_i . k^_j),
+// so with X the solution of (I + A) X = (w_i exp(l_i) k^_i | w_i v_i), X = (W | V'):     U = V' - W S,
+//     S_next = exp(l_L) S + sum_j exp(l_L - l_j) k^_j u_j^T,
+//     o_i    = exp(l_i) S^T q^_i + sum_{j<=i} exp(l_i - l_j) (q^_i . k^_j) u_j.
+// Every exponent is <= 0 and no quotient of decays is formed.
+//   prepare (chunk, head side by side): W, V', the factors k~_j = exp(l_L - l_j) k^_j (transposed), the pairs' weights in o
+//   states  (request, head, 16 columns e): U and the state in front of every chunk, chunk after chunk
+//   outputs (chunk, head, 64 columns): o
+// Float32 throughout, products on float32 matrix products. Scratch is padded: DP = D rounded up to a multiple of 64 that
+// four waves share evenly (64, 128 or 256), EP = E rounded up to a multiple of 16, zeros beyond D, E and a chunk's rows. A
+// chunk's table entry is {request, first row, rows, unused}.
+constexpr int DL = 64;
+constexpr int DL_PAD = DL + 1;
+constexpr int DL_ROW = DL + 4;          // row stride of the triangular matrix: 16-byte reads of a row
+typedef __attribute__((__vector_size__(16 * sizeof(float)))) float delta_floatx16;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float delta_floatx4;
+__device__ __forceinline__ int tile_row(int v, int lane) { return 8 * (v / 4) + 4 * (lane / 32) + v % 4; }
+
+template <typename X>
+__global__ void __launch_bounds__(256)
+delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __restrict__ beta, int64_t ldb,
+                           const X* __restrict__ decay, int64_t lda, const float* __restrict__ a_log,
+                           const float* __restrict__ dt_bias, float* __restrict__ w_out, float* __restrict__ v_out,
+                           float* __restrict__ k_out, float* __restrict__ pairs, float* __restrict__ q_factor,
+                           float* __restrict__ totals, const int4* __restrict__ chunks, int H, int G, int D, int E, int DP,
+                           int EP, float q_scale, float unit_eps) {
+  __shared__ float l_s[DL], beta_s[DL], q_unit[DL], k_unit[DL];
+  __shared__ float q_s[DL][DL_PAD], k_s[DL][DL_PAD];     // [row][d of this pass]
+  __shared__ __attribute__((aligned(16))) float a_s[DL][DL_ROW];
+  const int chunk = blockIdx.x, head = blockIdx.y;
+  const int4 entry = chunks[chunk];
+  const int first = entry.y, rows = entry.z;
+  const int shared_head = head / (H / G);
+  const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64;
+  const int64_t q_at = static_cast<int64_t>(shared_head) * D, k_at = static_cast<int64_t>(G + shared_head) * D;
+  const int64_t place = static_cast<int64_t>(chunk) * H + head;
+  if (wave == 0) {
+    const bool in = lane < rows;
+    const int64_t t = first + min(lane, rows - 1);
+    float l = in ? -expf(a_log[head]) * softplusf(to_float(decay[t * lda + head]) + dt_bias[head]) : 0.f;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float before = __shfl_up(l, o, 64);
+      if (lane >= o) l += before;
+    }
+    l_s[lane] = l;
+    beta_s[lane] = in ? sigmoidf(to_float(beta[t * ldb + head])) : 0.f;
+  }
+  // k . k and q . k of the chunk's rows (a wave: 32 rows i by 32 rows j), and the sums of squares (four threads a row)
+  const int ib = 32 * (wave / 2), jb = 32 * (wave % 2);
+  const int sum_row = tid / 4, sum_part = tid % 4;
+  delta_floatx16 kk = {}, qk = {};
+  float q_sq = 0.f, k_sq = 0.f;
+  for (int n0 = 0; n0 < D; n0 += DL) {
+    __syncthreads();
+    for (int j = wave; j < DL; j += 4) {
+      const bool in = j < rows && n0 + lane < D;
+      const X* row = qkv + static_cast<int64_t>(first + j) * ld + n0 + lane;
+      q_s[j][lane] = in ? to_float(row[q_at]) : 0.f;
+      k_s[j][lane] = in ? to_float(row[k_at]) : 0.f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const float q = q_s[sum_row][4 * i + sum_part], k = k_s[sum_row][4 * i + sum_part];
+      q_sq += q * q;
+      k_sq += k * k;
+    }
+    if (jb <= ib) {
+      for (int n = 0; n < DL; n += 2) {
+        const float other = k_s[jb + lane % 32][n + lane / 32];
+        kk = __builtin_amdgcn_mfma_f32_32x32x2f32(k_s[ib + lane % 32][n + lane / 32], other, kk, 0, 0, 0);
+        qk = __builtin_amdgcn_mfma_f32_32x32x2f32(q_s[ib + lane % 32][n + lane / 32], other, qk, 0, 0, 0);
+      }
+    }
+  }
+  q_sq += __shfl_xor(q_sq, 1, 64);
+  k_sq += __shfl_xor(k_sq, 1, 64);
+  q_sq += __shfl_xor(q_sq, 2, 64);
+  k_sq += __shfl_xor(k_sq, 2, 64);
+  if (sum_part == 0) {
+    q_unit[sum_row] = q_scale / sqrtf(q_sq + unit_eps);
+    k_unit[sum_row] = 1.f / sqrtf(k_sq + unit_eps);
+  }
+  __syncthreads();
+  const float l_end = l_s[DL - 1];                       // (rows beyond the chunk add nothing)
+  float* pair = pairs + place * DL * DL;
+#pragma unroll
+  for (int v = 0; v < 16; ++v) {
+    const int i = ib + tile_row(v, lane), j = jb + lane % 32;
+    const float fade = j <= i && i < rows ? expf(l_s[i] - l_s[j]) * k_unit[j] : 0.f;
+    a_s[i][j] = j < i ? fade * beta_s[i] * k_unit[i] * kk[v] : 0.f;
+    pair[i * DL + j] = fade * q_unit[i] * qk[v];
+  }
+  if (tid < DL) q_factor[place * DL + tid] = expf(l_s[tid]) * q_unit[tid];
+  if (tid == 0) totals[place] = expf(l_end);
+  __syncthreads();
+  // (I + A) X = B, a thread a column of B, forward substitution with the column in registers
+  for (int c = tid; c < DP + EP; c += 256) {
+    const bool key = c < DP;
+    const int col = key ? c : c - DP;
+    const bool in = key ? col < D : col < E;
+    const X* from = qkv + static_cast<int64_t>(first) * ld +
+                    (key ? k_at + col : 2 * static_cast<int64_t>(G) * D + static_cast<int64_t>(head) * E + col);
+    float x[DL];
+#pragma unroll
+    for (int i = 0; i < DL; ++i) x[i] = in && i < rows ? to_float(from[static_cast<int64_t>(i) * ld]) : 0.f;
+    if (key) {
+      float* to = k_out + (place * DP + col) * DL;
+#pragma unroll
+      for (int i = 0; i < DL; i += 4) {
+        float4 k4;
+        k4.x = x[i] * k_unit[i] * expf(l_end - l_s[i]);
+        k4.y = x[i + 1] * k_unit[i + 1] * expf(l_end - l_s[i + 1]);
+        k4.z = x[i + 2] * k_unit[i + 2] * expf(l_end - l_s[i + 2]);
+        k4.w = x[i + 3] * k_unit[i + 3] * expf(l_end - l_s[i + 3]);
+        *reinterpret_cast<float4*>(to + i) = k4;
+      }
+    }
+    float* to = key ? w_out + place * DL * DP + col : v_out + place * DL * EP + col;
+    const int stride = key ? DP : EP;
+#pragma unroll
+    for (int i = 0; i < DL; ++i) {
+      float acc = beta_s[i] * x[i] * (key ? k_unit[i] * expf(l_s[i]) : 1.f);
+#pragma unroll
+      for (int j = 0; j < i; j += 4) {
+        const float4 a = *reinterpret_cast<const float4*>(&a_s[i][j]);       // (zero from the diagonal on)
+        acc -= a.x * x[j];
+        if (j + 1 < i) acc -= a.y * x[j + 1];
+        if (j + 2 < i) acc -= a.z * x[j + 2];
+        if (j + 3 < i) acc -= a.w * x[j + 3];
+      }
+      x[i] = acc;
+      to[static_cast<int64_t>(i) * stride] = acc;
+    }
+  }
+}
+
+// blockIdx = (request, head, 16 columns e). Wave w keeps rows d = 16 TILES w .. of the state's 16 columns as TILES tiles of
+// 16 x 16 in the products' own result layout: lane (g = lane / 16, c = lane % 16) holds rows 4 g + v and column c of a tile,
+// which is also what the second operand of v_mfma_f32_16x16x4_f32 takes if the four products of a step of 16 summed indexes
+// take index 4 g + t from lane group g at product t. So neither the state nor U moves between lanes; W and k~ are read in the
+// same order, 16 bytes a lane. The four waves' shares of W S meet in LDS (two sets of places in turn: one barrier a chunk),
+// and every wave adds them up for itself.
+template <int TILES>
+__global__ void __launch_bounds__(256)
+delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restrict__ v_in, const float* __restrict__ k_in,
+                          const float* __restrict__ totals, float* __restrict__ u_out, float* __restrict__ scratch,
+                          float* __restrict__ state, const int32_t* __restrict__ first_chunk,
+                          const int32_t* __restrict__ state_slots, int H, int D, int E, int EP) {
+  constexpr int DP = 64 * TILES;
+  __shared__ __attribute__((aligned(16))) float share[2][4][4][64 * 4];        // [turn][wave][tile of rows][lane, v]
+  const int b = blockIdx.x, head = blockIdx.y, e0 = blockIdx.z * 16;
+  const int begin = first_chunk[b], end = first_chunk[b + 1];
+  if (begin >= end) return;
+  const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
+  const int g = lane / 16, c = lane % 16;
+  const int d0 = 16 * TILES * wave;
+  const bool column = e0 + c < E;
+  float* own = state + (static_cast<int64_t>(state_slots[b]) * H + head) * D * E + e0 + c;
+  delta_floatx4 s[TILES];
+#pragma unroll
+  for (int i = 0; i < TILES; ++i)
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+      const int d = d0 + 16 * i + 4 * g + v;
+      s[i][v] = column && d < D ? own[static_cast<int64_t>(d) * E] : 0.f;
+    }
+  delta_floatx4 w4[4][TILES], k4[TILES][4];
+  float v4[4][4];
+  auto fetch_w = [&](int64_t place) {
+    const float* p = w_in + place * DL * DP + d0 + 4 * g;
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int i = 0; i < TILES; ++i) w4[m][i] = *reinterpret_cast<const delta_floatx4*>(p + (16 * m + c) * DP + 16 * i);
+  };
+  auto fetch_kv = [&](int64_t place) {
+    const float* p = k_in + (place * DP + d0 + c) * DL + 4 * g;
+#pragma unroll
+    for (int i = 0; i < TILES; ++i)
+#pragma unroll
+      for (int m = 0; m < 4; ++m) k4[i][m] = *reinterpret_cast<const delta_floatx4*>(p + 16 * i * DL + 16 * m);
+    const float* q = v_in + place * DL * EP + e0 + c;
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int v = 0; v < 4; ++v) v4[m][v] = q[(16 * m + 4 * g + v) * EP];
+  };
+  fetch_w(static_cast<int64_t>(begin) * H + head);
+  fetch_kv(static_cast<int64_t>(begin) * H + head);
+  for (int chunk = begin; chunk < end; ++chunk) {
+    const int64_t place = static_cast<int64_t>(chunk) * H + head;
+    const int64_t next = static_cast<int64_t>(min(chunk + 1, end - 1)) * H + head;
+    const float total = totals[place];
+    delta_floatx4 part[4] = {};
+#pragma unroll
+    for (int i = 0; i < TILES; ++i)
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int m = 0; m < 4; ++m) part[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(w4[m][i][t], s[i][t], part[m], 0, 0, 0);
+    fetch_w(next);
+    float(*at)[4][256] = share[(chunk - begin) & 1];
+#pragma unroll
+    for (int m = 0; m < 4; ++m) *reinterpret_cast<delta_floatx4*>(&at[wave][m][4 * lane]) = part[m];
+    // the state in front of the chunk, for the outputs
+    if (column) {
+      float* to = scratch + place * D * E + e0 + c;
+#pragma unroll
+      for (int i = 0; i < TILES; ++i)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+          const int d = d0 + 16 * i + 4 * g + v;
+          if (d < D) to[static_cast<int64_t>(d) * E] = s[i][v];
+        }
+    }
+    __syncthreads();
+    float u[4][4];
+#pragma unroll
+    for (int m = 0; m < 4; ++m) {
+      delta_floatx4 sum = *reinterpret_cast<const delta_floatx4*>(&at[0][m][4 * lane]);
+#pragma unroll
+      for (int w = 1; w < 4; ++w) {
+        const delta_floatx4 more = *reinterpret_cast<const delta_floatx4*>(&at[w][m][4 * lane]);
+#pragma unroll
+        for (int v = 0; v < 4; ++v) sum[v] += more[v];
+      }
+#pragma unroll
+      for (int v = 0; v < 4; ++v) u[m][v] = v4[m][v] - sum[v];
+    }
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+      if (m == wave) {
+        float* to = u_out + place * DL * EP + e0 + c;
+#pragma unroll
+        for (int v = 0; v < 4; ++v) to[(16 * m + 4 * g + v) * EP] = u[m][v];
+      }
+#pragma unroll
+    for (int i = 0; i < TILES; ++i)
+#pragma unroll
+      for (int v = 0; v < 4; ++v) s[i][v] *= total;
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int i = 0; i < TILES; ++i) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[i][m][t], u[m][t], s[i], 0, 0, 0);
+    fetch_kv(next);
+  }
+  if (column) {
+#pragma unroll
+    for (int i = 0; i < TILES; ++i)
+#pragma unroll
+      for (int v = 0; v < 4; ++v) {
+        const int d = d0 + 16 * i + 4 * g + v;
+        if (d < D) own[static_cast<int64_t>(d) * E] = s[i][v];
+      }
+  }
+}
+
+// blockIdx = (chunk, head, 64 columns e); a wave: 32 rows i by 32 columns
+template <typename X>
+__global__ void __launch_bounds__(256)
+delta_chunk_outputs_kernel(const X* __restrict__ qkv, int64_t ld, const float* __restrict__ q_factor,
+                           const float* __restrict__ pairs, const float* __restrict__ u_in, const float* __restrict__ scratch,
+                           float* __restrict__ out, const int4* __restrict__ chunks, int H, int G, int D, int E, int EP) {
+  __shared__ float a_s[DL][DL_PAD];     // a tile of q [i][d], then the pairs' weights [i][j]
+  __shared__ float b_s[DL][DL_PAD];     // a tile of the state [d][e], then U [j][e]
+  __shared__ float f_s[DL];
+  const int chunk = blockIdx.x, head = blockIdx.y, e0 = blockIdx.z * 64;
+  const int4 entry = chunks[chunk];
+  const int first = entry.y, rows = entry.z;
+  const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
+  const int64_t place = static_cast<int64_t>(chunk) * H + head;
+  const int64_t q_at = static_cast<int64_t>(head / (H / G)) * D;
+  if (threadIdx.x < DL) f_s[threadIdx.x] = q_factor[place * DL + threadIdx.x];
+  const int ib = 32 * (wave / 2), pb = 32 * (wave % 2);
+  const float* s_in = scratch + place * D * E;
+  delta_floatx16 y = {};
+  for (int n0 = 0; n0 < D; n0 += DL) {
+    __syncthreads();
+    for (int j = wave; j < DL; j += 4) {
+      a_s[j][lane] = (j < rows && n0 + lane < D) ? to_float(qkv[static_cast<int64_t>(first + j) * ld + q_at + n0 + lane]) : 0.f;
+      b_s[j][lane] = (n0 + j < D && e0 + lane < E) ? s_in[static_cast<int64_t>(n0 + j) * E + e0 + lane] : 0.f;
+    }
+    __syncthreads();
+    for (int n = 0; n < DL; n += 2)
+      y = __builtin_amdgcn_mfma_f32_32x32x2f32(a_s[ib + lane % 32][n + lane / 32], b_s[n + lane / 32][pb + lane % 32], y, 0, 0, 0);
+  }
+#pragma unroll
+  for (int v = 0; v < 16; ++v) y[v] *= f_s[ib + tile_row(v, lane)];
+  __syncthreads();
+  for (int j = wave; j < DL; j += 4) {
+    a_s[j][lane] = pairs[place * DL * DL + j * DL + lane];
+    b_s[j][lane] = e0 + lane < E ? u_in[(place * DL + j) * EP + e0 + lane] : 0.f;
+  }
+  __syncthreads();
+  for (int j = 0; j < ib + 32; j += 2)
+    y = __builtin_amdgcn_mfma_f32_32x32x2f32(a_s[ib + lane % 32][j + lane / 32], b_s[j + lane / 32][pb + lane % 32], y, 0, 0, 0);
+#pragma unroll
+  for (int v = 0; v < 16; ++v) {
+    const int i = ib + tile_row(v, lane), col = e0 + pb + lane % 32;
+    if (i < rows && col < E) out[(static_cast<int64_t>(first + i) * H + head) * E + col] = y[v];
+  }
+}
+
+bool bad_shape(int H, int G, int D, int E, int64_t ld, int64_t ldb, int64_t lda) {
+  return H < 1 || G < 1 || H % G != 0 || D < 1 || E < 1 || D > 256 || H > 65535 || ldb < H || lda < H ||
+         ld < 2 * static_cast<int64_t>(G) * D + static_cast<int64_t>(H) * E;
+}
+
+}  // namespace
+
+// the largest key size a head may have
+extern "C" int distie_delta_scan_max_dim() { return 256; }
+
+extern "C" int distie_delta_scan(const void* qkv, int dtype, int64_t ld, const void* beta, int64_t ldb, const void* decay,
+                                 int64_t lda, const float* a_log, const float* dt_bias, float* state, float* out,
+                                 const int32_t* cu_q, const int32_t* state_slots, int B, int H, int G, int D, int E,
+                                 float q_scale, float unit_eps, hipStream_t stream) {
+  if (B <= 0) return 0;
+  if (bad_shape(H, G, D, E, ld, ldb, lda)) return DISTIE_BAD_ARGUMENT;
+  const dim3 grid(B, H, (E + 63) / 64);
+#define DISTIE_DELTA(PARTS, ROWS)                                                                                     \
+  DISTIE_DISPATCH(dtype, X, (delta_scan_kernel<X, PARTS, ROWS><<<grid, 64 * PARTS, 0, stream>>>(                      \
+      static_cast<const X*>(qkv), ld, static_cast<const X*>(beta), ldb, static_cast<const X*>(decay), lda, a_log,     \
+      dt_bias, state, out, cu_q, state_slots, H, G, D, E, q_scale, unit_eps)))
+  if (D <= 64) {
+    DISTIE_DELTA(4, 16);
+  } else if (D <= 128) {
+    DISTIE_DELTA(4, 32);
+  } else {
+    DISTIE_DELTA(8, 32);
+  }
+#undef DISTIE_DELTA
+  return launch_status();
+}
+
+extern "C" int distie_delta_scan_chunk_rows() { return DL; }
+extern "C" int distie_delta_scan_padded_dim(int D) { return D <= 64 ? 64 : (D <= 128 ? 128 : 256); }
+
+// chunks: int32 [count][4] = {request, first row, rows (1..64), 0}, the chunks of a request one after the other;
+// first_chunk: int32 [B + 1]. Float32 scratch, DP = distie_delta_scan_padded_dim(D), EP = E rounded up to a multiple of 16:
+// w [count, H, 64, DP], v and u [count, H, 64, EP], k [count, H, DP, 64], pairs [count, H, 64, 64], q_factor [count, H, 64],
+// totals [count, H], states [count, H, D, E].
+extern "C" int distie_delta_scan_chunked(const void* qkv, int dtype, int64_t ld, const void* beta, int64_t ldb,
+                                         const void* decay, int64_t lda, const float* a_log, const float* dt_bias,
+                                         float* state, float* out, float* w, float* v, float* u, float* k, float* pairs,
+                                         float* q_factor, float* totals, float* states, const void* chunks,
+                                         const int32_t* first_chunk, const int32_t* state_slots, int count, int B, int H,
+                                         int G, int D, int E, float q_scale, float unit_eps, hipStream_t stream) {
+  if (B <= 0 || count <= 0) return 0;
+  if (bad_shape(H, G, D, E, ld, ldb, lda)) return DISTIE_BAD_ARGUMENT;
+  const int DP = distie_delta_scan_padded_dim(D), EP = (E + 15) / 16 * 16;
+  const int4* table = static_cast<const int4*>(chunks);
+  int status = 0;
+  DISTIE_DISPATCH(dtype, X, (delta_chunk_prepare_kernel<X><<<dim3(count, H), 256, 0, stream>>>(
+      static_cast<const X*>(qkv), ld, static_cast<const X*>(beta), ldb, static_cast<const X*>(decay), lda, a_log, dt_bias, w, v,
+      k, pairs, q_factor, totals, table, H, G, D, E, DP, EP, q_scale, unit_eps)));
+  if ((status = launch_status()) != 0) return status;
+  const dim3 grid(B, H, EP / 16);
+#define DISTIE_DELTA_STATES(TILES)                                                                                    \
+  delta_chunk_states_kernel<TILES><<<grid, 256, 0, stream>>>(w, v, k, totals, u, states, state, first_chunk, state_slots, H, \
+                                                             D, E, EP)
+  if (DP == 64) {
+    DISTIE_DELTA_STATES(1);
+  } else if (DP == 128) {
+    DISTIE_DELTA_STATES(2);
+  } else {
+    DISTIE_DELTA_STATES(4);
+  }
+#undef DISTIE_DELTA_STATES
+  if ((status = launch_status()) != 0) return status;
+  DISTIE_DISPATCH(dtype, X, (delta_chunk_outputs_kernel<X><<<dim3(count, H, (E + 63) / 64), 256, 0, stream>>>(
+      static_cast<const X*>(qkv), ld, q_factor, pairs, u, states, out, table, H, G, D, E, EP)));
+  return launch_status();
+}

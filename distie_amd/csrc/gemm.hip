@@ -416,7 +416,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_packed_kernel(const bf16_t* _
         if (n >= half) continue;
         float gate = acc[i], u = up[i];
         if (bias != nullptr) { gate += bias[n]; u += bias[half + n]; }
-        y[static_cast<int64_t>(r) * half + n] = from_float<Y>(gate_activation(gate, rotary.act) * u);
+        y[static_cast<int64_t>(r) * half + n] = from_float<Y>(gated_value(gate, u, rotary.act, rotary.limit, rotary.slope, rotary.up_shift));
       }
     }
   } else if constexpr (MODE == PK_ROTARY) {
@@ -488,13 +488,15 @@ static int packed_waves(int K) {
 
 // y: as distie_gemm_skinny_bf16 (the same cut along K: slices go to other workgroups, hence to other
 // compute units, which a product with few rows of W needs to pull its bytes fast enough);
-// gated: [M, N / 2] of y_dtype, never cut. Up to 256 rows of x, in groups of 16.
+// gated: [M, N / 2] of y_dtype, never cut. Up to 256 rows of x, in groups of 16. limit, slope, up_shift: of the clamped
+// activation (5 above the low eight bits of `gated`).
 extern "C" int distie_gemm_packed_bf16(const void* x, const void* w_packed, const float* bias, void* y, int y_dtype,
-                                       int M, int N, int K, int gated, hipStream_t stream) {
+                                       int M, int N, int K, int gated, float limit, float slope, float up_shift,
+                                       hipStream_t stream) {
   if (M <= 0) return 0;
   const int act = gated >> 8;           // the activation on the gate, above the low eight bits
   gated &= 0xff;
-  if (M > 256 || N <= 0 || K <= 0 || K % 8 != 0 || (gated && N % 2 != 0) || act < 0 || act > 4) return DISTIE_BAD_ARGUMENT;
+  if (M > 256 || N <= 0 || K <= 0 || K % 8 != 0 || (gated && N % 2 != 0) || act < 0 || act > 5 || (act == 5 && !(limit > 0.f))) return DISTIE_BAD_ARGUMENT;
   int slices = 1, k_per_slice = (K + SK_KSTEP - 1) / SK_KSTEP * SK_KSTEP;
   if (!gated) skinny_plan(N, K, &slices, &k_per_slice);
   if (slices > 1 && y_dtype != DISTIE_F32) return DISTIE_BAD_ARGUMENT;
@@ -504,6 +506,7 @@ extern "C" int distie_gemm_packed_bf16(const void* x, const void* w_packed, cons
   const bf16_t* wb = static_cast<const bf16_t*>(w_packed);
   RotaryOut none = {};
   none.act = act;
+  none.limit = limit, none.slope = slope, none.up_shift = up_shift;
   if (gated && M <= 8) {
     // The gated product is not cut along K (the activation needs the whole sum), so a row block's K goes to the four
     // waves of a workgroup, which add their sums through LDS: up to 8 rows of x that is faster than one wave a row
@@ -621,7 +624,8 @@ constexpr int WD_MAX_BLOCKS = 6;
 // sum over K, which this kernel cuts into slices, so it is left to the kernel that adds the slices.
 struct HeadRows {
   int heads, kv_heads, dim;
-  int act;                    // gated products only: the activation on the gate (gate_activation)
+  int act;                    // gated products only: the activation on the gate (gate_activation, gated_value)
+  float limit, slope, up_shift;
 };
 
 template <typename Y, int MODE, int MB, int WD_WAVES>
@@ -749,7 +753,7 @@ __global__ __launch_bounds__(64 * WD_WAVES) void gemm_packed_wide_kernel(const b
         for (int i = 0; i < 4; ++i) {
           float gate = acc[b][i], u = up[i];
           if (bias != nullptr && n0 + i < half) { gate += bias[n0 + i]; u += bias[half + n0 + i]; }
-          v[i] = gate_activation(gate, head_rows.act) * u;
+          v[i] = gated_value(gate, u, head_rows.act, head_rows.limit, head_rows.slope, head_rows.up_shift);
         }
 #pragma unroll
         for (int i = 0; i < 4; ++i)
@@ -850,13 +854,13 @@ static int packed_wide_launch(const bf16_t* x, const bf16_t* w, const float* bia
 
 extern "C" int distie_gemm_packed_wide_bf16(const void* x, const void* w_packed, const float* bias, void* y,
                                             int y_dtype, int M, int N, int K, int gated, int pass_blocks,
-                                            hipStream_t stream) {
+                                            float limit, float slope, float up_shift, hipStream_t stream) {
   if (M <= 0) return 0;
   const int act = gated >> 8;           // the activation on the gate, above the low eight bits
   gated &= 0xff;
-  if (M > 256 || N <= 0 || K <= 0 || K % 8 != 0 || (gated && N % 2 != 0) || act < 0 || act > 4) return DISTIE_BAD_ARGUMENT;
+  if (M > 256 || N <= 0 || K <= 0 || K % 8 != 0 || (gated && N % 2 != 0) || act < 0 || act > 5 || (act == 5 && !(limit > 0.f))) return DISTIE_BAD_ARGUMENT;
   return packed_wide_launch(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w_packed), bias, y, y_dtype, M, N,
-                            K, gated ? PK_GATED : PK_PLAIN, pass_blocks, stream, HeadRows{0, 0, 0, act});
+                            K, gated ? PK_GATED : PK_PLAIN, pass_blocks, stream, HeadRows{0, 0, 0, act, limit, slope, up_shift});
 }
 
 // The stacked q/k/v product alone, on the ROTARY copy of its weight, for 17 rows of x and more against a weight large

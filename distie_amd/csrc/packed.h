@@ -19,6 +19,7 @@ struct RotaryOut {
   bf16_t* v_cache;            // [pages, kv_heads, D, block_size]
   int heads, kv_heads, dim, block_size, write;
   int act;                    // gated products only: the activation on the gate (see gate_activation)
+  float limit, slope, up_shift;      // of the clamped one (see gated_value)
 };
 
 // The activation on the gate of a gated product: 0 silu; else 1 + the kind as `distie_activation` numbers them
@@ -29,6 +30,14 @@ static __device__ __forceinline__ float gate_activation(float z, int act) {
   if (act == 3) return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
   const float p = fmaxf(z, 0.f);
   return act == 1 ? p * p : p;
+}
+
+// gate and up of one hidden value put together. act 5: g = min(gate, limit), u = clamp(up, -limit, limit),
+// g * sigmoid(slope * g) * (u + up_shift); else the activation of the gate times up.
+static __device__ __forceinline__ float gated_value(float gate, float up, int act, float limit, float slope, float up_shift) {
+  if (act != 5) return gate_activation(gate, act) * up;
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.f + expf(-slope * g)) * (u + up_shift);
 }
 
 static __device__ __forceinline__ uint2 pack_bf16x4(const float v[4]) {

@@ -704,10 +704,57 @@ __global__ void lru_chunk_apply_kernel(const float* __restrict__ a, const float*
 constexpr int ROUTE_MAX_EXPERTS = 1024;
 constexpr int ROUTE_MAX_TOP = 32;
 
+// Scoring 3: experts are chosen by sigmoid(z) + correction, among the `kept` strongest of `groups` groups of neighbours
+// (by the sum of a group's two largest choice scores), and weighted by scale * sigmoid(z) / (the chosen ones' sum).
+// `shared` (any scoring): the router has one row more than experts; the sigmoid of its logit goes behind a row's weights.
+struct RouteRule {
+  const float* correction;
+  int groups, kept;
+  float scale;
+  int shared;
+};
+
+// logits z -> choice scores in z, sigmoids in `own`; -inf for the experts of groups that are not kept. By the whole block
+// (`strength`: a float a group).
+__device__ __forceinline__ void choice_scores(float* z, float* own, float* strength, int E, const RouteRule& rule) {
+  for (int e = threadIdx.x; e < E; e += blockDim.x) {
+    const float s = 1.f / (1.f + expf(-z[e]));
+    own[e] = s;
+    z[e] = rule.correction != nullptr ? s + rule.correction[e] : s;
+  }
+  __syncthreads();
+  if (rule.groups <= 1 || rule.kept >= rule.groups) return;
+  const int size = E / rule.groups;
+  for (int g = threadIdx.x; g < rule.groups; g += blockDim.x) {
+    float first = -INFINITY, second = -INFINITY;
+    for (int e = g * size; e < (g + 1) * size; ++e) {
+      const float v = z[e];
+      if (v > first) second = first, first = v;
+      else second = fmaxf(second, v);
+    }
+    strength[g] = size > 1 ? first + second : first;
+  }
+  __syncthreads();
+  for (int g = threadIdx.x; g < rule.groups; g += blockDim.x) {
+    int ahead = 0;                                    // groups that come before this one (the lower index among equals)
+    for (int o = 0; o < rule.groups; ++o) ahead += strength[o] > strength[g] || (strength[o] == strength[g] && o < g) ? 1 : 0;
+    if (ahead >= rule.kept)
+      for (int e = g * size; e < (g + 1) * size; ++e) z[e] = -INFINITY;
+  }
+  __syncthreads();
+}
+
 // the weights of the chosen experts from their logits (largest first): softmax over those alone (scoring 0), each one's
-// own sigmoid (1), or the softmax over all experts (2; `rest`: the sum of exp(z - the largest z) over those not chosen)
+// own sigmoid (1), or the softmax over all experts (2; `rest`: the sum of exp(z - the largest z) over those not chosen);
+// scoring 3 hands in the chosen experts' sigmoids
 __device__ __forceinline__ void write_route_weights(const float* chosen, float* __restrict__ out, int top, int scoring,
-                                                    float rest) {
+                                                    float rest, float scale) {
+  if (scoring == 3) {
+    float sum = 0.f;
+    for (int k = 0; k < top; ++k) sum += chosen[k];
+    for (int k = 0; k < top; ++k) out[k] = chosen[k] / (sum + 1e-20f) * scale;
+    return;
+  }
   if (scoring == 1) {
     for (int k = 0; k < top; ++k) out[k] = 1.f / (1.f + expf(-chosen[k]));
     return;
@@ -728,15 +775,15 @@ __device__ __forceinline__ float rest_of_softmax(const float* z, int E, int lane
 template <typename X, typename W>
 __global__ void __launch_bounds__(256)
 route_topk_kernel(const X* __restrict__ x, const W* __restrict__ weight, const float* __restrict__ bias,
-                  int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int scoring) {
+                  int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int scoring, RouteRule rule) {
   extern __shared__ float xs[];                       // the token's row as float32
-  __shared__ float z[ROUTE_MAX_EXPERTS];
+  __shared__ float z[ROUTE_MAX_EXPERTS + 1], own[ROUTE_MAX_EXPERTS], strength[ROUTE_MAX_EXPERTS];
   __shared__ float chosen[ROUTE_MAX_TOP];
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
   for (int c = threadIdx.x; c < C; c += blockDim.x) xs[c] = to_float(x[t * C + c]);
   __syncthreads();
-  for (int e = wave; e < E; e += 4) {
+  for (int e = wave; e < E + rule.shared; e += 4) {
     const W* w = weight + static_cast<int64_t>(e) * C;
     float acc = 0.f;
     for (int c0 = lane; c0 < C; c0 += 64 * 8) {
@@ -751,6 +798,8 @@ route_topk_kernel(const X* __restrict__ x, const W* __restrict__ weight, const f
     if (lane == 0) z[e] = acc + (bias != nullptr ? bias[e] : 0.f);
   }
   __syncthreads();
+  if (scoring == 3) choice_scores(z, own, strength, E, rule);
+  gates += t * (top + rule.shared);
   if (wave != 0) return;
   float peak = 0.f;                                   // the largest logit
   for (int k = 0; k < top; ++k) {
@@ -771,13 +820,16 @@ route_topk_kernel(const X* __restrict__ x, const W* __restrict__ weight, const f
     if (k == 0) peak = best;
     if (lane == 0) {
       experts[t * top + k] = at;
-      chosen[k] = best;
+      chosen[k] = scoring == 3 ? own[at] : best;
     }
     if (at % 64 == lane) z[at] = -INFINITY;           // the lane that reads this place takes it out itself
   }
   float rest = 0.f;
   if (scoring == 2) rest = rest_of_softmax(z, E, lane, peak);
-  if (lane == 0) write_route_weights(chosen, gates + t * top, top, scoring, rest);
+  if (lane == 0) {
+    write_route_weights(chosen, gates, top, scoring, rest, rule.scale);
+    if (rule.shared) gates[top] = 1.f / (1.f + expf(-z[E]));
+  }
 }
 
 // The same for bfloat16 rows and weights whose width is a multiple of 8: a thread takes 16-byte pieces of the token's
@@ -797,28 +849,30 @@ __device__ __forceinline__ void unpack8(const uint4& raw, float v[8]) {
 // One row's router by one block of 256 threads: the chosen experts (largest logit first) and their weights end up in
 // `ids` and `weights` (LDS), for every thread of the block to read.
 struct RouteScratch {
-  float z[ROUTE_MAX_EXPERTS];
+  float z[ROUTE_MAX_EXPERTS + 1];
+  float own[ROUTE_MAX_EXPERTS], strength[ROUTE_MAX_EXPERTS];
   float part[4][ROUTE_GROUP];
   float chosen[ROUTE_MAX_TOP];
   int ids[ROUTE_MAX_TOP];
-  float weights[ROUTE_MAX_TOP];
+  float weights[ROUTE_MAX_TOP + 1];           // the shared expert's behind those of the chosen
 };
 
 template <int GROUP>                                   // experts worked on side by side: 16, or 8 where there are no more
 __device__ __forceinline__ void route_row_bf16(const bf16_t* __restrict__ x_row, const bf16_t* __restrict__ weight,
                                                const float* __restrict__ bias, int C, int E, int top, int scoring,
-                                               RouteScratch& lds) {
+                                               const RouteRule& rule, RouteScratch& lds) {
   static_assert(GROUP <= ROUTE_GROUP, "the scratch holds ROUTE_GROUP sums a wave");
   const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
   const int pieces = C / 8;
-  for (int e0 = 0; e0 < E; e0 += GROUP) {
+  const int rows = E + rule.shared;
+  for (int e0 = 0; e0 < rows; e0 += GROUP) {
     float acc[GROUP] = {};
     for (int p = threadIdx.x; p < pieces; p += 256) {
       uint4 raw[GROUP];
       const uint4 mine = *reinterpret_cast<const uint4*>(x_row + 8 * p);
 #pragma unroll
       for (int g = 0; g < GROUP; ++g)
-        raw[g] = *reinterpret_cast<const uint4*>(weight + static_cast<int64_t>(min(e0 + g, E - 1)) * C + 8 * p);
+        raw[g] = *reinterpret_cast<const uint4*>(weight + static_cast<int64_t>(min(e0 + g, rows - 1)) * C + 8 * p);
       float xv[8];
       unpack8(mine, xv);
 #pragma unroll
@@ -835,13 +889,14 @@ __device__ __forceinline__ void route_row_bf16(const bf16_t* __restrict__ x_row,
       if (lane == 0) lds.part[wave][g] = total;
     }
     __syncthreads();
-    if (threadIdx.x < GROUP && e0 + threadIdx.x < E) {
+    if (threadIdx.x < GROUP && e0 + threadIdx.x < rows) {
       const int e = e0 + threadIdx.x;
       lds.z[e] = lds.part[0][threadIdx.x] + lds.part[1][threadIdx.x] + lds.part[2][threadIdx.x] + lds.part[3][threadIdx.x] +
                  (bias != nullptr ? bias[e] : 0.f);
     }
     __syncthreads();
   }
+  if (scoring == 3) choice_scores(lds.z, lds.own, lds.strength, E, rule);
   if (wave == 0) {
     float peak = 0.f;
     for (int k = 0; k < top; ++k) {
@@ -861,31 +916,33 @@ __device__ __forceinline__ void route_row_bf16(const bf16_t* __restrict__ x_row,
       if (k == 0) peak = best;
       if (lane == 0) {
         lds.ids[k] = at;
-        lds.chosen[k] = best;
+        lds.chosen[k] = scoring == 3 ? lds.own[at] : best;
       }
       if (at % 64 == lane) lds.z[at] = -INFINITY;
     }
     float rest = 0.f;
     if (scoring == 2) rest = rest_of_softmax(lds.z, E, lane, peak);
-    if (lane == 0) write_route_weights(lds.chosen, lds.weights, top, scoring, rest);
+    if (lane == 0) {
+      write_route_weights(lds.chosen, lds.weights, top, scoring, rest, rule.scale);
+      if (rule.shared) lds.weights[top] = 1.f / (1.f + expf(-lds.z[E]));
+    }
   }
   __syncthreads();
 }
 
 __global__ void __launch_bounds__(256)
 route_topk_bf16_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ weight, const float* __restrict__ bias,
-                       int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int scoring) {
+                       int32_t* __restrict__ experts, float* __restrict__ gates, int C, int E, int top, int scoring,
+                       RouteRule rule) {
   __shared__ RouteScratch lds;
   const int64_t t = blockIdx.x;
-  if (E <= 8) {
-    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, lds);
+  if (E + rule.shared <= 8) {
+    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   } else {
-    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, lds);
+    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   }
-  if (threadIdx.x < top) {
-    experts[t * top + threadIdx.x] = lds.ids[threadIdx.x];
-    gates[t * top + threadIdx.x] = lds.weights[threadIdx.x];
-  }
+  if (threadIdx.x < top) experts[t * top + threadIdx.x] = lds.ids[threadIdx.x];
+  if (threadIdx.x < top + rule.shared) gates[t * (top + rule.shared) + threadIdx.x] = lds.weights[threadIdx.x];
 }
 
 // hidden [T, ld]: the columns [e * F, (e + 1) * F) of expert e times the row's weight for e, zero if e was not chosen
@@ -932,15 +989,17 @@ __global__ void route_scale_bf16x8_kernel(bf16_t* __restrict__ hidden, int64_t l
 // (E x F), then every expert's up columns; `slices` partial sums lie `stride` elements apart. For the expert e that owns
 // column c, chosen by the row with weight w: g and u times w if `on_input`, clamped if limit > 0 (g from above, u on both
 // sides), hidden = g * sigmoid(slope * g) * (u + up_shift), times w unless `on_input`; zero if the row did not choose e.
+// Both halves may end with columns of one more expert that every row uses (width > routed = E x F): its weight stands
+// behind those of a row's chosen experts (`gate_ld` weights a row).
 // V columns a thread (V > 1: F a multiple of V, rows aligned to V values). blockIdx.y walks the rows, so a row's choice is
 // the same for the whole block and is read once; blockIdx.x and the thread give the columns.
 constexpr int GLU_ROWS = 4;
 
 template <int V, typename X, typename O>
 __global__ void route_glu_kernel(const X* __restrict__ gate_up, int64_t ld, int slices, int64_t stride,
-                                 const int32_t* __restrict__ experts, const float* __restrict__ gates, int top, int F,
-                                 int width, float limit, float slope, float up_shift, int on_input, O* __restrict__ out,
-                                 int64_t T) {
+                                 const int32_t* __restrict__ experts, const float* __restrict__ gates, int gate_ld, int top,
+                                 int F, int routed, int width, float limit, float slope, float up_shift, int on_input,
+                                 O* __restrict__ out, int64_t T) {
   // Blocks go to the chip's eight dies in turn by their number (blockIdx.x fastest): with the columns taken from
   // blockIdx.x alone, the blocks of one expert's columns would all land on the same die, and where most rows choose the
   // same experts two dies would do the reading for all. The block row shifts the columns, so every die gets its share.
@@ -958,9 +1017,11 @@ __global__ void route_glu_kernel(const X* __restrict__ gate_up, int64_t ld, int 
     for (int r = 0; r < GLU_ROWS; ++r) {
       w[r] = 0.f, chosen[r] = false;
       const int64_t t = t0 + r;
-      if (t < T) {
+      if (t < T && c >= routed) {
+        w[r] = gates[t * gate_ld + top], chosen[r] = true;
+      } else if (t < T) {
         for (int k = 0; k < top; ++k)
-          if (experts[t * top + k] == e) w[r] = gates[t * top + k], chosen[r] = true;
+          if (experts[t * top + k] == e) w[r] = gates[t * gate_ld + k], chosen[r] = true;
       }
     }
 #pragma unroll
@@ -995,7 +1056,8 @@ template <int V, typename X, typename O>
 __global__ void __launch_bounds__(256)
 route_topk_glu_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ weight, const float* __restrict__ bias, int C,
                       int E, int top, int scoring, const X* __restrict__ gate_up, int64_t ld, int slices, int64_t stride,
-                      int F, int width, float limit, float slope, float up_shift, int on_input, O* __restrict__ out) {
+                      int F, int routed, int width, float limit, float slope, float up_shift, int on_input, RouteRule rule,
+                      O* __restrict__ out) {
   __shared__ RouteScratch lds;
   const int64_t t = blockIdx.y;
   const int c = V * static_cast<int>(blockIdx.x * blockDim.x + threadIdx.x);
@@ -1006,16 +1068,17 @@ route_topk_glu_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w
     sum_values<V>(gate_up + t * ld + c, slices, stride, g);
     sum_values<V>(gate_up + t * ld + width + c, slices, stride, u);
   }
-  if (E <= 8) {
-    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, lds);
+  if (E + rule.shared <= 8) {
+    route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   } else {
-    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, lds);
+    route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   }
   if (c >= width) return;
   const int e = c / F;
   float w = 0.f;
   bool chosen = false;
-  for (int k = 0; k < top; ++k)
+  if (c >= routed) w = lds.weights[top], chosen = true;
+  for (int k = 0; k < top && !chosen; ++k)
     if (lds.ids[k] == e) w = lds.weights[k], chosen = true;
   float h[V] = {};
   if (chosen) {
@@ -1222,18 +1285,25 @@ extern "C" int distie_lru_scan_chunked(const float* a, const float* x, float* st
   return launch_status();
 }
 
-// scoring: 0 softmax over the chosen, 1 sigmoid, 2 softmax over all experts
+static bool bad_rule(const RouteRule& rule, int E, int top) {
+  return rule.groups < 1 || E % rule.groups != 0 || rule.kept < 1 || rule.kept > rule.groups ||
+         top > E / rule.groups * rule.kept || rule.shared < 0 || rule.shared > 1;
+}
+
+// scoring: 0 softmax over the chosen, 1 sigmoid, 2 softmax over all experts, 3 sigmoids' shares (see RouteRule; the other
+// scorings take no correction, one group and scale 1). gates: [T, top + shared].
 extern "C" int distie_route_topk(const void* x, int x_dtype, const void* weight, int w_dtype, const float* bias,
                                  int32_t* experts, float* gates, int T, int C, int E, int top, int scoring,
-                                 hipStream_t stream) {
+                                 const float* correction, int groups, int kept, float scale, int shared, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (C < 1 || E < 1 || scoring < 0 || scoring > 2 || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP ||
+  const RouteRule rule = {correction, groups, kept, scale, shared};
+  if (C < 1 || E < 1 || scoring < 0 || scoring > 3 || bad_rule(rule, E, top) || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP ||
       static_cast<size_t>(C) * sizeof(float) > 96 * 1024)
     return DISTIE_BAD_ARGUMENT;
   if (x_dtype == DISTIE_BF16 && w_dtype == DISTIE_BF16 && C % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(weight) % 16 == 0) {
     route_topk_bf16_kernel<<<T, 256, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(weight), bias,
-                                                  experts, gates, C, E, top, scoring);
+                                                  experts, gates, C, E, top, scoring, rule);
     return launch_status();
   }
   const size_t lds = static_cast<size_t>(C) * sizeof(float);
@@ -1243,7 +1313,7 @@ extern "C" int distie_route_topk(const void* x, int x_dtype, const void* weight,
                             hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
       return DISTIE_BAD_ARGUMENT;
     route_topk_kernel<X, W><<<T, 256, lds, stream>>>(static_cast<const X*>(x), static_cast<const W*>(weight), bias,
-                                                     experts, gates, C, E, top, scoring);
+                                                     experts, gates, C, E, top, scoring, rule);
   }));
   return launch_status();
 }
@@ -1267,24 +1337,27 @@ extern "C" int distie_route_scale(void* hidden, int dtype, int64_t ld, const int
 }
 
 // gate_up: [T, ld] of `dtype`, or `slices` float32 partial sums [slices, T, ld]; out: [T, E * F] of `out_dtype`.
-// limit <= 0: no clamps.
+// limit <= 0: no clamps. shared_width: columns at the end of both halves of gate_up (and of out) that every row uses, with
+// the weight gates[t, top] (gates are then [T, top + 1]).
 extern "C" int distie_route_glu(const void* gate_up, int dtype, int64_t ld, int slices, const int32_t* experts,
                                 const float* gates, int T, int top, int E, int F, float limit, float slope, float up_shift,
-                                int on_input, void* out, int out_dtype, hipStream_t stream) {
+                                int on_input, int shared_width, void* out, int out_dtype, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (top < 1 || E < 1 || F < 1 || slices < 1 || (slices > 1 && dtype != DISTIE_F32) || ld < 2 * static_cast<int64_t>(E) * F)
+  if (top < 1 || E < 1 || F < 1 || slices < 1 || (slices > 1 && dtype != DISTIE_F32) || shared_width < 0 ||
+      ld < 2 * (static_cast<int64_t>(E) * F + shared_width))
     return DISTIE_BAD_ARGUMENT;
-  const int width = E * F;
+  const int routed = E * F, width = routed + shared_width, gate_ld = top + (shared_width > 0 ? 1 : 0);
   const int64_t stride = static_cast<int64_t>(T) * ld;
   const bool aligned = reinterpret_cast<uintptr_t>(gate_up) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
-  const int V = aligned && F % 8 == 0 && ld % 8 == 0 ? 8 : (aligned && F % 4 == 0 && ld % 4 == 0 ? 4 : 1);
+  const int step = F | shared_width;           // a multiple of what both are multiples of (powers of two)
+  const int V = aligned && step % 8 == 0 && ld % 8 == 0 ? 8 : (aligned && step % 4 == 0 && ld % 4 == 0 ? 4 : 1);
   const int per_row = width / V;
   const int threads = per_row >= 256 ? 256 : (per_row > 64 ? 128 : 64);
   const int row_groups = (T + GLU_ROWS - 1) / GLU_ROWS;
   const dim3 grid((per_row + threads - 1) / threads, row_groups < 32768 ? row_groups : 32768);
 #define DISTIE_ROUTE_GLU(V)                                                                                           \
   DISTIE_DISPATCH(dtype, X, DISTIE_DISPATCH(out_dtype, O, (route_glu_kernel<V, X, O><<<grid, threads, 0, stream>>>(   \
-      static_cast<const X*>(gate_up), ld, slices, stride, experts, gates, top, F, width, limit, slope, up_shift,      \
+      static_cast<const X*>(gate_up), ld, slices, stride, experts, gates, gate_ld, top, F, routed, width, limit, slope, up_shift, \
       on_input, static_cast<O*>(out), T))))
   if (V == 8) {
     DISTIE_ROUTE_GLU(8);
@@ -1300,22 +1373,26 @@ extern "C" int distie_route_glu(const void* gate_up, int dtype, int64_t ld, int 
 // `distie_route_topk` (bfloat16 rows and weights) and `distie_route_glu` in one launch; for steps of few rows.
 extern "C" int distie_route_topk_glu(const void* x, const void* weight, const float* bias, int C, int scoring,
                                      const void* gate_up, int dtype, int64_t ld, int slices, int T, int top, int E, int F,
-                                     float limit, float slope, float up_shift, int on_input, void* out, int out_dtype,
-                                     hipStream_t stream) {
+                                     float limit, float slope, float up_shift, int on_input, const float* correction,
+                                     int groups, int kept, float scale, int shared, int shared_width, void* out,
+                                     int out_dtype, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (C < 8 || scoring < 0 || scoring > 2 || C % 8 || E < 1 || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP || F < 1 || slices < 1 ||
-      T > 65535 || (slices > 1 && dtype != DISTIE_F32) || ld < 2 * static_cast<int64_t>(E) * F ||
+  const RouteRule rule = {correction, groups, kept, scale, shared};
+  if (shared_width < 0 || (shared_width > 0 && !shared) || bad_rule(rule, E, top)) return DISTIE_BAD_ARGUMENT;
+  if (C < 8 || scoring < 0 || scoring > 3 || C % 8 || E < 1 || E > ROUTE_MAX_EXPERTS || top < 1 || top > E || top > ROUTE_MAX_TOP || F < 1 || slices < 1 ||
+      T > 65535 || (slices > 1 && dtype != DISTIE_F32) || ld < 2 * (static_cast<int64_t>(E) * F + shared_width) ||
       reinterpret_cast<uintptr_t>(x) % 16 != 0 || reinterpret_cast<uintptr_t>(weight) % 16 != 0)
     return DISTIE_BAD_ARGUMENT;
-  const int width = E * F;
+  const int routed = E * F, width = routed + shared_width;
   const int64_t stride = static_cast<int64_t>(T) * ld;
   const bool aligned = reinterpret_cast<uintptr_t>(gate_up) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
-  const int V = aligned && F % 8 == 0 && ld % 8 == 0 ? 8 : (aligned && F % 4 == 0 && ld % 4 == 0 ? 4 : 1);
+  const int step = F | shared_width;
+  const int V = aligned && step % 8 == 0 && ld % 8 == 0 ? 8 : (aligned && step % 4 == 0 && ld % 4 == 0 ? 4 : 1);
   const dim3 grid((width / V + 255) / 256, T);
 #define DISTIE_ROUTE_TOPK_GLU(V)                                                                                          \
   DISTIE_DISPATCH(dtype, X, DISTIE_DISPATCH(out_dtype, O, (route_topk_glu_kernel<V, X, O><<<grid, 256, 0, stream>>>(       \
       static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(weight), bias, C, E, top, scoring,                        \
-      static_cast<const X*>(gate_up), ld, slices, stride, F, width, limit, slope, up_shift, on_input, static_cast<O*>(out)))))
+      static_cast<const X*>(gate_up), ld, slices, stride, F, routed, width, limit, slope, up_shift, on_input, rule, static_cast<O*>(out)))))
   if (V == 8) {
     DISTIE_ROUTE_TOPK_GLU(8);
   } else if (V == 4) {

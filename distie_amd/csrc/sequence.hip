@@ -264,8 +264,8 @@ __global__ void conv_state_kernel(const X* __restrict__ x, int64_t ldx, int taps
 // ---------------------------------------------------------------------------------------------------
 // Behind the stacked projection of attention: product [T, ld] holds q (H heads of D), then k (G heads of D) and
 // v (G heads of E) unless `has_kv` is 0. Each channel goes through its short convolution (taps 0: none); the
-// first 2 * pairs dimensions of every q and k head are turned by the token's angle (pair (j, j + pairs); cosine
-// and sine from `table` [T, pairs, 2], both times `magnitude`); q goes to q_out [T, H, DP] (zeros beyond D), k
+// first 2 * pairs dimensions of every q and k head are turned by the token's angle (pair (j, j + pairs), or (2j, 2j + 1)
+// with `neighbours`; cosine and sine from `table` [T, pairs, 2], both times `magnitude`); q goes to q_out [T, H, DP] (zeros beyond D), k
 // and v to the token's slot of the cache, k [pages, G, P, DP], v [pages, G, DP, P] (what lies beyond D and E there
 // was zero when the cache was made and is never written).
 // One block a (token, head): q heads, then k heads, then v heads. A thread owns its channels alone, so for a request
@@ -279,7 +279,8 @@ __global__ void conv_rope_kv_write_kernel(const X* __restrict__ product, int64_t
                                           const int32_t* __restrict__ state_slots, int H, int G, int D, int E, int DP,
                                           int block_size, int has_kv, int write, const int32_t* __restrict__ positions,
                                           float temp_coef, int temp_every, const float* __restrict__ q_norm,
-                                          const float* __restrict__ k_norm, float norm_eps, int slices, int64_t stride, int v_base) {
+                                          const float* __restrict__ k_norm, float norm_eps, int slices, int64_t stride, int v_base,
+                                          int neighbours) {
   // slices > 1 (taps 0 only): the product is partial sums that lie `stride` elements apart, added in order while read
   const int64_t t = blockIdx.x;
   const int head = blockIdx.y;
@@ -327,8 +328,8 @@ __global__ void conv_rope_kv_write_kernel(const X* __restrict__ product, int64_t
   int d0 = -1, d1 = -1;
   if (j < DP - pairs) {
     if (j < pairs) {
-      d0 = j;
-      d1 = j + pairs;
+      d0 = neighbours ? 2 * j : j;
+      d1 = neighbours ? 2 * j + 1 : j + pairs;
       x0 = value(base + d0);
       x1 = value(base + d1);
     } else {
@@ -443,11 +444,40 @@ __global__ void activation_kernel(const I* __restrict__ in, int slices, int64_t 
 // v (H x E). state float32 [slots, H, D, E]. A block owns 64 columns e of one head of one request and walks the
 // request's rows in order; thread (e, part) keeps rows d = part, part + PARTS, ... of its column in registers,
 // the PARTS partial sums of a column meet in LDS.
-template <typename X, int PARTS, int ROWS>
+// SILU false: q, k and v are the product's columns as they are; the first 2 * pairs dimensions of every q and k head are
+// turned by the row's angles (`table` [T, pairs, 2]; pair (j, j + pairs), or (2j, 2j + 1) with `neighbours`), and k is
+// multiplied by k_scale.
+struct ScanTurn {
+  const float2* table;
+  int pairs, neighbours;
+  float k_scale;
+};
+
+// dimension d of the q or k head whose columns begin at `head`, row t; SILU: the column itself (silu is the caller's)
+template <bool SILU, typename X>
+__device__ __forceinline__ float scan_value(const X* __restrict__ head, int d, int64_t t, const ScanTurn& turn) {
+  const float x = to_float(head[d]);
+  if constexpr (!SILU) {
+    if (d < 2 * turn.pairs) {
+      const bool first = turn.neighbours ? d % 2 == 0 : d < turn.pairs;
+      const int j = turn.neighbours ? d / 2 : (first ? d : d - turn.pairs);
+      const int step = turn.neighbours ? 1 : turn.pairs;
+      const float other = to_float(head[first ? d + step : d - step]);
+      const float2 cs = turn.table[t * turn.pairs + j];
+      return first ? x * cs.x - other * cs.y : x * cs.x + other * cs.y;
+    }
+  }
+  return x;
+}
+
+template <bool SILU>
+__device__ __forceinline__ float scan_act(float x) { return SILU ? siluf(x) : x; }
+
+template <bool SILU, typename X, int PARTS, int ROWS>
 __global__ void __launch_bounds__(64 * PARTS)
 decay_scan_kernel(const X* __restrict__ product, int64_t ld, float* __restrict__ state, const float* __restrict__ decay,
                   float* __restrict__ out, const int32_t* __restrict__ cu_q, const int32_t* __restrict__ state_slots,
-                  int H, int D, int E) {
+                  int H, int D, int E, ScanTurn turn) {
   __shared__ float q_s[PARTS * ROWS], k_s[PARTS * ROWS];
   __shared__ float partial[PARTS][64];
   const int b = blockIdx.x, head = blockIdx.y;
@@ -466,10 +496,10 @@ decay_scan_kernel(const X* __restrict__ product, int64_t ld, float* __restrict__
     const X* row = product + static_cast<int64_t>(t) * ld;
     __syncthreads();
     for (int d = threadIdx.x; d < D; d += blockDim.x) {
-      q_s[d] = siluf(to_float(row[head * D + d]));
-      k_s[d] = siluf(to_float(row[(H + head) * D + d]));
+      q_s[d] = scan_act<SILU>(scan_value<SILU>(row + head * D, d, t, turn));
+      k_s[d] = scan_act<SILU>(scan_value<SILU>(row + (H + head) * D, d, t, turn)) * (SILU ? 1.f : turn.k_scale);
     }
-    const float v = e < E ? siluf(to_float(row[2 * H * D + head * E + e])) : 0.f;
+    const float v = e < E ? scan_act<SILU>(to_float(row[2 * H * D + head * E + e])) : 0.f;
     __syncthreads();
     float o = 0.f;
 #pragma unroll
@@ -674,6 +704,7 @@ __global__ void causal_conv_bf16_taps_kernel(const bf16_t* __restrict__ x, int64
 // single dimensions). The blocks behind them: v for 16 tokens each; a thread owns one channel of v and, where
 // the 16 tokens lie side by side in one page, writes their values as one run of 32 bytes (the cache keeps v with
 // the key index innermost).
+// `neighbours`: the eight pairs of an item are (2j, 2j + 1), its sixteen dimensions lie side by side.
 // NORM: every q and k head first goes through x / sqrt(mean(x^2) + norm_eps) * weight over its D values (behind the
 // convolution, in front of the rotation): a first walk over the items leaves each item's sum of squares in LDS, and
 // an item of the second walk adds up those of its head, in their order.
@@ -696,7 +727,7 @@ __global__ void conv_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ produc
                                                int DP, int block_size, int has_kv, int write,
                                                const int32_t* __restrict__ positions, float temp_coef, int temp_every,
                                                const float* __restrict__ q_norm, const float* __restrict__ k_norm,
-                                               float norm_eps) {
+                                               float norm_eps, int neighbours) {
   extern __shared__ float squares[];                     // NORM: [heads of q and k, items of a head]
   const int N = H * D + (has_kv ? G * (D + E) : 0);
   if (static_cast<int>(blockIdx.x) >= T) {
@@ -773,13 +804,13 @@ __global__ void conv_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ produc
     for (int item = threadIdx.x; item < turned * per_head; item += blockDim.x) {
       const int j8 = item % per_head;
       const int base = item / per_head * D;
-      const int d0 = j8 < pair8 ? 8 * j8 : 2 * pairs + 8 * (j8 - pair8);
+      const int d0 = j8 < pair8 ? (neighbours ? 16 : 8) * j8 : 2 * pairs + 8 * (j8 - pair8);
       float x[8] = {}, self[8], sq = 0.f;
       if (d0 < D) conv8(product, ld, own, weight, taps, t, i, base + d0, N, x, self);
 #pragma unroll
       for (int e = 0; e < 8; ++e) sq += x[e] * x[e];
       if (j8 < pair8) {
-        conv8(product, ld, own, weight, taps, t, i, base + d0 + pairs, N, x, self);
+        conv8(product, ld, own, weight, taps, t, i, base + d0 + (neighbours ? 8 : pairs), N, x, self);
 #pragma unroll
         for (int e = 0; e < 8; ++e) sq += x[e] * x[e];
       }
@@ -805,7 +836,7 @@ __global__ void conv_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ produc
       }
     }
     if (j8 < pair8) {
-      const int d0 = 8 * j8, d1 = d0 + pairs;
+      const int d0 = (neighbours ? 16 : 8) * j8, d1 = d0 + (neighbours ? 8 : pairs);
       float x0[8], x1[8], s0[8], s1[8], a[8], c[8];
       conv8(product, ld, own, weight, taps, t, i, base + d0, N, x0, s0);
       conv8(product, ld, own, weight, taps, t, i, base + d1, N, x1, s1);
@@ -816,10 +847,20 @@ __global__ void conv_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ produc
 #pragma unroll
         for (int e = 0; e < 8; ++e) x0[e] *= r * w0[e], x1[e] *= r * w1[e];
       }
-      const float4* angles = reinterpret_cast<const float4*>(table + t * pairs + d0);       // (cos, sin) x 8
+      const float4* angles = reinterpret_cast<const float4*>(table + t * pairs + 8 * j8);   // (cos, sin) x 8
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const float4 cs = angles[e];
+        if (neighbours) {
+          // pairs 2e and 2e + 1 of the item are values 4e .. 4e + 3 of (x0, x1): all four in one half
+          const float* v = e < 2 ? x0 + 4 * e : x1 + 4 * (e - 2);
+          float* to = e < 2 ? a + 4 * e : c + 4 * (e - 2);
+          to[0] = v[0] * (cs.x * magnitude) - v[1] * (cs.y * magnitude);
+          to[1] = v[1] * (cs.x * magnitude) + v[0] * (cs.y * magnitude);
+          to[2] = v[2] * (cs.z * magnitude) - v[3] * (cs.w * magnitude);
+          to[3] = v[3] * (cs.z * magnitude) + v[2] * (cs.w * magnitude);
+          continue;
+        }
         a[2 * e] = x0[2 * e] * (cs.x * magnitude) - x1[2 * e] * (cs.y * magnitude);
         c[2 * e] = x1[2 * e] * (cs.x * magnitude) + x0[2 * e] * (cs.y * magnitude);
         a[2 * e + 1] = x0[2 * e + 1] * (cs.z * magnitude) - x1[2 * e + 1] * (cs.w * magnitude);
@@ -1026,10 +1067,10 @@ __device__ __forceinline__ void decay_powers(float* pw, float rate, int count) {
   }
 }
 
-template <typename X>
+template <bool SILU, typename X>
 __global__ void __launch_bounds__(256)
 scan_chunk_sums_kernel(const X* __restrict__ product, int64_t ld, const float* __restrict__ decay, float* __restrict__ scratch,
-                       const int4* __restrict__ chunks, int H, int D, int E) {
+                       const int4* __restrict__ chunks, int H, int D, int E, ScanTurn turn) {
   extern __shared__ float lds[];
   float* Ks = lds;                       // [64][D], each row times its power of the decay
   float* Vs = Ks + SCAN_L * D;           // [64][64]
@@ -1049,12 +1090,12 @@ scan_chunk_sums_kernel(const X* __restrict__ product, int64_t ld, const float* _
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
-        k[u] = j < len ? to_float(product[(row0 + j) * ld + (H + head) * D + d]) : 0.f;
+        k[u] = j < len ? scan_value<SILU>(product + (row0 + j) * ld + (H + head) * D, d, row0 + j, turn) : 0.f;
       }
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
-        Ks[j * D + d] = j < len ? pw[len - 1 - j] * siluf(k[u]) : 0.f;
+        Ks[j * D + d] = j < len ? pw[len - 1 - j] * (SILU ? siluf(k[u]) : k[u] * turn.k_scale) : 0.f;
       }
     }
     float v[SCAN_BATCH];
@@ -1064,7 +1105,7 @@ scan_chunk_sums_kernel(const X* __restrict__ product, int64_t ld, const float* _
       v[u] = (j < len && e0 + col < E) ? to_float(product[(row0 + j) * ld + 2 * H * D + head * E + e0 + col]) : 0.f;
     }
 #pragma unroll
-    for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = siluf(v[u]);
+    for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = scan_act<SILU>(v[u]);
   }
   __syncthreads();
   const int tx = threadIdx.x % 16, ty = threadIdx.x / 16;
@@ -1136,11 +1177,11 @@ __global__ void scan_chunk_states_kernel(float* __restrict__ scratch, float* __r
   *own = S;
 }
 
-template <typename X>
+template <bool SILU, typename X>
 __global__ void __launch_bounds__(256)
 scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float* __restrict__ decay,
                           const float* __restrict__ scratch, float* __restrict__ out, const int4* __restrict__ chunks,
-                          int H, int D, int E) {
+                          int H, int D, int E, ScanTurn turn) {
   extern __shared__ float lds[];
   float* Qt = lds;                       // [D][68]: Qt[d][i]
   float* Kt = Qt + D * SCAN_PAD;         // [D][68]; once the scores are made, the state in front of the chunk [D][64]
@@ -1160,14 +1201,14 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
         const X* row = product + (row0 + j) * ld;
-        q[u] = j < len ? to_float(row[head * D + d]) : 0.f;
-        k[u] = j < len ? to_float(row[(H + head) * D + d]) : 0.f;
+        q[u] = j < len ? scan_value<SILU>(row + head * D, d, row0 + j, turn) : 0.f;
+        k[u] = j < len ? scan_value<SILU>(row + (H + head) * D, d, row0 + j, turn) : 0.f;
       }
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
-        Qt[d * SCAN_PAD + j] = siluf(q[u]);
-        Kt[d * SCAN_PAD + j] = siluf(k[u]);
+        Qt[d * SCAN_PAD + j] = scan_act<SILU>(q[u]);
+        Kt[d * SCAN_PAD + j] = SILU ? siluf(k[u]) : k[u] * turn.k_scale;
       }
     }
     float v[SCAN_BATCH];
@@ -1177,7 +1218,7 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
       v[u] = (j < len && e0 + col < E) ? to_float(product[(row0 + j) * ld + 2 * H * D + head * E + e0 + col]) : 0.f;
     }
 #pragma unroll
-    for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = siluf(v[u]);
+    for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = scan_act<SILU>(v[u]);
   }
   __syncthreads();
   const int tx = threadIdx.x % 16, ty = threadIdx.x / 16;
@@ -1361,7 +1402,9 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
                                          const int32_t* cu_q, const int32_t* token_request, const int32_t* state_slots,
                                          int T, int H, int G, int D, int E, int DP, int block_size, int has_kv, int write,
                                          const int32_t* positions, float temp_coef, int temp_every, const float* q_norm,
-                                         const float* k_norm, float norm_eps, int slices, int q_dtype, hipStream_t stream) {
+                                         const float* k_norm, float norm_eps, int slices, int q_dtype, int neighbours,
+                                         hipStream_t stream) {
+  // neighbours: the rotation's pairs are (2j, 2j + 1) instead of (j, j + pairs)
   // slices > 1: `product` is float32 partial sums [slices, T, ld] (no convolution then); q_out is of `q_dtype`
   // temp_every >= 1: q of the token at position p times 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)
   // has_kv 2: the product holds no columns of v; the values are the columns of k as they are (E is D, no convolution)
@@ -1384,7 +1427,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
   const int64_t stride = static_cast<int64_t>(T) * ld;
   const bool normed = q_norm != nullptr || k_norm != nullptr;
   const int norm_items = (has_kv ? H + G : H) * ((DP - pairs) / 8);
-  if ((!tied || (normed && DP <= 512)) && (!normed || (static_cast<size_t>(norm_items) * sizeof(float) <= 48 * 1024 && D % 8 == 0 && pairs % 4 == 0 &&
+  if ((!tied || (normed && DP <= 512 && !neighbours)) && (!normed || (static_cast<size_t>(norm_items) * sizeof(float) <= 48 * 1024 && D % 8 == 0 && pairs % 4 == 0 &&
                    reinterpret_cast<uintptr_t>(q_norm) % 16 == 0 && reinterpret_cast<uintptr_t>(k_norm) % 16 == 0)) &&
       dtype == DISTIE_BF16 && q_dtype == DISTIE_BF16 && (weight == nullptr || w_dtype == DISTIE_BF16) && (!write || cache_dtype == DISTIE_BF16) &&
       T >= 32 && D % 8 == 0 && E % 8 == 0 && DP % 8 == 0 && pairs % 8 == 0 && ld % 8 == 0 &&
@@ -1393,7 +1436,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
     // with head norms a thread walks its items twice: as many threads as items (up to 512), so that it has one
     const int threads8 = normed && items <= 512 ? (items + 63) / 64 * 64 : (items > 128 ? 256 : (items > 64 ? 128 : 64));
     const int v_blocks = has_kv && (write || taps > 1) ? (T + VGROUP - 1) / VGROUP * G : 0;
-    if (normed && taps == 0 && DP <= 512) {
+    if (normed && taps == 0 && DP <= 512 && !neighbours) {
       const int64_t units = static_cast<int64_t>(T) * (has_kv ? H + G : H);
       int lanes = 1;
       while (8 * lanes < DP) lanes *= 2;
@@ -1411,7 +1454,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
         static_cast<const bf16_t*>(product), ld, static_cast<const bf16_t*>(weight), taps, state,                         \
         static_cast<const float2*>(table), pairs, magnitude, static_cast<bf16_t*>(q_out), static_cast<bf16_t*>(k_cache),  \
         static_cast<bf16_t*>(v_cache), slots, cu_q, token_request, state_slots, T, H, G, D, E, DP, block_size, has_kv,    \
-        write, positions, temp_coef, temp_every, q_norm, k_norm, norm_eps)
+        write, positions, temp_coef, temp_every, q_norm, k_norm, norm_eps, neighbours)
     if (normed) {
       DISTIE_CONV_ROPE_BF16(true, static_cast<size_t>(norm_items) * sizeof(float));
     } else {
@@ -1432,7 +1475,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
             static_cast<const float*>(product), ld, nullptr, taps, state, static_cast<const float2*>(table),
             pairs, magnitude, static_cast<Q*>(q_out), static_cast<C*>(k_cache), static_cast<C*>(v_cache), slots, cu_q,
             token_request, state_slots, H, G, D, E, DP, block_size, has_kv, write, positions, temp_coef, temp_every,
-            q_norm, k_norm, norm_eps, slices, stride, v_base)));
+            q_norm, k_norm, norm_eps, slices, stride, v_base, neighbours)));
     return launch_status();
   }
   DISTIE_DISPATCH(dtype, X, DISTIE_DISPATCH(w_dtype, W, DISTIE_DISPATCH(cache_dtype, C,
@@ -1440,7 +1483,7 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
           static_cast<const X*>(product), ld, static_cast<const W*>(weight), taps, state, static_cast<const float2*>(table),
           pairs, magnitude, static_cast<X*>(q_out), static_cast<C*>(k_cache), static_cast<C*>(v_cache), slots, cu_q,
           token_request, state_slots, H, G, D, E, DP, block_size, has_kv, write, positions, temp_coef, temp_every,
-          q_norm, k_norm, norm_eps, slices, stride, v_base))));
+          q_norm, k_norm, norm_eps, slices, stride, v_base, neighbours))));
   return launch_status();
 }
 
@@ -1515,15 +1558,25 @@ extern "C" int distie_activation(const void* in, int in_dtype, int slices, void*
 // the largest per-head key size the scan takes (rows of the state a thread keeps: PARTS x ROWS)
 extern "C" int distie_decay_scan_max_dim() { return 256; }
 
+// silu: q, k and v are the silu of the product's columns; else the columns as they are, q and k turned by `table` ([T,
+// pairs, 2]; null: not turned) and k times k_scale (see ScanTurn)
 extern "C" int distie_decay_scan(const void* product, int dtype, int64_t ld, float* state, const float* decay, float* out,
-                                 const int32_t* cu_q, const int32_t* state_slots, int B, int H, int D, int E,
-                                 hipStream_t stream) {
+                                 const int32_t* cu_q, const int32_t* state_slots, int B, int H, int D, int E, int silu,
+                                 const void* table, int pairs, int neighbours, float k_scale, hipStream_t stream) {
   if (B <= 0) return 0;
+  if (pairs < 0 || 2 * pairs > D || (pairs > 0 && (table == nullptr || silu))) return DISTIE_BAD_ARGUMENT;
+  const ScanTurn turn = {static_cast<const float2*>(table), pairs, neighbours, k_scale};
   if (H < 1 || D < 1 || E < 1 || D > 256 || ld < static_cast<int64_t>(H) * (2 * D + E)) return DISTIE_BAD_ARGUMENT;
   const dim3 grid(B, H, (E + 63) / 64);
 #define DISTIE_SCAN(PARTS, ROWS)                                                                                     \
-  DISTIE_DISPATCH(dtype, X, decay_scan_kernel<X, PARTS, ROWS><<<grid, 64 * PARTS, 0, stream>>>(                      \
-      static_cast<const X*>(product), ld, state, decay, out, cu_q, state_slots, H, D, E))
+  DISTIE_DISPATCH(dtype, X, {                                                                                        \
+    if (silu)                                                                                                        \
+      decay_scan_kernel<true, X, PARTS, ROWS><<<grid, 64 * PARTS, 0, stream>>>(                                      \
+          static_cast<const X*>(product), ld, state, decay, out, cu_q, state_slots, H, D, E, turn);                  \
+    else                                                                                                             \
+      decay_scan_kernel<false, X, PARTS, ROWS><<<grid, 64 * PARTS, 0, stream>>>(                                     \
+          static_cast<const X*>(product), ld, state, decay, out, cu_q, state_slots, H, D, E, turn);                  \
+  })
   if (D <= 32) {
     DISTIE_SCAN(4, 8);
   } else if (D <= 64) {
@@ -1552,9 +1605,12 @@ static int more_lds(K kernel, size_t lds) {
 // request_chunks: int32 [B + 1], the first chunk of every request; scratch: float32 [num_chunks, H, D, E]
 extern "C" int distie_decay_scan_chunked(const void* product, int dtype, int64_t ld, float* state, const float* decay,
                                          float* out, float* scratch, const int32_t* chunks, const int32_t* request_chunks,
-                                         const int32_t* state_slots, int num_chunks, int B, int H, int D, int E,
+                                         const int32_t* state_slots, int num_chunks, int B, int H, int D, int E, int silu,
+                                         const void* turn_table, int pairs, int neighbours, float k_scale,
                                          hipStream_t stream) {
   if (B <= 0 || num_chunks <= 0) return 0;
+  if (pairs < 0 || 2 * pairs > D || (pairs > 0 && (turn_table == nullptr || silu))) return DISTIE_BAD_ARGUMENT;
+  const ScanTurn turn = {static_cast<const float2*>(turn_table), pairs, neighbours, k_scale};
   if (H < 1 || D < 4 || E < 4 || D % 4 || E % 4 || D > 128 || ld < static_cast<int64_t>(H) * (2 * D + E))
     return DISTIE_BAD_ARGUMENT;
   const dim3 grid(num_chunks, H, (E + 63) / 64);
@@ -1563,17 +1619,18 @@ extern "C" int distie_decay_scan_chunked(const void* product, int dtype, int64_t
   const size_t lds_out = (2 * static_cast<size_t>(D) * SCAN_PAD + SCAN_L * SCAN_PAD + SCAN_L * 64 + SCAN_L + 2) * sizeof(float);
   int status = 0;
   DISTIE_DISPATCH(dtype, X, {
-    if ((status = more_lds(scan_chunk_sums_kernel<X>, lds_sums)) != 0) return status;
-    scan_chunk_sums_kernel<X><<<grid, 256, lds_sums, stream>>>(static_cast<const X*>(product), ld, decay, scratch, table, H, D, E);
+    const auto kernel = silu ? scan_chunk_sums_kernel<true, X> : scan_chunk_sums_kernel<false, X>;
+    if ((status = more_lds(kernel, lds_sums)) != 0) return status;
+    kernel<<<grid, 256, lds_sums, stream>>>(static_cast<const X*>(product), ld, decay, scratch, table, H, D, E, turn);
   });
   if ((status = launch_status()) != 0) return status;
   scan_chunk_states_kernel<<<dim3(B, H, (D * E + 255) / 256), 256, 0, stream>>>(scratch, state, decay, table, request_chunks,
                                                                                state_slots, H, D, E);
   if ((status = launch_status()) != 0) return status;
   DISTIE_DISPATCH(dtype, X, {
-    if ((status = more_lds(scan_chunk_outputs_kernel<X>, lds_out)) != 0) return status;
-    scan_chunk_outputs_kernel<X><<<grid, 256, lds_out, stream>>>(static_cast<const X*>(product), ld, decay, scratch, out, table,
-                                                                H, D, E);
+    const auto kernel = silu ? scan_chunk_outputs_kernel<true, X> : scan_chunk_outputs_kernel<false, X>;
+    if ((status = more_lds(kernel, lds_out)) != 0) return status;
+    kernel<<<grid, 256, lds_out, stream>>>(static_cast<const X*>(product), ld, decay, scratch, out, table, H, D, E, turn);
   });
   return launch_status();
 }

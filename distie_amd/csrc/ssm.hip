@@ -328,21 +328,29 @@ __global__ void gate_rmsnorm_kernel(const float* __restrict__ x, const W* __rest
   }
 }
 
+// act(g) * u; kind 4: g and u clamped (g from above, u on both sides) and g * sigmoid(slope * g) * (u + up_shift)
+__device__ __forceinline__ float glu_value(float g, float u, int kind, float limit, float slope, float up_shift) {
+  if (kind != 4) return activate(g, kind) * u;
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + expf(-slope * g)) * (u + up_shift);
+}
+
 // out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i], the input a sum of `slices` partial sums
 template <typename X, typename O>
 __global__ void glu_mul_kernel(const X* __restrict__ gate_up, int slices, int64_t slice_stride, O* __restrict__ out,
-                               int rows, int inter, int kind) {
+                               int rows, int inter, int kind, float limit, float slope, float up_shift) {
   const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (i >= static_cast<int64_t>(rows) * inter) return;
   const int64_t t = i / inter, c = i % inter;
   const float g = sum_strided(gate_up + t * 2 * inter + c, slices, slice_stride);
   const float u = sum_strided(gate_up + t * 2 * inter + inter + c, slices, slice_stride);
-  out[i] = from_float<O>(activate(g, kind) * u);
+  out[i] = from_float<O>(glu_value(g, u, kind, limit, slope, up_shift));
 }
 
 // bfloat16 in and out, one slice, inter a multiple of 8: 16-byte loads and stores
 __global__ void glu_mul_bf16x8_kernel(const uint4* __restrict__ gate_up, uint4* __restrict__ out, int64_t rows,
-                                      int inter8, int kind) {
+                                      int inter8, int kind, float limit, float slope, float up_shift) {
   const int64_t total = rows * inter8;
   for (int64_t i = blockIdx.x * static_cast<int64_t>(blockDim.x) + threadIdx.x; i < total;
        i += static_cast<int64_t>(gridDim.x) * blockDim.x) {
@@ -356,8 +364,8 @@ __global__ void glu_mul_bf16x8_kernel(const uint4* __restrict__ gate_up, uint4* 
     for (int e = 0; e < 4; ++e) {
       const float g0 = __uint_as_float(gw[e] << 16), g1 = __uint_as_float(gw[e] & 0xffff0000u);
       const float u0 = __uint_as_float(uw[e] << 16), u1 = __uint_as_float(uw[e] & 0xffff0000u);
-      const bf16_t lo = static_cast<bf16_t>(activate(g0, kind) * u0);
-      const bf16_t hi = static_cast<bf16_t>(activate(g1, kind) * u1);
+      const bf16_t lo = static_cast<bf16_t>(glu_value(g0, u0, kind, limit, slope, up_shift));
+      const bf16_t hi = static_cast<bf16_t>(glu_value(g1, u1, kind, limit, slope, up_shift));
       ow[e] = static_cast<uint32_t>(__builtin_bit_cast(uint16_t, lo)) |
               (static_cast<uint32_t>(__builtin_bit_cast(uint16_t, hi)) << 16);
     }
@@ -443,21 +451,23 @@ extern "C" int distie_gate_rmsnorm(const float* x, const void* weight, int w_dty
 }
 
 extern "C" int distie_glu_mul(const void* gate_up, int in_dtype, int slices, void* out, int dtype, int rows, int inter,
-                              int kind, hipStream_t stream) {
+                              int kind, float limit, float slope, float up_shift, hipStream_t stream) {
+  // kind 4: the clamped one (limit, slope and up_shift are its own)
   if (rows <= 0 || inter <= 0) return 0;
-  if (kind < 0 || kind > 3 || slices < 1) return DISTIE_BAD_ARGUMENT;
+  if (kind < 0 || kind > 4 || slices < 1 || (kind == 4 && !(limit > 0.f))) return DISTIE_BAD_ARGUMENT;
   if (in_dtype == DISTIE_BF16 && dtype == DISTIE_BF16 && slices == 1 && inter % 8 == 0 &&
       reinterpret_cast<uintptr_t>(gate_up) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0) {
     const int64_t pieces = static_cast<int64_t>(rows) * (inter / 8);
     const int blocks8 = static_cast<int>(pieces / 256 + 1 < 16384 ? pieces / 256 + 1 : 16384);
     glu_mul_bf16x8_kernel<<<blocks8, 256, 0, stream>>>(static_cast<const uint4*>(gate_up), static_cast<uint4*>(out), rows,
-                                                       inter / 8, kind);
+                                                       inter / 8, kind, limit, slope, up_shift);
     return launch_status();
   }
   const int64_t count = static_cast<int64_t>(rows) * inter;
   const int64_t blocks = (count + 255) / 256;
   if (blocks > 0x7fffffff) return DISTIE_BAD_ARGUMENT;
   DISTIE_DISPATCH(in_dtype, X, DISTIE_DISPATCH(dtype, O, glu_mul_kernel<X, O><<<static_cast<unsigned>(blocks), 256, 0, stream>>>(
-      static_cast<const X*>(gate_up), slices, static_cast<int64_t>(rows) * 2 * inter, static_cast<O*>(out), rows, inter, kind)));
+      static_cast<const X*>(gate_up), slices, static_cast<int64_t>(rows) * 2 * inter, static_cast<O*>(out), rows, inter, kind, limit, slope,
+      up_shift)));
   return launch_status();
 }

@@ -20,7 +20,7 @@ import numpy as np
 import torch
 
 from ..csrc import build
-from .interface import BatchMeta, Ops
+from .interface import BatchMeta, Ops, RouteRule
 
 _log = logging.getLogger(__name__)
 
@@ -303,8 +303,8 @@ class HipOps(Ops):
         o.distie_gemm_skinny_slices.argtypes = [_I, _I, _I]
         o.distie_gemm_skinny_bf16.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _P]
         o.distie_pack_rows.argtypes = [_P, _P, _P, _I, _I, _P]
-        o.distie_gemm_packed_bf16.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _P]
-        o.distie_gemm_packed_wide_bf16.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P]
+        o.distie_gemm_packed_bf16.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _F, _P]
+        o.distie_gemm_packed_wide_bf16.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P]
         o.distie_gemm_packed_wide_slices.argtypes = [_I, _I]
         o.distie_gemm_packed_wide_qkv_bf16.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
         o.distie_gemm_packed_rotary_bf16.argtypes = [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
@@ -317,7 +317,7 @@ class HipOps(Ops):
         o.distie_causal_conv.argtypes = [_P, _I, _L, _P, _I, _I, _P, _P, _I, _L, _I, _P, _P, _P, _P, _I, _I, _P]
         o.distie_conv_state.argtypes = [_P, _I, _L, _I, _P, _P, _P, _I, _I, _I, _P]
         o.distie_conv_rope_kv_write.argtypes = [_P, _I, _L, _P, _I, _I, _P, _P, _I, _F, _P, _P, _P, _I, _P, _P, _P, _P,
-                                                _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _F, _I, _P, _P, _F, _I, _I, _P]
+                                                _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _F, _I, _P, _P, _F, _I, _I, _I, _P]
         o.distie_sigmoid_gate.argtypes = [_P, _I, _I, _I, _P, _I, _L, _P, _I, _I, _I, _P]
         o.distie_rmsnorm_gate.argtypes = [_P, _P, _I, _F, _P, _I, _L, _P, _I, _I, _I, _I, _I, _I, _P]
         o.distie_norm_chain.argtypes = [_P, _I, _I, _P, _P, _I, _I, _P, _F, _F, _P, _F, _P, _P, _F, _P, _I, _P, _I, _I, _P]
@@ -326,15 +326,18 @@ class HipOps(Ops):
         o.distie_lru_gates.argtypes = [_P, _I, _L, _P, _P, _P, _P, _I, _P, _F, _P, _P, _I, _I, _I, _P]
         o.distie_lru_scan.argtypes = [_P, _P, _P, _P, _I, _L, _I, _P, _I, _P, _P, _I, _I, _P]
         o.distie_lru_scan_chunked.argtypes = [_P, _P, _P, _P, _P, _P, _P, _I, _L, _I, _P, _I, _P, _P, _P, _I, _I, _I, _P]
-        o.distie_route_topk.argtypes = [_P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _P]
-        o.distie_route_glu.argtypes = [_P, _I, _L, _I, _P, _P, _I, _I, _I, _I, _F, _F, _F, _I, _P, _I, _P]
-        o.distie_route_topk_glu.argtypes = [_P, _P, _P, _I, _I, _P, _I, _L, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P, _I, _P]
+        o.distie_route_topk.argtypes = [_P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _P, _I, _I, _F, _I, _P]
+        o.distie_route_glu.argtypes = [_P, _I, _L, _I, _P, _P, _I, _I, _I, _I, _F, _F, _F, _I, _I, _P, _I, _P]
+        o.distie_route_topk_glu.argtypes = [_P, _P, _P, _I, _I, _P, _I, _L, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P, _I, _I, _F, _I, _I, _P, _I, _P]
         o.distie_softcap_f32.argtypes = [_P, _L, _F, _P]
         o.distie_route_scale.argtypes = [_P, _I, _L, _P, _P, _I, _I, _I, _I, _P]
         o.distie_scale_f32.argtypes = [_P, _L, _F, _P]
         o.distie_activation.argtypes = [_P, _I, _I, _P, _I, _L, _I, _P]
-        o.distie_decay_scan.argtypes = [_P, _I, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P]
-        o.distie_decay_scan_chunked.argtypes = [_P, _I, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P]
+        o.distie_decay_scan.argtypes = [_P, _I, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P]
+        o.distie_decay_scan_chunked.argtypes = [_P, _I, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P]
+        o.distie_delta_scan.argtypes = [_P, _I, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _P]
+        o.distie_delta_scan_chunked.argtypes = [_P, _I, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P,
+                                                _P, _I, _I, _I, _I, _I, _I, _F, _F, _P]
         o.distie_latent_norm_rope_write.argtypes = [_P, _I, _L, _I, _P, _I, _P, _F, _I, _P, _F, _I, _P, _I, _P, _P, _I, _P,
                                                     _I, _I, _I, _I, _P]
         o.distie_latent_queries.argtypes = [_P, _I, _I, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _P]
@@ -345,7 +348,7 @@ class HipOps(Ops):
         o.distie_ssm_scan_chunked.argtypes = [_P, _I, _L, _P, _L, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I,
                                               _I, _I, _P]
         o.distie_gate_rmsnorm.argtypes = [_P, _P, _I, _F, _P, _I, _L, _P, _I, _I, _I, _I, _I, _P]
-        o.distie_glu_mul.argtypes = [_P, _I, _I, _P, _I, _I, _I, _I, _P]
+        o.distie_glu_mul.argtypes = [_P, _I, _I, _P, _I, _I, _I, _I, _F, _F, _F, _P]
         o.distie_group_chain.argtypes = [_P, _I, _I, _P, _F, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P, _I, _P, _P, _P]
         o.distie_token_shift.argtypes = [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _P]
         o.distie_wkv_scan.argtypes = [_P, _P, _P, _P, _I, _L, _P, _I, _L, _I, _P, _P, _P, _P, _P, _F, _P, _I, _P, _P, _I, _I,
@@ -615,7 +618,20 @@ class HipOps(Ops):
         else the product, then `glu_mul`."""
         if kind not in self.ACTIVATIONS:
             raise KernelError(f"linear_glu: no activation named {kind!r}")
-        gated = 1 if kind == "silu" else 1 | ((self.ACTIVATIONS[kind] + 1) << 8)
+        return self._linear_gated(x, gate_up_weight, 1 if kind == "silu" else 1 | ((self.ACTIVATIONS[kind] + 1) << 8),
+                                  lambda product: self.glu_mul(product, kind))
+
+    CLAMPED = 5                      # the clamped activation, as the packed products number what stands on the gate
+
+    def linear_clamped_glu(self, x, gate_up_weight, limit, slope, up_shift):
+        if not limit > 0:
+            raise KernelError("linear_clamped_glu: the limit must be positive")
+        return self._linear_gated(self.dense(x), gate_up_weight, 1 | (self.CLAMPED << 8),
+                                  lambda product: self.clamped_glu(product, limit, slope, up_shift),
+                                  (float(limit), float(slope), float(up_shift)))
+
+    def _linear_gated(self, x, gate_up_weight, gated, apart, clamp=(0.0, 1.0, 0.0)):
+        """`gated`: 1, and above the low eight bits what stands on the gate; `apart`: the same on a finished product."""
         packed = getattr(gate_up_weight, "_distie_gated", None)
         if isinstance(x, PendingNorm) and packed is not None and gate_up_weight.shape[1] == x.shape[1]:
             N, K = gate_up_weight.shape
@@ -625,7 +641,7 @@ class HipOps(Ops):
             return self._norm_product(x, packed, None, out, gated, N)
         x = self.dense(x)
         if packed is None or x.dtype != torch.bfloat16 or x.shape[0] > self._packed_rows(x.shape[0], *gate_up_weight.shape):
-            return self.glu_mul(self.linear(x, gate_up_weight), kind)
+            return apart(self.linear(x, gate_up_weight))
         self._own(x)
         M, K = x.shape
         N = gate_up_weight.shape[0]
@@ -636,11 +652,11 @@ class HipOps(Ops):
         out = torch.empty((M, N // 2), dtype=x.dtype, device=self.device)
         if M <= self.ONE_WAVE_MAX_ROWS:
             _check(self._ops.distie_gemm_packed_bf16(x.data_ptr(), packed.data_ptr(), None, out.data_ptr(), _code(out),
-                                                     M, N, K, gated, self._stream()), "gemm_packed_bf16")
+                                                     M, N, K, gated, *clamp, self._stream()), "gemm_packed_bf16")
         else:
             _check(self._ops.distie_gemm_packed_wide_bf16(
                 x.data_ptr(), packed.data_ptr(), None, out.data_ptr(), _code(out), M, N, K, gated,
-                self._pass_blocks(M, N * K), self._stream()), "gemm_packed_wide_bf16")
+                self._pass_blocks(M, N * K), *clamp, self._stream()), "gemm_packed_wide_bf16")
         return out
 
     def linear_rope_kv_write(self, x, weight, bias, meta, group, k_cache, v_cache, inv_freq, num_heads, num_kv_heads,
@@ -853,7 +869,7 @@ class HipOps(Ops):
                 out = torch.empty((slices, M, N), dtype=torch.float32, device=self.device)
             _check(self._ops.distie_gemm_packed_wide_bf16(
                 x.data_ptr(), packed.data_ptr(), bias.data_ptr() if bias is not None else None, out.data_ptr(),
-                _code(out), M, N, K, 0, self._pass_blocks(M, N * K), self._stream()),
+                _code(out), M, N, K, 0, self._pass_blocks(M, N * K), 0.0, 1.0, 0.0, self._stream()),
                 "gemm_packed_wide_bf16")
             if slices == 1:
                 return out
@@ -870,7 +886,7 @@ class HipOps(Ops):
             if packed is not None:
                 _check(self._ops.distie_gemm_packed_bf16(
                     x.data_ptr(), packed.data_ptr(), bias.data_ptr() if bias is not None else None, out.data_ptr(),
-                    _code(out), M, N, K, 0, self._stream()), "gemm_packed_bf16")
+                    _code(out), M, N, K, 0, 0.0, 1.0, 0.0, self._stream()), "gemm_packed_bf16")
             else:
                 _check(self._ops.distie_gemm_skinny_bf16(
                     x.data_ptr(), weight.data_ptr(), bias.data_ptr() if bias is not None else None, out.data_ptr(),
@@ -949,8 +965,8 @@ class HipOps(Ops):
     def paged_attention(self, qkv, meta: BatchMeta, group, k_cache, v_cache, num_heads, num_kv_heads, head_dim,
                         scale, window, extras=None):
         """The matrix-core kernels and the tiled float32 kernel compute attention with plain scores (a sink in the
-        denominator they take); a step whose `extras` bend the scores goes to the wave-per-token kernel, which takes
-        slopes and a cap as well (any types and sizes)."""
+        denominator they take, and chunks instead of a window); a step whose `extras` bend the scores goes to the
+        wave-per-token kernel, which takes slopes and a cap as well (any types and sizes)."""
         if not scale > 0:
             raise KernelError(f"paged_attention: the scale of the scores must be positive, not {scale}")
         qkv = self.dense(qkv)
@@ -973,6 +989,10 @@ class HipOps(Ops):
                 if vector.dtype != torch.float32 or tuple(vector.shape) != (num_heads,):
                     raise KernelError(f"paged_attention: {name} must be float32 [num_heads]")
         sinks_ptr = sinks.data_ptr() if sinks is not None else None
+        chunk = extras.chunk if extras is not None else 0
+        if chunk and (window or extras.mixes_heads):
+            raise KernelError("paged_attention: chunks do not go with a window or with mixed heads")
+        reach = -int(chunk) if chunk else int(window or 0)       # as the kernels take it: a window, or minus the chunks' size
         if extras is not None and extras.mixes_heads:
             self._mixed_attention(qkv, meta, table, rows_ptr, k_cache, v_cache, out, num_heads, num_kv_heads, head_dim, scale,
                                   window, extras)
@@ -983,18 +1003,18 @@ class HipOps(Ops):
             # how the step is launched, and its buffers for partial results, are the same for every layer
             # with these sizes: worked out once per step (the layers run one after the other, so they can
             # share the buffers)
-            key = ("attention", int(window or 0), num_heads, num_kv_heads, head_dim, meta.max_kv, meta.all_decode,
+            key = ("attention", reach, num_heads, num_kv_heads, head_dim, meta.max_kv, meta.all_decode,
                    meta.singles_bound, self.PREFILL_PARTS, self.PREFILL_WORKGROUPS, self.DECODE_WAVES, self.DECODE_MAX_RUNS,
                    self.DECODE_SHARED_BELOW)
             plan = meta.scratch.get(key)
             if plan is None or plan["cu_q"] is not meta.host_cu_q:
-                plan = meta.scratch[key] = self._attention_plan(lib, meta, T, num_heads, num_kv_heads, head_dim, window)
+                plan = meta.scratch[key] = self._attention_plan(lib, meta, T, num_heads, num_kv_heads, head_dim, abs(reach))
             if plan["decode"]:
                 _check(lib.distie_attention_decode_bf16(
                     qkv.data_ptr(), qkv.shape[1], k_cache.data_ptr(), v_cache.data_ptr(), meta.kv_len.data_ptr(),
                     meta.cu_q.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr, out.data_ptr(),
                     plan["decode_o"].data_ptr(), plan["decode_ml"].data_ptr(), meta.num_requests, num_heads,
-                    num_kv_heads, meta.block_size, float(scale), int(window or 0), plan["split_len"],
+                    num_kv_heads, meta.block_size, float(scale), reach, plan["split_len"],
                     plan["max_splits"], 1 if meta.all_decode else 0,
                     plan["run_len"].data_ptr() if plan["run_len"] is not None else None, sinks_ptr, self._stream()),
                     "attention_decode_bf16")
@@ -1003,7 +1023,7 @@ class HipOps(Ops):
                 _check(lib.distie_attention_prefill_bf16(
                     qkv.data_ptr(), qkv.shape[1], k_cache.data_ptr(), v_cache.data_ptr(), meta.positions.data_ptr(),
                     meta.cu_q.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr, out.data_ptr(), T, meta.num_requests,
-                    num_heads, num_kv_heads, meta.block_size, float(scale), int(window or 0),
+                    num_heads, num_kv_heads, meta.block_size, float(scale), reach,
                     2 if plan["decode"] else 1, meta.token_request.data_ptr(),
                     plan["prefill_o"].data_ptr() if parts > 1 else None,
                     plan["prefill_ml"].data_ptr() if parts > 1 else None, parts, sinks_ptr, self._stream()),
@@ -1013,16 +1033,16 @@ class HipOps(Ops):
         if plain and f32 and meta.max_q >= self.PREFILL_F32_MIN_TOKENS and meta.block_size % 16 == 0 and \
                 qkv.shape[1] % 4 == 0 and lib.distie_attention_prefill_f32_fits():
             # portions of prompts in float32: the tiled kernel on float32 matrix products takes the whole step
-            key = ("attention_f32", int(window or 0), num_heads, head_dim, meta.max_kv, self.PREFILL_PARTS,
+            key = ("attention_f32", reach, num_heads, head_dim, meta.max_kv, self.PREFILL_PARTS,
                    self.PREFILL_WORKGROUPS)
             plan = meta.scratch.get(key)
             if plan is None:
-                plan = meta.scratch[key] = self._prefill_parts(meta, T, num_heads, head_dim, window)
+                plan = meta.scratch[key] = self._prefill_parts(meta, T, num_heads, head_dim, abs(reach))
             parts = plan["parts"]
             _check(lib.distie_attention_prefill_f32(
                 qkv.data_ptr(), qkv.shape[1], k_cache.data_ptr(), v_cache.data_ptr(), meta.positions.data_ptr(),
                 meta.cu_q.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr, out.data_ptr(), T, meta.num_requests,
-                num_heads, num_kv_heads, meta.block_size, float(scale), int(window or 0), 1,
+                num_heads, num_kv_heads, meta.block_size, float(scale), reach, 1,
                 meta.token_request.data_ptr(), plan["prefill_o"].data_ptr() if parts > 1 else None,
                 plan["prefill_ml"].data_ptr() if parts > 1 else None, parts, sinks_ptr, self._stream()),
                 "attention_prefill_f32")
@@ -1030,7 +1050,7 @@ class HipOps(Ops):
         _check(lib.distie_attention_generic(
             qkv.data_ptr(), _code(qkv), qkv.shape[1], k_cache.data_ptr(), v_cache.data_ptr(), _code(k_cache),
             meta.positions.data_ptr(), meta.token_request.data_ptr(), table.data_ptr(), table.shape[1], rows_ptr,
-            out.data_ptr(), T, num_heads, num_kv_heads, meta.block_size, float(scale), int(window or 0),
+            out.data_ptr(), T, num_heads, num_kv_heads, meta.block_size, float(scale), reach,
             slopes.data_ptr() if slopes is not None else None, cap, sinks_ptr, self._stream()), "attention_generic")
         return out
 
@@ -1272,7 +1292,7 @@ class HipOps(Ops):
 
     def conv_rope_kv_write(self, product, conv_weight, state, meta, group, k_cache, v_cache, inv_freq, magnitude,
                            num_heads, num_kv_heads, dim, value_dim, padded_dim, has_kv, write, q_temp=None, qk_norm=None,
-                           keys_are_values=False):
+                           keys_are_values=False, neighbours=False):
         # without a filter the kernel adds up a product's partial sums itself while it reads them
         slices, q_dtype = 1, None
         if isinstance(product, PartialSums) and conv_weight is None:
@@ -1318,7 +1338,7 @@ class HipOps(Ops):
             meta.state_slots.data_ptr(), T, num_heads, num_kv_heads, dim, value_dim, padded_dim, meta.block_size,
             2 if keys_are_values else (1 if has_kv else 0), 1 if write else 0, meta.positions.data_ptr(), float(q_temp[0]) if q_temp else 0.0,
             int(q_temp[1]) if q_temp else 0, ptr(q_norm), ptr(k_norm) if has_kv else None, float(norm_eps),
-            slices, _CODES[q_dtype], self._stream()), "conv_rope_kv_write")
+            slices, _CODES[q_dtype], 1 if neighbours else 0, self._stream()), "conv_rope_kv_write")
         if taps > 1:
             if not meta.all_decode:
                 # (requests that bring one row had their state moved on by the kernel above)
@@ -1374,7 +1394,10 @@ class HipOps(Ops):
                                                       device=self.device)
         return count, packed, scratch
 
-    def decay_scan(self, product, state, decay, meta, num_heads, dim, value_dim):
+    def decay_scan(self, product, state, decay, meta, num_heads, dim, value_dim, act="silu", k_scale=1.0, inv_freq=None,
+                   neighbours=False):
+        if act not in ("silu", None) or (act is not None and (inv_freq is not None or k_scale != 1.0)):
+            raise KernelError("decay_scan: silu on q, k and v, or no activation with a rotation and a scale of k")
         product = self.dense(product)
         self._own(product, state, decay)
         T, W = product.shape
@@ -1384,6 +1407,13 @@ class HipOps(Ops):
             raise KernelError("decay_scan: the state is float32 [slots, heads, dim, value_dim]")
         if decay.dtype != torch.float32 or tuple(decay.shape) != (num_heads,):
             raise KernelError("decay_scan: decay must be float32 [heads]")
+        if dim > self._ops.distie_decay_scan_max_dim():
+            raise KernelError(f"decay_scan: heads of up to {self._ops.distie_decay_scan_max_dim()} dimensions")
+        pairs = 0 if inv_freq is None else inv_freq.shape[0]
+        if 2 * pairs > dim:
+            raise KernelError("decay_scan: the rotation turns more dimensions than a head has")
+        table = self._rope_table(meta, inv_freq) if pairs else None
+        turn = (1 if act else 0, table.data_ptr() if pairs else None, pairs, 1 if neighbours else 0, float(k_scale))
         out = torch.empty((T, num_heads * value_dim), dtype=torch.float32, device=self.device)
         if not self.captured and meta.host_cu_q is not None and meta.max_q >= self.SCAN_CHUNKED_MIN_ROWS and \
                 dim % 4 == 0 and value_dim % 4 == 0 and dim <= self._ops.distie_decay_scan_chunked_max_dim():
@@ -1394,12 +1424,13 @@ class HipOps(Ops):
             _check(self._ops.distie_decay_scan_chunked(
                 product.data_ptr(), _code(product), W, state.data_ptr(), decay.data_ptr(), out.data_ptr(),
                 scratch.data_ptr(), packed.data_ptr(), packed.data_ptr() + 16 * count, meta.state_slots.data_ptr(),
-                count, meta.num_requests, num_heads, dim, value_dim, self._stream()), "decay_scan_chunked")
+                count, meta.num_requests, num_heads, dim, value_dim, *turn, self._stream()), "decay_scan_chunked")
             _mark_written(state)
             return out
         _check(self._ops.distie_decay_scan(product.data_ptr(), _code(product), W, state.data_ptr(), decay.data_ptr(),
                                            out.data_ptr(), meta.cu_q.data_ptr(), meta.state_slots.data_ptr(),
-                                           meta.num_requests, num_heads, dim, value_dim, self._stream()), "decay_scan")
+                                           meta.num_requests, num_heads, dim, value_dim, *turn, self._stream()),
+               "decay_scan")
         _mark_written(state)
         return out
 
@@ -1801,26 +1832,41 @@ class HipOps(Ops):
         _mark_written(state)
         return out
 
-    SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_all": 2}
+    SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_all": 2, "sigmoid_share": 3}
+    NO_RULE = RouteRule()
 
-    def route_topk(self, x, weight, bias, top, scoring="softmax"):
+    def _route_rule(self, rule, scoring, experts):
+        """The rule's numbers as the kernels take them: (correction, groups, kept, scale, shared)."""
+        rule = rule or self.NO_RULE
+        if scoring != "sigmoid_share" and (rule.correction is not None or rule.groups != 1 or rule.scale != 1.0):
+            raise KernelError("a router's correction, groups and scale go with the scoring sigmoid_share")
+        self._own(rule.correction)
+        if rule.correction is not None and (rule.correction.dtype != torch.float32 or tuple(rule.correction.shape) != (experts,)):
+            raise KernelError("a router's correction is float32 [experts]")
+        return (rule.correction.data_ptr() if rule.correction is not None else None, int(rule.groups), int(rule.kept),
+                float(rule.scale), 1 if rule.shared else 0)
+
+    def route_topk(self, x, weight, bias, top, scoring="softmax", rule=None):
         if scoring not in self.SCORINGS:
             raise KernelError(f"route_topk: no scoring named {scoring!r}")
         x = self.dense(x)
         self._own(x, weight, bias)
         T, C = x.shape
-        E = weight.shape[0]
-        if tuple(weight.shape) != (E, C) or (bias is not None and (bias.dtype != torch.float32 or tuple(bias.shape) != (E,))):
-            raise KernelError("route_topk: weight [experts, C], bias float32 [experts]")
+        rows = weight.shape[0]
+        shared = 1 if rule is not None and rule.shared else 0
+        E = rows - shared
+        if tuple(weight.shape) != (rows, C) or (bias is not None and (bias.dtype != torch.float32 or tuple(bias.shape) != (rows,))):
+            raise KernelError("route_topk: weight [experts (+ 1 with a shared one), C], bias float32 with a number a row")
+        numbers = self._route_rule(rule, scoring, E)
         experts = torch.empty((T, top), dtype=torch.int32, device=self.device)
-        gates = torch.empty((T, top), dtype=torch.float32, device=self.device)
+        gates = torch.empty((T, top + shared), dtype=torch.float32, device=self.device)
         _check(self._ops.distie_route_topk(x.data_ptr(), _code(x), weight.data_ptr(), _code(weight),
                                            bias.data_ptr() if bias is not None else None, experts.data_ptr(),
-                                           gates.data_ptr(), T, C, E, int(top), self.SCORINGS[scoring],
+                                           gates.data_ptr(), T, C, E, int(top), self.SCORINGS[scoring], *numbers,
                                            self._stream()), "route_topk")
         return experts, gates
 
-    def route_glu(self, gate_up, experts, gates, num_experts, width, limit, slope, up_shift, on_input):
+    def route_glu(self, gate_up, experts, gates, num_experts, width, limit, slope, up_shift, on_input, shared_width=0):
         if isinstance(gate_up, (PendingNorm, PendingProduct)):
             gate_up = self.dense(gate_up)
         slices, source, dtype, ld = 1, gate_up, gate_up.dtype, gate_up.shape[1]
@@ -1835,22 +1881,25 @@ class HipOps(Ops):
         self._own(source, experts, gates)
         source = gate_up if source is None else source
         T, top = experts.shape
-        if experts.dtype != torch.int32 or gates.dtype != torch.float32 or gates.shape != experts.shape or \
-                gate_up.shape[0] != T or gate_up.shape[1] != 2 * num_experts * width:
-            raise KernelError("route_glu: experts int32 and gates float32 [T, top], gate_up [T, 2 * experts * width]")
+        total = num_experts * width + shared_width
+        if experts.dtype != torch.int32 or gates.dtype != torch.float32 or \
+                tuple(gates.shape) != (T, top + (1 if shared_width else 0)) or \
+                gate_up.shape[0] != T or gate_up.shape[1] != 2 * total:
+            raise KernelError("route_glu: experts int32 and gates float32 [T, top] (one more with a shared expert), gate_up "
+                              "[T, 2 * (experts * width + shared_width)]")
         if limit is not None and not limit > 0:
             raise KernelError("route_glu: the limit must be positive")
-        out = torch.empty((T, num_experts * width), dtype=dtype, device=self.device)
+        out = torch.empty((T, total), dtype=dtype, device=self.device)
         _check(self._ops.distie_route_glu(source.data_ptr(), _code(source), ld, slices, experts.data_ptr(),
                                           gates.data_ptr(), T, top, num_experts, width, float(limit or 0.0), float(slope),
-                                          float(up_shift), 1 if on_input else 0, out.data_ptr(), _code(out),
-                                          self._stream()), "route_glu")
+                                          float(up_shift), 1 if on_input else 0, int(shared_width), out.data_ptr(),
+                                          _code(out), self._stream()), "route_glu")
         return out
 
     FUSED_ROUTE_ROWS = 64       # up to so many rows every block works out its row's choice itself
 
     def route_experts_glu(self, x, router_weight, router_bias, top, scoring, gate_up, num_experts, width, limit, slope,
-                          up_shift, on_input):
+                          up_shift, on_input, rule=None, shared_width=0):
         if scoring not in self.SCORINGS:
             raise KernelError(f"route_experts_glu: no scoring named {scoring!r}")
         x = self.dense(x)
@@ -1858,25 +1907,27 @@ class HipOps(Ops):
         if T > self.FUSED_ROUTE_ROWS or x.dtype != torch.bfloat16 or router_weight.dtype != torch.bfloat16 or C % 8 or \
                 x.data_ptr() % 16 or router_weight.data_ptr() % 16 or not x.is_contiguous():
             return super().route_experts_glu(x, router_weight, router_bias, top, scoring, gate_up, num_experts, width,
-                                             limit, slope, up_shift, on_input)
+                                             limit, slope, up_shift, on_input, rule, shared_width)
         if isinstance(gate_up, (PendingNorm, PendingProduct)):
             gate_up = self.dense(gate_up)
         slices, source, dtype = 1, gate_up, gate_up.dtype
         if isinstance(gate_up, PartialSums):
             slices, source = gate_up.slices, gate_up.data
         self._own(x, router_weight, router_bias, source)
-        if tuple(router_weight.shape) != (num_experts, C) or not 1 <= top <= num_experts or gate_up.shape[0] != T or \
-                gate_up.shape[1] != 2 * num_experts * width or \
-                (router_bias is not None and (router_bias.dtype != torch.float32 or tuple(router_bias.shape) != (num_experts,))):
+        numbers = self._route_rule(rule, scoring, num_experts)
+        rows, total = num_experts + numbers[-1], num_experts * width + shared_width
+        if tuple(router_weight.shape) != (rows, C) or not 1 <= top <= num_experts or gate_up.shape[0] != T or \
+                gate_up.shape[1] != 2 * total or (shared_width and not numbers[-1]) or \
+                (router_bias is not None and (router_bias.dtype != torch.float32 or tuple(router_bias.shape) != (rows,))):
             raise KernelError("route_experts_glu: x [T, C], router [E, C], bias float32 [E], gate_up [T, 2 * E * width]")
         if limit is not None and not limit > 0:
             raise KernelError("route_experts_glu: the limit must be positive")
-        out = torch.empty((T, num_experts * width), dtype=dtype, device=self.device)
+        out = torch.empty((T, total), dtype=dtype, device=self.device)
         _check(self._ops.distie_route_topk_glu(
             x.data_ptr(), router_weight.data_ptr(), router_bias.data_ptr() if router_bias is not None else None, C,
             self.SCORINGS[scoring], source.data_ptr(), _code(source), gate_up.shape[1], slices, T, int(top),
-            num_experts, width, float(limit or 0.0), float(slope), float(up_shift), 1 if on_input else 0, out.data_ptr(),
-            _code(out), self._stream()), "route_topk_glu")
+            num_experts, width, float(limit or 0.0), float(slope), float(up_shift), 1 if on_input else 0, *numbers,
+            int(shared_width), out.data_ptr(), _code(out), self._stream()), "route_topk_glu")
         return out
 
     def softcap(self, x, cap):
@@ -1911,6 +1962,52 @@ class HipOps(Ops):
         out = torch.empty(tuple(x.shape), dtype=dtype, device=self.device)
         _check(self._ops.distie_activation(source.data_ptr(), _code(source), slices, out.data_ptr(), _code(out), out.numel(),
                                            self.ACTIVATIONS[kind], self._stream()), "activation")
+        return out
+
+    # ---- the gated delta rule (csrc/delta.hip)
+    def delta_scan(self, qkv, beta, decay, a_log, dt_bias, state, meta, num_heads, num_kv_heads, dim, value_dim, q_scale,
+                   unit_eps):
+        qkv = self.dense(qkv)
+        H, G, D, E = num_heads, num_kv_heads, dim, value_dim
+        q_ptr, ld = self._rows_view(qkv, qkv.shape[1])
+        b_ptr, ldb = self._rows_view(beta, H)
+        d_ptr, ldd = self._rows_view(decay, H)
+        self._own(a_log, dt_bias, state)
+        T = qkv.shape[0]
+        if T != meta.num_tokens or qkv.shape[1] < 2 * G * D + H * E or H % G or beta.shape[0] != T or decay.shape[0] != T or \
+                beta.dtype != qkv.dtype or decay.dtype != qkv.dtype:
+            raise KernelError("delta_scan: q, k, v and the logits do not match the batch or the head counts")
+        if D > self._ops.distie_delta_scan_max_dim():
+            raise KernelError(f"delta_scan: keys of up to {self._ops.distie_delta_scan_max_dim()} dimensions a head")
+        if state.dtype != torch.float32 or tuple(state.shape[1:]) != (H, D, E):
+            raise KernelError("delta_scan: the state is float32 [slots, heads, dim, value_dim]")
+        for vector in (a_log, dt_bias):
+            if vector.dtype != torch.float32 or tuple(vector.shape) != (H,):
+                raise KernelError("delta_scan: a_log and dt_bias are float32 [heads]")
+        out = torch.empty((T, H * E), dtype=torch.float32, device=self.device)
+        if not self.captured and meta.host_cu_q is not None and meta.max_q >= self.SCAN_CHUNKED_MIN_ROWS:
+            # portions of prompts: chunks of rows, the triangular systems of all chunks side by side
+            rows = self._ops.distie_delta_scan_chunk_rows()
+            count, packed, states = self._scan_chunks(meta, rows, H, D, E)
+            DP, EP = self._ops.distie_delta_scan_padded_dim(D), -(-E // 16) * 16
+            key = ("delta_scratch", count, H, DP, EP)
+            held = meta.scratch.get(key)
+            if held is None:
+                held = meta.scratch[key] = [torch.empty((count, H, *shape), dtype=torch.float32, device=self.device)
+                                            for shape in ((rows, DP), (rows, EP), (rows, EP), (DP, rows), (rows, rows), (rows,),
+                                                          ())]
+            _check(self._ops.distie_delta_scan_chunked(
+                q_ptr, _code(qkv), ld, b_ptr, ldb, d_ptr, ldd, a_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr(),
+                out.data_ptr(), *(t.data_ptr() for t in held), states.data_ptr(), packed.data_ptr(),
+                packed.data_ptr() + 16 * count, meta.state_slots.data_ptr(), count, meta.num_requests, H, G, D, E,
+                float(q_scale), float(unit_eps), self._stream()), "delta_scan_chunked")
+            _mark_written(state)
+            return out
+        _check(self._ops.distie_delta_scan(
+            q_ptr, _code(qkv), ld, b_ptr, ldb, d_ptr, ldd, a_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr(),
+            out.data_ptr(), meta.cu_q.data_ptr(), meta.state_slots.data_ptr(), meta.num_requests, H, G, D, E, float(q_scale),
+            float(unit_eps), self._stream()), "delta_scan")
+        _mark_written(state)
         return out
 
     # ---- a state with one decay a head and token, attention over a shared latent (csrc/ssm.hip, csrc/latent.hip)
@@ -2058,6 +2155,14 @@ class HipOps(Ops):
             return self.silu_mul(gate_up)
         if kind not in self.ACTIVATIONS:
             raise KernelError(f"glu_mul: no activation named {kind!r}")
+        return self._glu_mul(gate_up, self.ACTIVATIONS[kind])
+
+    def clamped_glu(self, gate_up, limit, slope, up_shift):
+        if not limit > 0:
+            raise KernelError("clamped_glu: the limit must be positive")
+        return self._glu_mul(gate_up, len(self.ACTIVATIONS), (float(limit), float(slope), float(up_shift)))
+
+    def _glu_mul(self, gate_up, kind, clamp=(0.0, 1.0, 0.0)):
         if isinstance(gate_up, (PendingNorm, PendingProduct)):
             gate_up = self.dense(gate_up)
         slices, source, dtype = 1, gate_up, gate_up.dtype
@@ -2067,7 +2172,7 @@ class HipOps(Ops):
         rows, two = gate_up.shape
         out = torch.empty((rows, two // 2), dtype=dtype, device=self.device)
         _check(self._ops.distie_glu_mul(source.data_ptr(), _code(source), slices, out.data_ptr(), _code(out), rows,
-                                        two // 2, self.ACTIVATIONS[kind], self._stream()), "glu_mul")
+                                        two // 2, kind, *clamp, self._stream()), "glu_mul")
         return out
 
     def silu_mul(self, gate_up):
