@@ -326,6 +326,35 @@ def netovik_config(size):
             "embedding": {"scale": 8.0}, "layers": layers}
 
 
+def mepapel_config(size):
+    """Groups of four layers: mixers side by side (attention in chunks of the window's size with filters, head norms and
+    neighbours turned, beside retention with half as many heads), a state-space layer (heads of 64 channels on twice the
+    width, a state of 128 rows, four taps) and two layers with the delta rule (keys shared by two heads, four taps); clamped
+    dense feed-forwards alternate with mixtures of eight experts of a quarter of the dense size in four groups, two a token
+    out of two groups, beside a shared one with a gate."""
+    z = DESIGN_SIZES[size]
+    layers = []
+    for i in range(z["layers"]):
+        mlp = {"kind": "dense", "ff": z["ff"], "limit": 7.0} if i % 2 == 0 else \
+            {"kind": "moe", "router": {"experts": 8, "top": 2, "groups": {"count": 4, "keep": 2}, "scale": 1.5},
+             "expert": {"ff": z["ff"] // 4}, "shared": {"ff": z["ff"] // 4}}
+        if i % 4 == 0:
+            half = max(1, z["heads"] // 2)
+            left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"], "conv": 4,
+                    "mask": {"size": z["window"]}, "rot": {"base": 500000.0, "dims": z["dim"]}, "scale": z["dim"] ** -0.5}
+            right = {"heads": half, "dim": z["dim"], "vdim": z["dim"], "rot": {"base": 10000.0, "dims": z["dim"]},
+                     "decay": [1.0 - 2.0 ** -(5 + 3 * h / max(1, half - 1)) for h in range(half)]}
+            layers.append({"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": mlp})
+        elif i % 4 == 1:
+            mixer = {"heads": 2 * z["width"] // 64, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}
+            layers.append({"type": "mamba2", "mixer": mixer, "mlp": mlp})
+        else:
+            mixer = {"heads": z["heads"], "kv_heads": z["heads"] // 2, "dim": z["dim"], "vdim": z["dim"], "conv": 4}
+            layers.append({"type": "delta", "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Mepapel", "vocab": DESIGN_VOCAB, "width": z["width"], "norm": {"eps": 1e-6},
+            "residual_mult": 0.5, "layers": layers}
+
+
 def qwen2_of_weights(size, layer_weights):
     """The Qwen2 decoder with the same width, depth and heads and a feed-forward sized so that its layers hold as many
     weights as the other design's layers do on average."""
@@ -345,7 +374,7 @@ def design_pair(design, size):
     from distie_amd.engine.model import Model
 
     config = {"sekazen": sekazen_config, "duparax": duparax_config, "dufelix": dufelix_config,
-              "netovik": netovik_config}[design](size)
+              "netovik": netovik_config, "mepapel": mepapel_config}[design](size)
     total = 0
     for name, spec in Model.declare(config_from_dict(config).model_spec()).items():
         if name.startswith("l"):
@@ -417,7 +446,7 @@ def main() -> int:
                         help="size the cache from free memory (the default for --shape 32b and --serve: 0.9)")
     parser.add_argument("--packed-weights", default=None, metavar="ROLES",
                         help="packed copies only for these products (qkv,attn_out,gate_up,down,head); 'none' for no copies")
-    parser.add_argument("--design", default=None, choices=["musutar", "duparax", "sekazen", "dufelix", "netovik"],
+    parser.add_argument("--design", default=None, choices=["musutar", "duparax", "sekazen", "dufelix", "netovik", "mepapel"],
                         help="instead of the workload above: this design beside a Qwen2 decoder of equal size, prefill and decode")
     parser.add_argument("--size", default=None, choices=sorted(DESIGN_SIZES), help="with --design: one size instead of all")
     args = parser.parse_args()

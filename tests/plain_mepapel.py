@@ -152,6 +152,18 @@ def delta_scan(q, k, v, beta, g):
     return out
 
 
+def write_squares(q, k, v, beta, g):
+    """The sum of the squares of what the tokens so far would add to an output without corrections."""
+    T, H, D = q.shape
+    state = torch.zeros(H, D, v.shape[2], dtype=torch.float64)
+    out = []
+    for t in range(T):
+        write = beta[t][:, None] * v[t]
+        state = (g[t] ** 2)[:, None, None] * state + (k[t] ** 2)[:, :, None] * (write ** 2)[:, None, :]
+        out.append((state * (q[t] ** 2)[:, :, None]).sum(1))
+    return torch.stack(out)
+
+
 def delta(h, w, p, m, eps, watch=None):
     T = h.shape[0]
     H, G, D, E = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])
@@ -163,7 +175,8 @@ def delta(h, w, p, m, eps, watch=None):
     g = torch.exp(-torch.exp(w[p + "A_log"]) * softplus(h @ w[p + "a"].T + w[p + "dt_bias"]))
     o = delta_scan(own(q), own(k), v.view(T, H, E), beta, g)
     if watch is not None:
-        watch("heads", o, delta_scan(own(q), own(k), v.view(T, H, E), beta, g) ** 2 + v.view(T, H, E) ** 2 / D ** 2)
+        # (the corrections depend on each other; the squares of an uncorrected write stand for its terms' size)
+        watch("heads", o, write_squares(own(q), own(k), v.view(T, H, E), beta, g))
     return (rms(o, eps) * w[p + "norm"]).reshape(T, H * E).mul(silu(h @ w[p + "g"].T)) @ w[p + "o"].T
 
 
