@@ -61,17 +61,27 @@ def in_portions(llm, rid, ids, cuts):
     return torch.cat(out)
 
 
-def check(got, want, dtype, what=""):
-    """float32: every row within the bound. bfloat16: norms behind the sub-layers make a row now and then more sensitive
-    to rounding than the others, so one row in twenty may pass the bound, none 2.5 times it (a wrong key, a lost state
-    or a sink left out moves a row by far more)."""
+def rounded_bound(folder, ids, want):
+    """For every row, how far bfloat16 may be off: the usual bound, or (a branch that nearly cancels in front of its norm makes
+    a row more sensitive to rounding than others) twice what the CPU test double is off in bfloat16, which rounds at the same
+    places."""
+    llm = LLM(folder, dtype="bfloat16", device="cpu", ops=TorchOps(), block_size=16, num_blocks=32, max_seqs=1, use_graphs=False)
+    err = mu.logit_error(whole(llm, "a", ids), want)
+    llm.close()
+    return (2 * err).clamp(min=mu.TOL[torch.bfloat16])
+
+
+def check(got, want, dtype, what="", bound=None):
+    """float32: every row within the bound. bfloat16 (`bound`: a bound for every row, see above): one row in twenty may pass
+    its bound, none 2.5 times it (a wrong key, a lost state or another expert moves a row by far more)."""
     err = mu.logit_error(got, want)
     tol = mu.TOL[DTYPES[dtype]]
-    worst = f"{what}: error {float(err.max())} at row {int(err.argmax())}"
     if dtype == "float32":
-        assert float(err.max()) < tol, worst
-    else:
-        assert float(err.max()) < 2.5 * tol and int((err > tol).sum()) <= max(1, len(err) // 20), worst
+        assert float(err.max()) < tol, f"{what}: error {float(err.max())} at row {int(err.argmax())}"
+        return
+    over = err / (tol if bound is None else bound)
+    worst = f"{what}: error {float(err[over.argmax()])} at row {int(over.argmax())}, {float(over.max())} times its bound"
+    assert float(over.max()) < 2.5 and int((over > 1).sum()) <= max(1, len(err) // 20), worst
 
 
 # nothing equal by accident: heads, head sizes, states, taps, chunks and feed-forwards of their own in every layer, every
@@ -201,8 +211,9 @@ def test_prompt_decode_and_portions(ops, folders, name):
         runs = {"whole": whole(llm, "a", ids), "token by token": in_portions(llm, "b", ids, []),
                 "portions": in_portions(llm, "c", ids, [2, 7, 3, 2, 13, 5, 2, 4]),
                 "a long portion, then tokens": in_portions(llm, "d", ids, [29])}
+        bound = rounded_bound(folder, ids, want) if dtype == "bfloat16" else None
         for what, got in runs.items():
-            check(got, want, dtype, f"{name} {dtype} {what}")
+            check(got, want, dtype, f"{name} {dtype} {what}", bound)
         llm.cache.check()
         assert not llm.cache.live()
 
@@ -256,7 +267,8 @@ def test_unequal_batches_and_reuse(ops, folders):
             llm.cache.check()
             turn += 1
         for i in prompts:
-            check(torch.cat(got[i]), want[i], dtype, f"request {i} {dtype}")
+            check(torch.cat(got[i]), want[i], dtype, f"request {i} {dtype}",
+                  rounded_bound(folder, prompts[i], want[i]) if dtype == "bfloat16" else None)
         assert not llm.cache.live() and llm.cache.free_pages() == [48] * len(llm.cache.groups)
 
 
@@ -402,7 +414,7 @@ def test_first_tokens_and_long_decoding(ops, folders):
         for dtype in dtypes:
             llm = engine(folder, ops, dtype, num_blocks=48)
             got = in_portions(llm, "a", ids, [1, 1, 1, 2])
-            check(got, want, dtype, f"{name} long decoding {dtype}")
+            check(got, want, dtype, f"{name} long decoding {dtype}", rounded_bound(folder, ids, want) if dtype == "bfloat16" else None)
             llm.cache.check()
             assert not llm.cache.live()
 
@@ -510,7 +522,8 @@ def test_trace_runner_and_command_line(folders, tmp_path):
         proc.stdin.close()
         assert proc.wait(timeout=60) == 0
         for r in reqs:
-            check(torch.cat(got[r]), want[r], dtype, f"request {r} {dtype}")
+            check(torch.cat(got[r]), want[r], dtype, f"request {r} {dtype}",
+                  rounded_bound(folder, reqs[r], want[r]) if dtype == "bfloat16" else None)
     prompts = [reqs["s"], reqs["q"][:9]]
     (tmp_path / "prompts.json").write_text(json.dumps(prompts))
     done = subprocess.run([sys.executable, "-m", "distie_amd.cli", "generate", "--model", str(folder), "--dtype", "fp32",
