@@ -121,7 +121,7 @@ typedef __attribute__((__vector_size__(4 * sizeof(float)))) float delta_floatx4;
 __device__ __forceinline__ int tile_row(int v, int lane) { return 8 * (v / 4) + 4 * (lane / 32) + v % 4; }
 
 template <typename X>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, 2)
 delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __restrict__ beta, int64_t ldb,
                            const X* __restrict__ decay, int64_t lda, const float* __restrict__ a_log,
                            const float* __restrict__ dt_bias, float* __restrict__ w_out, float* __restrict__ v_out,
@@ -129,6 +129,7 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
                            float* __restrict__ totals, const int4* __restrict__ chunks, int H, int G, int D, int E, int DP,
                            int EP, float q_scale, float unit_eps) {
   __shared__ float l_s[DL], beta_s[DL], q_unit[DL], k_unit[DL];
+  __shared__ float in_factor[DL], out_factor[DL];        // w_i exp(l_i) and exp(l_L - l_i), each over the length of k_i
   __shared__ float q_s[DL][DL_PAD], k_s[DL][DL_PAD];     // [row][d of this pass]
   __shared__ __attribute__((aligned(16))) float a_s[DL][DL_ROW];
   const int chunk = blockIdx.x, head = blockIdx.y;
@@ -157,11 +158,23 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
   float q_sq = 0.f, k_sq = 0.f;
   for (int n0 = 0; n0 < D; n0 += DL) {
     __syncthreads();
-    for (int j = wave; j < DL; j += 4) {
-      const bool in = j < rows && n0 + lane < D;
-      const X* row = qkv + static_cast<int64_t>(first + j) * ld + n0 + lane;
-      q_s[j][lane] = in ? to_float(row[q_at]) : 0.f;
-      k_s[j][lane] = in ? to_float(row[k_at]) : 0.f;
+    {
+      // a tile's loads are under way together: addresses clamped into the step's rows, what does not belong is dropped
+      const X* from = qkv + static_cast<int64_t>(first) * ld + min(n0 + lane, D - 1);
+      X q[16], k[16];
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const int64_t at = static_cast<int64_t>(min(wave + 4 * r, rows - 1)) * ld;
+        q[r] = from[at + q_at];
+        k[r] = from[at + k_at];
+      }
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const int j = wave + 4 * r;
+        const bool in = j < rows && n0 + lane < D;
+        q_s[j][lane] = in ? to_float(q[r]) : 0.f;
+        k_s[j][lane] = in ? to_float(k[r]) : 0.f;
+      }
     }
     __syncthreads();
 #pragma unroll
@@ -196,7 +209,12 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
     a_s[i][j] = j < i ? fade * beta_s[i] * k_unit[i] * kk[v] : 0.f;
     pair[i * DL + j] = fade * q_unit[i] * qk[v];
   }
-  if (tid < DL) q_factor[place * DL + tid] = expf(l_s[tid]) * q_unit[tid];
+  if (tid < DL) {
+    const float l = expf(l_s[tid]);
+    q_factor[place * DL + tid] = l * q_unit[tid];
+    in_factor[tid] = beta_s[tid] * k_unit[tid] * l;
+    out_factor[tid] = k_unit[tid] * expf(l_end - l_s[tid]);
+  }
   if (tid == 0) totals[place] = expf(l_end);
   __syncthreads();
   // (I + A) X = B, a thread a column of B, forward substitution with the column in registers
@@ -208,16 +226,20 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
                     (key ? k_at + col : 2 * static_cast<int64_t>(G) * D + static_cast<int64_t>(head) * E + col);
     float x[DL];
 #pragma unroll
-    for (int i = 0; i < DL; ++i) x[i] = in && i < rows ? to_float(from[static_cast<int64_t>(i) * ld]) : 0.f;
+    for (int i = 0; i < DL; ++i) x[i] = to_float(from[in ? min(i, rows - 1) * ld : 0]);      // (every load under way together)
+    if (!in) {
+#pragma unroll
+      for (int i = 0; i < DL; ++i) x[i] = 0.f;
+    }
     if (key) {
       float* to = k_out + (place * DP + col) * DL;
 #pragma unroll
       for (int i = 0; i < DL; i += 4) {
         float4 k4;
-        k4.x = x[i] * k_unit[i] * expf(l_end - l_s[i]);
-        k4.y = x[i + 1] * k_unit[i + 1] * expf(l_end - l_s[i + 1]);
-        k4.z = x[i + 2] * k_unit[i + 2] * expf(l_end - l_s[i + 2]);
-        k4.w = x[i + 3] * k_unit[i + 3] * expf(l_end - l_s[i + 3]);
+        k4.x = i < rows ? x[i] * out_factor[i] : 0.f;
+        k4.y = i + 1 < rows ? x[i + 1] * out_factor[i + 1] : 0.f;
+        k4.z = i + 2 < rows ? x[i + 2] * out_factor[i + 2] : 0.f;
+        k4.w = i + 3 < rows ? x[i + 3] * out_factor[i + 3] : 0.f;
         *reinterpret_cast<float4*>(to + i) = k4;
       }
     }
@@ -225,15 +247,17 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
     const int stride = key ? DP : EP;
 #pragma unroll
     for (int i = 0; i < DL; ++i) {
-      float acc = beta_s[i] * x[i] * (key ? k_unit[i] * expf(l_s[i]) : 1.f);
+      // (rows beyond the chunk have no factor; four sums, so that a sum need not wait for the one before)
+      float acc = x[i] * (key ? in_factor[i] : beta_s[i]), more[3] = {};
 #pragma unroll
       for (int j = 0; j < i; j += 4) {
         const float4 a = *reinterpret_cast<const float4*>(&a_s[i][j]);       // (zero from the diagonal on)
         acc -= a.x * x[j];
-        if (j + 1 < i) acc -= a.y * x[j + 1];
-        if (j + 2 < i) acc -= a.z * x[j + 2];
-        if (j + 3 < i) acc -= a.w * x[j + 3];
+        if (j + 1 < i) more[0] -= a.y * x[j + 1];
+        if (j + 2 < i) more[1] -= a.z * x[j + 2];
+        if (j + 3 < i) more[2] -= a.w * x[j + 3];
       }
+      acc += more[0] + (more[1] + more[2]);
       x[i] = acc;
       to[static_cast<int64_t>(i) * stride] = acc;
     }
@@ -247,7 +271,7 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
 // same order, 16 bytes a lane. The four waves' shares of W S meet in LDS (two sets of places in turn: one barrier a chunk),
 // and every wave adds them up for itself.
 template <int TILES>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, 1)
 delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restrict__ v_in, const float* __restrict__ k_in,
                           const float* __restrict__ totals, float* __restrict__ u_out, float* __restrict__ scratch,
                           float* __restrict__ state, const int32_t* __restrict__ first_chunk,
@@ -270,41 +294,48 @@ delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restric
       const int d = d0 + 16 * i + 4 * g + v;
       s[i][v] = column && d < D ? own[static_cast<int64_t>(d) * E] : 0.f;
     }
-  delta_floatx4 w4[4][TILES], k4[TILES][4];
-  float v4[4][4];
-  auto fetch_w = [&](int64_t place) {
+  // What a chunk needs is asked for while the chunk in front of it is worked on, into the other of two sets of registers
+  // (wider states have registers for one set only: asked for as soon as the set is free).
+  constexpr int SETS = TILES <= 2 ? 2 : 1;
+  delta_floatx4 w4[SETS][4][TILES], k4[SETS][TILES][4];
+  float v4[SETS][4][4], total_of[SETS];
+  auto fetch_w = [&](int set, int chunk) {
+    const int64_t place = static_cast<int64_t>(min(chunk, end - 1)) * H + head;
     const float* p = w_in + place * DL * DP + d0 + 4 * g;
 #pragma unroll
     for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int i = 0; i < TILES; ++i) w4[m][i] = *reinterpret_cast<const delta_floatx4*>(p + (16 * m + c) * DP + 16 * i);
+      for (int i = 0; i < TILES; ++i) w4[set][m][i] = *reinterpret_cast<const delta_floatx4*>(p + (16 * m + c) * DP + 16 * i);
   };
-  auto fetch_kv = [&](int64_t place) {
-    const float* p = k_in + (place * DP + d0 + c) * DL + 4 * g;
-#pragma unroll
-    for (int i = 0; i < TILES; ++i)
-#pragma unroll
-      for (int m = 0; m < 4; ++m) k4[i][m] = *reinterpret_cast<const delta_floatx4*>(p + 16 * i * DL + 16 * m);
+  auto fetch_kv = [&](int set, int chunk) {
+    const int64_t place = static_cast<int64_t>(min(chunk, end - 1)) * H + head;
     const float* q = v_in + place * DL * EP + e0 + c;
 #pragma unroll
     for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int v = 0; v < 4; ++v) v4[m][v] = q[(16 * m + 4 * g + v) * EP];
+      for (int v = 0; v < 4; ++v) v4[set][m][v] = q[(16 * m + 4 * g + v) * EP];
+    total_of[set] = totals[place];
+    const float* p = k_in + (place * DP + d0 + c) * DL + 4 * g;
+#pragma unroll
+    for (int i = 0; i < TILES; ++i)
+#pragma unroll
+      for (int m = 0; m < 4; ++m) k4[set][i][m] = *reinterpret_cast<const delta_floatx4*>(p + 16 * i * DL + 16 * m);
   };
-  fetch_w(static_cast<int64_t>(begin) * H + head);
-  fetch_kv(static_cast<int64_t>(begin) * H + head);
-  for (int chunk = begin; chunk < end; ++chunk) {
+  auto work = [&](int chunk, int set) {
     const int64_t place = static_cast<int64_t>(chunk) * H + head;
-    const int64_t next = static_cast<int64_t>(min(chunk + 1, end - 1)) * H + head;
-    const float total = totals[place];
+    if constexpr (SETS == 2) {
+      fetch_w(1 - set, chunk + 1);
+      fetch_kv(1 - set, chunk + 1);
+      __builtin_amdgcn_sched_barrier(0);
+    }
     delta_floatx4 part[4] = {};
 #pragma unroll
     for (int i = 0; i < TILES; ++i)
 #pragma unroll
       for (int t = 0; t < 4; ++t)
 #pragma unroll
-        for (int m = 0; m < 4; ++m) part[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(w4[m][i][t], s[i][t], part[m], 0, 0, 0);
-    fetch_w(next);
+        for (int m = 0; m < 4; ++m) part[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(w4[set][m][i][t], s[i][t], part[m], 0, 0, 0);
+    if constexpr (SETS == 1) fetch_w(0, chunk + 1);
     float(*at)[4][256] = share[(chunk - begin) & 1];
 #pragma unroll
     for (int m = 0; m < 4; ++m) *reinterpret_cast<delta_floatx4*>(&at[wave][m][4 * lane]) = part[m];
@@ -331,7 +362,7 @@ delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restric
         for (int v = 0; v < 4; ++v) sum[v] += more[v];
       }
 #pragma unroll
-      for (int v = 0; v < 4; ++v) u[m][v] = v4[m][v] - sum[v];
+      for (int v = 0; v < 4; ++v) u[m][v] = v4[set][m][v] - sum[v];
     }
 #pragma unroll
     for (int m = 0; m < 4; ++m)
@@ -343,14 +374,22 @@ delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restric
 #pragma unroll
     for (int i = 0; i < TILES; ++i)
 #pragma unroll
-      for (int v = 0; v < 4; ++v) s[i][v] *= total;
+      for (int v = 0; v < 4; ++v) s[i][v] *= total_of[set];
 #pragma unroll
     for (int m = 0; m < 4; ++m)
 #pragma unroll
       for (int t = 0; t < 4; ++t)
 #pragma unroll
-        for (int i = 0; i < TILES; ++i) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[i][m][t], u[m][t], s[i], 0, 0, 0);
-    fetch_kv(next);
+        for (int i = 0; i < TILES; ++i) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[set][i][m][t], u[m][t], s[i], 0, 0, 0);
+    if constexpr (SETS == 1) fetch_kv(0, chunk + 1);
+  };
+  fetch_w(0, begin);
+  fetch_kv(0, begin);
+  for (int chunk = begin; chunk < end; chunk += SETS) {
+    work(chunk, 0);
+    if constexpr (SETS == 2) {
+      if (chunk + 1 < end) work(chunk + 1, 1);
+    }
   }
   if (column) {
 #pragma unroll
@@ -384,9 +423,20 @@ delta_chunk_outputs_kernel(const X* __restrict__ qkv, int64_t ld, const float* _
   delta_floatx16 y = {};
   for (int n0 = 0; n0 < D; n0 += DL) {
     __syncthreads();
-    for (int j = wave; j < DL; j += 4) {
-      a_s[j][lane] = (j < rows && n0 + lane < D) ? to_float(qkv[static_cast<int64_t>(first + j) * ld + q_at + n0 + lane]) : 0.f;
-      b_s[j][lane] = (n0 + j < D && e0 + lane < E) ? s_in[static_cast<int64_t>(n0 + j) * E + e0 + lane] : 0.f;
+    const X* q_from = qkv + static_cast<int64_t>(first) * ld + q_at + min(n0 + lane, D - 1);
+    const float* s_from = s_in + min(e0 + lane, E - 1);
+    X q[16];
+    float s[16];
+#pragma unroll
+    for (int r = 0; r < 16; ++r) {
+      q[r] = q_from[static_cast<int64_t>(min(wave + 4 * r, rows - 1)) * ld];
+      s[r] = s_from[static_cast<int64_t>(min(n0 + wave + 4 * r, D - 1)) * E];
+    }
+#pragma unroll
+    for (int r = 0; r < 16; ++r) {
+      const int j = wave + 4 * r;
+      a_s[j][lane] = j < rows && n0 + lane < D ? to_float(q[r]) : 0.f;
+      b_s[j][lane] = n0 + j < D && e0 + lane < E ? s[r] : 0.f;
     }
     __syncthreads();
     for (int n = 0; n < DL; n += 2)
@@ -394,10 +444,17 @@ delta_chunk_outputs_kernel(const X* __restrict__ qkv, int64_t ld, const float* _
   }
 #pragma unroll
   for (int v = 0; v < 16; ++v) y[v] *= f_s[ib + tile_row(v, lane)];
+  float p[16], u[16];
+#pragma unroll
+  for (int r = 0; r < 16; ++r) {
+    p[r] = pairs[place * DL * DL + (wave + 4 * r) * DL + lane];
+    u[r] = u_in[(place * DL + wave + 4 * r) * EP + min(e0 + lane, EP - 1)];
+  }
   __syncthreads();
-  for (int j = wave; j < DL; j += 4) {
-    a_s[j][lane] = pairs[place * DL * DL + j * DL + lane];
-    b_s[j][lane] = e0 + lane < E ? u_in[(place * DL + j) * EP + e0 + lane] : 0.f;
+#pragma unroll
+  for (int r = 0; r < 16; ++r) {
+    a_s[wave + 4 * r][lane] = p[r];
+    b_s[wave + 4 * r][lane] = e0 + lane < E ? u[r] : 0.f;
   }
   __syncthreads();
   for (int j = 0; j < ib + 32; j += 2)

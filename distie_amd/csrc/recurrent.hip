@@ -857,7 +857,7 @@ struct RouteScratch {
   float weights[ROUTE_MAX_TOP + 1];           // the shared expert's behind those of the chosen
 };
 
-template <int GROUP>                                   // experts worked on side by side: 16, or 8 where there are no more
+template <int GROUP>                                   // experts worked on side by side: 16, or 8 or 12 where there are no more
 __device__ __forceinline__ void route_row_bf16(const bf16_t* __restrict__ x_row, const bf16_t* __restrict__ weight,
                                                const float* __restrict__ bias, int C, int E, int top, int scoring,
                                                const RouteRule& rule, RouteScratch& lds) {
@@ -938,6 +938,8 @@ route_topk_bf16_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ 
   const int64_t t = blockIdx.x;
   if (E + rule.shared <= 8) {
     route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
+  } else if (E + rule.shared <= 12) {
+    route_row_bf16<12>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   } else {
     route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   }
@@ -1070,6 +1072,8 @@ route_topk_glu_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w
   }
   if (E + rule.shared <= 8) {
     route_row_bf16<8>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
+  } else if (E + rule.shared <= 12) {
+    route_row_bf16<12>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   } else {
     route_row_bf16<ROUTE_GROUP>(x + t * C, weight, bias, C, E, top, scoring, rule, lds);
   }

@@ -484,8 +484,22 @@ decay_scan_kernel(const X* __restrict__ product, int64_t ld, float* __restrict__
   const int lane = threadIdx.x % 64, part = threadIdx.x / 64;
   const int e = blockIdx.z * 64 + lane;
   const int first = cu_q[b], last = cu_q[b + 1];
+  if (first >= last) return;
   const float rate = decay[head];
   float* own = state + (static_cast<int64_t>(state_slots[b]) * H + head) * D * E;
+  // a row's values are asked for before the row in front of it (for the first row: the state) is worked on
+  static_assert(PARTS * ROWS <= 64 * PARTS, "a thread fetches one dimension of q and k");
+  float nq = 0.f, nk = 0.f, nv = 0.f;
+  auto fetch = [&](int t) {
+    const X* row = product + static_cast<int64_t>(t) * ld;
+    const int d = threadIdx.x;
+    if (d < D) {
+      nq = scan_value<SILU>(row + head * D, d, t, turn);
+      nk = scan_value<SILU>(row + (H + head) * D, d, t, turn);
+    }
+    nv = e < E ? to_float(row[2 * H * D + head * E + e]) : 0.f;
+  };
+  fetch(first);
   float s[ROWS];
 #pragma unroll
   for (int r = 0; r < ROWS; ++r) {
@@ -493,13 +507,13 @@ decay_scan_kernel(const X* __restrict__ product, int64_t ld, float* __restrict__
     s[r] = (d < D && e < E) ? own[static_cast<int64_t>(d) * E + e] : 0.f;
   }
   for (int t = first; t < last; ++t) {
-    const X* row = product + static_cast<int64_t>(t) * ld;
     __syncthreads();
-    for (int d = threadIdx.x; d < D; d += blockDim.x) {
-      q_s[d] = scan_act<SILU>(scan_value<SILU>(row + head * D, d, t, turn));
-      k_s[d] = scan_act<SILU>(scan_value<SILU>(row + (H + head) * D, d, t, turn)) * (SILU ? 1.f : turn.k_scale);
+    if (threadIdx.x < D) {
+      q_s[threadIdx.x] = scan_act<SILU>(nq);
+      k_s[threadIdx.x] = scan_act<SILU>(nk) * (SILU ? 1.f : turn.k_scale);
     }
-    const float v = e < E ? scan_act<SILU>(to_float(row[2 * H * D + head * E + e])) : 0.f;
+    const float v = scan_act<SILU>(nv);
+    if (t + 1 < last) fetch(t + 1);
     __syncthreads();
     float o = 0.f;
 #pragma unroll
@@ -1003,6 +1017,199 @@ head_norm_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ product, int64_t 
   }
 }
 
+// Filters of TAPS = 2, 3 or 4 taps, head norms, rotation and cache write in one walk: a run of `lanes` lanes (a power of two,
+// DP / 8 rounded up; DP at most 512) owns one q or k head of CONV_ROWS rows of the step, a lane eight neighbouring
+// dimensions. The lane keeps its filters and the last TAPS - 1 inputs in registers, so a row of the product is read once for
+// all the rows that see it; where a row is its request's first of the step, the inputs before it come from the request's
+// state. The head's sum of squares is a sum over its lanes; a pair of the rotation lies in the lane itself
+// (`neighbours`) or in the lane pairs / 8 away. The blocks from `qk_blocks` on write v: 16 rows each, one channel a thread.
+constexpr int CONV_ROWS = 4;
+
+template <int TAPS>
+__global__ void __launch_bounds__(256)
+conv_head_norm_rope_kv_write_bf16_kernel(const bf16_t* __restrict__ product, int64_t ld, const bf16_t* __restrict__ weight,
+                                         float* __restrict__ state, const float2* __restrict__ table, int pairs,
+                                         float magnitude, bf16_t* __restrict__ q_out, bf16_t* __restrict__ k_cache,
+                                         bf16_t* __restrict__ v_cache, const int32_t* __restrict__ slots,
+                                         const int32_t* __restrict__ cu_q, const int32_t* __restrict__ token_request,
+                                         const int32_t* __restrict__ state_slots, int T, int H, int G, int D, int E, int DP,
+                                         int block_size, int has_kv, int write, const int32_t* __restrict__ positions,
+                                         float temp_coef, int temp_every, const float* __restrict__ q_norm,
+                                         const float* __restrict__ k_norm, float norm_eps, int qk_blocks, int lanes,
+                                         int neighbours) {
+  const int N = H * D + (has_kv ? G * (D + E) : 0);
+  if (static_cast<int>(blockIdx.x) >= qk_blocks) {
+    const int t0 = (static_cast<int>(blockIdx.x) - qk_blocks) / G * VGROUP;
+    const int g = (static_cast<int>(blockIdx.x) - qk_blocks) % G;
+    const int n = min(VGROUP, T - t0);
+    const int64_t slot0 = write ? slots[t0] : 0;
+    bool together = write && n == VGROUP && block_size % 8 == 0 && slot0 % block_size % 8 == 0 &&
+                    slot0 % block_size + VGROUP <= block_size;
+    if (write) {
+#pragma unroll
+      for (int k = 1; k < VGROUP; ++k) together = together && slots[min(t0 + k, T - 1)] == slot0 + k;
+    }
+    uint16_t* cache = reinterpret_cast<uint16_t*>(v_cache);
+    for (int e = threadIdx.x; e < E; e += blockDim.x) {
+      const int c = (H + G) * D + g * E + e;
+      float w[TAPS], x[VGROUP], before[TAPS - 1];          // before[m]: row t0 - 1 - m
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) w[j] = to_float(weight[static_cast<int64_t>(c) * TAPS + j]);
+#pragma unroll
+      for (int k = 0; k < VGROUP; ++k) x[k] = to_float(product[static_cast<int64_t>(t0 + min(k, n - 1)) * ld + c]);
+#pragma unroll
+      for (int m = 0; m < TAPS - 1; ++m) before[m] = to_float(product[static_cast<int64_t>(max(t0 - 1 - m, 0)) * ld + c]);
+      uint32_t bits[VGROUP];
+#pragma unroll
+      for (int k = 0; k < VGROUP; ++k) {
+        const int b = token_request[t0 + min(k, n - 1)];
+        const int first = cu_q[b];
+        const int i = t0 + min(k, n - 1) - first;
+        float* own = state + static_cast<int64_t>(state_slots[b]) * (TAPS - 1) * N + c;
+        const bool single = k < n && cu_q[b + 1] - first == 1;
+        float sum = 0.f;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) {
+          const int back = TAPS - 1 - j;
+          float v = back <= k ? x[k - back < 0 ? 0 : k - back] : before[back - k - 1 < 0 ? 0 : back - k - 1];
+          if (back > i) v = own[static_cast<int64_t>(TAPS - 1 - (back - i)) * N];
+          sum += w[j] * v;
+          if (single && j > 0) own[static_cast<int64_t>(j - 1) * N] = v;       // its inputs move on by this row
+        }
+        bits[k] = bf16_bits(sum);
+      }
+      if (!write) continue;
+      if (together) {
+        uint16_t* dst = cache + ((slot0 / block_size * G + g) * DP + e) * block_size + slot0 % block_size;
+        *reinterpret_cast<uint4*>(dst) = uint4{bits[0] | (bits[1] << 16), bits[2] | (bits[3] << 16),
+                                               bits[4] | (bits[5] << 16), bits[6] | (bits[7] << 16)};
+        *reinterpret_cast<uint4*>(dst + 8) = uint4{bits[8] | (bits[9] << 16), bits[10] | (bits[11] << 16),
+                                                   bits[12] | (bits[13] << 16), bits[14] | (bits[15] << 16)};
+      } else {
+#pragma unroll
+        for (int k = 0; k < VGROUP; ++k) {
+          if (k >= n) break;
+          const int64_t slot = slots[t0 + k];
+          cache[((slot / block_size * G + g) * DP + e) * block_size + slot % block_size] = static_cast<uint16_t>(bits[k]);
+        }
+      }
+    }
+    return;
+  }
+  const int turned = has_kv ? H + G : H;
+  const int lane = threadIdx.x % 64 % lanes;
+  const int groups = (T + CONV_ROWS - 1) / CONV_ROWS;
+  const int64_t count = static_cast<int64_t>(groups) * turned;
+  const int64_t unit = (static_cast<int64_t>(blockIdx.x) * 4 + threadIdx.x / 64) * (64 / lanes) + threadIdx.x % 64 / lanes;
+  const int64_t mine = min(unit, count - 1);
+  const int head = static_cast<int>(mine % turned);
+  const int t0 = static_cast<int>(mine / turned) * CONV_ROWS;
+  const int d0 = 8 * lane;
+  const bool inside = unit < count && d0 < D;              // the others only take part in the exchanges
+  const int c0 = head * D + min(d0, D - 8);
+  float w[TAPS][8], norm[8];
+  {
+    float flat[8 * TAPS];
+#pragma unroll
+    for (int q = 0; q < TAPS; ++q) unpack_bf16x8(load16(weight + static_cast<int64_t>(c0) * TAPS + 8 * q), flat + 8 * q);
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) w[j][e] = flat[e * TAPS + j];
+  }
+  const float* norm_weight = head < H ? q_norm : k_norm;
+  if (norm_weight != nullptr) load_f32x8(norm_weight + min(d0, D - 8), norm);
+  // all rows of the product that the run may need, under way together
+  uint4 raw[CONV_ROWS + TAPS - 1];
+#pragma unroll
+  for (int r = 0; r < CONV_ROWS + TAPS - 1; ++r)
+    raw[r] = load16(product + static_cast<int64_t>(min(max(t0 + r - (TAPS - 1), 0), T - 1)) * ld + c0);
+#pragma unroll
+  for (int r = 0; r < CONV_ROWS; ++r) {
+    const int t = t0 + r;
+    const int at = min(t, T - 1);
+    const int b = token_request[at];
+    const int first = cu_q[b];
+    const int i = at - first;
+    float* own = state + static_cast<int64_t>(state_slots[b]) * (TAPS - 1) * N + c0;
+    const bool single = inside && t < T && cu_q[b + 1] - first == 1;
+    float x[8] = {};
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      const int back = TAPS - 1 - j;
+      float v[8];
+      unpack_bf16x8(raw[r + j], v);
+      if (back > i) load_f32x8(own + static_cast<int64_t>(TAPS - 1 - (back - i)) * N, v);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] += w[j][e] * v[e];
+      if (single && j > 0) {                               // a request that brings one row: its inputs move on by that row
+        float4* to = reinterpret_cast<float4*>(own + static_cast<int64_t>(j - 1) * N);
+        to[0] = float4{v[0], v[1], v[2], v[3]};
+        to[1] = float4{v[4], v[5], v[6], v[7]};
+      }
+    }
+    if (!inside) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] = 0.f;
+    }
+    float sq = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sq += x[e] * x[e];
+    for (int o = lanes / 2; o > 0; o >>= 1) sq += __shfl_xor(sq, o, 64);
+    if (norm_weight != nullptr) {
+      const float scale = 1.f / sqrtf(sq / D + norm_eps);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] *= scale * norm[e];
+    }
+    float out[8];
+    if (neighbours) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) out[e] = x[e];
+      if (d0 < 2 * pairs) {                                // (pairs a multiple of 4: all of the lane's pairs turn, or none)
+        const float4* angles = reinterpret_cast<const float4*>(table + static_cast<int64_t>(at) * pairs + d0 / 2);
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+          const float4 cs = angles[e];
+          const float* v = x + 4 * e;
+          out[4 * e] = v[0] * (cs.x * magnitude) - v[1] * (cs.y * magnitude);
+          out[4 * e + 1] = v[1] * (cs.x * magnitude) + v[0] * (cs.y * magnitude);
+          out[4 * e + 2] = v[2] * (cs.z * magnitude) - v[3] * (cs.w * magnitude);
+          out[4 * e + 3] = v[3] * (cs.z * magnitude) + v[2] * (cs.w * magnitude);
+        }
+      }
+    } else {
+      const int shift = pairs / 8;                         // lanes [0, shift) hold the first halves, [shift, 2 shift) the second
+      const int partner = threadIdx.x % 64 - lane + (lane < shift ? lane + shift : (lane < 2 * shift ? lane - shift : lane));
+      float other[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) other[e] = __shfl(x[e], partner, 64), out[e] = x[e];
+      if (lane < 2 * shift) {
+        const bool lower = lane < shift;
+        const float4* angles = reinterpret_cast<const float4*>(table + static_cast<int64_t>(at) * pairs + 8 * (lower ? lane : lane - shift));
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float4 cs = angles[e];
+          const float s0 = lower ? -cs.y : cs.y, s1 = lower ? -cs.w : cs.w;
+          out[2 * e] = x[2 * e] * (cs.x * magnitude) + other[2 * e] * (s0 * magnitude);
+          out[2 * e + 1] = x[2 * e + 1] * (cs.z * magnitude) + other[2 * e + 1] * (s1 * magnitude);
+        }
+      }
+    }
+    if (t >= T || unit >= count) continue;
+    if (head < H) {
+      if (d0 >= DP) continue;
+      const float qt = query_temperature(positions, t, temp_coef, temp_every);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) out[e] *= qt;
+      *reinterpret_cast<uint4*>(q_out + (static_cast<int64_t>(t) * H + head) * DP + d0) = pack_bf16x8(out);
+    } else if (write && d0 < D) {
+      const int64_t slot = slots[t];
+      bf16_t* dst = k_cache + ((slot / block_size * G + (head - H)) * block_size + slot % block_size) * DP;
+      *reinterpret_cast<uint4*>(dst + d0) = pack_bf16x8(out);
+    }
+  }
+}
+
 // out = x * sigmoid(gates), eight a thread
 __global__ void sigmoid_gate_bf16x8_kernel(const bf16_t* __restrict__ x, int ldh, int E, const bf16_t* __restrict__ gates,
                                            int64_t ldg, bf16_t* __restrict__ out, int width, int64_t T) {
@@ -1051,10 +1258,14 @@ __global__ void activation_bf16x8_kernel(const uint4* __restrict__ in, uint4* __
 //   sums:     P[d][e]   = sum_j w^(L-1-j) k_j[d] v_j[e]                      (each chunk alone)
 //   states:   S_next    = w^L S + P, chunk after chunk; S (the state in front) takes P's place in the scratch
 //   outputs:  o_i[e]    = w^(i+1) sum_d q_i[d] S[d][e] + sum_{j<=i} w^(i-j) (q_i . k_j) v_j[e]
-// Only non-negative powers occur, so nothing grows with the chunk's length. Float32 throughout, FMAs on tiles
-// held in LDS; a chunk's table entry is {request, first row, rows, unused}.
+// Only non-negative powers occur, so nothing grows with the chunk's length. Float32 throughout: tiles in LDS,
+// products on v_mfma_f32_32x32x2_f32 (a lane gives A[row = lane % 32][k = lane / 32] and B[k = lane / 32][column = lane % 32]
+// and holds, in register v, the sum for row scan_row(v, lane) and column lane % 32); dimensions beyond D up to DP, the next
+// multiple of 32, are zeros. A chunk's table entry is {request, first row, rows, unused}.
 constexpr int SCAN_L = 64;
-constexpr int SCAN_PAD = 68;      // row stride of the transposed tiles: keeps 16-byte reads aligned
+constexpr int SCAN_PAD = SCAN_L + 1;   // row stride of the tiles: an odd number of words
+typedef __attribute__((__vector_size__(16 * sizeof(float)))) float scan_floatx16;
+__device__ __forceinline__ int scan_row(int v, int lane) { return 8 * (v / 4) + 4 * (lane / 32) + v % 4; }
 constexpr int SCAN_BATCH = 8;     // loads a thread has under way while it fills a tile
 
 __device__ __forceinline__ void decay_powers(float* pw, float rate, int count) {
@@ -1072,8 +1283,9 @@ __global__ void __launch_bounds__(256)
 scan_chunk_sums_kernel(const X* __restrict__ product, int64_t ld, const float* __restrict__ decay, float* __restrict__ scratch,
                        const int4* __restrict__ chunks, int H, int D, int E, ScanTurn turn) {
   extern __shared__ float lds[];
-  float* Ks = lds;                       // [64][D], each row times its power of the decay
-  float* Vs = Ks + SCAN_L * D;           // [64][64]
+  const int DP = (D + 31) / 32 * 32;
+  float* Ks = lds;                       // [64][DP], each row times its power of the decay
+  float* Vs = Ks + SCAN_L * DP;          // [64][64]
   float* pw = Vs + SCAN_L * 64;          // [65]
   const int c = blockIdx.x, head = blockIdx.y, e0 = blockIdx.z * 64;
   const int4 chunk = chunks[c];
@@ -1085,17 +1297,17 @@ scan_chunk_sums_kernel(const X* __restrict__ product, int64_t ld, const float* _
   // time (a load that waits for the one before it costs a trip to memory each; no division by D in the loop).
   const int col = threadIdx.x % 64, sub = threadIdx.x / 64;
   for (int j0 = sub; j0 < SCAN_L; j0 += 4 * SCAN_BATCH) {
-    for (int d = col; d < D; d += 64) {
+    for (int d = col; d < DP; d += 64) {
       float k[SCAN_BATCH];
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
-        k[u] = j < len ? scan_value<SILU>(product + (row0 + j) * ld + (H + head) * D, d, row0 + j, turn) : 0.f;
+        k[u] = j < len && d < D ? scan_value<SILU>(product + (row0 + j) * ld + (H + head) * D, d, row0 + j, turn) : 0.f;
       }
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
-        Ks[j * D + d] = j < len ? pw[len - 1 - j] * (SILU ? siluf(k[u]) : k[u] * turn.k_scale) : 0.f;
+        Ks[j * DP + d] = j < len ? pw[len - 1 - j] * (SILU ? siluf(k[u]) : k[u] * turn.k_scale) : 0.f;
       }
     }
     float v[SCAN_BATCH];
@@ -1108,36 +1320,22 @@ scan_chunk_sums_kernel(const X* __restrict__ product, int64_t ld, const float* _
     for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = scan_act<SILU>(v[u]);
   }
   __syncthreads();
-  const int tx = threadIdx.x % 16, ty = threadIdx.x / 16;
-  float acc[2][4][4] = {};
-#pragma unroll 4
-  for (int j = 0; j < len; ++j) {
-    const float4 v4 = *reinterpret_cast<const float4*>(Vs + j * 64 + 4 * tx);
-    const float v[4] = {v4.x, v4.y, v4.z, v4.w};
+  // a wave: tiles of 32 dimensions d by 32 columns e
+  const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
+  float* dst = scratch + (static_cast<int64_t>(c) * H + head) * D * E;
+  for (int tile = wave; tile < DP / 16; tile += 4) {
+    const int db = 32 * (tile / 2), eb = 32 * (tile % 2);
+    scan_floatx16 acc = {};
+#pragma unroll 8
+    for (int j = 0; j < SCAN_L; j += 2)
+      acc = __builtin_amdgcn_mfma_f32_32x32x2f32(Ks[(j + lane / 32) * DP + db + lane % 32], Vs[(j + lane / 32) * 64 + eb + lane % 32],
+                                                 acc, 0, 0, 0);
 #pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      const int d0 = 4 * ty + 64 * s;
-      if (d0 >= D) break;
-      const float4 k4 = *reinterpret_cast<const float4*>(Ks + j * D + d0);
-      const float k[4] = {k4.x, k4.y, k4.z, k4.w};
-#pragma unroll
-      for (int a = 0; a < 4; ++a)
-#pragma unroll
-        for (int b = 0; b < 4; ++b) acc[s][a][b] += k[a] * v[b];
+    for (int v = 0; v < 16; ++v) {
+      const int d = db + scan_row(v, lane), e = e0 + eb + lane % 32;
+      if (d < D && e < E) dst[static_cast<int64_t>(d) * E + e] = acc[v];
     }
   }
-  float* dst = scratch + (static_cast<int64_t>(c) * H + head) * D * E;
-#pragma unroll
-  for (int s = 0; s < 2; ++s)
-#pragma unroll
-    for (int a = 0; a < 4; ++a) {
-      const int d = 4 * ty + 64 * s + a;
-      if (d >= D) continue;
-      const int e = e0 + 4 * tx;                          // E is a multiple of 4: four columns are there or none
-      if (e < E)
-        *reinterpret_cast<float4*>(dst + static_cast<int64_t>(d) * E + e) =
-            float4{acc[s][a][0], acc[s][a][1], acc[s][a][2], acc[s][a][3]};
-    }
 }
 
 __global__ void scan_chunk_states_kernel(float* __restrict__ scratch, float* __restrict__ state, const float* __restrict__ decay,
@@ -1183,10 +1381,11 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
                           const float* __restrict__ scratch, float* __restrict__ out, const int4* __restrict__ chunks,
                           int H, int D, int E, ScanTurn turn) {
   extern __shared__ float lds[];
-  float* Qt = lds;                       // [D][68]: Qt[d][i]
-  float* Kt = Qt + D * SCAN_PAD;         // [D][68]; once the scores are made, the state in front of the chunk [D][64]
-  float* At = Kt + D * SCAN_PAD;         // [64][68]: At[j][i] = w^(i-j) q_i . k_j for j <= i
-  float* Vs = At + SCAN_L * SCAN_PAD;    // [64][64]
+  const int DP = (D + 31) / 32 * 32;
+  float* Qt = lds;                       // [DP][65]: Qt[d][i]
+  float* Kt = Qt + DP * SCAN_PAD;        // [DP][65]; once the scores are made, the state in front of the chunk [DP][64]
+  float* As = Kt + DP * SCAN_PAD;        // [64][65]: As[i][j] = w^(i-j) q_i . k_j for j <= i
+  float* Vs = As + SCAN_L * SCAN_PAD;    // [64][64]
   float* pw = Vs + SCAN_L * 64;          // [66]
   const int c = blockIdx.x, head = blockIdx.y, e0 = blockIdx.z * 64;
   const int4 chunk = chunks[c];
@@ -1195,14 +1394,14 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
   decay_powers(pw, decay[head], SCAN_L + 2);
   const int col = threadIdx.x % 64, sub = threadIdx.x / 64;
   for (int j0 = sub; j0 < SCAN_L; j0 += 4 * SCAN_BATCH) {
-    for (int d = col; d < D; d += 64) {
+    for (int d = col; d < DP; d += 64) {
       float q[SCAN_BATCH], k[SCAN_BATCH];
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
         const X* row = product + (row0 + j) * ld;
-        q[u] = j < len ? scan_value<SILU>(row + head * D, d, row0 + j, turn) : 0.f;
-        k[u] = j < len ? scan_value<SILU>(row + (H + head) * D, d, row0 + j, turn) : 0.f;
+        q[u] = j < len && d < D ? scan_value<SILU>(row + head * D, d, row0 + j, turn) : 0.f;
+        k[u] = j < len && d < D ? scan_value<SILU>(row + (H + head) * D, d, row0 + j, turn) : 0.f;
       }
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
@@ -1221,31 +1420,25 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
     for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = scan_act<SILU>(v[u]);
   }
   __syncthreads();
-  const int tx = threadIdx.x % 16, ty = threadIdx.x / 16;
-  float s4[4][4] = {};
-  if (tx <= ty) {
+  // the pairs' weights: a wave 32 rows i by 32 rows j (nothing above the diagonal)
+  const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
+  const int ib = 32 * (wave / 2), jb = 32 * (wave % 2);
+  scan_floatx16 pair = {};
+  if (jb <= ib) {
 #pragma unroll 8
-    for (int d = 0; d < D; ++d) {
-      const float4 q4 = *reinterpret_cast<const float4*>(Qt + d * SCAN_PAD + 4 * ty);
-      const float4 k4 = *reinterpret_cast<const float4*>(Kt + d * SCAN_PAD + 4 * tx);
-      const float q[4] = {q4.x, q4.y, q4.z, q4.w}, k[4] = {k4.x, k4.y, k4.z, k4.w};
-#pragma unroll
-      for (int a = 0; a < 4; ++a)
-#pragma unroll
-        for (int b = 0; b < 4; ++b) s4[a][b] += q[a] * k[b];
-    }
+    for (int d = 0; d < DP; d += 2)
+      pair = __builtin_amdgcn_mfma_f32_32x32x2f32(Qt[(d + lane / 32) * SCAN_PAD + ib + lane % 32],
+                                                  Kt[(d + lane / 32) * SCAN_PAD + jb + lane % 32], pair, 0, 0, 0);
   }
 #pragma unroll
-  for (int a = 0; a < 4; ++a)
-#pragma unroll
-    for (int b = 0; b < 4; ++b) {
-      const int i = 4 * ty + a, j = 4 * tx + b;
-      At[j * SCAN_PAD + i] = j <= i ? pw[i - j] * s4[a][b] : 0.f;
-    }
+  for (int v = 0; v < 16; ++v) {
+    const int i = ib + scan_row(v, lane), j = jb + lane % 32;
+    As[i * SCAN_PAD + j] = j <= i ? pw[i - j] * pair[v] : 0.f;
+  }
   __syncthreads();
   float* Ss = Kt;
   const float* src = scratch + (static_cast<int64_t>(c) * H + head) * D * E;
-  for (int d0 = sub; d0 < D; d0 += 4 * SCAN_BATCH) {
+  for (int d0 = sub; d0 < DP; d0 += 4 * SCAN_BATCH) {
     float t[SCAN_BATCH];
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u) {
@@ -1254,40 +1447,26 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
     }
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u)
-      if (d0 + 4 * u < D) Ss[(d0 + 4 * u) * 64 + col] = t[u];
+      if (d0 + 4 * u < DP) Ss[(d0 + 4 * u) * 64 + col] = t[u];
   }
   __syncthreads();
-  float o[4][4] = {}, r[4][4] = {};
+  // a wave: 32 rows i by 32 columns e; the state's share times the row's power, then the chunk's own rows
+  const int eb = 32 * (wave % 2);
+  scan_floatx16 o = {};
 #pragma unroll 8
-  for (int d = 0; d < D; ++d) {
-    const float4 q4 = *reinterpret_cast<const float4*>(Qt + d * SCAN_PAD + 4 * ty);
-    const float4 t4 = *reinterpret_cast<const float4*>(Ss + d * 64 + 4 * tx);
-    const float q[4] = {q4.x, q4.y, q4.z, q4.w}, t[4] = {t4.x, t4.y, t4.z, t4.w};
+  for (int d = 0; d < DP; d += 2)
+    o = __builtin_amdgcn_mfma_f32_32x32x2f32(Qt[(d + lane / 32) * SCAN_PAD + ib + lane % 32],
+                                             Ss[(d + lane / 32) * 64 + eb + lane % 32], o, 0, 0, 0);
 #pragma unroll
-    for (int a = 0; a < 4; ++a)
+  for (int v = 0; v < 16; ++v) o[v] *= pw[ib + scan_row(v, lane) + 1];
+#pragma unroll 8
+  for (int j = 0; j < ib + 32; j += 2)
+    o = __builtin_amdgcn_mfma_f32_32x32x2f32(As[(ib + lane % 32) * SCAN_PAD + j + lane / 32],
+                                             Vs[(j + lane / 32) * 64 + eb + lane % 32], o, 0, 0, 0);
 #pragma unroll
-      for (int b = 0; b < 4; ++b) r[a][b] += q[a] * t[b];
-  }
-  const int reach = min(len, 4 * ty + 4);
-#pragma unroll 4
-  for (int j = 0; j < reach; ++j) {
-    const float4 a4 = *reinterpret_cast<const float4*>(At + j * SCAN_PAD + 4 * ty);
-    const float4 v4 = *reinterpret_cast<const float4*>(Vs + j * 64 + 4 * tx);
-    const float w[4] = {a4.x, a4.y, a4.z, a4.w}, v[4] = {v4.x, v4.y, v4.z, v4.w};
-#pragma unroll
-    for (int a = 0; a < 4; ++a)
-#pragma unroll
-      for (int b = 0; b < 4; ++b) o[a][b] += w[a] * v[b];
-  }
-#pragma unroll
-  for (int a = 0; a < 4; ++a) {
-    const int i = 4 * ty + a;
-    if (i >= len) continue;
-    const int e = e0 + 4 * tx;
-    const float w = pw[i + 1];
-    if (e < E)
-      *reinterpret_cast<float4*>(out + ((row0 + i) * H + head) * E + e) =
-          float4{o[a][0] + w * r[a][0], o[a][1] + w * r[a][1], o[a][2] + w * r[a][2], o[a][3] + w * r[a][3]};
+  for (int v = 0; v < 16; ++v) {
+    const int i = ib + scan_row(v, lane), e = e0 + eb + lane % 32;
+    if (i < len && e < E) out[((row0 + i) * H + head) * E + e] = o[v];
   }
 }
 
@@ -1447,6 +1626,28 @@ extern "C" int distie_conv_rope_kv_write(const void* product, int dtype, int64_t
           static_cast<const bf16_t*>(product), ld, static_cast<const float2*>(table), pairs, magnitude,
           static_cast<bf16_t*>(q_out), static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), slots, T, H, G, D, E, DP,
           block_size, has_kv, write, positions, temp_coef, temp_every, q_norm, k_norm, norm_eps, qk_blocks, lanes, v_base);
+      return launch_status();
+    }
+    if (normed && taps >= 2 && taps <= 4 && !tied && DP <= 512 && D >= 8 && reinterpret_cast<uintptr_t>(weight) % 16 == 0) {
+      const int64_t units = static_cast<int64_t>((T + CONV_ROWS - 1) / CONV_ROWS) * (has_kv ? H + G : H);
+      int lanes = 1;
+      while (8 * lanes < DP) lanes *= 2;
+      const int per_block = 4 * (64 / lanes);
+      const int qk_blocks = static_cast<int>((units + per_block - 1) / per_block);
+#define DISTIE_CONV_HEADS(TAPS)                                                                                          \
+      conv_head_norm_rope_kv_write_bf16_kernel<TAPS><<<qk_blocks + v_blocks, 256, 0, stream>>>(                           \
+          static_cast<const bf16_t*>(product), ld, static_cast<const bf16_t*>(weight), state,                             \
+          static_cast<const float2*>(table), pairs, magnitude, static_cast<bf16_t*>(q_out), static_cast<bf16_t*>(k_cache), \
+          static_cast<bf16_t*>(v_cache), slots, cu_q, token_request, state_slots, T, H, G, D, E, DP, block_size, has_kv,   \
+          write, positions, temp_coef, temp_every, q_norm, k_norm, norm_eps, qk_blocks, lanes, neighbours)
+      if (taps == 2) {
+        DISTIE_CONV_HEADS(2);
+      } else if (taps == 3) {
+        DISTIE_CONV_HEADS(3);
+      } else {
+        DISTIE_CONV_HEADS(4);
+      }
+#undef DISTIE_CONV_HEADS
       return launch_status();
     }
 #define DISTIE_CONV_ROPE_BF16(NORM, LDS)                                                                                 \
@@ -1611,12 +1812,12 @@ extern "C" int distie_decay_scan_chunked(const void* product, int dtype, int64_t
   if (B <= 0 || num_chunks <= 0) return 0;
   if (pairs < 0 || 2 * pairs > D || (pairs > 0 && (turn_table == nullptr || silu))) return DISTIE_BAD_ARGUMENT;
   const ScanTurn turn = {static_cast<const float2*>(turn_table), pairs, neighbours, k_scale};
-  if (H < 1 || D < 4 || E < 4 || D % 4 || E % 4 || D > 128 || ld < static_cast<int64_t>(H) * (2 * D + E))
-    return DISTIE_BAD_ARGUMENT;
+  if (H < 1 || D < 1 || E < 1 || D > 128 || ld < static_cast<int64_t>(H) * (2 * D + E)) return DISTIE_BAD_ARGUMENT;
+  const int DP = (D + 31) / 32 * 32;
   const dim3 grid(num_chunks, H, (E + 63) / 64);
   const int4* table = reinterpret_cast<const int4*>(chunks);
-  const size_t lds_sums = (static_cast<size_t>(SCAN_L) * D + SCAN_L * 64 + SCAN_L + 1) * sizeof(float);
-  const size_t lds_out = (2 * static_cast<size_t>(D) * SCAN_PAD + SCAN_L * SCAN_PAD + SCAN_L * 64 + SCAN_L + 2) * sizeof(float);
+  const size_t lds_sums = (static_cast<size_t>(SCAN_L) * DP + SCAN_L * 64 + SCAN_L + 1) * sizeof(float);
+  const size_t lds_out = (2 * static_cast<size_t>(DP) * SCAN_PAD + SCAN_L * SCAN_PAD + SCAN_L * 64 + SCAN_L + 2) * sizeof(float);
   int status = 0;
   DISTIE_DISPATCH(dtype, X, {
     const auto kernel = silu ? scan_chunk_sums_kernel<true, X> : scan_chunk_sums_kernel<false, X>;

@@ -1416,7 +1416,7 @@ class HipOps(Ops):
         turn = (1 if act else 0, table.data_ptr() if pairs else None, pairs, 1 if neighbours else 0, float(k_scale))
         out = torch.empty((T, num_heads * value_dim), dtype=torch.float32, device=self.device)
         if not self.captured and meta.host_cu_q is not None and meta.max_q >= self.SCAN_CHUNKED_MIN_ROWS and \
-                dim % 4 == 0 and value_dim % 4 == 0 and dim <= self._ops.distie_decay_scan_chunked_max_dim():
+                dim <= self._ops.distie_decay_scan_chunked_max_dim():
             # portions of prompts: chunks of rows side by side instead of one row after the other. Which rows form
             # a chunk is worked out here from the step's row counts (known on the host outside captured steps).
             count, packed, scratch = self._scan_chunks(meta, self._ops.distie_decay_scan_chunk_rows(), num_heads, dim,
