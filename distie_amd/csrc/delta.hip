@@ -111,14 +111,36 @@ delta_scan_kernel(const X* __restrict__ qkv, int64_t ld, const X* __restrict__ b
 //   states  (request, head, 16 columns e): U and the state in front of every chunk, chunk after chunk
 //   outputs (chunk, head, 64 columns): o
 // Float32 throughout, products on float32 matrix products. Scratch is padded: DP = D rounded up to a multiple of 64 that
-// four waves share evenly (64, 128 or 256), EP = E rounded up to a multiple of 16, zeros beyond D, E and a chunk's rows. A
-// chunk's table entry is {request, first row, rows, unused}.
+// four waves share evenly (64, 128 or 256), EP = E rounded up to a multiple of 16, zeros beyond D, E and a chunk's rows. It
+// lies in tiles of 16 x 16 in the order in which a wave of `states` holds them, lane (g = lane / 16, c = lane % 16) four
+// neighbouring values, so that the wave reads and writes a tile as one run of 1,024 bytes:
+//   W       [chunk, head][rows / 16][DP / 16]:    lane holds row c, columns 4 g ..
+//   k~      [chunk, head][DP / 16][rows / 16]:    lane holds dimension c, rows 4 g ..
+//   V', U   [chunk, head][EP / 16][rows / 16]:    lane holds rows 4 g .., column c
+//   states  [chunk, head][EP / 16][DP / 16]:      lane holds dimensions 4 g .., column c
+// A chunk's table entry is {request, first row, rows, unused}.
 constexpr int DL = 64;
 constexpr int DL_PAD = DL + 1;
 constexpr int DL_ROW = DL + 4;          // row stride of the triangular matrix: 16-byte reads of a row
 typedef __attribute__((__vector_size__(16 * sizeof(float)))) float delta_floatx16;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float delta_floatx4;
 __device__ __forceinline__ int tile_row(int v, int lane) { return 8 * (v / 4) + 4 * (lane / 32) + v % 4; }
+
+// a[k] of thread q of four neighbours <-> a[q] of thread k
+__device__ __forceinline__ void transpose_quad(float a[4]) {
+  const int q = threadIdx.x % 4;
+  const auto swap = [](float& low, float& high, bool upper, float partner) {
+    if (upper) low = partner;
+    else high = partner;
+  };
+  const auto near = [](float x) { return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(x), 0xB1, 0xf, 0xf, true)); };
+  const auto far = [](float x) { return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(x), 0x4E, 0xf, 0xf, true)); };
+  const bool odd = q & 1, upper = q & 2;
+  swap(a[0], a[1], odd, near(odd ? a[0] : a[1]));
+  swap(a[2], a[3], odd, near(odd ? a[2] : a[3]));
+  swap(a[0], a[2], upper, far(upper ? a[0] : a[2]));
+  swap(a[1], a[3], upper, far(upper ? a[1] : a[3]));
+}
 
 template <typename X>
 __global__ void __launch_bounds__(256, 2)
@@ -232,7 +254,7 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
       for (int i = 0; i < DL; ++i) x[i] = 0.f;
     }
     if (key) {
-      float* to = k_out + (place * DP + col) * DL;
+      float* to = k_out + (place * DP + col / 16 * 16) * DL + col % 16 * 4;
 #pragma unroll
       for (int i = 0; i < DL; i += 4) {
         float4 k4;
@@ -240,11 +262,9 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
         k4.y = i + 1 < rows ? x[i + 1] * out_factor[i + 1] : 0.f;
         k4.z = i + 2 < rows ? x[i + 2] * out_factor[i + 2] : 0.f;
         k4.w = i + 3 < rows ? x[i + 3] * out_factor[i + 3] : 0.f;
-        *reinterpret_cast<float4*>(to + i) = k4;
+        *reinterpret_cast<float4*>(to + i / 16 * 256 + i / 4 % 4 * 64) = k4;
       }
     }
-    float* to = key ? w_out + place * DL * DP + col : v_out + place * DL * EP + col;
-    const int stride = key ? DP : EP;
 #pragma unroll
     for (int i = 0; i < DL; ++i) {
       // (rows beyond the chunk have no factor; four sums, so that a sum need not wait for the one before)
@@ -259,7 +279,20 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
       }
       acc += more[0] + (more[1] + more[2]);
       x[i] = acc;
-      to[static_cast<int64_t>(i) * stride] = acc;
+    }
+    if (key) {
+      // four neighbouring columns change places with four rows: a thread then holds one row's four columns
+      float* to = w_out + place * DL * DP + col / 16 * 256 + col / 4 % 4 * 64 + tid % 4 * 4;
+#pragma unroll
+      for (int i = 0; i < DL; i += 4) {
+        transpose_quad(x + i);
+        *reinterpret_cast<float4*>(to + i / 16 * (DP / 16) * 256 + i % 16 * 4) = float4{x[i], x[i + 1], x[i + 2], x[i + 3]};
+      }
+    } else {
+      float* to = v_out + (place * EP + col / 16 * 16) * DL + col % 16 * 4;
+#pragma unroll
+      for (int i = 0; i < DL; i += 4)
+        *reinterpret_cast<float4*>(to + i / 16 * 256 + i / 4 % 4 * 64) = float4{x[i], x[i + 1], x[i + 2], x[i + 3]};
     }
   }
 }
@@ -267,8 +300,8 @@ delta_chunk_prepare_kernel(const X* __restrict__ qkv, int64_t ld, const X* __res
 // blockIdx = (request, head, 16 columns e). Wave w keeps rows d = 16 TILES w .. of the state's 16 columns as TILES tiles of
 // 16 x 16 in the products' own result layout: lane (g = lane / 16, c = lane % 16) holds rows 4 g + v and column c of a tile,
 // which is also what the second operand of v_mfma_f32_16x16x4_f32 takes if the four products of a step of 16 summed indexes
-// take index 4 g + t from lane group g at product t. So neither the state nor U moves between lanes; W and k~ are read in the
-// same order, 16 bytes a lane. The four waves' shares of W S meet in LDS (two sets of places in turn: one barrier a chunk),
+// take index 4 g + t from lane group g at product t. So neither the state nor U moves between lanes; W and k~ lie in that
+// order too. The four waves' shares of W S meet in LDS (two sets of places in turn: one barrier a chunk),
 // and every wave adds them up for itself.
 template <int TILES>
 __global__ void __launch_bounds__(256, 1)
@@ -298,31 +331,40 @@ delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restric
   // (wider states have registers for one set only: asked for as soon as the set is free).
   constexpr int SETS = TILES <= 2 ? 2 : 1;
   delta_floatx4 w4[SETS][4][TILES], k4[SETS][TILES][4];
-  float v4[SETS][4][4], total_of[SETS];
+  delta_floatx4 v4[SETS][4];
+  float total_of[SETS];
   auto fetch_w = [&](int set, int chunk) {
     const int64_t place = static_cast<int64_t>(min(chunk, end - 1)) * H + head;
-    const float* p = w_in + place * DL * DP + d0 + 4 * g;
+    const float* p = w_in + place * DL * DP + TILES * wave * 256 + 4 * lane;
 #pragma unroll
     for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int i = 0; i < TILES; ++i) w4[set][m][i] = *reinterpret_cast<const delta_floatx4*>(p + (16 * m + c) * DP + 16 * i);
+      for (int i = 0; i < TILES; ++i) w4[set][m][i] = *reinterpret_cast<const delta_floatx4*>(p + (m * (DP / 16) + i) * 256);
   };
   auto fetch_kv = [&](int set, int chunk) {
     const int64_t place = static_cast<int64_t>(min(chunk, end - 1)) * H + head;
-    const float* q = v_in + place * DL * EP + e0 + c;
+    const float* q = v_in + (place * EP + e0) * DL + 4 * lane;
 #pragma unroll
-    for (int m = 0; m < 4; ++m)
-#pragma unroll
-      for (int v = 0; v < 4; ++v) v4[set][m][v] = q[(16 * m + 4 * g + v) * EP];
+    for (int m = 0; m < 4; ++m) v4[set][m] = *reinterpret_cast<const delta_floatx4*>(q + m * 256);
     total_of[set] = totals[place];
-    const float* p = k_in + (place * DP + d0 + c) * DL + 4 * g;
+    const float* p = k_in + (place * DP + d0) * DL + 4 * lane;
 #pragma unroll
     for (int i = 0; i < TILES; ++i)
 #pragma unroll
-      for (int m = 0; m < 4; ++m) k4[set][i][m] = *reinterpret_cast<const delta_floatx4*>(p + 16 * i * DL + 16 * m);
+      for (int m = 0; m < 4; ++m) k4[set][i][m] = *reinterpret_cast<const delta_floatx4*>(p + (4 * i + m) * 256);
+  };
+  delta_floatx4 mine = {};                                 // the rows of U that this wave hands on: tile `wave`
+  auto store_u = [&](int chunk) {
+    *reinterpret_cast<delta_floatx4*>(u_out + ((static_cast<int64_t>(chunk) * H + head) * EP + e0) * DL + wave * 256 + 4 * lane) = mine;
   };
   auto work = [&](int chunk, int set) {
     const int64_t place = static_cast<int64_t>(chunk) * H + head;
+    // stores first, so that they are a chunk old when the next wait for loads comes: the state in front of the chunk, and the
+    // chunk before's U
+    float* to = scratch + (place * EP + e0) * DP + TILES * wave * 256 + 4 * lane;
+#pragma unroll
+    for (int i = 0; i < TILES; ++i) *reinterpret_cast<delta_floatx4*>(to + i * 256) = s[i];
+    if (chunk > begin) store_u(chunk - 1);
     if constexpr (SETS == 2) {
       fetch_w(1 - set, chunk + 1);
       fetch_kv(1 - set, chunk + 1);
@@ -339,17 +381,6 @@ delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restric
     float(*at)[4][256] = share[(chunk - begin) & 1];
 #pragma unroll
     for (int m = 0; m < 4; ++m) *reinterpret_cast<delta_floatx4*>(&at[wave][m][4 * lane]) = part[m];
-    // the state in front of the chunk, for the outputs
-    if (column) {
-      float* to = scratch + place * D * E + e0 + c;
-#pragma unroll
-      for (int i = 0; i < TILES; ++i)
-#pragma unroll
-        for (int v = 0; v < 4; ++v) {
-          const int d = d0 + 16 * i + 4 * g + v;
-          if (d < D) to[static_cast<int64_t>(d) * E] = s[i][v];
-        }
-    }
     __syncthreads();
     float u[4][4];
 #pragma unroll
@@ -366,11 +397,8 @@ delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restric
     }
 #pragma unroll
     for (int m = 0; m < 4; ++m)
-      if (m == wave) {
-        float* to = u_out + place * DL * EP + e0 + c;
 #pragma unroll
-        for (int v = 0; v < 4; ++v) to[(16 * m + 4 * g + v) * EP] = u[m][v];
-      }
+      for (int v = 0; v < 4; ++v) mine[v] = m == wave ? u[m][v] : mine[v];
 #pragma unroll
     for (int i = 0; i < TILES; ++i)
 #pragma unroll
@@ -391,6 +419,7 @@ delta_chunk_states_kernel(const float* __restrict__ w_in, const float* __restric
       if (chunk + 1 < end) work(chunk + 1, 1);
     }
   }
+  store_u(end - 1);
   if (column) {
 #pragma unroll
     for (int i = 0; i < TILES; ++i)
@@ -407,7 +436,8 @@ template <typename X>
 __global__ void __launch_bounds__(256)
 delta_chunk_outputs_kernel(const X* __restrict__ qkv, int64_t ld, const float* __restrict__ q_factor,
                            const float* __restrict__ pairs, const float* __restrict__ u_in, const float* __restrict__ scratch,
-                           float* __restrict__ out, const int4* __restrict__ chunks, int H, int G, int D, int E, int EP) {
+                           float* __restrict__ out, const int4* __restrict__ chunks, int H, int G, int D, int E, int DP,
+                           int EP) {
   __shared__ float a_s[DL][DL_PAD];     // a tile of q [i][d], then the pairs' weights [i][j]
   __shared__ float b_s[DL][DL_PAD];     // a tile of the state [d][e], then U [j][e]
   __shared__ float f_s[DL];
@@ -419,43 +449,53 @@ delta_chunk_outputs_kernel(const X* __restrict__ qkv, int64_t ld, const float* _
   const int64_t q_at = static_cast<int64_t>(head / (H / G)) * D;
   if (threadIdx.x < DL) f_s[threadIdx.x] = q_factor[place * DL + threadIdx.x];
   const int ib = 32 * (wave / 2), pb = 32 * (wave % 2);
-  const float* s_in = scratch + place * D * E;
+  const float* s_in = scratch + place * DP * EP;
+  // four tiles of the wave's 16 columns -> rows of b_s
+  auto spread = [&](const float4 tiles[4]) {
+#pragma unroll
+    for (int m = 0; m < 4; ++m) {
+      const int row = 16 * m + 4 * (lane / 16), col = 16 * wave + lane % 16;
+      b_s[row][col] = tiles[m].x;
+      b_s[row + 1][col] = tiles[m].y;
+      b_s[row + 2][col] = tiles[m].z;
+      b_s[row + 3][col] = tiles[m].w;
+    }
+  };
   delta_floatx16 y = {};
   for (int n0 = 0; n0 < D; n0 += DL) {
     __syncthreads();
     const X* q_from = qkv + static_cast<int64_t>(first) * ld + q_at + min(n0 + lane, D - 1);
-    const float* s_from = s_in + min(e0 + lane, E - 1);
     X q[16];
-    float s[16];
+    float4 s[4];
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      q[r] = q_from[static_cast<int64_t>(min(wave + 4 * r, rows - 1)) * ld];
-      s[r] = s_from[static_cast<int64_t>(min(n0 + wave + 4 * r, D - 1)) * E];
-    }
+    for (int r = 0; r < 16; ++r) q[r] = q_from[static_cast<int64_t>(min(wave + 4 * r, rows - 1)) * ld];
+    // a wave: the 16 columns 16 wave .., four tiles of 16 dimensions (zeros beyond D, up to DP)
+    const float* s_from = s_in + static_cast<int64_t>(min(e0 + 16 * wave, EP - 16)) * DP + n0 / 16 * 256 + 4 * lane;
+#pragma unroll
+    for (int m = 0; m < 4; ++m) s[m] = *reinterpret_cast<const float4*>(s_from + m * 256);
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int j = wave + 4 * r;
       a_s[j][lane] = j < rows && n0 + lane < D ? to_float(q[r]) : 0.f;
-      b_s[j][lane] = n0 + j < D && e0 + lane < E ? s[r] : 0.f;
     }
+    spread(s);
     __syncthreads();
     for (int n = 0; n < DL; n += 2)
       y = __builtin_amdgcn_mfma_f32_32x32x2f32(a_s[ib + lane % 32][n + lane / 32], b_s[n + lane / 32][pb + lane % 32], y, 0, 0, 0);
   }
 #pragma unroll
   for (int v = 0; v < 16; ++v) y[v] *= f_s[ib + tile_row(v, lane)];
-  float p[16], u[16];
+  float p[16];
+  float4 u[4];
 #pragma unroll
-  for (int r = 0; r < 16; ++r) {
-    p[r] = pairs[place * DL * DL + (wave + 4 * r) * DL + lane];
-    u[r] = u_in[(place * DL + wave + 4 * r) * EP + min(e0 + lane, EP - 1)];
-  }
+  for (int r = 0; r < 16; ++r) p[r] = pairs[place * DL * DL + (wave + 4 * r) * DL + lane];
+  const float* u_from = u_in + (place * EP + min(e0 + 16 * wave, EP - 16)) * DL + 4 * lane;
+#pragma unroll
+  for (int m = 0; m < 4; ++m) u[m] = *reinterpret_cast<const float4*>(u_from + m * 256);
   __syncthreads();
 #pragma unroll
-  for (int r = 0; r < 16; ++r) {
-    a_s[wave + 4 * r][lane] = p[r];
-    b_s[wave + 4 * r][lane] = e0 + lane < E ? u[r] : 0.f;
-  }
+  for (int r = 0; r < 16; ++r) a_s[wave + 4 * r][lane] = p[r];
+  spread(u);
   __syncthreads();
   for (int j = 0; j < ib + 32; j += 2)
     y = __builtin_amdgcn_mfma_f32_32x32x2f32(a_s[ib + lane % 32][j + lane / 32], b_s[j + lane / 32][pb + lane % 32], y, 0, 0, 0);
@@ -502,9 +542,9 @@ extern "C" int distie_delta_scan_chunk_rows() { return DL; }
 extern "C" int distie_delta_scan_padded_dim(int D) { return D <= 64 ? 64 : (D <= 128 ? 128 : 256); }
 
 // chunks: int32 [count][4] = {request, first row, rows (1..64), 0}, the chunks of a request one after the other;
-// first_chunk: int32 [B + 1]. Float32 scratch, DP = distie_delta_scan_padded_dim(D), EP = E rounded up to a multiple of 16:
-// w [count, H, 64, DP], v and u [count, H, 64, EP], k [count, H, DP, 64], pairs [count, H, 64, 64], q_factor [count, H, 64],
-// totals [count, H], states [count, H, D, E].
+// first_chunk: int32 [B + 1]. Float32 scratch, DP = distie_delta_scan_padded_dim(D), EP = E rounded up to a multiple of 16
+// (numbers of elements; for their order see above): w [count, H, 64, DP], v and u [count, H, 64, EP], k [count, H, DP, 64], pairs [count, H, 64, 64], q_factor [count, H, 64],
+// totals [count, H], states [count, H, DP, EP].
 extern "C" int distie_delta_scan_chunked(const void* qkv, int dtype, int64_t ld, const void* beta, int64_t ldb,
                                          const void* decay, int64_t lda, const float* a_log, const float* dt_bias,
                                          float* state, float* out, float* w, float* v, float* u, float* k, float* pairs,
@@ -534,6 +574,6 @@ extern "C" int distie_delta_scan_chunked(const void* qkv, int dtype, int64_t ld,
 #undef DISTIE_DELTA_STATES
   if ((status = launch_status()) != 0) return status;
   DISTIE_DISPATCH(dtype, X, (delta_chunk_outputs_kernel<X><<<dim3(count, H, (E + 63) / 64), 256, 0, stream>>>(
-      static_cast<const X*>(qkv), ld, q_factor, pairs, u, states, out, table, H, G, D, E, EP)));
+      static_cast<const X*>(qkv), ld, q_factor, pairs, u, states, out, table, H, G, D, E, DP, EP)));
   return launch_status();
 }

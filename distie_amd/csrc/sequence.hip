@@ -470,6 +470,22 @@ __device__ __forceinline__ float scan_value(const X* __restrict__ head, int d, i
   return x;
 }
 
+// The same for many rows at one dimension: which other dimension it is turned with, which of a row's angles, and the sign of
+// the other's share (0: it is not turned; what is read is then dropped).
+struct TurnedDim {
+  int other, pair;
+  float sign;
+};
+__device__ __forceinline__ TurnedDim turned_dim(int d, const ScanTurn& turn) {
+  if (d >= 2 * turn.pairs) return TurnedDim{d, 0, 0.f};
+  const bool first = turn.neighbours ? d % 2 == 0 : d < turn.pairs;
+  const int step = turn.neighbours ? 1 : turn.pairs;
+  return TurnedDim{first ? d + step : d - step, turn.neighbours ? d / 2 : (first ? d : d - turn.pairs), first ? -1.f : 1.f};
+}
+__device__ __forceinline__ float turned_value(float x, float other, const float2& cs, const TurnedDim& by) {
+  return by.sign == 0.f ? x : x * cs.x + by.sign * other * cs.y;
+}
+
 template <bool SILU>
 __device__ __forceinline__ float scan_act(float x) { return SILU ? siluf(x) : x; }
 
@@ -1298,23 +1314,35 @@ scan_chunk_sums_kernel(const X* __restrict__ product, int64_t ld, const float* _
   const int col = threadIdx.x % 64, sub = threadIdx.x / 64;
   for (int j0 = sub; j0 < SCAN_L; j0 += 4 * SCAN_BATCH) {
     for (int d = col; d < DP; d += 64) {
-      float k[SCAN_BATCH];
+      float k[SCAN_BATCH], other[SCAN_BATCH];
+      float2 cs[SCAN_BATCH];
+      const TurnedDim by = turned_dim(min(d, D - 1), turn);
+      // (addresses clamped into the chunk, so that every load is under way before the first is used)
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
-        const int j = j0 + 4 * u;
-        k[u] = j < len && d < D ? scan_value<SILU>(product + (row0 + j) * ld + (H + head) * D, d, row0 + j, turn) : 0.f;
+        const int64_t t = row0 + min(j0 + 4 * u, len - 1);
+        const X* from = product + t * ld + (H + head) * D;
+        k[u] = to_float(from[min(d, D - 1)]);
+        if constexpr (!SILU) {
+          other[u] = to_float(from[by.other]);
+          cs[u] = turn.pairs > 0 ? turn.table[t * turn.pairs + by.pair] : float2{1.f, 0.f};
+        }
       }
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
-        Ks[j * DP + d] = j < len ? pw[len - 1 - j] * (SILU ? siluf(k[u]) : k[u] * turn.k_scale) : 0.f;
+        float value;
+        if constexpr (SILU) value = siluf(k[u]);
+        else value = turned_value(k[u], other[u], cs[u], by) * turn.k_scale;
+        Ks[j * DP + d] = j < len && d < D ? pw[len - 1 - j] * value : 0.f;
       }
     }
     float v[SCAN_BATCH];
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u) {
       const int j = j0 + 4 * u;
-      v[u] = (j < len && e0 + col < E) ? to_float(product[(row0 + j) * ld + 2 * H * D + head * E + e0 + col]) : 0.f;
+      v[u] = to_float(product[(row0 + min(j, len - 1)) * ld + 2 * H * D + head * E + min(e0 + col, E - 1)]);
+      if (j >= len || e0 + col >= E) v[u] = 0.f;
     }
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = scan_act<SILU>(v[u]);
@@ -1395,26 +1423,42 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
   const int col = threadIdx.x % 64, sub = threadIdx.x / 64;
   for (int j0 = sub; j0 < SCAN_L; j0 += 4 * SCAN_BATCH) {
     for (int d = col; d < DP; d += 64) {
-      float q[SCAN_BATCH], k[SCAN_BATCH];
+      float q[SCAN_BATCH], k[SCAN_BATCH], other_q[SCAN_BATCH], other_k[SCAN_BATCH];
+      float2 cs[SCAN_BATCH];
+      const TurnedDim by = turned_dim(min(d, D - 1), turn);
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
-        const int j = j0 + 4 * u;
-        const X* row = product + (row0 + j) * ld;
-        q[u] = j < len && d < D ? scan_value<SILU>(row + head * D, d, row0 + j, turn) : 0.f;
-        k[u] = j < len && d < D ? scan_value<SILU>(row + (H + head) * D, d, row0 + j, turn) : 0.f;
+        const int64_t t = row0 + min(j0 + 4 * u, len - 1);
+        const X* from = product + t * ld + head * D;
+        q[u] = to_float(from[min(d, D - 1)]);
+        k[u] = to_float(from[H * D + min(d, D - 1)]);
+        if constexpr (!SILU) {
+          other_q[u] = to_float(from[by.other]);
+          other_k[u] = to_float(from[H * D + by.other]);
+          cs[u] = turn.pairs > 0 ? turn.table[t * turn.pairs + by.pair] : float2{1.f, 0.f};
+        }
       }
 #pragma unroll
       for (int u = 0; u < SCAN_BATCH; ++u) {
         const int j = j0 + 4 * u;
-        Qt[d * SCAN_PAD + j] = scan_act<SILU>(q[u]);
-        Kt[d * SCAN_PAD + j] = SILU ? siluf(k[u]) : k[u] * turn.k_scale;
+        const bool in = j < len && d < D;
+        float q_value, k_value;
+        if constexpr (SILU) {
+          q_value = siluf(q[u]), k_value = siluf(k[u]);
+        } else {
+          q_value = turned_value(q[u], other_q[u], cs[u], by);
+          k_value = turned_value(k[u], other_k[u], cs[u], by) * turn.k_scale;
+        }
+        Qt[d * SCAN_PAD + j] = in ? q_value : 0.f;
+        Kt[d * SCAN_PAD + j] = in ? k_value : 0.f;
       }
     }
     float v[SCAN_BATCH];
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u) {
       const int j = j0 + 4 * u;
-      v[u] = (j < len && e0 + col < E) ? to_float(product[(row0 + j) * ld + 2 * H * D + head * E + e0 + col]) : 0.f;
+      v[u] = to_float(product[(row0 + min(j, len - 1)) * ld + 2 * H * D + head * E + min(e0 + col, E - 1)]);
+      if (j >= len || e0 + col >= E) v[u] = 0.f;
     }
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u) Vs[(j0 + 4 * u) * 64 + col] = scan_act<SILU>(v[u]);
@@ -1443,7 +1487,8 @@ scan_chunk_outputs_kernel(const X* __restrict__ product, int64_t ld, const float
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u) {
       const int d = d0 + 4 * u;
-      t[u] = (d < D && e0 + col < E) ? src[static_cast<int64_t>(d) * E + e0 + col] : 0.f;
+      t[u] = src[static_cast<int64_t>(min(d, D - 1)) * E + min(e0 + col, E - 1)];
+      if (d >= D || e0 + col >= E) t[u] = 0.f;
     }
 #pragma unroll
     for (int u = 0; u < SCAN_BATCH; ++u)

@@ -1988,8 +1988,8 @@ class HipOps(Ops):
         if not self.captured and meta.host_cu_q is not None and meta.max_q >= self.SCAN_CHUNKED_MIN_ROWS:
             # portions of prompts: chunks of rows, the triangular systems of all chunks side by side
             rows = self._ops.distie_delta_scan_chunk_rows()
-            count, packed, states = self._scan_chunks(meta, rows, H, D, E)
             DP, EP = self._ops.distie_delta_scan_padded_dim(D), -(-E // 16) * 16
+            count, packed, states = self._scan_chunks(meta, rows, H, DP, EP)
             key = ("delta_scratch", count, H, DP, EP)
             held = meta.scratch.get(key)
             if held is None:
