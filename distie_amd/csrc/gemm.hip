@@ -488,7 +488,7 @@ static int packed_waves(int K) {
 
 // y: as distie_gemm_skinny_bf16 (the same cut along K: slices go to other workgroups, hence to other
 // compute units, which a product with few rows of W needs to pull its bytes fast enough);
-// gated: [M, N / 2] of y_dtype, never cut. Up to 256 rows of x, in groups of 16. limit, slope, up_shift: of the clamped
+// gated 1: [M, N / 2] of y_dtype, never cut; gated 2: a plain product, [M, N] of y_dtype, never cut. Up to 256 rows of x, in groups of 16. limit, slope, up_shift: of the clamped
 // activation (5 above the low eight bits of `gated`).
 extern "C" int distie_gemm_packed_bf16(const void* x, const void* w_packed, const float* bias, void* y, int y_dtype,
                                        int M, int N, int K, int gated, float limit, float slope, float up_shift,
@@ -496,9 +496,11 @@ extern "C" int distie_gemm_packed_bf16(const void* x, const void* w_packed, cons
   if (M <= 0) return 0;
   const int act = gated >> 8;           // the activation on the gate, above the low eight bits
   gated &= 0xff;
-  if (M > 256 || N <= 0 || K <= 0 || K % 8 != 0 || (gated && N % 2 != 0) || act < 0 || act > 5 || (act == 5 && !(limit > 0.f))) return DISTIE_BAD_ARGUMENT;
+  if (M > 256 || N <= 0 || K <= 0 || K % 8 != 0 || (gated == 1 && N % 2 != 0) || gated > 2 || act < 0 || act > 5 || (act == 5 && !(limit > 0.f))) return DISTIE_BAD_ARGUMENT;
   int slices = 1, k_per_slice = (K + SK_KSTEP - 1) / SK_KSTEP * SK_KSTEP;
-  if (!gated) skinny_plan(N, K, &slices, &k_per_slice);
+  const bool whole = gated == 2;        // plain, the whole K in one workgroup: its waves share it and add their sums in LDS
+  if (whole) gated = 0;
+  if (!gated && !whole) skinny_plan(N, K, &slices, &k_per_slice);
   if (slices > 1 && y_dtype != DISTIE_F32) return DISTIE_BAD_ARGUMENT;
   const int row_blocks = gated ? (N / 2 + 7) / 8 : (N + 15) / 16;
   dim3 grid(row_blocks, slices, (M + 15) / 16);
@@ -517,6 +519,12 @@ extern "C" int distie_gemm_packed_bf16(const void* x, const void* w_packed, cons
                                     xb, wb, bias, static_cast<Y*>(y), M, N, K, k_per_slice / 32, none)));
   } else if (gated) {
     DISTIE_DISPATCH(y_dtype, Y, (gemm_packed_kernel<Y, PK_GATED, 1><<<grid, 64, 0, stream>>>(
+                                    xb, wb, bias, static_cast<Y*>(y), M, N, K, k_per_slice / 32, none)));
+  } else if (whole && K >= 4096) {
+    DISTIE_DISPATCH(y_dtype, Y, (gemm_packed_kernel<Y, PK_PLAIN, 8><<<grid, 512, 0, stream>>>(
+                                    xb, wb, bias, static_cast<Y*>(y), M, N, K, k_per_slice / 32, none)));
+  } else if (whole) {
+    DISTIE_DISPATCH(y_dtype, Y, (gemm_packed_kernel<Y, PK_PLAIN, 4><<<grid, 256, 0, stream>>>(
                                     xb, wb, bias, static_cast<Y*>(y), M, N, K, k_per_slice / 32, none)));
   } else {
     DISTIE_DISPATCH(y_dtype, Y, (gemm_packed_kernel<Y, PK_PLAIN, 1><<<grid, 64, 0, stream>>>(

@@ -107,19 +107,36 @@ constexpr int SSM_PAD = SSM_L + 1;
 typedef __attribute__((__vector_size__(16 * sizeof(float)))) float ssm_floatx16;
 __device__ __forceinline__ int tile_row(int v, int lane) { return 8 * (v / 4) + 4 * (lane / 32) + v % 4; }
 
-// d_j and l_j of a chunk's rows for one head, into LDS (thread 0 adds the logarithms in order)
+// A 64 x 64 tile of a chunk into LDS: rows j, columns n of `from` (row stride ld), zeros where n >= columns or j >= rows. The
+// sixteen elements a thread brings are asked for together: addresses are clamped into what is there, the rest is dropped.
+template <typename X>
+__device__ __forceinline__ void stage_tile(float (*tile)[SSM_PAD], const X* __restrict__ from, int64_t ld, int rows, int columns) {
+  const int n = threadIdx.x % 64, part = threadIdx.x / 64;
+  X raw[16];
+#pragma unroll
+  for (int r = 0; r < 16; ++r) raw[r] = from[static_cast<int64_t>(min(part + 4 * r, rows - 1)) * ld + min(n, columns - 1)];
+#pragma unroll
+  for (int r = 0; r < 16; ++r) {
+    const int j = part + 4 * r;
+    tile[j][n] = j < rows && n < columns ? to_float(raw[r]) : 0.f;
+  }
+}
+
+// d_j and l_j of a chunk's rows for one head, into LDS (the running sums by the first wave, one row a lane)
 template <typename X>
 __device__ __forceinline__ void chunk_decays(const X* __restrict__ dt, int64_t ldd, int first, int rows, int head,
                                              float bias, float rate, float* d_s, float* l_s) {
-  for (int j = threadIdx.x; j < SSM_L; j += blockDim.x)
-    d_s[j] = j < rows ? softplusf(to_float(dt[static_cast<int64_t>(first + j) * ldd + head]) + bias) : 0.f;
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    float l = 0.f;
-    for (int j = 0; j < SSM_L; ++j) {
-      l += rate * d_s[j];
-      l_s[j] = l;
+  if (threadIdx.x < SSM_L) {
+    const int j = threadIdx.x;
+    const float d = softplusf(to_float(dt[static_cast<int64_t>(first + min(j, rows - 1)) * ldd + head]) + bias);
+    d_s[j] = j < rows ? d : 0.f;
+    float l = j < rows ? rate * d : 0.f;
+#pragma unroll
+    for (int o = 1; o < SSM_L; o <<= 1) {
+      const float before = __shfl_up(l, o, 64);
+      if (j >= o) l += before;
     }
+    l_s[j] = l;
   }
   __syncthreads();
 }
@@ -140,12 +157,11 @@ ssm_chunk_sums_kernel(const X* __restrict__ xbc, int64_t ld, const X* __restrict
   chunk_decays(dt, ldd, first, rows, head, dt_bias[head], -expf(a_log[head]), d_s, l_s);
   const float l_end = l_s[rows - 1];
   if (threadIdx.x == 0 && blockIdx.z == 0) totals[static_cast<int64_t>(chunk) * H + head] = expf(l_end);
-  for (int i = threadIdx.x; i < SSM_L * 64; i += 256) {
-    const int j = i / 64, p = i % 64;
-    x_s[j][p] = (j < rows && p0 + p < P)
-                    ? expf(l_end - l_s[j]) * d_s[j] * to_float(xbc[static_cast<int64_t>(first + j) * ld + head * P + p0 + p])
-                    : 0.f;
-  }
+  if (threadIdx.x < SSM_L) d_s[threadIdx.x] *= expf(l_end - l_s[threadIdx.x]);
+  stage_tile(x_s, xbc + static_cast<int64_t>(first) * ld + head * P + p0, ld, rows, P - p0);
+  __syncthreads();
+#pragma unroll
+  for (int r = 0; r < 16; ++r) x_s[threadIdx.x / 64 + 4 * r][threadIdx.x % 64] *= d_s[threadIdx.x / 64 + 4 * r];
   const int64_t b_at = static_cast<int64_t>(H) * P + static_cast<int64_t>(group) * N;
   float* u = scratch + (static_cast<int64_t>(chunk) * H + head) * N * P;
   // a wave: 32 rows n by 32 columns p of the pass's 64 x 64, on float32 matrix products over the rows j
@@ -153,10 +169,7 @@ ssm_chunk_sums_kernel(const X* __restrict__ xbc, int64_t ld, const X* __restrict
   const int nb = 32 * (wave / 2), pb = 32 * (wave % 2);
   for (int n0 = 0; n0 < N; n0 += SSM_L) {
     __syncthreads();
-    for (int i = threadIdx.x; i < SSM_L * SSM_L; i += 256) {
-      const int j = i / SSM_L, n = i % SSM_L;
-      b_s[j][n] = (j < rows && n0 + n < N) ? to_float(xbc[static_cast<int64_t>(first + j) * ld + b_at + n0 + n]) : 0.f;
-    }
+    stage_tile(b_s, xbc + static_cast<int64_t>(first) * ld + b_at + n0, ld, rows, N - n0);
     __syncthreads();
     ssm_floatx16 acc = {};
     for (int j = 0; j < SSM_L; j += 2)
@@ -210,12 +223,8 @@ ssm_chunk_pairs_kernel(const X* __restrict__ xbc, int64_t ld, float* __restrict_
   ssm_floatx16 acc = {};
   for (int n0 = 0; n0 < N; n0 += SSM_L) {
     __syncthreads();
-    for (int i = threadIdx.x; i < SSM_L * SSM_L; i += 256) {
-      const int j = i / SSM_L, n = i % SSM_L;
-      const bool in = j < rows && n0 + n < N;
-      b_s[j][n] = in ? to_float(xbc[static_cast<int64_t>(first + j) * ld + b_at + n0 + n]) : 0.f;
-      c_s[j][n] = in ? to_float(xbc[static_cast<int64_t>(first + j) * ld + c_at + n0 + n]) : 0.f;
-    }
+    stage_tile(b_s, xbc + static_cast<int64_t>(first) * ld + b_at + n0, ld, rows, N - n0);
+    stage_tile(c_s, xbc + static_cast<int64_t>(first) * ld + c_at + n0, ld, rows, N - n0);
     __syncthreads();
     for (int n = 0; n < SSM_L; n += 2)
       acc = __builtin_amdgcn_mfma_f32_32x32x2f32(c_s[ib + lane % 32][n + lane / 32], b_s[jb + lane % 32][n + lane / 32],
@@ -251,7 +260,8 @@ ssm_chunk_outputs_kernel(const X* __restrict__ xbc, int64_t ld, const X* __restr
 #pragma unroll
   for (int r = 0; r < SSM_L / 4; ++r) {
     const int i = part + 4 * r, j = col;
-    a_s[i][j] = (j <= i && i < rows) ? pair[i * SSM_L + j] * expf(l_s[i] - l_s[j]) * d_s[j] : 0.f;
+    const float weight = pair[i * SSM_L + j];                      // (read whether it counts or not: sixteen loads together)
+    a_s[i][j] = (j <= i && i < rows) ? weight * expf(l_s[i] - l_s[j]) * d_s[j] : 0.f;
   }
   // a wave: 32 rows i by 32 columns p of the outputs
   const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
@@ -259,24 +269,15 @@ ssm_chunk_outputs_kernel(const X* __restrict__ xbc, int64_t ld, const X* __restr
   ssm_floatx16 y = {};                 // the state's share: sum_n C_i[n] S[n][p]
   for (int n0 = 0; n0 < N; n0 += SSM_L) {
     __syncthreads();
-    for (int i = threadIdx.x; i < SSM_L * SSM_L; i += 256) {
-      const int j = i / SSM_L, n = i % SSM_L;
-      t_s[j][n] = (j < rows && n0 + n < N) ? to_float(xbc[static_cast<int64_t>(first + j) * ld + c_at + n0 + n]) : 0.f;
-    }
-    for (int i = threadIdx.x; i < SSM_L * 64; i += 256) {
-      const int n = i / 64, p = i % 64;
-      u_s[n][p] = (n0 + n < N && p0 + p < P) ? s_in[static_cast<int64_t>(n0 + n) * P + p0 + p] : 0.f;
-    }
+    stage_tile(t_s, xbc + static_cast<int64_t>(first) * ld + c_at + n0, ld, rows, N - n0);
+    stage_tile(u_s, s_in + static_cast<int64_t>(n0) * P + p0, P, N - n0, P - p0);
     __syncthreads();
     for (int n = 0; n < SSM_L; n += 2)
       y = __builtin_amdgcn_mfma_f32_32x32x2f32(t_s[ib + lane % 32][n + lane / 32], u_s[n + lane / 32][pb + lane % 32], y,
                                                0, 0, 0);
   }
   __syncthreads();
-  for (int i = threadIdx.x; i < SSM_L * 64; i += 256) {
-    const int j = i / 64, p = i % 64;
-    t_s[j][p] = (j < rows && p0 + p < P) ? to_float(xbc[static_cast<int64_t>(first + j) * ld + head * P + p0 + p]) : 0.f;
-  }
+  stage_tile(t_s, xbc + static_cast<int64_t>(first) * ld + head * P + p0, ld, rows, P - p0);
   __syncthreads();
   // the chunk's own rows: sum_{j <= i} a[i][j] x_j[p]; rows j beyond the wave's last i have weight zero
   ssm_floatx16 own = {};

@@ -925,6 +925,26 @@ class HipOps(Ops):
         """May return `PartialSums` (see there)."""
         return self._linear(x, weight, bias, x.dtype, partial_ok=True, lazy=True)
 
+    def linear_dense(self, x, weight, bias=None):
+        """Steps of up to ONE_WAVE_MAX_ROWS rows: the packed product with the whole K in one workgroup, which writes the
+        finished values (cut into slices, a kernel that adds them up would have to follow)."""
+        x = self.dense(x)
+        packed = getattr(weight, "_distie_packed", None)
+        M, K = x.shape
+        N = weight.shape[0]
+        if packed is None or x.dtype != torch.bfloat16 or M > self.ONE_WAVE_MAX_ROWS or K % 8 or weight.shape[1] != K:
+            return self.dense(self.linear(x, weight, bias))
+        self._own(x, bias)
+        if bias is not None and (bias.dtype != torch.float32 or bias.shape[0] != N):
+            raise KernelError("linear: bias must be float32 [N]")
+        if packed.numel() != self._packed_elements(N, K, False):
+            raise KernelError("linear: the packed copy does not belong to this weight")
+        out = torch.empty((M, N), dtype=x.dtype, device=self.device)
+        _check(self._ops.distie_gemm_packed_bf16(
+            x.data_ptr(), packed.data_ptr(), bias.data_ptr() if bias is not None else None, out.data_ptr(), _code(out), M, N, K,
+            2, 0.0, 1.0, 0.0, self._stream()), "gemm_packed_bf16")
+        return out
+
     def linear_f32out(self, x, weight, bias=None, scale=1.0, partial=False):
         if partial and scale == 1.0:
             return self._linear(x, weight, bias, torch.float32, partial_ok=True)

@@ -179,6 +179,11 @@ class Ops(abc.ABC):
         its own; any other tensor as it is. For parts that compute on the values themselves."""
         return x
 
+    def linear_dense(self, x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """dense(linear(x, weight, bias)), for parts that read the values themselves (several operations read columns of
+        one stacked product); an implementation may choose another kernel than for a product that one operation reads."""
+        return self.dense(self.linear(x, weight, bias))
+
     def prepare_linear(self, weight: torch.Tensor, gated: bool = False, rotary=None, role: Optional[str] = None) -> None:
         """Called once for every weight of a `linear` after it is loaded (`gated`: the weight of a
         `linear_silu_mul`; `rotary = (num_heads, num_kv_heads, head_dim)`: the stacked q/k/v weight

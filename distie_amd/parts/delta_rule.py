@@ -90,7 +90,7 @@ class GatedDeltaRule(Mixer):
 
     def forward(self, ops, x, ctx, cache, writes_cache: bool):
         H, channels = self.num_heads, self.conv_channels
-        product = ops.dense(ops.linear(x, self.in_weight))
+        product = ops.linear_dense(x, self.in_weight)
         history = cache["conv"] if self.taps > 1 else None
         qkv = ops.causal_conv(product[:, :channels], self.conv_weight, history, ctx.meta, act="silu")
         behind = channels + self.inner

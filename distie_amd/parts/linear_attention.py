@@ -54,7 +54,7 @@ class DecayLinearAttention(Mixer):
         ops.prepare_linear(self.out_weight, role="attn_out")
 
     def forward(self, ops, x, ctx, cache, writes_cache: bool):
-        product = ops.dense(ops.linear(x, self.in_weight))
+        product = ops.linear_dense(x, self.in_weight)
         mixed = ops.decay_scan(product, cache["state"], self.decay, ctx.meta, self.num_heads, self.head_dim, self.value_dim)
         first = self.num_heads * (2 * self.head_dim + self.value_dim)
         gates = product[:, first:first + self.num_heads * self.value_dim]
@@ -117,7 +117,7 @@ class Retention(Mixer):
         ops.prepare_linear(self.out_weight, role="attn_out")
 
     def forward(self, ops, x, ctx, cache, writes_cache: bool):
-        product = ops.dense(ops.linear(x, self.in_weight))
+        product = ops.linear_dense(x, self.in_weight)
         mixed = ops.decay_scan(product, cache["state"], self.decay, ctx.meta, self.num_heads, self.head_dim,
                                self.value_dim, act=None, k_scale=self.k_scale, inv_freq=self.position.rotary(),
                                neighbours=self.neighbours)
@@ -185,7 +185,7 @@ class GatedLinearAttention(Mixer):
         ops.prepare_linear(self.out_weight, role="attn_out")
 
     def forward(self, ops, x, ctx, cache, writes_cache: bool):
-        product = ops.dense(ops.linear(x, self.in_weight))
+        product = ops.linear_dense(x, self.in_weight)
         first = self.num_heads * (2 * self.head_dim + self.value_dim)
         behind = first + self.num_heads * self.value_dim
         low = product[:, behind:behind + self.decay_rank]

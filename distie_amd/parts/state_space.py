@@ -77,7 +77,7 @@ class StateSpaceDuality(Mixer):
 
     def forward(self, ops, x, ctx, cache, writes_cache: bool):
         inner, channels = self.inner, self.conv_channels
-        product = ops.dense(ops.linear(x, self.in_weight))
+        product = ops.linear_dense(x, self.in_weight)
         history = cache["conv"] if self.taps > 1 else None
         xbc = ops.causal_conv(product[:, inner:inner + channels], self.conv_weight, history, ctx.meta,
                               bias=self.conv_bias, act="silu")
