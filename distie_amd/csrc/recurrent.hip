@@ -705,7 +705,7 @@ constexpr int ROUTE_MAX_EXPERTS = 1024;
 constexpr int ROUTE_MAX_TOP = 32;
 
 // Scoring 3: experts are chosen by sigmoid(z) + correction, among the `kept` strongest of `groups` groups of neighbours
-// (by the sum of a group's two largest choice scores), and weighted by scale * sigmoid(z) / (the chosen ones' sum).
+// (a group counts by its two best choice scores added up), and weighted by scale * sigmoid(z) / (the chosen ones' sum).
 // `shared` (any scoring): the router has one row more than experts; the sigmoid of its logit goes behind a row's weights.
 struct RouteRule {
   const float* correction;

@@ -113,9 +113,9 @@ class RouteRule:
     shared expert (with any scoring).
 
     s = sigmoid(z); choice score = s + correction. With `groups` > 1 the experts form that many groups of neighbours; a
-    group counts by the sum of its two largest choice scores (of its only one), and experts outside the `kept` strongest
-    groups are never chosen. The `top` experts with the largest choice scores are weighted by scale * s / (sum of the chosen
-    experts' s + 1e-20). `shared`: the router's weight has one row more than there are experts, and the sigmoid of its
+    group counts by its two best choice scores added up (its only one, if it has no more), and experts outside the
+    `kept` strongest groups are never chosen. The `top` best of the rest are chosen and weighted by scale * s / (sum of
+    the chosen experts' s + 1e-20). `shared`: the router's weight has one row more than there are experts, and the sigmoid of its
     logit is handed out behind the chosen experts' weights."""
 
     correction: Optional[torch.Tensor] = None       # float32 [E] on the device

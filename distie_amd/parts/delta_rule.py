@@ -2,19 +2,20 @@
 per head that forgets by a factor computed from the token and corrects what it holds under the token's key.
 
 q and k (kv_heads heads of head_dim) and v (num_heads heads of value_dim) are projections of the mixer's input; every
-channel of the three goes through a causal convolution over time (`<q|k|v>.conv` [channels, taps], the last column is the
-current token's, zeros before the start) and silu. Head h uses q/k head h // (num_heads / kv_heads). Both become unit
-vectors, x / sqrt(sum(x^2) + 1e-6), and q is multiplied by head_dim^(-1/2) besides. With
+channel of the three is filtered over time (`<q|k|v>.conv` [channels, taps], oldest row first; rows in front of a request's
+first are zero) and goes through silu. num_heads / kv_heads value heads in a row share a q/k head. With k^ and q^ the
+vectors of length one, x / sqrt(x . x + 1e-6), q^ times head_dim^(-1/2) besides, and two numbers a head and token,
 
-    beta = sigmoid(W_b h),        a = exp(-exp(A_log) * softplus(W_a h + dt_bias))        (a number each per head)
+    w = sigmoid(b),    b from W_b,        ln f = -exp(A_log) * softplus(a + dt_bias),    a from W_a,
 
-a head turns its state S (head_dim x value_dim) and reads it, the current token's write included:
+a head's state S (head_dim x value_dim) goes from token t - 1 to t, and is read behind that, by
 
-    S <- a S,        u = beta * (v - S^T k),        S <- S + k u^T,        o = S^T q.
+    S_t = f_t (1 - w_t k^_t k^_t^T) S_(t-1) + w_t k^_t v_t^T,        o_t = S_t^T q^_t:
 
-Every head's o goes through an RMS norm over its value_dim columns (weight `norm` [value_dim], the same for all heads), the
-heads side by side are multiplied by silu(W_g h) and projected by `o`. The state starts at zero and is float32 [num_heads,
-head_dim, value_dim] for each request; the convolution's last taps - 1 inputs are state as well. Everything behind the
+what stood under k^_t is replaced, by the part w_t, with v_t. Every head's o goes through an RMS norm over its value_dim
+columns (weight `norm` [value_dim], the same for all heads), then the gate's silu (from W_g), then `o`. For each request the
+mixer keeps S, float32 [num_heads, head_dim, value_dim] and zero in the beginning, and the taps - 1 newest rows in front of
+the filters. Everything behind the
 projections and convolutions is float32 in either precision: unit norms, beta, the decay, the state and every sum into it,
 the norm and the gate. The six projections are one matrix product: their weights are stacked at load (q, k, v, g, b, a, and
 rows of zeros up to a multiple of 16).

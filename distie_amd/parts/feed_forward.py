@@ -105,7 +105,7 @@ class RoutedExperts(FeedForward):
     instead of the product's own epilogue and a scaling behind it. `scoring` "sigmoid_share": with s = sigmoid(z) the
     experts are chosen by s, or by s + correction (`correction`: the tensor `correction` [E]), and weighted by s over the
     sum of the chosen experts' s, times `weight_scale`. `groups` and `groups_kept`: the experts form that many groups of
-    neighbours, a group counts by the sum of its two largest choice scores, and only the experts of the groups_kept
+    neighbours, a group counts by its two best experts' choice scores added up, and only the experts of the groups_kept
     strongest groups can be chosen. `shared_gate` (with `route_in_hidden`): the shared expert counts with weight
     sigmoid(w . x), w the tensor `shared.sg` [1, C]; its logit is one more row of the router.
 

@@ -72,8 +72,8 @@ class Retention(Mixer):
 
         S_t = decay_h * S_(t-1) + k_t v_t^T,        o_t = S_t^T q_t.
 
-    Every head's o is divided by its root mean square (no weight), the heads side by side are multiplied by silu(W_g h) and
-    projected by W_o. The state starts at zero and is float32 [heads, dim, value_dim] for each request; rotation, scale,
+    A head's o is RMS-normed without a weight; gate (silu, from W_g) and output projection follow. For each request the
+    mixer keeps S, float32 [heads, dim, value_dim] and zero in the beginning; rotation, scale,
     state, sums and norm are float32 in either precision. The four projections are one matrix product: their weights
     are stacked at load."""
 
